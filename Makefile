@@ -12,7 +12,10 @@ LIB     ?= $(LIBDIR)/libturboinfer_amd.so
 
 COMMON  := -std=c++20 -O3 -fPIC -Iinclude -Iturboinfer_amd/csrc/kernels -Wall -Wno-unused-result -Wno-unused-value
 EXTRA   ?=
-DEVFLAGS:= $(COMMON) --offload-arch=$(ARCH) -fno-gpu-rdc $(EXTRA)
+# no packed-fp32 instructions (some of their forms have given wrong results on MI355X); the host pass
+# does not know the feature and says so
+NOPKF32 := -Xclang -target-feature -Xclang -packed-fp32-ops
+DEVFLAGS:= $(COMMON) --offload-arch=$(ARCH) -fno-gpu-rdc $(NOPKF32) $(EXTRA)
 
 KERN    := $(wildcard turboinfer_amd/csrc/kernels/*.hip)
 HOST    := $(wildcard turboinfer_amd/csrc/host/*.cpp)
@@ -50,7 +53,7 @@ $(BUILD)/k_%.o: turboinfer_amd/csrc/kernels/%.hip $(HDRS)
 
 $(BUILD)/h_%.o: turboinfer_amd/csrc/host/%.cpp $(HDRS)
 	@mkdir -p $(BUILD)
-	$(HIPCC) $(COMMON) -ffp-contract=off -x hip --offload-arch=$(ARCH) -c $< -o $@
+	$(HIPCC) $(COMMON) -ffp-contract=off -x hip --offload-arch=$(ARCH) $(NOPKF32) -c $< -o $@
 
 # C++20 drop-in API (turboinfer::core / model / optimize): host code over the C-ABI only
 $(BUILD)/a_%.o: turboinfer_amd/csrc/api/%.cpp $(HDRS)

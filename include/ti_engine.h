@@ -19,6 +19,8 @@
 #include <stddef.h>
 #include <stdint.h>
 
+#include "ti_stack.h"
+
 #ifdef __cplusplus
 extern "C" {
 #endif
@@ -38,6 +40,28 @@ typedef struct ti_engine_config {
   int32_t attn_splits;     /* 0 = auto */
 } ti_engine_config;
 
+/* ---------------------------------------------------------------- layer-stack models
+ * A model given layer by layer (config.json "layers"), each with its own sizes, run in order with an
+ * optional looped range (config.json "loop").  Every loop pass of a layer is a run with its own cache.
+ * Each sublayer is x += post_norm(f(pre_norm(x))). */
+enum ti_mixer { TI_MIX_LATENT = 0 };        /* latent attention (ti_stack.h)                     */
+enum ti_mlp { TI_MLP_NONE = 0, TI_MLP_MOE = 1 };
+typedef struct ti_stack_layer {
+  int32_t mixer;
+  int32_t heads, dim, rot_dim, vdim, q_rank, kv_rank;
+  int32_t rot_dims;        /* leading dimensions of the rotated part that turn (<= rot_dim, even)    */
+  float rot_base, scale;
+  int32_t mlp;
+  int32_t experts, top, ff;
+} ti_stack_layer;
+typedef struct ti_stack_config {
+  int32_t vocab, width, layers;
+  int32_t loop_start, loop_stop, loop_times;   /* loop_times 0: no loop (layers run once each)      */
+  float eps, emb_scale;
+  int32_t dtype;           /* ti_dtype: bf16 weights / activations / cache, or everything fp32       */
+  int32_t max_seq, max_batch, device;
+} ti_stack_config;
+
 enum ti_slot {
   TI_W_Q = 0, TI_W_K, TI_W_V, TI_W_O, TI_W_GATE, TI_W_UP, TI_W_DOWN, /* per layer, [K][N] */
   TI_W_LM_HEAD,                                                    /* [hidden][vocab]   */
@@ -48,6 +72,24 @@ enum ti_slot {
 
 int ti_engine_create(const ti_engine_config* cfg, ti_engine** out);
 int ti_engine_destroy(ti_engine* e);
+/* A layer-stack engine: every other call of this header that is not about llama weights (set_tensor*,
+ * set_fold, set_qkv_attn, time_kernel, stamp_steps) works on it as on a llama engine. */
+int ti_engine_create_stack(const ti_stack_config* cfg, const ti_stack_layer* layers, ti_engine** out);
+/* Its weights, by checkpoint name: number of tensors, the i-th one's name and shape (cols 1: a vector),
+ * and upload of one from host fp32 [rows][cols].  All must be set before the first step. */
+int ti_engine_weight_count(ti_engine* e);
+int ti_engine_weight_info(ti_engine* e, int i, char* name, int name_len, int* rows, int* cols);
+int ti_engine_set_weight(ti_engine* e, const char* name, const float* data, int rows, int cols);
+/* Build an engine from a model folder (config.json + model.safetensors): the architecture key of
+ * config.json picks the model class.  max_seq KV slots per stream, max_batch streams. */
+int ti_engine_load(const char* dir, int dtype, int max_seq, int max_batch, int device, ti_engine** out);
+/* Sizes of an engine (a layer-stack engine reports runs as layers and its first layer's heads). */
+int ti_engine_describe(ti_engine* e, ti_engine_config* out);
+/* Prompt tokens [0, n) of stream `slot` at positions pos0 + i through the prefill path; want lists
+ * n_want places (ascending) whose next-token logits [n_want][vocab] are returned.  layers_out
+ * (nullable, layer-stack engines): the residual after every layer run, [runs][n][width]. */
+int ti_engine_prefill(ti_engine* e, int slot, const int32_t* tokens, int n, int pos0, const int32_t* want, int n_want,
+                      float* logits, float* layers_out);
 int ti_engine_get_stream(ti_engine* e, void** stream);
 int ti_engine_memory(ti_engine* e, size_t* weight_bytes, size_t* kv_bytes);
 

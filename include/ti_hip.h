@@ -387,7 +387,8 @@ int ti_hbm_calibrate(size_t bytes, int reps, double* read_gbps, double* copy_gbp
  * 0.1f*((offset + i) % 100) (inference_engine.cpp:1444-1448, 1509-1512) with offset
  * placeholder_first on step 0 and 0 afterwards.
  * fold_x non-NULL: also fold_x[m][i] = fp16(h[m][i] * fold_w[i]) and fold_ss[m] = sum_i
- * h[m][i]^2, the TI_X_F16_FOLDED input (n_ss = 1) of the first layer's projection. */
+ * h[m][i]^2, the TI_X_F16_FOLDED input (n_ss = 1) of the first layer's projection.
+ * emb_kind 1 / 2: h = fp32(emb row) * emb_scale from a bf16 / fp32 table (no fold_x, no placeholder). */
 typedef struct ti_step_args {
   const uint16_t* emb;               /* [vocab][hidden] fp16 */
   float* h;                          /* [M][hidden] */
@@ -402,6 +403,9 @@ typedef struct ti_step_args {
   const float* fold_w;               /* [hidden] (with fold_x) */
   uint16_t* fold_x;                  /* [M][hidden] fp16, nullable */
   float* fold_ss;                    /* [M] */
+  int32_t emb_kind;                  /* 0: fp16 table (above); 1: bf16, 2: fp32, both scaled by emb_scale */
+  float emb_scale;
+  float* h0;                         /* nullable [M][hidden]: a second copy of the embedding row (emb_kind > 0) */
 } ti_step_args;
 int ti_step_begin(const ti_step_args* a, ti_stream_t s);
 

@@ -40,7 +40,8 @@ def test_gemm_max_rows(L):
 
 def test_exports_every_declared_symbol(L):
     declared = header_functions(os.path.join(ROOT, "include", "ti_hip.h")) + \
-        header_functions(os.path.join(ROOT, "include", "ti_engine.h"))
+        header_functions(os.path.join(ROOT, "include", "ti_engine.h")) + \
+        header_functions(os.path.join(ROOT, "include", "ti_stack.h"))
     assert len(declared) >= 50
     missing = [f for f in declared if not hasattr(L, f)]
     assert not missing, missing

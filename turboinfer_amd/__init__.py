@@ -55,7 +55,8 @@ class StepArgs(C.Structure):
                 ("placeholder_first", C.c_int32), ("in_tokens", C.c_void_p), ("n_in", C.c_void_p),
                 ("argmax", C.c_void_p), ("out_tokens", C.c_void_p), ("pos", C.c_void_p),
                 ("base_pos", C.c_void_p), ("step_ctr", C.c_void_p), ("fold_w", C.c_void_p),
-                ("fold_x", C.c_void_p), ("fold_ss", C.c_void_p)]
+                ("fold_x", C.c_void_p), ("fold_ss", C.c_void_p), ("emb_kind", C.c_int32),
+                ("emb_scale", C.c_float), ("h0", C.c_void_p)]
 
 
 class EngineConfig(C.Structure):
@@ -66,7 +67,49 @@ class EngineConfig(C.Structure):
                 ("attn_splits", C.c_int32)]
 
 
-# Every symbol declared in include/ti_hip.h and include/ti_engine.h (checked by tests).
+DT_BF16, DT_F32 = 0, 1              # ti_dtype (include/ti_stack.h)
+MLP_NONE, MLP_MOE = 0, 1            # ti_mlp (include/ti_engine.h)
+(DE_F32, DE_T, DE_SWIGLU, DE_ROPE, DE_GATE, DE_LOGITS, DE_KFRAG, DE_VFRAG) = range(8)
+NORM_LAYER, NORM_RMS = 0, 1
+
+
+class StackLayer(C.Structure):
+    """ti_stack_layer (include/ti_engine.h)."""
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "rot_dims")] + \
+        [("rot_base", C.c_float), ("scale", C.c_float)] + [(n, C.c_int32) for n in ("mlp", "experts", "top", "ff")]
+
+
+class StackConfig(C.Structure):
+    """ti_stack_config (include/ti_engine.h)."""
+    _fields_ = [(n, C.c_int32) for n in ("vocab", "width", "layers", "loop_start", "loop_stop", "loop_times")] + \
+        [("eps", C.c_float), ("emb_scale", C.c_float)] + [(n, C.c_int32) for n in ("dtype", "max_seq", "max_batch", "device")]
+
+
+class DenseArgs(C.Structure):
+    """ti_dense_args (include/ti_stack.h)."""
+    _fields_ = [("w", C.c_void_p), ("w_batch", C.c_int64), ("a", C.c_void_p), ("a_batch", C.c_int64), ("out", C.c_void_p),
+                ("o_batch", C.c_int64)] + \
+        [(n, C.c_int32) for n in ("lda", "ldo", "M", "N", "K", "batch", "epi", "dtype")] + \
+        [("add", C.c_void_p), ("rope_cs", C.c_void_p), ("pos", C.c_void_p), ("head_w", C.c_int32), ("rot_off", C.c_int32),
+         ("gate", C.c_void_p), ("gate_ld", C.c_int32), ("key_blocks", C.c_int32), ("argmax", C.c_void_p),
+         ("step_ctr", C.c_void_p), ("advance", C.c_int32), ("tile_rows", C.c_int32), ("max_tiles", C.c_int32),
+         ("tiles", C.c_void_p), ("n_tiles", C.c_void_p), ("rows_in", C.c_void_p), ("rows_out", C.c_void_p),
+         ("row_div", C.c_int32)]
+
+
+class RownormArgs(C.Structure):
+    """ti_rownorm_args (include/ti_stack.h)."""
+    _fields_ = [(n, C.c_void_p) for n in ("x", "y", "parts", "part_w", "post_w", "post_b", "w", "b", "xn", "x0", "cat")] + \
+        [("eps", C.c_float)] + [(n, C.c_int32) for n in ("M", "H", "ldy", "ldn", "ldc", "top", "kind", "dtype")]
+
+
+class RouteArgs(C.Structure):
+    """ti_route_args (include/ti_stack.h)."""
+    _fields_ = [("logits", C.c_void_p)] + [(n, C.c_int32) for n in ("ld", "M", "E", "top")] + \
+        [(n, C.c_void_p) for n in ("idx", "wgt", "list", "tiles", "n_tiles")] + [("tile_rows", C.c_int32)]
+
+
+# Every symbol declared in include/ti_hip.h, ti_engine.h and ti_stack.h (checked by tests).
 EXPORTED = [
     "ti_last_error", "ti_device_count", "ti_init", "ti_device_name", "ti_malloc", "ti_free", "ti_memcpy_h2d",
     "ti_memcpy_d2h", "ti_memcpy_d2d", "ti_memset", "ti_stream_create", "ti_stream_destroy", "ti_stream_sync",
@@ -89,6 +132,10 @@ EXPORTED = [
     "ti_gemm_fold_partials", "ti_engine_set_stop", "ti_engine_counters",
     "ti_qkv_attn_partials", "ti_qkv_attn_part_o_elems", "ti_qkv_attn_part_ml_elems", "ti_engine_set_qkv_attn",
     "ti_qkv_attn_xchg_bytes", "ti_qkv_attn_supported", "ti_qkv_attn_error_offset",
+    "ti_engine_create_stack", "ti_engine_weight_count", "ti_engine_weight_info", "ti_engine_set_weight", "ti_engine_load",
+    "ti_engine_describe", "ti_engine_prefill", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
+    "ti_stack_convert", "ti_stack_fill", "ti_dense", "ti_dense_args_bytes", "ti_rownorm", "ti_route", "ti_route_max_tiles",
+    "ti_latent_prep", "ti_latent_prepare", "ti_latent_attn_decode", "ti_latent_attn_splits", "ti_latent_attn_prefill",
 ]
 
 _lib = None
@@ -211,6 +258,26 @@ def lib() -> C.CDLL:
             L.ti_engine_stamp_steps.argtypes = [vp, i32, i32, vp, vp, C.POINTER(C.c_int)]
         L.ti_hbm_calibrate.argtypes = [sz, i32, C.POINTER(C.c_double), C.POINTER(C.c_double), vp]
         L.ti_gemm_kernel_name.argtypes = [i32, i32, i32, i32, i32, C.c_char_p, i32]
+        if hasattr(L, "ti_engine_create_stack"):
+            L.ti_engine_create_stack.argtypes = [C.POINTER(StackConfig), C.POINTER(StackLayer), C.POINTER(vp)]
+            L.ti_engine_weight_count.argtypes = [vp]
+            L.ti_engine_weight_info.argtypes = [vp, i32, C.c_char_p, i32, C.POINTER(C.c_int), C.POINTER(C.c_int)]
+            L.ti_engine_set_weight.argtypes = [vp, C.c_char_p, vp, i32, i32]
+            L.ti_engine_load.argtypes = [C.c_char_p, i32, i32, i32, i32, C.POINTER(vp)]
+            L.ti_engine_describe.argtypes = [vp, C.POINTER(EngineConfig)]
+            L.ti_engine_prefill.argtypes = [vp, i32, vp, i32, i32, vp, i32, vp, vp]
+            L.ti_stack_kpad.argtypes = [i32, i32]
+            L.ti_stack_weight_bytes.argtypes = [i32, i32, i32]
+            L.ti_stack_weight_bytes.restype = sz
+            L.ti_stack_pack.argtypes = [vp, i64, i64, i32, i32, vp, i32, vp, vp]
+            L.ti_stack_convert.argtypes = [vp, u64, i32, vp, vp]
+            L.ti_stack_fill.argtypes = [u64, C.c_uint32, u64, f32, i32, vp, vp]
+            L.ti_dense.argtypes = [C.POINTER(DenseArgs), vp]
+            L.ti_dense_args_bytes.restype = sz
+            L.ti_rownorm.argtypes = [C.POINTER(RownormArgs), vp]
+            L.ti_route.argtypes = [C.POINTER(RouteArgs), vp]
+            L.ti_route_max_tiles.argtypes = [i32, i32, i32, i32]
+            L.ti_latent_attn_splits.argtypes = [i32, i32, i32]
         L.ti_rope_table.argtypes = [vp, i32, i32, f32, vp]
         L.ti_sample_token.argtypes = [vp, i32, f32, i32, f32, f32, C.POINTER(C.c_int), C.POINTER(C.c_float)]
         _lib = L
@@ -360,6 +427,65 @@ class Engine:
         h = C.c_void_p()
         check(lib().ti_engine_create(C.byref(self.cfg), C.byref(h)))
         self.h = h
+
+    @classmethod
+    def _adopt(cls, handle) -> "Engine":
+        e = cls.__new__(cls)
+        e.h = handle
+        e.cfg = EngineConfig()
+        check(lib().ti_engine_describe(handle, C.byref(e.cfg)))
+        return e
+
+    @classmethod
+    def load(cls, model_dir, dtype="bfloat16", max_seq=2048, max_batch=1, device=0) -> "Engine":
+        """Engine of a model folder (config.json + model.safetensors; ti_engine_load)."""
+        h = C.c_void_p()
+        check(lib().ti_engine_load(os.fsencode(model_dir), {"bfloat16": DT_BF16, "float32": DT_F32}[dtype], max_seq,
+                                   max_batch, device, C.byref(h)))
+        return cls._adopt(h)
+
+    @classmethod
+    def stack(cls, config: dict, dtype="bfloat16", max_seq=2048, max_batch=1, device=0) -> "Engine":
+        """Layer-stack engine (ti_engine_create_stack) of a config.json-shaped dictionary, weights not set."""
+        lp = config.get("loop") or {}
+        c = StackConfig(config["vocab"], config["width"], len(config["layers"]), lp.get("start", 0), lp.get("stop", 0),
+                        lp.get("times", 0), config["norm"]["eps"], config["embedding"]["scale"],
+                        {"bfloat16": DT_BF16, "float32": DT_F32}[dtype], max_seq, max_batch, device)
+        ls = (StackLayer * len(config["layers"]))()
+        for d, l in zip(ls, config["layers"]):
+            m, f = l["mixer"], l.get("mlp")
+            for k in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "scale"):
+                setattr(d, k, m[k])
+            d.rot_dims, d.rot_base = m["rot"].get("dims", m["rot_dim"]), m["rot"]["base"]
+            if f:
+                d.mlp, d.experts, d.top, d.ff = MLP_MOE, f["router"]["experts"], f["router"]["top"], f["expert"]["ff"]
+        h = C.c_void_p()
+        check(lib().ti_engine_create_stack(C.byref(c), ls, C.byref(h)))
+        return cls._adopt(h)
+
+    def weights(self):
+        """[(name, rows, cols)] of a layer-stack engine (cols 1: a vector)."""
+        out = []
+        for i in range(lib().ti_engine_weight_count(self.h)):
+            name, r, c = C.create_string_buffer(256), C.c_int(), C.c_int()
+            check(lib().ti_engine_weight_info(self.h, i, name, 256, C.byref(r), C.byref(c)))
+            out.append((name.value.decode(), r.value, c.value))
+        return out
+
+    def set_weight(self, name, data):
+        a = np.ascontiguousarray(data, np.float32)
+        check(lib().ti_engine_set_weight(self.h, name.encode(), _ptr(a), a.shape[0], a.shape[1] if a.ndim > 1 else 1))
+
+    def prefill(self, slot, tokens, pos0=0, want=None, want_layers=False):
+        """Prompt tokens of one stream slot through the prefill path (ti_engine_prefill): logits at the
+        places `want` (default: the last), with want_layers also the residual after every layer run."""
+        t = np.ascontiguousarray(tokens, np.int32)
+        w = np.ascontiguousarray([t.size - 1] if want is None else want, np.int32)
+        logits = np.zeros((w.size, self.cfg.vocab), np.float32)
+        lay = np.zeros((self.cfg.layers, t.size, self.cfg.hidden), np.float32) if want_layers else None
+        check(lib().ti_engine_prefill(self.h, slot, _ptr(t), t.size, pos0, _ptr(w), w.size, _ptr(logits),
+                                      None if lay is None else _ptr(lay)))
+        return (logits, lay) if want_layers else logits
 
     def close(self):
         if getattr(self, "h", None):

@@ -18,6 +18,7 @@
 #include <stdexcept>
 
 #include "api_common.hpp"
+#include "model_registry.hpp"
 #include "ti_engine.h"
 #include "ti_hip.h"
 
@@ -237,6 +238,7 @@ class InferenceEngineImpl {
   ti_engine_config cfg{};
   int capacity = 1;      // streams one device call holds
   bool compat = false;
+  bool stack = false;    // a registered layer-stack architecture
   std::mt19937 rng;
   size_t total_generations = 0, total_tokens = 0, total_forward_passes = 0;
   float total_time_ms = 0.0f, peak_tps = 0.0f;
@@ -363,7 +365,22 @@ class InferenceEngineImpl {
     check(ti_engine_synth(eng, 0x7475726269ull, 0.0f), "ti_engine_synth");
   }
 
+  // A registered layer-stack architecture (model_registry.cpp): bf16, or fp32 throughout with
+  // extra_params["turboinfer.float32"] = "1" / TI_FLOAT32=1.
+  void build_stack(const ModelData& m, const InferenceConfig& c) {
+    const ModelMetadata& md = m.metadata();
+    const int dtype = engine_option(md, "turboinfer.float32", "TI_FLOAT32", 0) ? TI_DT_F32 : TI_DT_BF16;
+    capacity = (int)std::max<size_t>(1, std::min<size_t>(c.max_batch_size, 64));
+    stack = true;
+    eng = api::build_stack_engine(m, dtype, (int)std::max<size_t>(1, c.max_sequence_length), capacity,
+                                  engine_option(md, "turboinfer.gpu_index", "TI_GPU_INDEX", 0));
+    check(ti_engine_describe(eng, &cfg), "ti_engine_describe");
+    if (cfg.vocab > kGenerateEos) check(ti_engine_set_stop(eng, kGenerateEos), "ti_engine_set_stop");
+  }
+
   void build(const ModelData& m, const InferenceConfig& c) {
+    if (api::is_stack_architecture(m.metadata().architecture) && !m.get_config_param("config.json").empty())
+      return build_stack(m, c);
     if (gguf_named(m)) {
       gguf_src = true;
       return build(from_gguf_names(m), c);
@@ -777,10 +794,14 @@ std::string InferenceEngine::performance_stats() const {
   if (im.total_time_ms > 0.0f)
     os << "  Average Tokens/Second: " << (im.total_tokens / (im.total_time_ms / 1000.0f)) << "\n";
   os << "  Peak Tokens/Second: " << im.peak_tps << "\n";
-  os << "  Device Memory: " << (memory_usage() / (1024.0 * 1024.0)) << " MB (weights " << (im.cfg.bits & ~(TI_BITS_G32 | TI_BITS_AFF))
-     << "-bit" << ((im.cfg.bits & TI_BITS_AFF) ? " affine group-32 blocks" : (im.cfg.bits & TI_BITS_G32) ? " group-32 blocks" : "") << ", fp16 KV, " << im.capacity
-     << " stream(s) x " << im.cfg.max_seq << " slots)\n";
-  os << "  Mode: " << (im.compat ? "reference_compat (plumbing model)" : "llama decode") << "\n";
+  if (im.stack)
+    os << "  Device Memory: " << (memory_usage() / (1024.0 * 1024.0)) << " MB (" << im.cfg.layers << " layer runs, "
+       << im.capacity << " stream(s) x " << im.cfg.max_seq << " slots)\n";
+  else
+    os << "  Device Memory: " << (memory_usage() / (1024.0 * 1024.0)) << " MB (weights " << (im.cfg.bits & ~(TI_BITS_G32 | TI_BITS_AFF))
+       << "-bit" << ((im.cfg.bits & TI_BITS_AFF) ? " affine group-32 blocks" : (im.cfg.bits & TI_BITS_G32) ? " group-32 blocks" : "") << ", fp16 KV, " << im.capacity
+       << " stream(s) x " << im.cfg.max_seq << " slots)\n";
+  os << "  Mode: " << (im.compat ? "reference_compat (plumbing model)" : im.stack ? "layer stack" : "llama decode") << "\n";
   return os.str();
 }
 

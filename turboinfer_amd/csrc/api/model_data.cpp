@@ -2,10 +2,12 @@
 // ModelLoader entry points.  Container semantics follow the reference's
 // src/model/model_loader.cpp:186-311; file parsing is SURVEY.md 8(f) rank 3 (not built).
 #include <algorithm>
+#include <filesystem>
 #include <fstream>
 #include <sstream>
 #include <stdexcept>
 
+#include "model_registry.hpp"
 #include "turboinfer/model/model_loader.hpp"
 
 namespace turboinfer {
@@ -95,6 +97,8 @@ bool ends_with(const std::string& s, const std::string& suffix) {
 ModelData ModelLoader::load(const std::string& file_path) { return load(file_path, detect_format(file_path)); }
 ModelData ModelLoader::load(const std::string& file_path, ModelFormat format) {
   if (format == ModelFormat::kGGUF) return load_gguf(file_path);
+  // config.json + safetensors folders of the registered architectures (model_registry.cpp)
+  if (format == ModelFormat::kSafeTensors && api::is_model_dir(file_path)) return api::load_model_dir(file_path);
   loader_off_path("load(" + file_path + ")");
 }
 // get_model_info (reference model_loader.cpp:596-633): for GGUF the header is checked and the
@@ -127,6 +131,7 @@ ModelFormat ModelLoader::detect_format(const std::string& file_path) {
   if (ends_with(file_path, ".safetensors")) return ModelFormat::kSafeTensors;
   if (ends_with(file_path, ".pt") || ends_with(file_path, ".pth")) return ModelFormat::kPyTorch;
   if (ends_with(file_path, ".onnx")) return ModelFormat::kONNX;
+  if (std::filesystem::is_directory(file_path) && api::is_model_dir(file_path)) return ModelFormat::kSafeTensors;
   throw std::runtime_error("Unknown model format: " + file_path);
 }
 

@@ -20,10 +20,12 @@
 #include <cstdlib>
 #include <cstring>
 #include <map>
+#include <memory>
 #include <utility>
 #include <vector>
 
 #include "ti_engine.h"
+#include "stack.hpp"
 #include "ti_hip.h"
 
 int ti_set_error(int code, const char* fmt, ...);
@@ -41,6 +43,8 @@ int ti_check_hip(hipError_t e, const char* what);
   } while (0)
 
 namespace {
+
+constexpr int kStackPrefillRows = 2048;   // prompt tokens per chunk of a layer-stack engine
 
 // tensor ids of the synthetic model: identical to oracle/ti_oracle.c
 constexpr uint32_t kTidEmb = 1, kTidOutNorm = 2, kTidLmHead = 3, kTidLayer0 = 16;
@@ -74,6 +78,7 @@ uint16_t host_half(float f) {
 
 struct ti_engine {
   ti_engine_config c{};
+  std::unique_ptr<ti_host::StackModel> stack;   // layer-stack models; NULL: llama (the members below)
   hipStream_t s = nullptr;
   std::vector<void*> allocs;
   std::vector<DevLayer> layer;
@@ -205,6 +210,7 @@ struct ti_engine {
   ~ti_engine() {
     for (auto& g : graphs) hipGraphExecDestroy(g.second);
     for (void* p : allocs) hipFree(p);
+    stack.reset();
     if (s) hipStreamDestroy(s);
   }
 };
@@ -385,11 +391,34 @@ bool qa_usable(ti_engine* e, int M) {
          ti_qkv_attn_supported(c.bits, c.hidden, c.heads, c.kv_heads, c.head_dim, sp);
 }
 
+// The embedding table of either kind of engine.
+void step_embedding(ti_engine* e, ti_step_args& sa) {
+  sa.emb = e->emb;
+  if (!e->stack) return;
+  const ti_stack_config& k = e->stack->c;
+  sa.emb = static_cast<const uint16_t*>(e->stack->emb);
+  sa.emb_kind = k.dtype == TI_DT_BF16 ? 1 : 2;
+  sa.emb_scale = k.emb_scale;
+  sa.h0 = e->stack->h0;
+}
+
+// Final norm + lm_head + argmax of n residual rows x (first token after a prefill, wanted prompt rows).
+int enqueue_head(ti_engine* e, int n, float* x) {
+  const ti_engine_config& c = e->c;
+  if (e->stack) return e->stack->head(x, n, e->logits, e->argmax);
+  ti_epilogue el{};
+  el.kind = TI_EPI_LOGITS_ARGMAX;
+  el.ldo = c.vocab;
+  el.out = e->logits;
+  el.argmax = e->argmax;
+  return gemm_rows(e, e->lm, n, x, TI_X_F32_RMSNORM, c.hidden, e->out_norm, el, 4, false);
+}
+
 // One decode step for streams [0, M) on e->s.  Graph-capturable (no host sync / alloc).
 int enqueue_step(ti_engine* e, int M, int advance) {
   const ti_engine_config& c = e->c;
   ti_step_args sa{};
-  sa.emb = e->emb;
+  step_embedding(e, sa);
   sa.h = e->h;
   sa.hidden = c.hidden;
   sa.M = M;
@@ -404,6 +433,19 @@ int enqueue_step(ti_engine* e, int M, int advance) {
   sa.pos = e->pos;
   sa.base_pos = e->base_pos;
   sa.step_ctr = e->step_ctr;
+  if (e->stack) {
+    TI_TRY(ti_step_begin(&sa, e->s));
+    ti_host::StackRows r;
+    r.M = M;
+    r.pos = e->pos;
+    r.h = e->h;
+    r.h0 = e->stack->h0;
+    TI_TRY(e->stack->forward(r, true, e->logits, e->argmax, e->step_ctr, advance));
+    if (e->samp_on)
+      TI_TRY(ti_sample_step_ws(e->logits, c.vocab, M, c.vocab, e->samp_t, e->samp_k, e->samp_p, e->draws, e->draw_cap,
+                               e->step_ctr, advance, e->n_in, e->argmax, e->lps, e->samp_ws, e->s));
+    return TI_OK;
+  }
   const int H = c.hidden, qd = e->qd(), kvd = e->kvd(), I = c.inter, V = c.vocab;
   // fold (M == 1): every rms_norm input is handed over as fx + ss partials by its producer
   const bool fold = fold_usable(e, M), part = part_usable(e, M), pk = packed_rows(e, M), qa = qa_usable(e, M);
@@ -583,14 +625,14 @@ static bool prefill_attn_on() {
   return on != 0;
 }
 
-int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base) {
+int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base, float* layers_out = nullptr, int layers_stride = 0) {
   const ti_engine_config& c = e->c;
   ++e->n_prefill_chunks;
   std::vector<int32_t> bp(rows);
   for (int j = 0; j < rows; ++j) bp[j] = base + t0 + j;
   TI_TRY(ti_memcpy_h2d(e->pf_base, bp.data(), (size_t)rows * 4, e->s));
   ti_step_args sa{};
-  sa.emb = e->emb;
+  step_embedding(e, sa);
   sa.h = e->h;
   sa.hidden = c.hidden;
   sa.M = rows;
@@ -606,6 +648,20 @@ int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base) {
   sa.base_pos = e->pf_base;
   sa.step_ctr = e->pf_zero;
   TI_TRY(ti_step_begin(&sa, e->s));
+  if (e->stack) {
+    TI_TRY(e->stack->ready());
+    ti_host::StackRows r;
+    r.M = rows;
+    r.pos = e->pos;
+    r.h = e->h;
+    r.h0 = e->stack->h0;
+    r.chunk = true;
+    r.slot = m;
+    r.pos0 = base + t0;
+    r.layers_out = layers_out;
+    r.layers_stride = (size_t)layers_stride;
+    return e->stack->forward(r, false, nullptr, nullptr, nullptr, 0);
+  }
   const int H = c.hidden, qd = e->qd(), kvd = e->kvd(), I = c.inter;
   for (int l = 0; l < c.layers; ++l) {
     DevLayer& L = e->layer[l];
@@ -659,6 +715,7 @@ int get_graph(ti_engine* e, int M, int advance, hipGraphExec_t* out) {
     *out = it->second;
     return TI_OK;
   }
+  if (e->stack) TI_TRY(e->stack->ready());
   TI_TRY(ti_gemm_prepare());
   E_CHECK(hipStreamBeginCapture(e->s, hipStreamCaptureModeThreadLocal), "hipStreamBeginCapture");
   const int rc = enqueue_step(e, M, advance);
@@ -801,6 +858,114 @@ int ti_engine_create(const ti_engine_config* cfg, ti_engine** out) {
   return TI_OK;
 }
 
+int ti_engine_create_stack(const ti_stack_config* cfg, const ti_stack_layer* layers, ti_engine** out) {
+  if (!cfg || !layers || !out) return ti_set_error(TI_ERR_ARG, "ti_engine_create_stack: null");
+  *out = nullptr;
+  TI_TRY(ti_host::StackModel::check(*cfg, layers));
+  DeviceScope bind_(cfg->device);
+  TI_TRY(ti_init(cfg->device));
+  TI_TRY(ti_latent_prepare());
+  auto e = std::make_unique<ti_engine>();
+  ti_engine_config& c = e->c;
+  c.vocab = cfg->vocab;
+  c.hidden = cfg->width;
+  c.heads = c.kv_heads = layers[0].heads;
+  c.head_dim = layers[0].dim + layers[0].rot_dim;
+  c.inter = layers[0].mlp == TI_MLP_MOE ? layers[0].ff * layers[0].top : 0;
+  c.rope_theta = layers[0].rot_base;
+  c.eps = cfg->eps;
+  c.bits = 16;
+  c.max_seq = cfg->max_seq;
+  c.max_batch = cfg->max_batch;
+  c.device = cfg->device;
+  if (hipStreamCreateWithFlags(&e->s, hipStreamNonBlocking) != hipSuccess)
+    return ti_check_hip(hipErrorUnknown, "hipStreamCreate");
+  const int B = c.max_batch, H = c.hidden;
+  e->pf_rows = std::min(kStackPrefillRows, std::max(16, c.max_seq));
+  e->rows_cap = std::max(B, e->pf_rows);
+  e->stack = std::make_unique<ti_host::StackModel>();
+  TI_TRY(e->stack->create(*cfg, layers, e->rows_cap, e->s));
+  c.layers = (int)e->stack->run.size();
+  e->weight_bytes = e->stack->weight_bytes;
+  e->kv_bytes = e->stack->kv_bytes;
+  const int R = e->rows_cap;
+  TI_TRY(e->alloc_t(&e->pf_ones, (size_t)R));
+  TI_TRY(e->alloc_t(&e->pf_zero, (size_t)1));
+  TI_TRY(e->alloc_t(&e->pf_base, (size_t)R));
+  TI_TRY(e->alloc_t(&e->h, (size_t)R * H));
+  TI_TRY(e->alloc_t(&e->h_last, (size_t)B * H));
+  TI_TRY(e->alloc_t(&e->logits, (size_t)B * c.vocab));
+  TI_TRY(e->alloc_t(&e->argmax, (size_t)R * TI_ARGMAX_SLOTS));
+  TI_TRY(e->alloc_t(&e->pos, (size_t)R));
+  TI_TRY(e->alloc_t(&e->base_pos, (size_t)B));
+  TI_TRY(e->alloc_t(&e->step_ctr, (size_t)1));
+  TI_TRY(e->alloc_t(&e->n_in, (size_t)B));
+  TI_TRY(ensure_io(e.get(), 8, 8));
+  const std::vector<int32_t> ones((size_t)R, 1);
+  TI_TRY(ti_memcpy_h2d(e->pf_ones, ones.data(), ones.size() * 4, e->s));
+  TI_TRY(ti_stream_sync(e->s));
+  *out = e.release();
+  return TI_OK;
+}
+
+int ti_engine_weight_count(ti_engine* e) { return e && e->stack ? (int)e->stack->weights.size() : 0; }
+
+int ti_engine_weight_info(ti_engine* e, int i, char* name, int name_len, int* rows, int* cols) {
+  if (!e || !e->stack || i < 0 || i >= (int)e->stack->weights.size() || (name && name_len < 1))
+    return ti_set_error(TI_ERR_ARG, "ti_engine_weight_info: bad arguments");
+  const ti_host::StackWeight& w = e->stack->weights[i];
+  if (name) {
+    std::strncpy(name, w.name.c_str(), (size_t)name_len - 1);
+    name[name_len - 1] = 0;
+  }
+  if (rows) *rows = w.rows;
+  if (cols) *cols = w.cols;
+  return TI_OK;
+}
+
+int ti_engine_set_weight(ti_engine* e, const char* name, const float* data, int rows, int cols) {
+  if (!e || !e->stack || !name) return ti_set_error(TI_ERR_ARG, "ti_engine_set_weight: not a layer-stack engine");
+  DeviceScope bind_(e);
+  return e->stack->set_weight(name, data, rows, cols);
+}
+
+int ti_engine_describe(ti_engine* e, ti_engine_config* out) {
+  if (!e || !out) return ti_set_error(TI_ERR_ARG, "ti_engine_describe: null");
+  *out = e->c;
+  return TI_OK;
+}
+
+int ti_engine_prefill(ti_engine* e, int slot, const int32_t* tokens, int n, int pos0, const int32_t* want, int n_want,
+                      float* logits, float* layers_out) {
+  if (!e || !tokens || n < 1 || n_want < 0 || (n_want && (!want || !logits)) || slot < 0 || slot >= e->c.max_batch || pos0 < 0 ||
+      pos0 + n > e->c.max_seq)
+    return ti_set_error(TI_ERR_ARG, "ti_engine_prefill: slot %d, %d tokens at %d", slot, n, pos0);
+  if (e->c.compat || (layers_out && !e->stack)) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_prefill: engine kind");
+  for (int i = 0; i < n_want; ++i)
+    if (want[i] < 0 || want[i] >= n || (i && want[i] <= want[i - 1]))
+      return ti_set_error(TI_ERR_ARG, "ti_engine_prefill: place %d of %d tokens", want[i], n);
+  DeviceScope bind_(e);
+  const ti_engine_config& c = e->c;
+  if (e->stack) TI_TRY(e->stack->ready());
+  const int pf = e->pf_rows > 0 ? e->pf_rows : std::min(e->rows_cap, 16), H = c.hidden, B = c.max_batch;
+  TI_TRY(ensure_io(e, n, 1));
+  TI_TRY(ti_memcpy_h2d(e->in_tokens + (size_t)slot * e->in_cap, tokens, (size_t)n * 4, e->s));
+  int w = 0;
+  for (int t0 = 0; t0 < n; t0 += pf) {
+    const int rows = std::min(pf, n - t0);
+    TI_TRY(enqueue_prefill(e, slot, t0, rows, pos0, layers_out ? layers_out + (size_t)t0 * H : nullptr, n));
+    while (w < n_want && want[w] < t0 + rows) {   // the wanted rows, as many at once as the logits buffer holds
+      int k = 0;
+      for (; k < B && w + k < n_want && want[w + k] < t0 + rows; ++k)
+        TI_TRY(ti_memcpy_d2d(e->h_last + (size_t)k * H, e->h + (size_t)(want[w + k] - t0) * H, (size_t)H * 4, e->s));
+      TI_TRY(enqueue_head(e, k, e->h_last));
+      TI_TRY(ti_memcpy_d2h(logits + (size_t)w * c.vocab, e->logits, (size_t)k * c.vocab * 4, e->s));
+      w += k;
+    }
+  }
+  return ti_stream_sync(e->s);
+}
+
 int ti_engine_destroy(ti_engine* e) {
   if (e) {
     DeviceScope bind_(e);
@@ -828,6 +993,7 @@ int ti_engine_memory(ti_engine* e, size_t* wb, size_t* kb) {
 int ti_engine_set_tensor(ti_engine* e, int slot, int layer, const float* data, int scale_mode) {
   if (!e || !data) return ti_set_error(TI_ERR_ARG, "ti_engine_set_tensor: null");
   DeviceScope bind_(e);
+  if (e->stack) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_set_tensor: layer-stack engines take ti_engine_set_weight");
   const ti_engine_config& c = e->c;
   const int H = c.hidden, I = c.inter, V = c.vocab;
   const bool per_layer = slot <= TI_W_DOWN || slot == TI_V_ATTN_NORM || slot == TI_V_FFN_NORM;
@@ -890,6 +1056,7 @@ static int set_tensor_blocks(ti_engine* e, int slot, int layer, const void* q, c
   if (!e || !q || !d) return ti_set_error(TI_ERR_ARG, "%s: null", fn);
   DeviceScope bind_(e);
   const ti_engine_config& c = e->c;
+  if (e->stack) return ti_set_error(TI_ERR_UNSUPPORTED, "%s: layer-stack engines take ti_engine_set_weight", fn);
   if (!(c.bits & TI_BITS_G32)) return ti_set_error(TI_ERR_ARG, "%s: engine bits %d lack TI_BITS_G32", fn, c.bits);
   if (((c.bits & TI_BITS_AFF) != 0) != (m != nullptr))
     return ti_set_error(TI_ERR_ARG, "%s: engine bits %d (%s blocks expected)", fn, c.bits,
@@ -936,6 +1103,7 @@ int ti_engine_synth(ti_engine* e, uint64_t seed, float norm_jitter) {
   if (!e) return ti_set_error(TI_ERR_ARG, "ti_engine_synth: null");
   DeviceScope bind_(e);
   const ti_engine_config& c = e->c;
+  if (e->stack) return e->stack->synth(seed, norm_jitter);
   if (c.compat) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_synth: compat engines take the reference model");
   if (c.bits & TI_BITS_G32)
     return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_synth: group-32 engines take their weights from ti_engine_set_tensor[_q]");
@@ -964,6 +1132,7 @@ int ti_engine_fill_kv(ti_engine* e, int stream, int n, uint64_t seed) {
   DeviceScope bind_(e);
   if (stream < 0 || stream >= e->c.max_batch || n < 0 || n > e->c.max_seq)
     return ti_set_error(TI_ERR_ARG, "ti_engine_fill_kv: stream %d n %d", stream, n);
+  if (e->stack) return e->stack->fill_kv(stream, n, seed);
   for (int l = 0; l < e->c.layers; ++l) {
     DevLayer& L = e->layer[l];
     TI_TRY(ti_fill_kv_uniform(seed, tid_kv(l, 0), n, e->c.kv_heads, e->c.head_dim, e->c.max_seq,
@@ -1026,13 +1195,7 @@ int ti_engine_generate(ti_engine* e, int n, const int32_t* prompts, const int32_
     if (last_in_prefill) {
       // one stream: its row in place, argmax slots cleared by the chunk's step_begin
       if (n > 1) TI_TRY(ti_memset(e->argmax, 0, (size_t)n * TI_ARGMAX_SLOTS * 8, e->s));
-      ti_epilogue el{};
-      el.kind = TI_EPI_LOGITS_ARGMAX;
-      el.ldo = c.vocab;
-      el.out = e->logits;
-      el.argmax = e->argmax;
-      const float* x = n > 1 ? e->h_last : e->h + (size_t)(last_rows - 1) * c.hidden;
-      TI_TRY(gemm_rows(e, e->lm, n, x, TI_X_F32_RMSNORM, c.hidden, e->out_norm, el, 4, false));
+      TI_TRY(enqueue_head(e, n, n > 1 ? e->h_last : e->h + (size_t)(last_rows - 1) * c.hidden));
     }
   }
   TI_TRY(ti_memcpy_h2d(e->step_ctr, &s0, 4, e->s));
@@ -1221,6 +1384,7 @@ std::vector<float> beam_top_p(const std::vector<float>& probs, float p) {
 // Copy slot `src`'s cache positions [0, n) into slot `dst`, every layer, K and V.
 int fork_slot(ti_engine* e, int src, int dst, int n) {
   const ti_engine_config& c = e->c;
+  if (e->stack) return e->stack->fork(src, dst, n);
   return ti_kv_copy_slots(e->kv_tab, 2 * c.layers, (int64_t)src * e->kv_stride, (int64_t)dst * e->kv_stride,
                           c.kv_heads, (int64_t)c.max_seq * c.head_dim, (int64_t)n * c.head_dim, e->s);
 }
@@ -1465,7 +1629,7 @@ int ti_engine_counters(ti_engine* e, uint64_t* decode_steps, uint64_t* prefill_c
 }
 
 int ti_engine_set_prefill(ti_engine* e, int rows) {
-  if (!e || e->c.compat || rows < 0 || rows > e->rows_cap || (rows > 0 && rows > ((e->c.bits & ~TI_BITS_G32) == 4 ? TI_GEMM_MAX_ROWS : 16)))
+  if (!e || e->c.compat || rows < 0 || rows > e->rows_cap || (rows > 0 && (!e->stack && rows > ((e->c.bits & ~TI_BITS_G32) == 4 ? TI_GEMM_MAX_ROWS : 16))))
     return ti_set_error(TI_ERR_ARG, "ti_engine_set_prefill: rows %d", rows);
   DeviceScope bind_(e);
   e->pf_rows = rows;
@@ -1598,6 +1762,7 @@ int ti_engine_last_tokens(ti_engine* e, int n, int32_t* tokens) {
 int ti_engine_time_kernel(ti_engine* e, int which, int n, int kv_len, int reps, double* avg_us, double* bytes) {
   if (!e || e->c.compat || !avg_us || !bytes || reps < 1 || n < 1 || n > e->c.max_batch || e->c.layers < 1)
     return ti_set_error(TI_ERR_ARG, "ti_engine_time_kernel: bad arguments");
+  if (e->stack) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_time_kernel: llama engines only");
   DeviceScope bind_(e);
   const ti_engine_config& c = e->c;
   const int H = c.hidden, I = c.inter, qd = e->qd(), kvd = e->kvd();
@@ -1799,6 +1964,7 @@ int ti_engine_stamp_steps(ti_engine* e, int steps, int cap, int32_t* info_out, d
   if (!e || e->replay_M < 1 || steps < 1 || steps > 256 || cap < 1 || !info_out || !t_out || !n_launch)
     return ti_set_error(TI_ERR_ARG, "ti_engine_stamp_steps: call ti_engine_replay_prepare first; 1 <= steps <= 256, "
                         "cap >= 1");
+  if (e->stack) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_stamp_steps: llama engines only");
   DeviceScope bind_(e);
   TI_TRY(ti_stream_sync(e->s));
   // pass 1: one step's launch list and grids; pass 2: `steps` steps back to back in one graph, every

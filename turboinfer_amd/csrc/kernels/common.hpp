@@ -108,6 +108,12 @@ __device__ __forceinline__ float group_sum(float v) {
   return v;
 }
 
+// monotone key of an fp32 value (greedy argmax keys: unsigned order = float order)
+__device__ __forceinline__ uint32_t float_order_key(float v) {
+  const uint32_t u = __builtin_bit_cast(uint32_t, v);
+  return (u & 0x80000000u) ? ~u : (u | 0x80000000u);
+}
+
 // ------------------------------------------------------- write-through (sc1) accesses
 // (persistent decode hand-offs, split merges: MI355X_MICROARCH.md "Hand-offs measured with sc1 loads")
 constexpr int kAuxSc1Load = 16;   // buffer aux bit 4 = sc1 on gfx950

@@ -1,0 +1,445 @@
+// dense.hip -- matrix products of the layer-stack models (ti_stack.h ti_dense): fragment-ordered
+// weights x row-major activations on MFMA, bf16 or fp32, with the consumer's first step fused into
+// the epilogue (SiLU * up, rotary pairs, head gates, logits + argmax, key / value fragments).
+//
+// Two kernels share the epilogue:
+//   * dense_skinny_kernel (M <= 64): HBM-bound weight streaming.  One workgroup per 16 output columns,
+//     its waves split k; each weight fragment is one contiguous KiB read once and multiplied with up
+//     to 4 row tiles; the waves' partial sums meet in LDS.
+//   * dense_tile_kernel (more rows): 4 waves as 2 x 2 over a BM x BN tile, activations staged through
+//     double-buffered LDS in fragment order, weight fragments straight from L2 into registers one
+//     k-stage (128 bytes) ahead.
+// Both take independent batches (per-head products) or grouped tiles (experts: a tile is up to
+// tile_rows entries of one expert's list, rows gathered and scattered through the list).
+#include <algorithm>
+
+#include "elem.hpp"
+
+namespace ti {
+
+__device__ __forceinline__ unsigned long long logit_key(float v, int n) {
+  return ((unsigned long long)float_order_key(v) << 32) | (unsigned long long)(0xFFFFFFFFu - (uint32_t)n);
+}
+
+// Four consecutive output columns n0.. of row m (out row mo); rows >= rows are padding.
+template <class T>
+__device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, int m, int mo, int rows, int n0, f32x4 v) {
+  constexpr int VEC = El<T>::VEC, KT = El<T>::KT;
+  const bool live = m < rows;
+  switch (a.epi) {
+    case TI_DE_F32: {
+      if (!live) return;
+      float* o = (float*)a.out + (size_t)batch * a.o_batch + (size_t)mo * a.ldo + n0;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (n0 + i < a.N) o[i] = a.add ? v[i] + a.add[n0 + i] : v[i];
+      return;
+    }
+    case TI_DE_T: {
+      if (!live) return;
+      T* o = (T*)a.out + (size_t)batch * a.o_batch + (size_t)mo * a.ldo + n0;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (n0 + i < a.N) o[i] = (T)v[i];
+      return;
+    }
+    case TI_DE_SWIGLU: {
+      if (!live) return;
+      T* o = (T*)a.out + (size_t)mo * a.ldo + (n0 >> 1);
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+        if (n0 + 2 * i < a.N) o[i] = (T)(v[2 * i] * sigmoidf(v[2 * i]) * v[2 * i + 1]);
+      return;
+    }
+    case TI_DE_ROPE: {
+      if (!live || n0 >= a.N) return;
+      const int r = n0 % a.head_w - a.rot_off;
+      if (r >= 0) {
+        const int pairs = (a.head_w - a.rot_off) >> 1;
+        const float* cs = a.rope_cs + ((size_t)a.pos[m] * pairs + (r >> 1)) * 2;
+        const f32x4 t = *(const f32x4*)cs;
+        v = (f32x4){v[0] * t[0] - v[1] * t[1], v[1] * t[0] + v[0] * t[1], v[2] * t[2] - v[3] * t[3],
+                    v[3] * t[2] + v[2] * t[3]};
+      }
+      *(typename El<T>::Q*)((T*)a.out + (size_t)mo * a.ldo + n0) = quad<T>(v);
+      return;
+    }
+    case TI_DE_GATE: {
+      if (!live) return;
+      const float g = a.gate[(size_t)m * a.gate_ld + batch];
+      T* o = (T*)a.out + (size_t)mo * a.ldo + (size_t)batch * a.N + n0;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (n0 + i < a.N) o[i] = (T)(v[i] * g);
+      return;
+    }
+    case TI_DE_KFRAG: {   // every row of the tile is written (padding rows repeat the last key)
+      if (n0 >= a.N) return;
+      const int h = n0 / a.head_w, d = n0 - h * a.head_w, dt = a.head_w / KT;
+      T* o = (T*)a.out + ((((size_t)h * a.key_blocks + (m >> 4)) * dt + d / KT) * 64 + ((d % KT) / VEC) * 16 + (m & 15)) * VEC +
+             d % VEC;
+      *(typename El<T>::Q*)o = quad<T>(v);
+      return;
+    }
+    default: return;
+  }
+}
+
+// TI_DE_VFRAG: four consecutive keys m0.. of column n.
+template <class T>
+__device__ __forceinline__ void dense_store_v(const ti_dense_args& a, int m0, int n, f32x4 v) {
+  constexpr int VEC = El<T>::VEC, KT = El<T>::KT;
+  if (n >= a.N) return;
+  const int h = n / a.head_w, d = n - h * a.head_w;
+  const int kb = m0 / KT, t = (m0 % KT) >> 4, g = (m0 & 15) >> 2, nkb = a.key_blocks * 16 / KT;
+  T* o = (T*)a.out + ((((size_t)h * (a.head_w >> 4) + (d >> 4)) * nkb + kb) * 64 + g * 16 + (d & 15)) * VEC + t * 4;
+  *(typename El<T>::Q*)o = quad<T>(v);
+}
+
+// Greedy argmax keys of a 16-column tile: lane l holds columns n0.. of row m = its (l & 15).
+__device__ __forceinline__ void dense_argmax(const ti_dense_args& a, int m, int rows, int n0, f32x4 v, int lane, int slot) {
+  unsigned long long key = 0ull;
+  if (m < rows) {
+    float* o = (float*)a.out + (size_t)m * a.ldo + n0;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (n0 + i < a.N) {
+        o[i] = v[i];
+        const unsigned long long k = logit_key(v[i], n0 + i);
+        key = k > key ? k : key;
+      }
+  }
+#pragma unroll
+  for (int o = 16; o < 64; o <<= 1) {
+    const unsigned long long other = __shfl_xor(key, o, kWave);
+    key = other > key ? other : key;
+  }
+  if (lane < 16 && key) atomicMax(a.argmax + (size_t)m * TI_ARGMAX_SLOTS + (slot & (TI_ARGMAX_SLOTS - 1)), key);
+}
+
+struct DenseSpan {   // what a workgroup works on
+  int rows, first, batch;
+  const void* w;
+};
+
+__device__ __forceinline__ bool dense_span(const ti_dense_args& a, int y, DenseSpan& s, size_t esize) {
+  if (a.tile_rows) {
+    if (y >= *a.n_tiles) return false;
+    const int e = a.tiles[4 * y];
+    s.first = a.tiles[4 * y + 1];
+    s.rows = a.tiles[4 * y + 2];
+    s.batch = 0;
+    s.w = (const char*)a.w + (size_t)e * a.w_batch * esize;
+  } else {
+    s.first = 0;
+    s.rows = a.M;
+    s.batch = y;
+    s.w = (const char*)a.w + (size_t)y * a.w_batch * esize;
+  }
+  return true;
+}
+__device__ __forceinline__ int row_in(const ti_dense_args& a, int p) { return a.rows_in ? a.rows_in[p] / a.row_div : p; }
+__device__ __forceinline__ int row_out(const ti_dense_args& a, int p) { return a.rows_out ? a.rows_out[p] : p; }
+
+template <class T, int MT, int W>
+__global__ __launch_bounds__(64 * W) void dense_skinny_kernel(const ti_dense_args a) {
+  typedef typename El<T>::V V;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, U = 8;
+  __shared__ f32x4 red[W][MT][64];
+  DenseSpan sp;
+  if (!dense_span(a, blockIdx.y, sp, sizeof(T))) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nt = blockIdx.x, nk = a.K / KT;
+  const V* wp = (const V*)sp.w + (size_t)nt * nk * 64 + lane;
+  const V* ap[MT];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) {
+    const int p = sp.first + min(mt * 16 + (lane & 15), sp.rows - 1);
+    ap[mt] = (const V*)((const T*)a.a + (size_t)sp.batch * a.a_batch + (size_t)row_in(a, p) * a.lda) + (lane >> 4);
+  }
+  f32x4 acc[MT];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) acc[mt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  int kt = wave;
+  for (; kt + (U - 1) * W < nk; kt += U * W) {
+    V wf[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) wf[u] = wp[(size_t)(kt + u * W) * 64];
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+      V af[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) af[u] = ap[mt][(kt + u * W) * (KT / VEC)];
+#pragma unroll
+      for (int u = 0; u < U; ++u) acc[mt] = mma(wf[u], af[u], acc[mt]);
+    }
+  }
+  for (; kt < nk; kt += W) {
+    const V wf = wp[(size_t)kt * 64];
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) acc[mt] = mma(wf, ap[mt][kt * (KT / VEC)], acc[mt]);
+  }
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) red[wave][mt][lane] = acc[mt];
+  __syncthreads();
+  for (int mt = wave; mt < MT; mt += W) {
+    f32x4 v = red[0][mt][lane];
+#pragma unroll
+    for (int w = 1; w < W; ++w) v += red[w][mt][lane];
+    const int m = mt * 16 + (lane & 15), n0 = nt * 16 + 4 * (lane >> 4);
+    if (a.epi == TI_DE_LOGITS)
+      dense_argmax(a, m, sp.rows, n0, v, lane, nt);
+    else
+      dense_store<T>(a, sp.batch, m, m < sp.rows ? row_out(a, sp.first + m) : 0, sp.rows, n0, v);
+  }
+  if (a.epi == TI_DE_LOGITS && a.step_ctr && nt == 0 && tid == 0) *a.step_ctr += a.advance;
+}
+
+template <class T, int BM, int BN, bool VF>
+__global__ __launch_bounds__(256) void dense_tile_kernel(const ti_dense_args a, int m_tiles, int n_tiles) {
+  typedef typename El<T>::V V;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, FM = BM / 32, FN = BN / 32;
+  __shared__ V as[2][BM / 16 * 2][64];
+  DenseSpan sp;
+  if (!dense_span(a, blockIdx.y, sp, sizeof(T))) return;
+  // consecutive workgroups go to the 8 XCDs in turn: give each XCD a contiguous run of tiles, row
+  // tiles fastest, so the weight columns a run shares stay in that XCD's L2
+  const int total = m_tiles * n_tiles, per = (total + 7) >> 3;
+  const int id = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
+  if (id >= total) return;
+  const int mtile = id % m_tiles, ntile = id / m_tiles, m_base = mtile * BM;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave & 1, wn = wave >> 1;
+  const int nk = a.K / KT, nst = nk >> 1, NT = (a.N + 15) >> 4;
+  const V* ap[FM];
+#pragma unroll
+  for (int i = 0; i < FM; ++i) {
+    const int f = i * 4 + wave;   // fragment (row tile f >> 1, k-tile f & 1) of the stage
+    const int p = sp.first + min(m_base + (f >> 1) * 16 + (lane & 15), sp.rows - 1);
+    ap[i] = (const V*)((const T*)a.a + (size_t)sp.batch * a.a_batch + (size_t)row_in(a, p) * a.lda) + (f & 1) * (KT / VEC) +
+            (lane >> 4);
+  }
+  const V* wp[FN];
+#pragma unroll
+  for (int j = 0; j < FN; ++j)
+    wp[j] = (const V*)sp.w + (size_t)min(ntile * (BN / 16) + wn * FN + j, NT - 1) * nk * 64 + lane;
+  f32x4 acc[FM][FN];
+#pragma unroll
+  for (int i = 0; i < FM; ++i)
+#pragma unroll
+    for (int j = 0; j < FN; ++j) acc[i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  V ar[FM], wc[FN][2], wx[FN][2];
+#pragma unroll
+  for (int i = 0; i < FM; ++i) ar[i] = ap[i][0];
+#pragma unroll
+  for (int j = 0; j < FN; ++j) {
+    wc[j][0] = wp[j][0];
+    wc[j][1] = wp[j][64];
+  }
+#pragma unroll
+  for (int i = 0; i < FM; ++i) as[0][i * 4 + wave][lane] = ar[i];
+  __syncthreads();
+  for (int s = 0; s < nst; ++s) {
+    const int nx = min(s + 1, nst - 1);
+#pragma unroll
+    for (int i = 0; i < FM; ++i) ar[i] = ap[i][nx * 2 * (KT / VEC)];
+#pragma unroll
+    for (int j = 0; j < FN; ++j) {
+      wx[j][0] = wp[j][(size_t)nx * 128];
+      wx[j][1] = wp[j][(size_t)nx * 128 + 64];
+    }
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      V af[FM];
+#pragma unroll
+      for (int i = 0; i < FM; ++i) af[i] = as[s & 1][(wm * FM + i) * 2 + kk][lane];
+#pragma unroll
+      for (int i = 0; i < FM; ++i)
+#pragma unroll
+        for (int j = 0; j < FN; ++j) acc[i][j] = VF ? mma(af[i], wc[j][kk], acc[i][j]) : mma(wc[j][kk], af[i], acc[i][j]);
+    }
+#pragma unroll
+    for (int i = 0; i < FM; ++i) as[(s + 1) & 1][i * 4 + wave][lane] = ar[i];
+#pragma unroll
+    for (int j = 0; j < FN; ++j) {
+      wc[j][0] = wx[j][0];
+      wc[j][1] = wx[j][1];
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < FM; ++i) {
+    const int mt = m_base + (wm * FM + i) * 16;
+    const int m = mt + (lane & 15);
+    const int mo = m < sp.rows ? row_out(a, sp.first + m) : 0;
+#pragma unroll
+    for (int j = 0; j < FN; ++j) {
+      const int nt = ntile * (BN / 16) + wn * FN + j;
+      if (nt >= NT) continue;
+      if (VF)
+        dense_store_v<T>(a, mt + 4 * (lane >> 4), nt * 16 + (lane & 15), acc[i][j]);
+      else if (a.epi == TI_DE_LOGITS)
+        dense_argmax(a, m, sp.rows, nt * 16 + 4 * (lane >> 4), acc[i][j], lane, nt);
+      else
+        dense_store<T>(a, sp.batch, m, mo, sp.rows, nt * 16 + 4 * (lane >> 4), acc[i][j]);
+    }
+  }
+  if (a.epi == TI_DE_LOGITS && a.step_ctr && id == 0 && tid == 0) *a.step_ctr += a.advance;
+}
+
+template <class T, int MT>
+int launch_skinny(const ti_dense_args& a, hipStream_t s) {
+  const int NT = (a.N + 15) / 16, y = a.tile_rows ? a.max_tiles : a.batch, nk = a.K / El<T>::KT;
+  if (nk >= 32)
+    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 8>), dim3(NT, y), dim3(512), 0, s, a);
+  else
+    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 4>), dim3(NT, y), dim3(256), 0, s, a);
+  TI_LAUNCH_CHECK("dense_skinny_kernel");
+  return TI_OK;
+}
+
+template <class T, int BM, int BN, bool VF>
+int launch_tile(const ti_dense_args& a, hipStream_t s) {
+  const int mt = a.tile_rows ? 1 : (a.M + BM - 1) / BM, nt = (a.N + BN - 1) / BN, per = (mt * nt + 7) / 8;
+  hipLaunchKernelGGL((dense_tile_kernel<T, BM, BN, VF>), dim3(per * 8, a.tile_rows ? a.max_tiles : a.batch), dim3(256), 0, s,
+                     a, mt, nt);
+  TI_LAUNCH_CHECK("dense_tile_kernel");
+  return TI_OK;
+}
+
+template <class T>
+int dispatch_dense(const ti_dense_args& a, hipStream_t s) {
+  if (a.epi == TI_DE_VFRAG) return launch_tile<T, 128, 64, true>(a, s);
+  if (a.epi == TI_DE_KFRAG) return launch_tile<T, 128, 64, false>(a, s);
+  if (a.tile_rows == 16) return launch_skinny<T, 1>(a, s);
+  if (a.tile_rows == 64) return launch_tile<T, 64, 64, false>(a, s);
+  if (a.M <= 16) return launch_skinny<T, 1>(a, s);
+  if (a.M <= 32) return launch_skinny<T, 2>(a, s);
+  if (a.M <= 64) return launch_skinny<T, 4>(a, s);
+  // the largest tile that still gives every CU a workgroup
+  auto wgs = [&](int bm, int bn) { return (long)((a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn) * a.batch; };
+  if (wgs(128, 128) >= 256) return launch_tile<T, 128, 128, false>(a, s);
+  if (wgs(128, 64) >= 256) return launch_tile<T, 128, 64, false>(a, s);
+  return launch_tile<T, 64, 64, false>(a, s);
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void stack_fill_kernel(uint64_t stream, uint64_t n, float scale, T* out) {
+  for (uint64_t i = (uint64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (uint64_t)gridDim.x * 256)
+    out[i] = (T)(scale * synth_unit(stream, i));
+}
+
+// fp32 source elements into fragment order (ti_stack_pack)
+template <class T>
+__global__ __launch_bounds__(256) void stack_pack_kernel(const float* src, int64_t rs, int64_t ks, int rows, int K, int nk,
+                                                         const int32_t* map, T* dst) {
+  constexpr int VEC = El<T>::VEC, KT = El<T>::KT;
+  const int64_t n = (int64_t)rows * K;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+    const int r = (int)(i / K), k = (int)(i - (int64_t)r * K), d = map ? map[r] : r;
+    dst[(((int64_t)(d >> 4) * nk + k / KT) * 64 + ((k % KT) / VEC) * 16 + (d & 15)) * VEC + k % VEC] = (T)src[r * rs + k * ks];
+  }
+}
+template <class T>
+__global__ __launch_bounds__(256) void stack_convert_kernel(const float* src, uint64_t n, T* dst) {
+  for (uint64_t i = (uint64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (uint64_t)gridDim.x * 256) dst[i] = (T)src[i];
+}
+
+}  // namespace ti
+
+extern "C" int ti_stack_kpad(int dtype, int K) {
+  const int u = dtype == TI_DT_BF16 ? 64 : 32;
+  return (K + u - 1) / u * u;
+}
+
+extern "C" size_t ti_stack_weight_bytes(int dtype, int N, int K) {
+  if (N < 1 || K < 1) return 0;
+  return (size_t)((N + 15) / 16 * 16) * ti_stack_kpad(dtype, K) * (dtype == TI_DT_BF16 ? 2 : 4);
+}
+
+extern "C" int ti_stack_pack(const float* src, int64_t rs, int64_t ks, int rows, int K, const int32_t* map, int dtype,
+                             void* dst, ti_stream_t stream) {
+  using namespace ti;
+  if (!src || !dst || rows < 1 || K < 1 || (dtype != TI_DT_BF16 && dtype != TI_DT_F32))
+    return ti_set_error(TI_ERR_ARG, "ti_stack_pack: bad arguments");
+  const unsigned g = (unsigned)std::min<int64_t>(((int64_t)rows * K + 255) / 256, 8192);
+  const int kp = ti_stack_kpad(dtype, K);
+  if (dtype == TI_DT_BF16)
+    hipLaunchKernelGGL(stack_pack_kernel<bf16>, dim3(g), dim3(256), 0, (hipStream_t)stream, src, rs, ks, rows, K,
+                       kp / El<bf16>::KT, map, (bf16*)dst);
+  else
+    hipLaunchKernelGGL(stack_pack_kernel<float>, dim3(g), dim3(256), 0, (hipStream_t)stream, src, rs, ks, rows, K,
+                       kp / El<float>::KT, map, (float*)dst);
+  TI_LAUNCH_CHECK("stack_pack_kernel");
+  return TI_OK;
+}
+
+extern "C" int ti_stack_convert(const float* src, uint64_t n, int dtype, void* dst, ti_stream_t stream) {
+  using namespace ti;
+  if (!src || !dst || (dtype != TI_DT_BF16 && dtype != TI_DT_F32)) return ti_set_error(TI_ERR_ARG, "ti_stack_convert: bad arguments");
+  if (n == 0) return TI_OK;
+  const unsigned g = (unsigned)std::min<uint64_t>((n + 255) / 256, 4096);
+  if (dtype == TI_DT_BF16)
+    hipLaunchKernelGGL(stack_convert_kernel<bf16>, dim3(g), dim3(256), 0, (hipStream_t)stream, src, n, (bf16*)dst);
+  else
+    hipLaunchKernelGGL(stack_convert_kernel<float>, dim3(g), dim3(256), 0, (hipStream_t)stream, src, n, (float*)dst);
+  TI_LAUNCH_CHECK("stack_convert_kernel");
+  return TI_OK;
+}
+
+extern "C" size_t ti_dense_args_bytes(void) { return sizeof(ti_dense_args); }
+
+extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->w || !a->a || !a->out || a->M < 1 || a->N < 1 || a->K < 1 || a->batch < 1)
+    return ti_set_error(TI_ERR_ARG, "ti_dense: bad arguments");
+  if (a->dtype != TI_DT_BF16 && a->dtype != TI_DT_F32) return ti_set_error(TI_ERR_ARG, "ti_dense: dtype %d", a->dtype);
+  const int vec = a->dtype == TI_DT_BF16 ? 8 : 4;
+  if (a->K != ti_stack_kpad(a->dtype, a->K) || a->lda % vec || a->a_batch % vec)
+    return ti_set_error(TI_ERR_ARG, "ti_dense: K %d / lda %d not padded", a->K, a->lda);
+  if ((!a->tile_rows && !a->rows_in && a->lda < a->K) || a->batch > 65535)
+    return ti_set_error(TI_ERR_ARG, "ti_dense: lda %d < K %d or batch %d", a->lda, a->K, a->batch);
+  if (a->tile_rows && ((a->tile_rows != 16 && a->tile_rows != 64) || !a->tiles || !a->n_tiles || a->max_tiles < 1 ||
+                       a->max_tiles > 65535 || a->batch != 1 || a->epi > TI_DE_SWIGLU || (a->rows_in && a->row_div < 1)))
+    return ti_set_error(TI_ERR_ARG, "ti_dense: grouped arguments");
+  if (!a->tile_rows && (a->rows_in || a->rows_out)) return ti_set_error(TI_ERR_ARG, "ti_dense: row lists need grouped tiles");
+  switch (a->epi) {
+    case TI_DE_F32: case TI_DE_T: break;
+    case TI_DE_SWIGLU:
+      if (a->N % 2 || a->batch != 1) return ti_set_error(TI_ERR_ARG, "ti_dense: SWIGLU N %d", a->N);
+      break;
+    case TI_DE_ROPE:
+      if (!a->rope_cs || !a->pos || a->head_w < 1 || a->N % a->head_w || a->head_w % 4 || a->rot_off % 4 || a->ldo % 4 ||
+          a->rot_off > a->head_w || a->batch != 1)
+        return ti_set_error(TI_ERR_ARG, "ti_dense: ROPE arguments");
+      break;
+    case TI_DE_GATE:
+      if (!a->gate || a->gate_ld < a->batch) return ti_set_error(TI_ERR_ARG, "ti_dense: GATE arguments");
+      break;
+    case TI_DE_LOGITS:
+      if (!a->argmax || a->batch != 1) return ti_set_error(TI_ERR_ARG, "ti_dense: LOGITS arguments");
+      break;
+    case TI_DE_KFRAG: case TI_DE_VFRAG: {
+      const int unit = a->epi == TI_DE_KFRAG ? 4 * vec : 16;
+      if (a->head_w < 1 || a->N % a->head_w || a->head_w % unit || a->batch != 1 || a->key_blocks % 8 ||
+          (long)a->key_blocks * 16 < ((long)a->M + 127) / 128 * 128)
+        return ti_set_error(TI_ERR_ARG, "ti_dense: key / value fragments: head_w %d, key_blocks %d, M %d", a->head_w,
+                            a->key_blocks, a->M);
+      break;
+    }
+    default: return ti_set_error(TI_ERR_ARG, "ti_dense: epilogue %d", a->epi);
+  }
+  return a->dtype == TI_DT_BF16 ? dispatch_dense<bf16>(*a, (hipStream_t)stream) : dispatch_dense<float>(*a, (hipStream_t)stream);
+}
+
+extern "C" int ti_stack_fill(uint64_t seed, uint32_t tid, uint64_t n, float scale, int dtype, void* out, ti_stream_t stream) {
+  using namespace ti;
+  if (!out || (dtype != TI_DT_BF16 && dtype != TI_DT_F32)) return ti_set_error(TI_ERR_ARG, "ti_stack_fill: bad arguments");
+  if (n == 0) return TI_OK;
+  const unsigned g = (unsigned)std::min<uint64_t>((n + 255) / 256, 4096);
+  const uint64_t st = synth_stream(seed, tid);
+  if (dtype == TI_DT_BF16)
+    hipLaunchKernelGGL(stack_fill_kernel<bf16>, dim3(g), dim3(256), 0, (hipStream_t)stream, st, n, scale, (bf16*)out);
+  else
+    hipLaunchKernelGGL(stack_fill_kernel<float>, dim3(g), dim3(256), 0, (hipStream_t)stream, st, n, scale, (float*)out);
+  TI_LAUNCH_CHECK("stack_fill_kernel");
+  return TI_OK;
+}

@@ -1,0 +1,67 @@
+// elem.hpp -- element types of the layer-stack kernels: bf16 and fp32 behind one fragment shape.
+//
+// A fragment is 64 lanes x 16 bytes (ti_stack.h): lane l holds row (l & 15) and VEC consecutive k
+// starting at VEC * (l >> 4) of a k-tile of KT.  bf16: one v_mfma_f32_16x16x32_bf16 per fragment
+// pair; fp32: four v_mfma_f32_16x16x4_f32, the i-th taking k = VEC * (l >> 4) + i from every lane
+// group (both operands use the same k order, so the sum is the same set of products).
+// Result of mma(a, b): lane l, register i = a-row 4 * (l >> 4) + i, b-row (l & 15).
+#pragma once
+
+#include "common.hpp"
+#include "ti_stack.h"
+
+namespace ti {
+
+typedef __bf16 bf16;
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
+
+template <class T>
+struct El;
+template <>
+struct El<bf16> {
+  static constexpr int VEC = 8, KT = 32;
+  typedef bf16x8 V;
+  typedef bf16x4 Q;   // 4 consecutive elements
+};
+template <>
+struct El<float> {
+  static constexpr int VEC = 4, KT = 16;
+  typedef f32x4 V;
+  typedef f32x4 Q;
+};
+
+__device__ __forceinline__ f32x4 mma(bf16x8 a, bf16x8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+__device__ __forceinline__ f32x4 mma(f32x4 a, f32x4 b, f32x4 c) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
+  return c;
+}
+
+template <class T>
+__device__ __forceinline__ typename El<T>::Q quad(f32x4 v) {
+  typename El<T>::Q q;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) q[i] = (T)v[i];
+  return q;
+}
+
+// block-wide sum of one float per thread; every thread gets it.  red: one float per wave.
+__device__ __forceinline__ float block_sum(float v, float* red) {
+  v = group_sum<64>(v);
+  const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  __syncthreads();   // red may still be read from the previous sum
+  if ((threadIdx.x & 63) == 0) red[wave] = v;
+  __syncthreads();
+  float s = 0.0f;
+  for (int i = 0; i < nw; ++i) s += red[i];
+  return s;
+}
+
+__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+}  // namespace ti

@@ -210,11 +210,6 @@ __device__ __forceinline__ void stage_x_generic(const GemvArgs& a, f16* xl, floa
 }
 
 // ------------------------------------------------------------------ epilogue
-__device__ __forceinline__ uint32_t float_order_key(float v) {
-  const uint32_t u = __builtin_bit_cast(uint32_t, v);
-  return (u & 0x80000000u) ? ~u : (u | 0x80000000u);
-}
-
 // Thread (l, i) holds y[m][n] of tile nt with m = 4*(l>>4) + i, n = l & 15 (the
 // v_mfma_f32_16x16x32 C layout, reduced over the 8 waves); l is the lane or, for M <= 4,
 // n alone.  Partners of the shuffles below (n ^ 1, n + 8) sit in the same 16-lane group.  `best` is the

@@ -1,0 +1,460 @@
+// latent_attn.hip -- attention over a shared low-rank latent (ti_stack.h): keys and values of every
+// head are linear images of one cached latent row per position, plus one rotated key part all heads
+// share.
+//
+//   * latent_prep_kernel: RMS norms of the query latent and the cached latent, rotary of the shared
+//     key part, cache append, sigmoid of the head gates -- one launch per layer.
+//   * latent_decode_kernel: the up-projections are carried over to the query and output side, so 16
+//     heads share every cached row: scores are one MFMA chain over [latent | rotated] with the heads as
+//     the MFMA columns, the weighted sum a second one over the latent part.  Keys are split over
+//     workgroups (splits) and over the waves of each.
+//   * latent_prefill_kernel: prompt chunks, keys and values expanded per head into MFMA fragments
+//     (dense.hip TI_DE_KFRAG / TI_DE_VFRAG); a wave owns 16 or 32 query rows of one head.
+// Scores, softmax and sums are fp32; the softmax denominator holds exp(sink) of the head once.
+#include <algorithm>
+
+#include "elem.hpp"
+
+namespace ti {
+
+template <class T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(const ti_latent_prep_args a) {
+  __shared__ float red[4];
+  const int m = blockIdx.x, tid = threadIdx.x, pos = a.pos[m];
+  const float* r = a.a32 + (size_t)m * a.lda;
+  float q2 = 0.0f, c2 = 0.0f;
+  for (int i = tid; i < a.q_rank; i += 256) q2 = fmaf(r[i], r[i], q2);
+  for (int i = tid; i < a.kv_rank; i += 256) c2 = fmaf(r[a.lat_off + i], r[a.lat_off + i], c2);
+  const float qi = 1.0f / sqrtf(block_sum(q2, red) / (float)a.q_rank + a.eps);
+  const float ci = 1.0f / sqrtf(block_sum(c2, red) / (float)a.kv_rank + a.eps);
+  T* cq = (T*)a.cq + (size_t)m * a.ldq;
+  for (int i = tid; i < a.q_rank; i += 256) cq[i] = (T)(r[i] * qi * a.q_w[i]);
+  T* row = (T*)a.cache + (size_t)m * a.slot_stride + (size_t)pos * (a.lat_p + a.rot_p);
+  for (int i = tid; i < a.lat_p; i += 256) row[i] = i < a.kv_rank ? (T)(r[a.lat_off + i] * ci * a.c_w[i]) : (T)0.0f;
+  for (int i = tid; i < a.rot_p / 2; i += 256) {
+    float u = 0.0f, v = 0.0f;
+    if (2 * i < a.rot_dim) u = r[a.rot_off + 2 * i];
+    if (2 * i + 1 < a.rot_dim) v = r[a.rot_off + 2 * i + 1];
+    const float2 cs = *(const float2*)(a.rope_cs + ((size_t)pos * (a.rot_p / 2) + i) * 2);
+    row[a.lat_p + 2 * i] = (T)(u * cs.x - v * cs.y);
+    row[a.lat_p + 2 * i + 1] = (T)(v * cs.x + u * cs.y);
+  }
+  for (int i = tid; i < a.heads; i += 256) a.gate[(size_t)m * a.heads + i] = sigmoidf(r[a.gate_off + i]);
+}
+
+// The VEC x VEC transpose a value fragment needs: in[j] = VEC consecutive value dims of key j of this
+// lane group; out(c) = dim c of the VEC keys.
+__device__ __forceinline__ bf16x8 gather_dim(const bf16x8* in, int c) {
+  const u32x4* d = (const u32x4*)in;
+  const uint32_t sel = (c & 1) ? 0x07060302u : 0x05040100u;   // the high or low halves of two dwords
+  u32x4 o;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) o[j] = __builtin_amdgcn_perm(d[2 * j + 1][c >> 1], d[2 * j][c >> 1], sel);
+  return __builtin_bit_cast(bf16x8, o);
+}
+
+// acc[c] += (value dims i * VEC + c, i = a-row) x (weights p of VEC-per-lane-group keys)
+__device__ __forceinline__ void mma_values(f32x4* acc, const bf16x8* vin, bf16x8 p) {
+#pragma unroll
+  for (int c = 0; c < 8; ++c) acc[c] = mma(gather_dim(vin, c), p, acc[c]);
+}
+__device__ __forceinline__ void mma_values(f32x4* acc, const f32x4* vin, f32x4 p) {
+#pragma unroll
+  for (int s = 0; s < 4; ++s)
+#pragma unroll
+    for (int c = 0; c < 4; ++c) acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(vin[s][c], p[s], acc[c], 0, 0, 0);
+}
+
+// Grid (splits, head tiles of 16, rows).  A block is 4 * KPW keys: wave w scores keys [w * KPW, +KPW),
+// then sums value dims of its groups (wave, wave + 4, ...; a group is 16 * VEC dims) over all of them.
+template <class T, int KPW, int GPW>
+__global__ __launch_bounds__(256) void latent_decode_kernel(const ti_latent_attn_args a) {
+  typedef typename El<T>::V V;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, KB = 4 * KPW, PLD = KB + 16 / (int)sizeof(T);
+  extern __shared__ char lds[];
+  const int split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
+  const int cw = a.lat_p + a.rot_p, nkt = cw / KT, lkt = a.lat_p / KT, G = a.lat_p / (16 * VEC) + (a.lat_p % (16 * VEC) != 0);
+  V* qf = (V*)lds;                                  // [nkt][64]
+  T* pb = (T*)(lds + (size_t)nkt * 1024);           // [16][PLD]
+  float* sm = (float*)(pb + 16 * PLD);              // [4][16] wave maxima, then [4][16] wave sums
+  const int pos = a.pos[m], head = ht * 16 + col;
+  const T* cache = (const T*)a.cache + (size_t)m * a.slot_stride;
+  for (int kt = wave; kt < nkt; kt += 4) {
+    V v = {};
+    if (head < a.heads)
+      v = kt < lkt ? *(const V*)((const T*)a.qa + ((size_t)m * a.heads + head) * a.lat_p + kt * KT + g * VEC)
+                   : *(const V*)((const T*)a.q + ((size_t)m * a.heads + head) * a.ldqr + a.qr_off + (kt - lkt) * KT + g * VEC);
+    qf[kt * 64 + lane] = v;
+  }
+  f32x4 o[GPW][VEC];
+#pragma unroll
+  for (int i = 0; i < GPW; ++i)
+#pragma unroll
+    for (int c = 0; c < VEC; ++c) o[i][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float mr = -INFINITY, lr = 0.0f;
+  const int nb = (pos + KB) / KB, bps = (nb + a.splits - 1) / a.splits, b0 = split * bps, b1 = min(nb, b0 + bps);
+  __syncthreads();
+  for (int b = b0; b < b1; ++b) {
+    const int k0 = b * KB + wave * KPW;
+    f32x4 s[KPW / 16];
+#pragma unroll
+    for (int t = 0; t < KPW / 16; ++t) s[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const V* kp = (const V*)(cache + (size_t)(k0 + col) * cw) + g;
+#pragma unroll 6
+    for (int kt = 0; kt < nkt; ++kt) {
+      const V q = qf[kt * 64 + lane];
+#pragma unroll
+      for (int t = 0; t < KPW / 16; ++t) s[t] = mma(kp[(size_t)t * 16 * cw / VEC + kt * 4], q, s[t]);
+    }
+    float mx = -INFINITY;
+#pragma unroll
+    for (int t = 0; t < KPW / 16; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        s[t][r] = k0 + t * 16 + 4 * g + r <= pos ? s[t][r] * a.scale : -INFINITY;
+        mx = fmaxf(mx, s[t][r]);
+      }
+    mx = xor32_max(xor16_max(mx));
+    if (lane < 16) sm[wave * 16 + col] = mx;
+    __syncthreads();
+    const float mn = fmaxf(fmaxf(mr, fmaxf(sm[col], sm[16 + col])), fmaxf(sm[32 + col], sm[48 + col]));
+    const float alpha = expf(mr - mn);   // (every block holds a visible key: mn is finite)
+    mr = mn;
+    lr *= alpha;
+#pragma unroll
+    for (int t = 0; t < KPW / 16; ++t) {
+      f32x4 p;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        p[r] = expf(s[t][r] - mn);
+        lr += p[r];
+      }
+      *(typename El<T>::Q*)(pb + col * PLD + wave * KPW + t * 16 + 4 * g) = quad<T>(p);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < GPW; ++i) {
+      const int gi = wave + 4 * i;
+      if (gi >= G) continue;
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) o[i][c] *= alpha;
+      const int d = gi * 16 * VEC + col * VEC, dc = min(d, a.lat_p - VEC);   // (dims past the latent: not stored)
+#pragma unroll 2
+      for (int kb = 0; kb < KB / KT; ++kb) {
+        const V p = *(const V*)(pb + col * PLD + kb * KT + g * VEC);
+        V vin[VEC];
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) vin[j] = *(const V*)(cache + (size_t)(b * KB + kb * KT + g * VEC + j) * cw + dc);
+        mma_values(o[i], vin, p);
+      }
+    }
+  }
+  lr = lane_xor<16>(lr) + lr;
+  lr = lane_xor<32>(lr) + lr;
+  __syncthreads();
+  if (lane < 16) sm[wave * 16 + col] = lr;
+  __syncthreads();
+  float l = sm[col] + sm[16 + col] + sm[32 + col] + sm[48 + col];
+  if (head >= a.heads) return;
+  const size_t row = a.splits > 1 ? (((size_t)m * a.splits + split) * a.heads + head) : (size_t)m * a.heads + head;
+  if (a.splits > 1) {
+    if (wave == 0 && lane < 16) {
+      a.part_ml[row * 2] = mr;
+      a.part_ml[row * 2 + 1] = l;
+    }
+    if (b0 >= b1) return;
+  } else {   // the whole row: the sink joins the denominator here
+    l += expf(a.sink[head] - mr);   // (a huge sink gives inf: weights 0)
+  }
+  const float inv = 1.0f / l;
+  T* out = (T*)(a.splits > 1 ? a.part_o : a.out) + row * a.lat_p;
+#pragma unroll
+  for (int i = 0; i < GPW; ++i) {
+    const int gi = wave + 4 * i;
+    if (gi >= G) continue;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = gi * 16 * VEC + (4 * g + r) * VEC;
+      if (d >= a.lat_p) continue;
+      V v;
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) v[c] = (T)(o[i][c][r] * inv);
+      *(V*)(out + d) = v;
+    }
+  }
+}
+
+template <class T>
+__global__ __launch_bounds__(128) void latent_merge_kernel(const ti_latent_attn_args a) {
+  typedef typename El<T>::V V;
+  constexpr int VEC = El<T>::VEC;
+  const int h = blockIdx.x, m = blockIdx.y;
+  const size_t row0 = (size_t)m * a.splits * a.heads + h;
+  float mx = a.sink[h];
+  for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, a.part_ml[(row0 + (size_t)s * a.heads) * 2]);
+  float den = expf(a.sink[h] - mx);
+  for (int s = 0; s < a.splits; ++s) {
+    const float* ml = a.part_ml + (row0 + (size_t)s * a.heads) * 2;
+    den += ml[1] * expf(ml[0] - mx);
+  }
+  for (int d = threadIdx.x * VEC; d < a.lat_p; d += 128 * VEC) {
+    float acc[VEC] = {};
+    for (int s = 0; s < a.splits; ++s) {
+      const size_t r = row0 + (size_t)s * a.heads;
+      const float w = a.part_ml[r * 2 + 1] * expf(a.part_ml[r * 2] - mx) / den;
+      if (w == 0.0f) continue;   // (a split without keys holds no partial)
+      const V v = *(const V*)((const T*)a.part_o + r * a.lat_p + d);
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) acc[c] = fmaf(w, (float)v[c], acc[c]);
+    }
+    V o;
+#pragma unroll
+    for (int c = 0; c < VEC; ++c) o[c] = (T)acc[c];
+    *(V*)((T*)a.out + ((size_t)m * a.heads + h) * a.lat_p + d) = o;
+  }
+}
+
+// ------------------------------------------------------------------ prompt chunks
+// Weights of 64 keys (4 key tiles, lane: query column, keys t * 16 + 4 g + r) x value fragments.
+__device__ __forceinline__ void pv_block(f32x4& acc, const bf16x8* vf, const f32x4* p) {
+#pragma unroll
+  for (int b = 0; b < 2; ++b) {
+    bf16x8 pf;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      pf[r] = (bf16)p[2 * b][r];
+      pf[4 + r] = (bf16)p[2 * b + 1][r];
+    }
+    acc = mma(vf[b], pf, acc);
+  }
+}
+__device__ __forceinline__ void pv_block(f32x4& acc, const f32x4* vf, const f32x4* p) {
+#pragma unroll
+  for (int t = 0; t < 4; ++t) acc = mma(vf[t], p[t], acc);
+}
+
+// Grid (row blocks of 4 * 16 * MQ, heads); a wave owns 16 * MQ rows.  The last row blocks (most keys)
+// start first.
+template <class T, int MQ, int NV>
+__global__ __launch_bounds__(256) void latent_prefill_kernel(const ti_latent_prefill_args a) {
+  typedef typename El<T>::V V;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, VB = 64 / KT;
+  extern __shared__ char lds[];
+  const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
+  const int row0 = ((int)(gridDim.x - 1 - blockIdx.x) * 4 + wave) * 16 * MQ;
+  if (row0 >= a.M) return;   // (no barrier below: waves are independent)
+  const int dkt = a.dim_p / KT, rkt = a.rot_p / KT, nkt = dkt + rkt, cw = a.lat_p + a.rot_p, nv = a.vdim_p >> 4;
+  V* qf = (V*)lds + (size_t)wave * nkt * MQ * 64;
+  for (int kt = 0; kt < nkt; ++kt)
+#pragma unroll
+    for (int q = 0; q < MQ; ++q) {
+      const int m = min(row0 + q * 16 + col, a.M - 1);
+      qf[(kt * MQ + q) * 64 + lane] =
+          *(const V*)((const T*)a.q + ((size_t)m * a.heads + h) * (a.dim_p + a.rot_p) + kt * KT + g * VEC);
+    }
+  const V* kf = (const V*)a.kfrag + (size_t)h * a.key_blocks * dkt * 64 + lane;
+  const V* vf = (const V*)a.vfrag + (size_t)h * nv * (a.key_blocks * 16 / KT) * 64 + lane;
+  const V* rp = (const V*)((const T*)a.cache + a.lat_p + (size_t)col * cw) + g;
+  f32x4 o[MQ][NV];
+  float mr[MQ], lr[MQ];
+#pragma unroll
+  for (int q = 0; q < MQ; ++q) {
+    mr[q] = a.sink[h];   // the sink: weight exp(sink - max), no value
+    lr[q] = g == 0 ? 1.0f : 0.0f;
+#pragma unroll
+    for (int v = 0; v < NV; ++v) o[q][v] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  }
+  const int last = a.pos0 + min(row0 + 16 * MQ, a.M) - 1;   // the wave's last position
+  for (int k0 = 0; k0 <= last; k0 += 64) {
+    f32x4 s[MQ][4];
+#pragma unroll
+    for (int q = 0; q < MQ; ++q)
+#pragma unroll
+      for (int t = 0; t < 4; ++t) s[q][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int kt = 0; kt < dkt; ++kt) {
+      V k[4];
+#pragma unroll
+      for (int t = 0; t < 4; ++t) k[t] = kf[((size_t)((k0 >> 4) + t) * dkt + kt) * 64];
+#pragma unroll
+      for (int q = 0; q < MQ; ++q) {
+        const V qv = qf[(kt * MQ + q) * 64 + lane];
+#pragma unroll
+        for (int t = 0; t < 4; ++t) s[q][t] = mma(k[t], qv, s[q][t]);
+      }
+    }
+    for (int kt = 0; kt < rkt; ++kt) {
+      V k[4];
+#pragma unroll
+      for (int t = 0; t < 4; ++t) k[t] = rp[(size_t)(k0 + t * 16) * cw / VEC + kt * 4];
+#pragma unroll
+      for (int q = 0; q < MQ; ++q) {
+        const V qv = qf[((dkt + kt) * MQ + q) * 64 + lane];
+#pragma unroll
+        for (int t = 0; t < 4; ++t) s[q][t] = mma(k[t], qv, s[q][t]);
+      }
+    }
+#pragma unroll
+    for (int q = 0; q < MQ; ++q) {
+      const int p = a.pos0 + row0 + q * 16 + col;
+      float mx = mr[q];
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          s[q][t][r] = k0 + t * 16 + 4 * g + r <= p ? s[q][t][r] * a.scale : -INFINITY;
+          mx = fmaxf(mx, s[q][t][r]);
+        }
+      mx = xor32_max(xor16_max(mx));
+      const float alpha = expf(mr[q] - mx);
+      mr[q] = mx;
+      float l = 0.0f;
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          s[q][t][r] = expf(s[q][t][r] - mx);
+          l += s[q][t][r];
+        }
+      lr[q] = lr[q] * alpha + l;
+#pragma unroll
+      for (int v = 0; v < NV; ++v) o[q][v] *= alpha;
+    }
+    const int nkb = a.key_blocks * 16 / KT;
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+      if (v < nv) {
+        V vv[VB];
+#pragma unroll
+        for (int b = 0; b < VB; ++b) vv[b] = vf[((size_t)v * nkb + k0 / KT + b) * 64];
+#pragma unroll
+        for (int q = 0; q < MQ; ++q) pv_block(o[q][v], vv, s[q]);
+      }
+    }
+  }
+#pragma unroll
+  for (int q = 0; q < MQ; ++q) {
+    const int m = row0 + q * 16 + col;
+    float l = lr[q];
+    l += lane_xor<16>(l);
+    l += lane_xor<32>(l);
+    if (m >= a.M) continue;
+    const float sc = a.gate[(size_t)m * a.heads + h] / l;
+    T* out = (T*)a.out + (size_t)m * a.ldo + (size_t)h * a.vdim;
+#pragma unroll
+    for (int v = 0; v < NV; ++v)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = v * 16 + 4 * g + r;
+        if (d < a.vdim) out[d] = (T)(o[q][v][r] * sc);
+      }
+  }
+}
+
+template <class T, int KPW>
+int launch_decode(const ti_latent_attn_args& a, hipStream_t s) {
+  constexpr int VEC = El<T>::VEC;
+  const int G = (a.lat_p + 16 * VEC - 1) / (16 * VEC), gpw = (G + 3) / 4;
+  const size_t lds = (size_t)(a.lat_p + a.rot_p) / El<T>::KT * 1024 + (size_t)16 * (4 * KPW + 16 / sizeof(T)) * sizeof(T) + 64 * 4;
+  const dim3 grid(a.splits, (a.heads + 15) / 16, a.M), blk(256);
+#define TI_LD(GPW) hipLaunchKernelGGL((latent_decode_kernel<T, KPW, GPW>), grid, blk, lds, s, a)
+  if (gpw == 1) TI_LD(1);
+  else if (gpw == 2) TI_LD(2);
+  else TI_LD(4);
+#undef TI_LD
+  TI_LAUNCH_CHECK("latent_decode_kernel");
+  if (a.splits > 1) {
+    hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(a.heads, a.M), dim3(128), 0, s, a);
+    TI_LAUNCH_CHECK("latent_merge_kernel");
+  }
+  return TI_OK;
+}
+
+template <class T>
+int launch_prefill(const ti_latent_prefill_args& a, hipStream_t s) {
+  const int nkt = (a.dim_p + a.rot_p) / El<T>::KT, nv = a.vdim_p / 16;
+  const bool two = (size_t)nkt * 2 * 1024 * 4 <= 81920 && nv <= 8 && a.M > 64;
+  const int mq = two ? 2 : 1;
+  const size_t lds = (size_t)nkt * mq * 1024 * 4;
+  if (lds > 163840 - 1024) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_prefill: head of %d + %d dims", a.dim_p, a.rot_p);
+  const dim3 grid((a.M + 64 * mq - 1) / (64 * mq), a.heads), blk(256);
+#define TI_LP(MQ, NV) hipLaunchKernelGGL((latent_prefill_kernel<T, MQ, NV>), grid, blk, lds, s, a)
+  if (two && nv <= 4) TI_LP(2, 4);
+  else if (two) TI_LP(2, 8);
+  else if (nv <= 4) TI_LP(1, 4);
+  else if (nv <= 8) TI_LP(1, 8);
+  else TI_LP(1, 16);
+#undef TI_LP
+  TI_LAUNCH_CHECK("latent_prefill_kernel");
+  return TI_OK;
+}
+
+// Kernels whose dynamic LDS can pass 64 KiB (before any graph capture).
+template <class T>
+int prepare() {
+  const void* k[] = {(const void*)latent_decode_kernel<T, 16, 1>, (const void*)latent_decode_kernel<T, 16, 2>,
+                     (const void*)latent_decode_kernel<T, 16, 4>, (const void*)latent_prefill_kernel<T, 2, 4>,
+                     (const void*)latent_prefill_kernel<T, 2, 8>, (const void*)latent_prefill_kernel<T, 1, 4>,
+                     (const void*)latent_prefill_kernel<T, 1, 8>, (const void*)latent_prefill_kernel<T, 1, 16>};
+  for (const void* f : k)
+    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 163840 - 1024), "latent attention LDS");
+  return TI_OK;
+}
+
+bool dtype_ok(int dt) { return dt == TI_DT_BF16 || dt == TI_DT_F32; }
+
+}  // namespace ti
+
+extern "C" int ti_latent_prepare(void) {
+  const int rc = ti::prepare<ti::bf16>();
+  return rc ? rc : ti::prepare<float>();
+}
+
+extern "C" int ti_latent_prep(const ti_latent_prep_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->a32 || !a->q_w || !a->c_w || !a->rope_cs || !a->pos || !a->cq || !a->cache || !a->gate || a->M < 1 ||
+      a->q_rank < 1 || a->kv_rank < 1 || a->rot_dim < 2 || a->rot_dim > a->rot_p || a->kv_rank > a->lat_p || a->ldq < a->q_rank ||
+      a->heads < 1 || !dtype_ok(a->dtype))
+    return ti_set_error(TI_ERR_ARG, "ti_latent_prep: bad arguments");
+  if (a->dtype == TI_DT_BF16)
+    hipLaunchKernelGGL(latent_prep_kernel<bf16>, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a);
+  else
+    hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a);
+  TI_LAUNCH_CHECK("latent_prep_kernel");
+  return TI_OK;
+}
+
+extern "C" int ti_latent_attn_splits(int M, int heads, int max_seq) {
+  // about one workgroup per CU, none with less than one 64-key block
+  const int wgs = M * ((heads + 15) / 16), cap = std::max(1, (max_seq + 63) / 64);
+  return std::max(1, std::min({cap, 64, (256 + wgs - 1) / std::max(1, wgs)}));
+}
+
+extern "C" int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->qa || !a->q || !a->cache || !a->pos || !a->sink || !a->out || a->M < 1 || a->M > 65535 || a->heads < 1 ||
+      a->splits < 1 || !dtype_ok(a->dtype) || (a->splits > 1 && (!a->part_o || !a->part_ml)))
+    return ti_set_error(TI_ERR_ARG, "ti_latent_attn_decode: bad arguments");
+  const int kt = a->dtype == TI_DT_BF16 ? 32 : 16, lim = a->dtype == TI_DT_BF16 ? 2048 : 1024;
+  if (a->lat_p < kt || a->lat_p % kt || a->rot_p < kt || a->rot_p % kt || a->seq_p % 128 || a->ldqr % (kt / 4) || a->qr_off % (kt / 4))
+    return ti_set_error(TI_ERR_ARG, "ti_latent_attn_decode: lat_p %d rot_p %d seq_p %d", a->lat_p, a->rot_p, a->seq_p);
+  if (a->lat_p > lim || (a->lat_p + a->rot_p) / kt * 1024 > 140000)
+    return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_decode: latent size %d (at most %d)", a->lat_p, lim);
+  hipStream_t s = (hipStream_t)stream;
+  if (a->dtype == TI_DT_BF16) return launch_decode<bf16, 16>(*a, s);
+  return launch_decode<float, 16>(*a, s);
+}
+
+extern "C" int ti_latent_attn_prefill(const ti_latent_prefill_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->q || !a->kfrag || !a->vfrag || !a->cache || !a->sink || !a->gate || !a->out || a->M < 1 || a->pos0 < 0 ||
+      a->heads < 1 || a->heads > 65535 || !dtype_ok(a->dtype))
+    return ti_set_error(TI_ERR_ARG, "ti_latent_attn_prefill: bad arguments");
+  const int kt = a->dtype == TI_DT_BF16 ? 32 : 16;
+  if (a->dim_p < kt || a->dim_p % kt || a->rot_p < kt || a->rot_p % kt || a->lat_p % kt || a->vdim_p % 16 || a->vdim > a->vdim_p ||
+      a->ldo < a->heads * a->vdim || a->key_blocks % 8 || (long)a->key_blocks * 16 < (long)a->pos0 + a->M)
+    return ti_set_error(TI_ERR_ARG, "ti_latent_attn_prefill: sizes");
+  if (a->vdim_p > 256) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_prefill: value size %d (at most 256)", a->vdim_p);
+  hipStream_t s = (hipStream_t)stream;
+  return a->dtype == TI_DT_BF16 ? launch_prefill<bf16>(*a, s) : launch_prefill<float>(*a, s);
+}

@@ -24,7 +24,7 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
   // loaded before the token is decided.
   constexpr int kPT = 4;   // pieces of 8 per thread
   const int H8 = a.hidden >> 3;
-  const bool vec = (a.hidden & 7) == 0 && H8 <= 256 * kPT && a.placeholder_first < 0;
+  const bool vec = (a.hidden & 7) == 0 && H8 <= 256 * kPT && a.placeholder_first < 0 && a.emb_kind == 0;
   float4 fw[kPT][2];
   if (vec && a.fold_x) {
 #pragma unroll
@@ -69,6 +69,15 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
     const size_t off = s == 0 ? (size_t)a.placeholder_first : 0;
     for (int i = tid; i < a.hidden; i += 256) {
       h[i] = 0.1f * (float)((off + (size_t)i) % 100);
+    }
+  } else if (a.emb_kind) {
+    const size_t r0 = (size_t)s_tok * a.hidden;
+    float* h0 = a.h0 ? a.h0 + (size_t)m * a.hidden : nullptr;
+    for (int i = tid; i < a.hidden; i += 256) {
+      const float v = a.emb_scale * (a.emb_kind == 1 ? __builtin_bit_cast(float, (uint32_t)a.emb[r0 + i] << 16)
+                                                     : ((const float*)a.emb)[r0 + i]);
+      h[i] = v;
+      if (h0) h0[i] = v;
     }
   } else if (vec) {
     const uint16_t* e = a.emb + (size_t)s_tok * a.hidden;
@@ -270,6 +279,8 @@ extern "C" int ti_step_begin(const ti_step_args* a, ti_stream_t stream) {
   if (a->n_in && !a->in_tokens) return ti_set_error(TI_ERR_ARG, "ti_step_begin: in_tokens required");
   if (a->fold_x && (!a->fold_w || !a->fold_ss || a->placeholder_first >= 0))
     return ti_set_error(TI_ERR_ARG, "ti_step_begin: fold_x needs fold_w, fold_ss and the embedding gather");
+  if (a->emb_kind < 0 || a->emb_kind > 2 || (a->emb_kind && (a->fold_x || a->placeholder_first >= 0)) || (a->h0 && !a->emb_kind))
+    return ti_set_error(TI_ERR_ARG, "ti_step_begin: emb_kind %d", a->emb_kind);
   hipLaunchKernelGGL(step_begin_kernel, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a,
                      ti_stamp_next(STAMP_BEGIN, a->M));
   TI_LAUNCH_CHECK("step_begin_kernel");

@@ -1,0 +1,233 @@
+// stack_ops.hip -- row kernels of the layer-stack models (ti_stack.h): residual + norms, expert
+// routing.  All arithmetic fp32.
+#include <algorithm>
+
+#include "elem.hpp"
+
+namespace ti {
+
+// A row of H values in LDS, normalised: mean and inverse deviation (layer norm) or inverse root mean
+// square (mean = 0).  The variance is the mean of the squared deviations (second pass over LDS).
+__device__ __forceinline__ float2 row_stats(const float* row, int H, float eps, int kind, float* red) {
+  float mean = 0.0f;
+  if (kind == TI_NORM_LAYER) {
+    float s = 0.0f;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) s += row[i];
+    mean = block_sum(s, red) / (float)H;
+  }
+  float q = 0.0f;
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    const float d = row[i] - mean;
+    q = fmaf(d, d, q);
+  }
+  const float var = block_sum(q, red) / (float)H;
+  return make_float2(mean, 1.0f / sqrtf(var + eps));
+}
+
+template <class T>
+__global__ __launch_bounds__(512) void rownorm_kernel(const ti_rownorm_args a) {
+  extern __shared__ float row[];
+  __shared__ float red[8];
+  const int m = blockIdx.x, H = a.H;
+  float* x = a.x + (size_t)m * H;
+  // (each thread touches only its own elements of `row` outside the reductions, which hold barriers)
+  if (a.y || a.parts) {
+    if (a.parts) {
+      const T* p = (const T*)a.parts + (size_t)m * a.top * a.ldy;
+      for (int i = threadIdx.x; i < H; i += blockDim.x) {
+        float v = 0.0f;
+        for (int k = 0; k < a.top; ++k) v = fmaf(a.part_w[(size_t)m * a.top + k], (float)p[(size_t)k * a.ldy + i], v);
+        row[i] = v;
+      }
+    } else {
+      for (int i = threadIdx.x; i < H; i += blockDim.x) row[i] = a.y[(size_t)m * a.ldy + i];
+    }
+    if (a.post_w) {
+      const float2 st = row_stats(row, H, a.eps, a.kind, red);
+      for (int i = threadIdx.x; i < H; i += blockDim.x) {
+        const float b = a.kind == TI_NORM_LAYER ? a.post_b[i] : 0.0f;
+        row[i] = x[i] + ((row[i] - st.x) * st.y * a.post_w[i] + b);
+      }
+    } else {
+      for (int i = threadIdx.x; i < H; i += blockDim.x) row[i] += x[i];
+    }
+    for (int i = threadIdx.x; i < H; i += blockDim.x) x[i] = row[i];
+  } else {
+    for (int i = threadIdx.x; i < H; i += blockDim.x) row[i] = x[i];
+  }
+  if (a.cat) {
+    T* c = (T*)a.cat + (size_t)m * a.ldc;
+    const float* x0 = a.x0 + (size_t)m * H;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      c[i] = (T)row[i];
+      c[H + i] = (T)x0[i];
+    }
+  }
+  if (a.xn) {
+    const float2 st = row_stats(row, H, a.eps, a.kind, red);
+    T* o = (T*)a.xn + (size_t)m * a.ldn;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      const float b = a.kind == TI_NORM_LAYER ? a.b[i] : 0.0f;
+      o[i] = (T)((row[i] - st.x) * st.y * a.w[i] + b);
+    }
+  }
+}
+
+// ------------------------------------------------------------------ expert routing
+constexpr int kMaxE = 1024, kMaxTop = 64;
+
+// One wave per row: softmax over the experts, the top scores by repeated maximum.  Lane l holds
+// experts l, l + 64, ...; a key orders by score, then by lower index.
+__device__ __forceinline__ void route_row(const ti_route_args& a, int m) {
+  constexpr int PER = kMaxE / 64;
+  const int lane = threadIdx.x & 63;
+  const float* z = a.logits + (size_t)m * a.ld;
+  float s[PER];
+  float mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = e < a.E ? z[e] : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
+  mx = wave_max_xor<64>(mx);
+  float sum = 0.0f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    s[i] = lane + 64 * i < a.E ? expf(s[i] - mx) : -1.0f;
+    sum += s[i] >= 0.0f ? s[i] : 0.0f;
+  }
+  sum = group_sum<64>(sum);
+  for (int k = 0; k < a.top; ++k) {
+    unsigned long long best = 0ull;
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (s[i] >= 0.0f) {
+        const unsigned long long key = ((unsigned long long)float_order_key(s[i]) << 32) |
+                                       (unsigned long long)(0xFFFFFFFFu - (uint32_t)(lane + 64 * i));
+        best = key > best ? key : best;
+      }
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const unsigned long long other = __shfl_xor(best, o, kWave);
+      best = other > best ? other : best;
+    }
+    // (no comparable score left, NaN logits: expert 0, never an index outside the table)
+    const int e = best ? (int)(0xFFFFFFFFu - (uint32_t)(best & 0xFFFFFFFFull)) : 0;
+    float v = 0.0f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (lane + 64 * i == e) {
+        v = s[i];
+        s[i] = -1.0f;
+      }
+    if (lane == (e & 63)) {
+      a.idx[(size_t)m * a.top + k] = e;
+      a.wgt[(size_t)m * a.top + k] = v / sum;
+    }
+  }
+}
+
+// One workgroup groups the M * top entries by expert: counts, a scan over the experts of entries and
+// tiles, then the lists.
+__device__ __forceinline__ void route_group(const ti_route_args& a) {
+  __shared__ int cnt[kMaxE], at[kMaxE], tl[kMaxE];
+  const int tid = threadIdx.x, nt = blockDim.x, n = a.M * a.top;
+  for (int e = tid; e < a.E; e += nt) cnt[e] = 0;
+  __syncthreads();
+  for (int p = tid; p < n; p += nt) atomicAdd(&cnt[a.idx[p]], 1);
+  __syncthreads();
+  if (tid < 64) {   // wave 0: exclusive scans over the experts, 64 at a time
+    int base = 0, tbase = 0;
+    for (int e0 = 0; e0 < a.E; e0 += 64) {
+      const int e = e0 + tid, c = e < a.E ? cnt[e] : 0, t = (c + a.tile_rows - 1) / a.tile_rows;
+      int ic = c, it = t;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int uc = __shfl_up(ic, o, 64), ut = __shfl_up(it, o, 64);
+        if (tid >= o) {
+          ic += uc;
+          it += ut;
+        }
+      }
+      if (e < a.E) {
+        at[e] = base + ic - c;
+        tl[e] = tbase + it - t;
+      }
+      base += __shfl(ic, 63, 64);
+      tbase += __shfl(it, 63, 64);
+    }
+    if (tid == 0) *a.n_tiles = tbase;
+  }
+  __syncthreads();
+  for (int e = tid; e < a.E; e += nt)
+    for (int i = 0, c = cnt[e]; i < c; i += a.tile_rows) {
+      int* t = a.tiles + 4 * (tl[e] + i / a.tile_rows);
+      t[0] = e;
+      t[1] = at[e] + i;
+      t[2] = min(a.tile_rows, c - i);
+      t[3] = 0;
+    }
+  __syncthreads();
+  for (int p = tid; p < n; p += nt) a.list[atomicAdd(&at[a.idx[p]], 1)] = p;
+}
+
+__global__ __launch_bounds__(256) void route_kernel(const ti_route_args a) {
+  const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (m < a.M) route_row(a, m);
+}
+__global__ __launch_bounds__(1024) void route_group_kernel(const ti_route_args a) { route_group(a); }
+// few rows: both steps in one workgroup
+__global__ __launch_bounds__(1024) void route_both_kernel(const ti_route_args a) {
+  for (int m = threadIdx.x >> 6; m < a.M; m += 16) route_row(a, m);
+  __threadfence_block();
+  __syncthreads();
+  route_group(a);
+}
+
+}  // namespace ti
+
+extern "C" int ti_rownorm(const ti_rownorm_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->x || a->M < 1 || a->H < 1 || a->H > 16128 || (a->kind != TI_NORM_LAYER && a->kind != TI_NORM_RMS) ||
+      (a->dtype != TI_DT_BF16 && a->dtype != TI_DT_F32))
+    return ti_set_error(TI_ERR_ARG, "ti_rownorm: bad arguments");
+  if ((a->y && a->parts) || ((a->y || a->parts) && a->ldy < a->H) || (a->parts && (!a->part_w || a->top < 1)) ||
+      (a->post_w && a->kind == TI_NORM_LAYER && !a->post_b) ||
+      (a->xn && (!a->w || a->ldn < a->H || (a->kind == TI_NORM_LAYER && !a->b))) ||
+      (a->cat && (!a->x0 || a->ldc < 2 * a->H)))
+    return ti_set_error(TI_ERR_ARG, "ti_rownorm: inconsistent arguments");
+  const int threads = a->H <= 1024 ? 256 : 512;
+  const size_t lds = (size_t)a->H * 4;
+  if (a->dtype == TI_DT_BF16)
+    hipLaunchKernelGGL(rownorm_kernel<bf16>, dim3(a->M), dim3(threads), lds, (hipStream_t)stream, *a);
+  else
+    hipLaunchKernelGGL(rownorm_kernel<float>, dim3(a->M), dim3(threads), lds, (hipStream_t)stream, *a);
+  TI_LAUNCH_CHECK("rownorm_kernel");
+  return TI_OK;
+}
+
+extern "C" int ti_route_max_tiles(int M, int E, int top, int tile_rows) {
+  if (M < 1 || E < 1 || top < 1 || tile_rows < 1) return 0;
+  const long n = (long)M * top;
+  // every expert with entries has at most one partly filled tile
+  return (int)(std::min<long>(E, n) + n / tile_rows);
+}
+
+extern "C" int ti_route(const ti_route_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->logits || !a->idx || !a->wgt || a->M < 1 || a->E < 1 || a->E > kMaxE || a->top < 1 || a->top > kMaxTop ||
+      a->top > a->E || a->ld < a->E)
+    return ti_set_error(TI_ERR_ARG, "ti_route: bad arguments (1 <= top <= experts <= %d, top <= %d)", kMaxE, kMaxTop);
+  if (a->tile_rows && (!a->list || !a->tiles || !a->n_tiles || a->tile_rows < 1))
+    return ti_set_error(TI_ERR_ARG, "ti_route: list / tiles");
+  hipStream_t s = (hipStream_t)stream;
+  if (a->tile_rows && a->M <= 64) {
+    hipLaunchKernelGGL(route_both_kernel, dim3(1), dim3(1024), 0, s, *a);
+  } else {
+    hipLaunchKernelGGL(route_kernel, dim3((a->M + 3) / 4), dim3(256), 0, s, *a);
+    if (a->tile_rows) hipLaunchKernelGGL(route_group_kernel, dim3(1), dim3(1024), 0, s, *a);
+  }
+  TI_LAUNCH_CHECK("route_kernel");
+  return TI_OK;
+}
