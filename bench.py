@@ -33,6 +33,14 @@ MODELS = {
     "tinyllama-1.1b": (32000, 2048, 22, 32, 4, 64, 5632, 8, 10000.0),
     "llama3-8b": (128256, 4096, 32, 32, 8, 128, 14336, 4, 500000.0),
 }
+# layer-stack models (architecture "Gegepel"): layer sizes of a real mixture-of-experts model, random weights
+STACKS = {
+    # name: (vocab, width, layers, loop (start, stop, times), mixer, experts, top, ff)
+    "gegepel-2k": (32000, 2048, 6, (2, 5, 2), dict(heads=16, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512), 64, 6, 1408),
+    "gegepel-4k": (32000, 4096, 4, (1, 3, 2), dict(heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512), 32, 4, 2816),
+    "gegepel-1k": (32000, 1024, 8, (2, 6, 2), dict(heads=8, dim=64, rot_dim=32, vdim=64, q_rank=512, kv_rank=256), 32, 4, 768),
+}
+MFMA_PEAK_TFS = 2500.0  # MI355X dense bf16 / fp16
 HBM_PEAK_GBS = 8000.0   # MI355X HBM3E spec peak (MI355X_MICROARCH.md, chip-level parameters)
 
 
@@ -165,6 +173,93 @@ def dry_run(g: "Group", args) -> int:
     return 0
 
 
+def stack_config(name: str) -> dict:
+    V, W, n, (l0, l1, t), mx, E, top, ff = STACKS[name]
+    mixer = dict(mx, rot=dict(base=10000.0, dims=mx["rot_dim"]), scale=(mx["dim"] + mx["rot_dim"]) ** -0.5)
+    layer = dict(type="latent_attention", mixer=mixer, mlp=dict(kind="moe", expert=dict(ff=ff), router=dict(experts=E, top=top)))
+    return dict(architecture="Gegepel", vocab=V, width=W, embedding=dict(scale=1.0), norm=dict(eps=1e-5), layers=[layer] * n,
+                loop=dict(start=l0, stop=l1, times=t))
+
+
+def stack_bench(args) -> int:
+    """Prefill and decode throughput of a layer-stack model (`--model gegepel-*`) beside the engine's llama
+    model at equal size: the same width, vocabulary, layer runs, heads of 128, and a dense feed-forward as
+    wide as the experts a token uses, fp16 weights (as many bytes per weight).  Both in this process, on
+    one GPU, timed in turn: decode is the replayed step graph at position kv - 1, prefill one prompt of
+    --prompt tokens to its last logits, each the best of --steps / 3 repetitions."""
+    import numpy as np
+    import turboinfer_amd as T
+    T.init(0)
+    name, L = args.model, args.kv
+    cfg = stack_config(name)
+    V, W, _, _, mx, E, top, ff = STACKS[name]
+    batches = [int(b) for b in args.stack_batches.split(",")]
+    prompts = [int(p) for p in args.stack_prompts.split(",")]
+    out = {"metric": "layer-stack decode / prefill tokens/s (one GPU) beside the llama engine at equal size", "value": None,
+           "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "vs_baseline": None, "dtype": "bf16",
+           "data": "synthetic (seeded random weights and cache)", "config": {"model": name, "kv": L}, "decode": [], "prefill": []}
+    seq = max(L, max(prompts))
+    rng = np.random.default_rng(args.seed)
+
+    def measure(e, hidden_runs):
+        dec, pre = {}, {}
+        for B in batches:
+            for s in range(B):
+                e.fill_kv(s, min(L, seq) - 1, args.seed + s)
+            e.replay_prepare(B, L, 1)
+            e.replay_run(args.warmup)
+            e.sync()
+            best = 1e9
+            for _ in range(3):
+                n = max(1, args.steps // 3)
+                t0 = time.perf_counter()
+                e.replay_run(n)
+                e.sync()
+                best = min(best, (time.perf_counter() - t0) / n)
+            dec[B] = best
+        for P in prompts:
+            t = rng.integers(0, V, P)
+            e.prefill(0, t)
+            best = 1e9
+            for _ in range(3):
+                t0 = time.perf_counter()
+                e.prefill(0, t)
+                best = min(best, time.perf_counter() - t0)
+            pre[P] = best
+        return dec, pre
+
+    e = T.Engine.stack(cfg, args.stack_dtype, max_seq=seq, max_batch=max(batches))
+    e.synth(args.seed, 0.0)
+    runs = e.cfg.layers
+    wb = e.memory()[0]
+    sd, sp = measure(e, runs)
+    e.close()
+    ld = lp = None
+    if not args.no_llama:
+        h = W // 128
+        e = T.Engine(V, W, runs, h, h, 128, top * ff, bits=16, max_seq=seq, max_batch=max(batches))
+        e.synth(args.seed, 0.0)
+        ld, lp = measure(e, runs)
+        lwb = e.memory()[0]
+        e.close()
+    for B in batches:
+        d = {"streams": B, "kv": L, "ms_per_step": round(sd[B] * 1e3, 4), "tokens_per_s": round(B / sd[B], 1)}
+        if ld:
+            d.update(llama_ms_per_step=round(ld[B] * 1e3, 4), llama_tokens_per_s=round(B / ld[B], 1))
+        out["decode"].append(d)
+    for P in prompts:
+        d = {"prompt": P, "ms": round(sp[P] * 1e3, 3), "tokens_per_s": round(P / sp[P], 1)}
+        if lp:
+            d.update(llama_ms=round(lp[P] * 1e3, 3), llama_tokens_per_s=round(P / lp[P], 1))
+        out["prefill"].append(d)
+    out["value"] = out["decode"][0]["tokens_per_s"]
+    out["ms_per_step"] = out["decode"][0]["ms_per_step"]
+    out["steps"], out["warmup"] = args.steps, args.warmup
+    out["config"].update(runs=runs, weight_bytes=wb, **({"llama_weight_bytes": lwb} if ld else {}))
+    print(json.dumps(out))
+    return 0
+
+
 def cpu_info() -> str:
     try:
         with open("/proc/cpuinfo") as f:
@@ -213,7 +308,12 @@ def main() -> int:
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--batch", type=int, default=1, help="decode streams per GPU")
     ap.add_argument("--kv", type=int, default=2048, help="KV length read per step")
-    ap.add_argument("--model", default="llama2-7b", choices=sorted(MODELS))
+    ap.add_argument("--model", default="llama2-7b", choices=sorted(MODELS) + sorted(STACKS),
+                    help="gegepel-*: the layer-stack benchmark (decode and prefill beside llama at equal size)")
+    ap.add_argument("--stack-batches", default="1,16,64", help="decode streams, layer-stack benchmark")
+    ap.add_argument("--stack-prompts", default="512,2048", help="prompt lengths, layer-stack benchmark")
+    ap.add_argument("--stack-dtype", default="bfloat16", choices=("bfloat16", "float32"))
+    ap.add_argument("--no-llama", action="store_true", help="layer-stack benchmark: without the llama side")
     ap.add_argument("--seed", type=int, default=0x7157)
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--kernel-reps", type=int, default=50)
@@ -224,6 +324,11 @@ def main() -> int:
                          "no engine; prints the JSON line with value null (tests)")
     args = ap.parse_args()
 
+    if args.model in STACKS:
+        if args.gpus != 1:
+            print("bench.py: the layer-stack benchmark runs on one GPU", file=sys.stderr)
+            return 2
+        return stack_bench(args)
     world_env = os.environ.get("WORLD_SIZE")
     if world_env is None and args.gpus > 1:
         return spawn_replicas(args.gpus, sys.argv[1:])

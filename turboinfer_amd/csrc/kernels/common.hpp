@@ -26,6 +26,14 @@ constexpr int kWave = 64;
 
 // ---------------------------------------------------------------- fp16 helpers
 __device__ __forceinline__ float h2f(uint16_t h) { return (float)__builtin_bit_cast(f16, h); }
+// fp16(fp32 product), the product rounded on its own: hipcc can fold a multiply into the conversion
+// (v_fma_mixlo_f16, one rounding less) for one use of the value and not for another, so that a value
+// and a sum over the same values disagree by an ulp
+__device__ __forceinline__ f16 mul_f16(float a, float b) {
+  float p = a * b;
+  asm("" : "+v"(p));
+  return (f16)p;
+}
 __device__ __forceinline__ uint16_t f2h(float f) { return __builtin_bit_cast(uint16_t, (f16)f); }
 
 // fp32 -> fp16 bits, round to nearest even with subnormals, in integer arithmetic: used where

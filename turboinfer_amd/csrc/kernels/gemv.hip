@@ -183,10 +183,10 @@ __device__ __forceinline__ void stage_x_generic(const GemvArgs& a, f16* xl, floa
         const float4 v0 = *(const float4*)(xr + 8 * k8), v1 = *(const float4*)(xr + 8 * k8 + 4);
         const float4 w0 = *(const float4*)(a.norm_w + 8 * k8), w1 = *(const float4*)(a.norm_w + 8 * k8 + 4);
         f16x8 h;
-        h[0] = (f16)((v0.x / rms) * w0.x); h[1] = (f16)((v0.y / rms) * w0.y);
-        h[2] = (f16)((v0.z / rms) * w0.z); h[3] = (f16)((v0.w / rms) * w0.w);
-        h[4] = (f16)((v1.x / rms) * w1.x); h[5] = (f16)((v1.y / rms) * w1.y);
-        h[6] = (f16)((v1.z / rms) * w1.z); h[7] = (f16)((v1.w / rms) * w1.w);
+        h[0] = mul_f16(v0.x / rms, w0.x); h[1] = mul_f16(v0.y / rms, w0.y);
+        h[2] = mul_f16(v0.z / rms, w0.z); h[3] = mul_f16(v0.w / rms, w0.w);
+        h[4] = mul_f16(v1.x / rms, w1.x); h[5] = mul_f16(v1.y / rms, w1.y);
+        h[6] = mul_f16(v1.z / rms, w1.z); h[7] = mul_f16(v1.w / rms, w1.w);
         *(f16x8*)(xl + m * xs + 8 * k8) = h;
       }
       __syncthreads();   // red reused by the next row
@@ -519,10 +519,10 @@ __global__ __launch_bounds__(kGemvThreads, 1) void gemv_wq_kernel(const u32x4* p
     float part = 0.0f;
     if (tid < K8) {
       f16x8 h;
-      h[0] = (f16)((v0.x / rms) * w0.x); h[1] = (f16)((v0.y / rms) * w0.y);
-      h[2] = (f16)((v0.z / rms) * w0.z); h[3] = (f16)((v0.w / rms) * w0.w);
-      h[4] = (f16)((v1.x / rms) * w1.x); h[5] = (f16)((v1.y / rms) * w1.y);
-      h[6] = (f16)((v1.z / rms) * w1.z); h[7] = (f16)((v1.w / rms) * w1.w);
+      h[0] = mul_f16(v0.x / rms, w0.x); h[1] = mul_f16(v0.y / rms, w0.y);
+      h[2] = mul_f16(v0.z / rms, w0.z); h[3] = mul_f16(v0.w / rms, w0.w);
+      h[4] = mul_f16(v1.x / rms, w1.x); h[5] = mul_f16(v1.y / rms, w1.y);
+      h[6] = mul_f16(v1.z / rms, w1.z); h[7] = mul_f16(v1.w / rms, w1.w);
       if constexpr (kRegPrep) part = int4_x_prep(h);
       *(f16x8*)(xl + 8 * tid) = h;
     }
@@ -2264,10 +2264,10 @@ __global__ __launch_bounds__(kGemvThreads) void rmsnorm_f16_kernel(const float* 
     const float4 v0 = *(const float4*)(xr + 8 * k8), v1 = *(const float4*)(xr + 8 * k8 + 4);
     const float4 w0 = *(const float4*)(w + 8 * k8), w1 = *(const float4*)(w + 8 * k8 + 4);
     f16x8 h;
-    h[0] = (f16)((v0.x / rms) * w0.x); h[1] = (f16)((v0.y / rms) * w0.y);
-    h[2] = (f16)((v0.z / rms) * w0.z); h[3] = (f16)((v0.w / rms) * w0.w);
-    h[4] = (f16)((v1.x / rms) * w1.x); h[5] = (f16)((v1.y / rms) * w1.y);
-    h[6] = (f16)((v1.z / rms) * w1.z); h[7] = (f16)((v1.w / rms) * w1.w);
+    h[0] = mul_f16(v0.x / rms, w0.x); h[1] = mul_f16(v0.y / rms, w0.y);
+    h[2] = mul_f16(v0.z / rms, w0.z); h[3] = mul_f16(v0.w / rms, w0.w);
+    h[4] = mul_f16(v1.x / rms, w1.x); h[5] = mul_f16(v1.y / rms, w1.y);
+    h[6] = mul_f16(v1.z / rms, w1.z); h[7] = mul_f16(v1.w / rms, w1.w);
     *(f16x8*)(y + (pk_kt > 0 ? TI_PACKED_INDEX(m, 8 * k8, pk_kt) : (size_t)m * ldy + 8 * k8)) = h;
   }
 }

@@ -99,7 +99,7 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
         f16x8 fx;
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          fx[j] = (f16)(v[j] * w[j]);
+          fx[j] = mul_f16(v[j], w[j]);
           ss = fmaf(v[j], v[j], ss);
         }
         *(f16x8*)(a.fold_x + (size_t)m * a.hidden + 8 * i8) = fx;

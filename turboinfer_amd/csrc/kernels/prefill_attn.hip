@@ -51,6 +51,7 @@ typedef _Float16 f16x4 __attribute__((ext_vector_type(4)));
 
 // fp32 x -> (hi, lo) fp16 with hi + lo = x to ~2^-22 relative
 __device__ __forceinline__ void pf_split(float x, _Float16& hi, _Float16& lo) {
+  asm("" : "+v"(x));   // one value for both roundings (ti::mul_f16's note)
   hi = (_Float16)x;
   lo = (_Float16)(x - (float)hi);
 }
@@ -287,8 +288,8 @@ __global__ __launch_bounds__(64, WPE) void attn_prefill_kernel(const float* __re
       uint32_t o[DV / 2];
 #pragma unroll
       for (int t = 0; t < DV / 2; ++t) {
-        const uint16_t lo = __builtin_bit_cast(uint16_t, (_Float16)(acc[2 * t][i] * inv));
-        const uint16_t hi = __builtin_bit_cast(uint16_t, (_Float16)(acc[2 * t + 1][i] * inv));
+        const uint16_t lo = __builtin_bit_cast(uint16_t, ti::mul_f16(acc[2 * t][i], inv));
+        const uint16_t hi = __builtin_bit_cast(uint16_t, ti::mul_f16(acc[2 * t + 1][i], inv));
         o[t] = lo | ((uint32_t)hi << 16);
       }
       if constexpr (HD == 128) *(ti::u32x4*)(dst + i * DV) = (ti::u32x4){o[0], o[1], o[2], o[3]};
@@ -556,8 +557,8 @@ __global__ __launch_bounds__(256 * HALVES, 1) void attn_prefill_wg_kernel(const 
       uint32_t o[DV / 2];
 #pragma unroll
       for (int t = 0; t < DV / 2; ++t) {
-        const uint16_t lo = __builtin_bit_cast(uint16_t, (_Float16)(acc[2 * t][i] * inv));
-        const uint16_t hi = __builtin_bit_cast(uint16_t, (_Float16)(acc[2 * t + 1][i] * inv));
+        const uint16_t lo = __builtin_bit_cast(uint16_t, ti::mul_f16(acc[2 * t][i], inv));
+        const uint16_t hi = __builtin_bit_cast(uint16_t, ti::mul_f16(acc[2 * t + 1][i], inv));
         o[t] = lo | ((uint32_t)hi << 16);
       }
       *(ti::u32x4*)(dst + i * DV) = (ti::u32x4){o[0], o[1], o[2], o[3]};
