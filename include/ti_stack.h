@@ -74,13 +74,20 @@ typedef struct ti_dense_args {
   int32_t* step_ctr;           /* TI_DE_LOGITS, nullable: += advance once                    */
   int32_t advance;
   /* grouped products (experts): tile t covers entries [first, first + rows) of expert e's list */
-  int32_t tile_rows;           /* 0 = not grouped; 16 or 64: rows a tile holds at most       */
+  int32_t tile_rows;           /* 0 = not grouped; 16 or 64: rows a tile holds at most; 1: tile t is
+                                  entry t alone, expert tiles[t] (or the routed one, below)   */
   int32_t max_tiles;           /* tiles launched; those at or past *n_tiles return at once   */
   const int32_t* tiles;        /* device [max_tiles][4] = expert, first, rows, -             */
   const int32_t* n_tiles;      /* device                                                     */
-  const int32_t* rows_in;      /* nullable: entry p reads activation row rows_in[p] / row_div */
+  const int32_t* rows_in;      /* entry p reads activation row (rows_in ? rows_in[p] : p) / row_div */
   const int32_t* rows_out;     /* nullable: entry p writes output row rows_out[p]            */
   int32_t row_div;
+  /* tile_rows 1: entry t = (row t / top, choice t % top) routed here from fp32 logits [.][route_e],
+   * route_e <= 64 (ti_route's choice), recorded in route_idx / route_wgt [max_tiles] */
+  int32_t route_e, top;
+  const float* route_logits;
+  int32_t* route_idx;
+  float* route_wgt;
 } ti_dense_args;
 int ti_dense(const ti_dense_args* a, ti_stream_t s);
 size_t ti_dense_args_bytes(void);
@@ -161,8 +168,9 @@ int ti_latent_prepare(void);
  * [0, pos[m]], softmax whose denominator also holds exp(sink[h]), out = weights . latents.
  * qa T [M][heads][lat_p] (the query carried through the key up-projection), qr T rows of `ldqr`
  * elements per (m, head) with the rotated part at qr_off.  out T [M][heads][lat_p].
- * splits > 1: part_o T [M][splits][heads][lat_p] and part_ml fp32 [M][splits][heads][2] are merged
- * into out by a second launch. */
+ * splits > 1 (at most 64): part_o T [M][splits][heads][lat_p] and part_ml fp32 [M][splits][heads][2]
+ * hold each split's normalised row and (max, sum); out non-NULL: a second launch merges them, NULL: left
+ * to ti_latent_attn_out. */
 typedef struct ti_latent_attn_args {
   const void* qa;
   const void* q;               /* T [M][heads][ldqr]; rotated part at qr_off                 */
@@ -178,6 +186,19 @@ typedef struct ti_latent_attn_args {
   int32_t M, heads, lat_p, rot_p, splits, seq_p, dtype;
 } ti_latent_attn_args;
 int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t s);
+/* Merge of the splits, value up-projection and head gate: out T [M][ldo], head h's vdim values at
+ * h * vdim.  w: fragment-ordered, w_batch elements per head ([vdim][lat_p]). */
+typedef struct ti_latent_out_args {
+  const void* part_o;
+  const float* part_ml;
+  const float* sink;
+  const void* w;
+  int64_t w_batch;
+  const float* gate;           /* [M][heads]                                                 */
+  void* out;
+  int32_t ldo, M, heads, lat_p, vdim, splits, dtype;
+} ti_latent_out_args;
+int ti_latent_attn_out(const ti_latent_out_args* a, ti_stream_t s);
 int ti_latent_attn_splits(int M, int heads, int max_seq);
 
 /* Prompt-chunk attention over keys and values expanded per head (TI_DE_KFRAG / TI_DE_VFRAG), rows

@@ -94,7 +94,8 @@ class DenseArgs(C.Structure):
          ("gate", C.c_void_p), ("gate_ld", C.c_int32), ("key_blocks", C.c_int32), ("argmax", C.c_void_p),
          ("step_ctr", C.c_void_p), ("advance", C.c_int32), ("tile_rows", C.c_int32), ("max_tiles", C.c_int32),
          ("tiles", C.c_void_p), ("n_tiles", C.c_void_p), ("rows_in", C.c_void_p), ("rows_out", C.c_void_p),
-         ("row_div", C.c_int32)]
+         ("row_div", C.c_int32), ("route_e", C.c_int32), ("top", C.c_int32), ("route_logits", C.c_void_p),
+         ("route_idx", C.c_void_p), ("route_wgt", C.c_void_p)]
 
 
 class RownormArgs(C.Structure):
@@ -135,7 +136,7 @@ EXPORTED = [
     "ti_engine_create_stack", "ti_engine_weight_count", "ti_engine_weight_info", "ti_engine_set_weight", "ti_engine_load",
     "ti_engine_describe", "ti_engine_prefill", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
     "ti_stack_convert", "ti_stack_fill", "ti_dense", "ti_dense_args_bytes", "ti_rownorm", "ti_route", "ti_route_max_tiles",
-    "ti_latent_prep", "ti_latent_prepare", "ti_latent_attn_decode", "ti_latent_attn_splits", "ti_latent_attn_prefill",
+    "ti_latent_prep", "ti_latent_prepare", "ti_latent_attn_decode", "ti_latent_attn_splits", "ti_latent_attn_prefill", "ti_latent_attn_out",
 ]
 
 _lib = None

@@ -86,6 +86,8 @@ int StackModel::check(const ti_stack_config& c, const ti_stack_layer* l) {
     const int lim = c.dtype == TI_DT_BF16 ? 2048 : 1024;
     if (L.vdim > 256 || ti_stack_kpad(c.dtype, L.kv_rank) > lim)
       return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: vdim %d (at most 256), kv_rank %d (at most %d)", i, L.vdim, L.kv_rank, lim);
+    if (L.q_rank + L.kv_rank + L.rot_dim + L.heads > 15996)
+      return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: q_rank + kv_rank + rot_dim + heads > 15996", i);
     if (L.mlp != TI_MLP_NONE && L.mlp != TI_MLP_MOE) return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: feed-forward %d", i, L.mlp);
     if (L.mlp == TI_MLP_MOE && (L.experts < 1 || L.experts > 1024 || L.top < 1 || L.top > L.experts || L.top > 64 || L.ff < 1))
       return ti_set_error(TI_ERR_ARG, "layer %d: %d experts, top %d, ff %d", i, L.experts, L.top, L.ff);
@@ -526,20 +528,41 @@ int StackModel::attention(const StackLayer& L, const StackRun& run, const StackR
     f.splits = ti_latent_attn_splits(M, k.heads, c.max_seq);
     f.seq_p = seq_p;
     f.dtype = c.dtype;
-    TI_TRY(ti_latent_attn_decode(&f, s_));
-    ti_dense_args dv{};
-    dv.batch = k.heads;
-    dv.N = k.vdim;
-    dv.w_batch = (int64_t)L.vdim_p * L.uv.kp;
-    dv.a_batch = L.lat_p;
-    dv.gate = gate_;
-    dv.gate_ld = k.heads;
-    TI_TRY(dense(L.uv, olat_, k.heads * L.lat_p, M, attn_, ldat, TI_DE_GATE, dv));
+    if (f.splits > 1) {
+      f.out = nullptr;
+      TI_TRY(ti_latent_attn_decode(&f, s_));
+      ti_latent_out_args u{};
+      u.part_o = part_o_;
+      u.part_ml = part_ml_;
+      u.sink = L.sink;
+      u.w = L.uv.p;
+      u.w_batch = (int64_t)L.vdim_p * L.uv.kp;
+      u.gate = gate_;
+      u.out = attn_;
+      u.ldo = ldat;
+      u.M = M;
+      u.heads = k.heads;
+      u.lat_p = L.lat_p;
+      u.vdim = k.vdim;
+      u.splits = f.splits;
+      u.dtype = c.dtype;
+      TI_TRY(ti_latent_attn_out(&u, s_));
+    } else {
+      TI_TRY(ti_latent_attn_decode(&f, s_));
+      ti_dense_args dv{};
+      dv.batch = k.heads;
+      dv.N = k.vdim;
+      dv.w_batch = (int64_t)L.vdim_p * L.uv.kp;
+      dv.a_batch = L.lat_p;
+      dv.gate = gate_;
+      dv.gate_ld = k.heads;
+      TI_TRY(dense(L.uv, olat_, k.heads * L.lat_p, M, attn_, ldat, TI_DE_GATE, dv));
+    }
   }
   return dense(L.o, attn_, ldat, M, y_, c.width, TI_DE_F32, {});
 }
 
-int StackModel::experts(const StackLayer& L, int M, bool /*direct*/) {
+int StackModel::experts(const StackLayer& L, int M) {
   const ti_stack_layer& k = L.c;
   const int W = c.width, ldx = kpad(W), ldact = kpad(k.ff);
   TI_TRY(dense(L.router, xn_, ldx, M, zr_, k.experts, TI_DE_F32, {}));
@@ -554,19 +577,39 @@ int StackModel::experts(const StackLayer& L, int M, bool /*direct*/) {
   ra.list = list_;
   ra.tiles = tiles_;
   ra.n_tiles = n_tiles_;
-  ra.tile_rows = M <= 64 ? 16 : 64;
-  TI_TRY(ti_route(&ra, s_));
   ti_dense_args g{};
-  g.tile_rows = ra.tile_rows;
-  g.max_tiles = ti_route_max_tiles(M, k.experts, k.top, ra.tile_rows);
-  g.tiles = tiles_;
-  g.n_tiles = n_tiles_;
-  g.rows_in = list_;
-  g.row_div = k.top;
   g.w_batch = (int64_t)up(2 * k.ff, 16) * L.gu.kp;
+  g.row_div = k.top;
+  // few rows: every (row, choice) entry is a tile of its own (an expert two rows share is read twice);
+  // with at most 64 experts the gate / up launch also does the routing
+  const bool direct = M == 1 || (long)M * k.top * 2 <= k.experts;
+  if (direct) {
+    g.tile_rows = 1;
+    g.max_tiles = M * k.top;
+    g.tiles = idx_;
+    if (k.experts <= 64) {
+      g.route_logits = zr_;
+      g.route_e = k.experts;
+      g.top = k.top;
+      g.route_idx = idx_;
+      g.route_wgt = wgt_;
+    } else {
+      TI_TRY(ti_route(&ra, s_));
+    }
+  } else {
+    ra.tile_rows = M <= 64 ? 16 : 64;
+    TI_TRY(ti_route(&ra, s_));
+    g.tile_rows = ra.tile_rows;
+    g.max_tiles = ti_route_max_tiles(M, k.experts, k.top, ra.tile_rows);
+    g.tiles = tiles_;
+    g.n_tiles = n_tiles_;
+    g.rows_in = list_;
+  }
   TI_TRY(dense(L.gu, xn_, ldx, M, act_, ldact, TI_DE_SWIGLU, g));
   g.rows_in = nullptr;
-  g.rows_out = list_;
+  g.row_div = 1;
+  g.route_logits = nullptr;
+  if (!direct) g.rows_out = list_;
   g.w_batch = (int64_t)up(W, 16) * L.down.kp;
   return dense(L.down, act_, ldact, M, parts_, W, TI_DE_T, g);
 }
@@ -628,7 +671,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
     parts = false;
     if (L.c.mlp == TI_MLP_MOE) {
       TI_TRY(rownorm(L.n2, nullptr));
-      TI_TRY(experts(L, M, false));
+      TI_TRY(experts(L, M));
       post = L.n2b;
       parts = true;
       top = L.c.top;

@@ -123,22 +123,43 @@ struct DenseSpan {   // what a workgroup works on
 };
 
 __device__ __forceinline__ bool dense_span(const ti_dense_args& a, int y, DenseSpan& s, size_t esize) {
-  if (a.tile_rows) {
+  s.batch = 0;
+  int e = 0;
+  if (a.tile_rows == 1) {
+    s.first = y;
+    s.rows = 1;
+    if (a.route_logits) {   // every wave finds the row's k-th expert itself; one workgroup records it
+      const int m = y / a.top, k = y - m * a.top;
+      float score;
+      route_top64(a.route_logits + (size_t)m * a.route_e, a.route_e, k + 1, score, [&](int i, int x) {
+        e = x;
+        return i < k;
+      });
+      if (blockIdx.x == 0 && (int)threadIdx.x == e) {
+        a.route_idx[y] = e;
+        a.route_wgt[y] = score;
+      }
+    } else {
+      e = a.tiles[y];
+    }
+    e = __builtin_amdgcn_readfirstlane(e);
+  } else if (a.tile_rows) {
     if (y >= *a.n_tiles) return false;
-    const int e = a.tiles[4 * y];
+    e = a.tiles[4 * y];
     s.first = a.tiles[4 * y + 1];
     s.rows = a.tiles[4 * y + 2];
-    s.batch = 0;
-    s.w = (const char*)a.w + (size_t)e * a.w_batch * esize;
   } else {
     s.first = 0;
     s.rows = a.M;
-    s.batch = y;
-    s.w = (const char*)a.w + (size_t)y * a.w_batch * esize;
+    s.batch = e = y;
   }
+  s.w = (const char*)a.w + (size_t)e * a.w_batch * esize;
   return true;
 }
-__device__ __forceinline__ int row_in(const ti_dense_args& a, int p) { return a.rows_in ? a.rows_in[p] / a.row_div : p; }
+__device__ __forceinline__ int row_in(const ti_dense_args& a, int p) {
+  const int r = a.rows_in ? a.rows_in[p] : p;
+  return a.row_div > 1 ? r / a.row_div : r;
+}
 __device__ __forceinline__ int row_out(const ti_dense_args& a, int p) { return a.rows_out ? a.rows_out[p] : p; }
 
 template <class T, int MT, int W>
@@ -148,36 +169,43 @@ __global__ __launch_bounds__(64 * W) void dense_skinny_kernel(const ti_dense_arg
   __shared__ f32x4 red[W][MT][64];
   DenseSpan sp;
   if (!dense_span(a, blockIdx.y, sp, sizeof(T))) return;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nt = blockIdx.x, nk = a.K / KT;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nt = blockIdx.x, nk = a.K / KT, z0 = blockIdx.z * MT * 16;
   const V* wp = (const V*)sp.w + (size_t)nt * nk * 64 + lane;
   const V* ap[MT];
 #pragma unroll
   for (int mt = 0; mt < MT; ++mt) {
-    const int p = sp.first + min(mt * 16 + (lane & 15), sp.rows - 1);
+    const int p = sp.first + min(z0 + mt * 16 + (lane & 15), sp.rows - 1);
     ap[mt] = (const V*)((const T*)a.a + (size_t)sp.batch * a.a_batch + (size_t)row_in(a, p) * a.lda) + (lane >> 4);
   }
   f32x4 acc[MT];
 #pragma unroll
   for (int mt = 0; mt < MT; ++mt) acc[mt] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  int kt = wave;
-  for (; kt + (U - 1) * W < nk; kt += U * W) {
-    V wf[U];
+  // n k-tiles of this wave: their weight fragments in flight together (kept to ~64 VGPRs: workgroups
+  // per CU hide more latency than a deeper wave)
+  auto batch = [&]<int N>(int kt) {
+    V wf[N];
 #pragma unroll
-    for (int u = 0; u < U; ++u) wf[u] = wp[(size_t)(kt + u * W) * 64];
+    for (int u = 0; u < N; ++u) wf[u] = wp[(size_t)(kt + u * W) * 64];
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt) {
-      V af[U];
+      V af[N];
 #pragma unroll
-      for (int u = 0; u < U; ++u) af[u] = ap[mt][(kt + u * W) * (KT / VEC)];
+      for (int u = 0; u < N; ++u) af[u] = ap[mt][(kt + u * W) * (KT / VEC)];
 #pragma unroll
-      for (int u = 0; u < U; ++u) acc[mt] = mma(wf[u], af[u], acc[mt]);
+      for (int u = 0; u < N; ++u) acc[mt] = mma(wf[u], af[u], acc[mt]);
     }
+  };
+  int kt = wave;
+  for (; kt + (U - 1) * W < nk; kt += U * W) batch.template operator()<U>(kt);
+  if (kt + 3 * W < nk) {
+    batch.template operator()<4>(kt);
+    kt += 4 * W;
   }
-  for (; kt < nk; kt += W) {
-    const V wf = wp[(size_t)kt * 64];
-#pragma unroll
-    for (int mt = 0; mt < MT; ++mt) acc[mt] = mma(wf, ap[mt][kt * (KT / VEC)], acc[mt]);
+  if (kt + W < nk) {
+    batch.template operator()<2>(kt);
+    kt += 2 * W;
   }
+  if (kt < nk) batch.template operator()<1>(kt);
 #pragma unroll
   for (int mt = 0; mt < MT; ++mt) red[wave][mt][lane] = acc[mt];
   __syncthreads();
@@ -185,13 +213,13 @@ __global__ __launch_bounds__(64 * W) void dense_skinny_kernel(const ti_dense_arg
     f32x4 v = red[0][mt][lane];
 #pragma unroll
     for (int w = 1; w < W; ++w) v += red[w][mt][lane];
-    const int m = mt * 16 + (lane & 15), n0 = nt * 16 + 4 * (lane >> 4);
+    const int m = z0 + mt * 16 + (lane & 15), n0 = nt * 16 + 4 * (lane >> 4);
     if (a.epi == TI_DE_LOGITS)
       dense_argmax(a, m, sp.rows, n0, v, lane, nt);
     else
       dense_store<T>(a, sp.batch, m, m < sp.rows ? row_out(a, sp.first + m) : 0, sp.rows, n0, v);
   }
-  if (a.epi == TI_DE_LOGITS && a.step_ctr && nt == 0 && tid == 0) *a.step_ctr += a.advance;
+  if (a.epi == TI_DE_LOGITS && a.step_ctr && nt == 0 && blockIdx.z == 0 && tid == 0) *a.step_ctr += a.advance;
 }
 
 template <class T, int BM, int BN, bool VF>
@@ -288,10 +316,11 @@ __global__ __launch_bounds__(256) void dense_tile_kernel(const ti_dense_args a, 
 template <class T, int MT>
 int launch_skinny(const ti_dense_args& a, hipStream_t s) {
   const int NT = (a.N + 15) / 16, y = a.tile_rows ? a.max_tiles : a.batch, nk = a.K / El<T>::KT;
+  const int z = a.tile_rows ? 1 : (a.M + 16 * MT - 1) / (16 * MT);
   if (nk >= 32)
-    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 8>), dim3(NT, y), dim3(512), 0, s, a);
+    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 8>), dim3(NT, y, z), dim3(512), 0, s, a);
   else
-    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 4>), dim3(NT, y), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 4>), dim3(NT, y, z), dim3(256), 0, s, a);
   TI_LAUNCH_CHECK("dense_skinny_kernel");
   return TI_OK;
 }
@@ -309,11 +338,16 @@ template <class T>
 int dispatch_dense(const ti_dense_args& a, hipStream_t s) {
   if (a.epi == TI_DE_VFRAG) return launch_tile<T, 128, 64, true>(a, s);
   if (a.epi == TI_DE_KFRAG) return launch_tile<T, 128, 64, false>(a, s);
-  if (a.tile_rows == 16) return launch_skinny<T, 1>(a, s);
+  if (a.tile_rows == 1 || a.tile_rows == 16) return launch_skinny<T, 1>(a, s);
   if (a.tile_rows == 64) return launch_tile<T, 64, 64, false>(a, s);
-  if (a.M <= 16) return launch_skinny<T, 1>(a, s);
-  if (a.M <= 32) return launch_skinny<T, 2>(a, s);
-  if (a.M <= 64) return launch_skinny<T, 4>(a, s);
+  // up to 64 rows: as many row tiles per workgroup as still leave two workgroups per CU
+  if (a.M <= 64) {
+    const long g = (long)((a.N + 15) / 16) * a.batch;
+    const int mt = (a.M + 15) / 16;
+    if (mt == 1 || g < 256) return launch_skinny<T, 1>(a, s);
+    if (mt == 2 || g < 512) return launch_skinny<T, 2>(a, s);
+    return launch_skinny<T, 4>(a, s);
+  }
   // the largest tile that still gives every CU a workgroup
   auto wgs = [&](int bm, int bn) { return (long)((a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn) * a.batch; };
   if (wgs(128, 128) >= 256) return launch_tile<T, 128, 128, false>(a, s);
@@ -397,9 +431,13 @@ extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
     return ti_set_error(TI_ERR_ARG, "ti_dense: K %d / lda %d not padded", a->K, a->lda);
   if ((!a->tile_rows && !a->rows_in && a->lda < a->K) || a->batch > 65535)
     return ti_set_error(TI_ERR_ARG, "ti_dense: lda %d < K %d or batch %d", a->lda, a->K, a->batch);
-  if (a->tile_rows && ((a->tile_rows != 16 && a->tile_rows != 64) || !a->tiles || !a->n_tiles || a->max_tiles < 1 ||
-                       a->max_tiles > 65535 || a->batch != 1 || a->epi > TI_DE_SWIGLU || (a->rows_in && a->row_div < 1)))
+  if (a->tile_rows && ((a->tile_rows != 1 && a->tile_rows != 16 && a->tile_rows != 64) || a->max_tiles < 1 || a->max_tiles > 65535 ||
+                       a->batch != 1 || a->epi > TI_DE_SWIGLU || (a->rows_in && a->row_div < 1) ||
+                       (a->tile_rows == 1 ? (!a->tiles && !a->route_logits) || a->rows_in || a->rows_out
+                                          : !a->tiles || !a->n_tiles || a->route_logits)))
     return ti_set_error(TI_ERR_ARG, "ti_dense: grouped arguments");
+  if (a->route_logits && (!a->route_idx || !a->route_wgt || a->route_e < 1 || a->route_e > 64 || a->top < 1 || a->top > a->route_e))
+    return ti_set_error(TI_ERR_ARG, "ti_dense: routing arguments");
   if (!a->tile_rows && (a->rows_in || a->rows_out)) return ti_set_error(TI_ERR_ARG, "ti_dense: row lists need grouped tiles");
   switch (a->epi) {
     case TI_DE_F32: case TI_DE_T: break;

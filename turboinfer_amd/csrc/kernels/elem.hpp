@@ -62,6 +62,33 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return s;
 }
 
+// All-reduce maximum over the wave (group_sum's lane exchanges).
+__device__ __forceinline__ float wave_max(float v) {
+  v = fmaxf(v, lane_xor<1>(v));
+  v = fmaxf(v, lane_xor<2>(v));
+  v = fmaxf(v, dpp_f<0x141>(v));
+  v = fmaxf(v, dpp_f<0x140>(v));
+  return xor32_max(xor16_max(v));
+}
+
+// Routing of one row over E <= 64 experts by one wave: the lane's softmax score (lane = expert), and
+// take(score) in turn for the best, second best, ... (lowest index first among equals) of `top`
+// choices; take returns false to stop.  NaN logits: expert 0.
+template <class F>
+__device__ __forceinline__ void route_top64(const float* z, int E, int top, float& score, F take) {
+  const int lane = threadIdx.x & 63;
+  const float v = lane < E ? z[lane] : -INFINITY;
+  const float mx = wave_max(v);
+  float p = lane < E ? expf(v - mx) : -1.0f;
+  score = p / group_sum<64>(lane < E ? p : 0.0f);
+  for (int k = 0; k < top; ++k) {
+    const unsigned long long best = __ballot(p == wave_max(p) && p >= 0.0f);
+    const int e = best ? __builtin_ctzll(best) : 0;
+    if (!take(k, e)) return;
+    if (lane == e) p = -1.0f;
+  }
+}
+
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 }  // namespace ti

@@ -18,20 +18,23 @@
 namespace ti {
 
 template <class T>
-__global__ __launch_bounds__(256) void latent_prep_kernel(const ti_latent_prep_args a) {
-  __shared__ float red[4];
-  const int m = blockIdx.x, tid = threadIdx.x, pos = a.pos[m];
-  const float* r = a.a32 + (size_t)m * a.lda;
+__global__ __launch_bounds__(512) void latent_prep_kernel(const ti_latent_prep_args a) {
+  extern __shared__ float r[];   // the fused projection's row
+  __shared__ float red[8];
+  const int m = blockIdx.x, tid = threadIdx.x, pos = a.pos[m], n4 = (a.gate_off + a.heads + 3) >> 2;
+  const f32x4* src = (const f32x4*)(a.a32 + (size_t)m * a.lda);
+  for (int i = tid; i < n4; i += 512) ((f32x4*)r)[i] = src[i];
+  __syncthreads();
   float q2 = 0.0f, c2 = 0.0f;
-  for (int i = tid; i < a.q_rank; i += 256) q2 = fmaf(r[i], r[i], q2);
-  for (int i = tid; i < a.kv_rank; i += 256) c2 = fmaf(r[a.lat_off + i], r[a.lat_off + i], c2);
+  for (int i = tid; i < a.q_rank; i += 512) q2 = fmaf(r[i], r[i], q2);
+  for (int i = tid; i < a.kv_rank; i += 512) c2 = fmaf(r[a.lat_off + i], r[a.lat_off + i], c2);
   const float qi = 1.0f / sqrtf(block_sum(q2, red) / (float)a.q_rank + a.eps);
   const float ci = 1.0f / sqrtf(block_sum(c2, red) / (float)a.kv_rank + a.eps);
   T* cq = (T*)a.cq + (size_t)m * a.ldq;
-  for (int i = tid; i < a.q_rank; i += 256) cq[i] = (T)(r[i] * qi * a.q_w[i]);
+  for (int i = tid; i < a.q_rank; i += 512) cq[i] = (T)(r[i] * qi * a.q_w[i]);
   T* row = (T*)a.cache + (size_t)m * a.slot_stride + (size_t)pos * (a.lat_p + a.rot_p);
-  for (int i = tid; i < a.lat_p; i += 256) row[i] = i < a.kv_rank ? (T)(r[a.lat_off + i] * ci * a.c_w[i]) : (T)0.0f;
-  for (int i = tid; i < a.rot_p / 2; i += 256) {
+  for (int i = tid; i < a.lat_p; i += 512) row[i] = i < a.kv_rank ? (T)(r[a.lat_off + i] * ci * a.c_w[i]) : (T)0.0f;
+  for (int i = tid; i < a.rot_p / 2; i += 512) {
     float u = 0.0f, v = 0.0f;
     if (2 * i < a.rot_dim) u = r[a.rot_off + 2 * i];
     if (2 * i + 1 < a.rot_dim) v = r[a.rot_off + 2 * i + 1];
@@ -39,7 +42,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const ti_latent_prep_a
     row[a.lat_p + 2 * i] = (T)(u * cs.x - v * cs.y);
     row[a.lat_p + 2 * i + 1] = (T)(v * cs.x + u * cs.y);
   }
-  for (int i = tid; i < a.heads; i += 256) a.gate[(size_t)m * a.heads + i] = sigmoidf(r[a.gate_off + i]);
+  for (int i = tid; i < a.heads; i += 512) a.gate[(size_t)m * a.heads + i] = sigmoidf(r[a.gate_off + i]);
 }
 
 // The VEC x VEC transpose a value fragment needs: in[j] = VEC consecutive value dims of key j of this
@@ -65,12 +68,14 @@ __device__ __forceinline__ void mma_values(f32x4* acc, const f32x4* vin, f32x4 p
     for (int c = 0; c < 4; ++c) acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(vin[s][c], p[s], acc[c], 0, 0, 0);
 }
 
-// Grid (splits, head tiles of 16, rows).  A block is 4 * KPW keys: wave w scores keys [w * KPW, +KPW),
-// then sums value dims of its groups (wave, wave + 4, ...; a group is 16 * VEC dims) over all of them.
-template <class T, int KPW, int GPW>
-__global__ __launch_bounds__(256) void latent_decode_kernel(const ti_latent_attn_args a) {
+// Grid (splits, head tiles of 16, rows).  A block is 64 keys: wave w scores keys [16 w, +16), then sums
+// value dims of its groups (wave, wave + 4, ...; a group is 16 * VEC dims) over all 64.  A wave's key
+// fragments of a block (NKU k-tiles at a time) and, with one group per wave, its value rows -- the same
+// cache lines -- are all in flight before the first product.
+template <class T, int GPW>
+__global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_attn_args a) {
   typedef typename El<T>::V V;
-  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, KB = 4 * KPW, PLD = KB + 16 / (int)sizeof(T);
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, KB = 64, NVB = KB / KT, PLD = KB + 16 / (int)sizeof(T), NKU = 18;
   extern __shared__ char lds[];
   const int split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
@@ -96,25 +101,32 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const ti_latent_attn
   const int nb = (pos + KB) / KB, bps = (nb + a.splits - 1) / a.splits, b0 = split * bps, b1 = min(nb, b0 + bps);
   __syncthreads();
   for (int b = b0; b < b1; ++b) {
-    const int k0 = b * KB + wave * KPW;
-    f32x4 s[KPW / 16];
-#pragma unroll
-    for (int t = 0; t < KPW / 16; ++t) s[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const int k0 = b * KB + wave * 16;
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
     const V* kp = (const V*)(cache + (size_t)(k0 + col) * cw) + g;
-#pragma unroll 6
-    for (int kt = 0; kt < nkt; ++kt) {
-      const V q = qf[kt * 64 + lane];
+    const T* vp = cache + (size_t)(b * KB + g * VEC) * cw;
+    V vin[GPW == 1 ? NVB : 1][VEC];
+    for (int kt0 = 0; kt0 < nkt; kt0 += NKU) {
+      V k[NKU];
 #pragma unroll
-      for (int t = 0; t < KPW / 16; ++t) s[t] = mma(kp[(size_t)t * 16 * cw / VEC + kt * 4], q, s[t]);
+      for (int u = 0; u < NKU; ++u) k[u] = kp[min(kt0 + u, nkt - 1) * 4];
+      if (GPW == 1 && kt0 == 0) {   // (dims past the latent: clamped, not stored)
+        const T* vd = vp + min(wave * 16 * VEC + col * VEC, a.lat_p - VEC);
+#pragma unroll
+        for (int kb = 0; kb < NVB; ++kb)
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) vin[kb][j] = *(const V*)(vd + (size_t)(kb * KT + j) * cw);
+      }
+#pragma unroll
+      for (int u = 0; u < NKU; ++u)
+        if (kt0 + u < nkt) s = mma(k[u], qf[(kt0 + u) * 64 + lane], s);
     }
     float mx = -INFINITY;
 #pragma unroll
-    for (int t = 0; t < KPW / 16; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        s[t][r] = k0 + t * 16 + 4 * g + r <= pos ? s[t][r] * a.scale : -INFINITY;
-        mx = fmaxf(mx, s[t][r]);
-      }
+    for (int r = 0; r < 4; ++r) {
+      s[r] = k0 + 4 * g + r <= pos ? s[r] * a.scale : -INFINITY;
+      mx = fmaxf(mx, s[r]);
+    }
     mx = xor32_max(xor16_max(mx));
     if (lane < 16) sm[wave * 16 + col] = mx;
     __syncthreads();
@@ -122,16 +134,13 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const ti_latent_attn
     const float alpha = expf(mr - mn);   // (every block holds a visible key: mn is finite)
     mr = mn;
     lr *= alpha;
+    f32x4 p;
 #pragma unroll
-    for (int t = 0; t < KPW / 16; ++t) {
-      f32x4 p;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        p[r] = expf(s[t][r] - mn);
-        lr += p[r];
-      }
-      *(typename El<T>::Q*)(pb + col * PLD + wave * KPW + t * 16 + 4 * g) = quad<T>(p);
+    for (int r = 0; r < 4; ++r) {
+      p[r] = expf(s[r] - mn);
+      lr += p[r];
     }
+    *(typename El<T>::Q*)(pb + col * PLD + wave * 16 + 4 * g) = quad<T>(p);
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < GPW; ++i) {
@@ -139,14 +148,18 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const ti_latent_attn
       if (gi >= G) continue;
 #pragma unroll
       for (int c = 0; c < VEC; ++c) o[i][c] *= alpha;
-      const int d = gi * 16 * VEC + col * VEC, dc = min(d, a.lat_p - VEC);   // (dims past the latent: not stored)
-#pragma unroll 2
-      for (int kb = 0; kb < KB / KT; ++kb) {
-        const V p = *(const V*)(pb + col * PLD + kb * KT + g * VEC);
-        V vin[VEC];
+      const T* vd = vp + min(gi * 16 * VEC + col * VEC, a.lat_p - VEC);
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) vin[j] = *(const V*)(cache + (size_t)(b * KB + kb * KT + g * VEC + j) * cw + dc);
-        mma_values(o[i], vin, p);
+      for (int kb = 0; kb < NVB; ++kb) {
+        const V p = *(const V*)(pb + col * PLD + kb * KT + g * VEC);
+        if constexpr (GPW == 1) {
+          mma_values(o[i], vin[kb], p);
+        } else {
+          V v[VEC];
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) v[j] = *(const V*)(vd + (size_t)(kb * KT + j) * cw);
+          mma_values(o[i], v, p);
+        }
       }
     }
   }
@@ -182,6 +195,98 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const ti_latent_attn
       for (int c = 0; c < VEC; ++c) v[c] = (T)(o[i][c][r] * inv);
       *(V*)(out + d) = v;
     }
+  }
+}
+
+// The splits' rows merged and carried through the value up-projection in one launch: grid (pairs of 16
+// value dims, heads, tiles of 16 rows).  The merged rows go to LDS in operand fragments: a thread sums
+// one 16-byte piece over a share of the splits (groups of threads share a piece when there are few),
+// then the waves split k.
+constexpr int kMaxSplits = 64;
+template <class T>
+__global__ __launch_bounds__(256) void latent_out_kernel(const ti_latent_out_args a) {
+  typedef typename El<T>::V V;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC;
+  extern __shared__ char lds[];
+  __shared__ float wt[16][kMaxSplits];
+  __shared__ f32x4 red[4][2][64];
+  const int h = blockIdx.y, m0 = blockIdx.z * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int rows = min(16, a.M - m0), S = a.splits, nk = a.lat_p / KT, NT = (a.vdim + 15) >> 4, nt0 = blockIdx.x * 2;
+  const int C = a.lat_p / VEC;   // pieces per row
+  V* xf = (V*)lds;               // [nk][64]
+  float* part = (float*)(lds + (size_t)nk * 1024);   // [256][VEC] partial pieces
+  const V* w0 = (const V*)a.w + ((size_t)h * (a.w_batch / VEC)) + (size_t)nt0 * nk * 64 + lane;
+  const V* w1 = nt0 + 1 < NT ? w0 + (size_t)nk * 64 : w0;
+  for (int m = wave; m < rows; m += 4) {
+    float mx = -INFINITY, l = 0.0f;
+    if (lane < S) {
+      const float2 ml = *(const float2*)(a.part_ml + (((size_t)(m0 + m) * S + lane) * a.heads + h) * 2);
+      mx = ml.x;
+      l = ml.y;
+    }
+    const float sink = a.sink[h], mm = fmaxf(wave_max(mx), sink), e = l > 0.0f ? l * expf(mx - mm) : 0.0f;
+    wt[m][lane] = e / (group_sum<64>(e) + expf(sink - mm));
+  }
+  __syncthreads();
+  const size_t sstride = (size_t)a.heads * a.lat_p;
+  // pieces in batches of 256 / SG threads' worth, SG threads per piece
+  int SG = 1;
+  while (SG < 8 && rows * C * SG * 2 <= 256 && SG * 2 <= S) SG *= 2;
+  const int per = 256 / SG, ss = (S + SG - 1) / SG, sg = tid / per;
+  for (int p0 = 0; p0 < rows * C; p0 += per) {
+    const int p = p0 + tid % per;
+    const bool live = p < rows * C;
+    const int m = live ? p / C : 0, c = live ? p - m * C : 0;
+    const T* po = (const T*)a.part_o + ((size_t)(m0 + m) * S * a.heads + h) * a.lat_p + c * VEC;
+    float x[VEC] = {};
+    const int s1 = min(S, (sg + 1) * ss);
+    for (int s0 = sg * ss; s0 < s1; s0 += 8) {
+      V v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v[u] = *(const V*)(po + (size_t)min(s0 + u, S - 1) * sstride);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const float f = s0 + u < s1 ? wt[m][s0 + u] : 0.0f;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) x[e] = f != 0.0f ? fmaf(f, (float)v[u][e], x[e]) : x[e];   // (empty split: no row)
+      }
+    }
+    if (SG > 1) {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) part[tid * VEC + e] = x[e];
+      __syncthreads();
+      if (sg == 0)
+        for (int g = 1; g < SG; ++g)
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) x[e] += part[(g * per + tid) * VEC + e];
+    }
+    if (live && sg == 0) {
+      V o;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o[e] = (T)x[e];
+      xf[(c >> 2) * 64 + (c & 3) * 16 + m] = o;
+    }
+  }
+  __syncthreads();
+  f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+  const int slot = (lane & 48) + min(lane & 15, rows - 1);
+  for (int kt = wave; kt < nk; kt += 4) {
+    const V wa = w0[(size_t)kt * 64], wb = w1[(size_t)kt * 64], x = xf[kt * 64 + slot];
+    acc[0] = mma(wa, x, acc[0]);
+    acc[1] = mma(wb, x, acc[1]);
+  }
+  red[wave][0][lane] = acc[0];
+  red[wave][1][lane] = acc[1];
+  __syncthreads();
+  if (wave < 2 && (lane & 15) < rows && nt0 + wave < NT) {
+    const int m = lane & 15;
+    const f32x4 v = (red[0][wave][lane] + red[1][wave][lane]) + (red[2][wave][lane] + red[3][wave][lane]);
+    const float gt = a.gate[(size_t)(m0 + m) * a.heads + h];
+    const int n0 = (nt0 + wave) * 16 + 4 * (lane >> 4);
+    T* o = (T*)a.out + (size_t)(m0 + m) * a.ldo + (size_t)h * a.vdim + n0;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (n0 + i < a.vdim) o[i] = (T)(v[i] * gt);
   }
 }
 
@@ -351,19 +456,17 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const ti_latent_pre
   }
 }
 
-template <class T, int KPW>
+template <class T>
 int launch_decode(const ti_latent_attn_args& a, hipStream_t s) {
   constexpr int VEC = El<T>::VEC;
   const int G = (a.lat_p + 16 * VEC - 1) / (16 * VEC), gpw = (G + 3) / 4;
-  const size_t lds = (size_t)(a.lat_p + a.rot_p) / El<T>::KT * 1024 + (size_t)16 * (4 * KPW + 16 / sizeof(T)) * sizeof(T) + 64 * 4;
+  const size_t lds = (size_t)(a.lat_p + a.rot_p) / El<T>::KT * 1024 + (size_t)16 * (64 + 16 / sizeof(T)) * sizeof(T) + 64 * 4;
   const dim3 grid(a.splits, (a.heads + 15) / 16, a.M), blk(256);
-#define TI_LD(GPW) hipLaunchKernelGGL((latent_decode_kernel<T, KPW, GPW>), grid, blk, lds, s, a)
-  if (gpw == 1) TI_LD(1);
-  else if (gpw == 2) TI_LD(2);
-  else TI_LD(4);
-#undef TI_LD
+  if (gpw == 1) hipLaunchKernelGGL((latent_decode_kernel<T, 1>), grid, blk, lds, s, a);
+  else if (gpw == 2) hipLaunchKernelGGL((latent_decode_kernel<T, 2>), grid, blk, lds, s, a);
+  else hipLaunchKernelGGL((latent_decode_kernel<T, 4>), grid, blk, lds, s, a);
   TI_LAUNCH_CHECK("latent_decode_kernel");
-  if (a.splits > 1) {
+  if (a.splits > 1 && a.out) {
     hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(a.heads, a.M), dim3(128), 0, s, a);
     TI_LAUNCH_CHECK("latent_merge_kernel");
   }
@@ -392,12 +495,12 @@ int launch_prefill(const ti_latent_prefill_args& a, hipStream_t s) {
 // Kernels whose dynamic LDS can pass 64 KiB (before any graph capture).
 template <class T>
 int prepare() {
-  const void* k[] = {(const void*)latent_decode_kernel<T, 16, 1>, (const void*)latent_decode_kernel<T, 16, 2>,
-                     (const void*)latent_decode_kernel<T, 16, 4>, (const void*)latent_prefill_kernel<T, 2, 4>,
+  const void* k[] = {(const void*)latent_decode_kernel<T, 1>, (const void*)latent_decode_kernel<T, 2>,
+                     (const void*)latent_decode_kernel<T, 4>, (const void*)latent_prefill_kernel<T, 2, 4>,
                      (const void*)latent_prefill_kernel<T, 2, 8>, (const void*)latent_prefill_kernel<T, 1, 4>,
-                     (const void*)latent_prefill_kernel<T, 1, 8>, (const void*)latent_prefill_kernel<T, 1, 16>};
+                     (const void*)latent_prefill_kernel<T, 1, 8>, (const void*)latent_out_kernel<T>, (const void*)latent_prefill_kernel<T, 1, 16>};
   for (const void* f : k)
-    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 163840 - 1024), "latent attention LDS");
+    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, f == (const void*)latent_out_kernel<T> ? 131072 : 163840 - 1024), "latent attention LDS");
   return TI_OK;
 }
 
@@ -414,26 +517,27 @@ extern "C" int ti_latent_prep(const ti_latent_prep_args* a, ti_stream_t stream) 
   using namespace ti;
   if (!a || !a->a32 || !a->q_w || !a->c_w || !a->rope_cs || !a->pos || !a->cq || !a->cache || !a->gate || a->M < 1 ||
       a->q_rank < 1 || a->kv_rank < 1 || a->rot_dim < 2 || a->rot_dim > a->rot_p || a->kv_rank > a->lat_p || a->ldq < a->q_rank ||
-      a->heads < 1 || !dtype_ok(a->dtype))
+      a->heads < 1 || a->lda % 4 || a->lda < a->gate_off + a->heads || a->lda > 16000 || !dtype_ok(a->dtype))
     return ti_set_error(TI_ERR_ARG, "ti_latent_prep: bad arguments");
+  const size_t lds = (size_t)a->lda * 4;
   if (a->dtype == TI_DT_BF16)
-    hipLaunchKernelGGL(latent_prep_kernel<bf16>, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a);
+    hipLaunchKernelGGL(latent_prep_kernel<bf16>, dim3(a->M), dim3(512), lds, (hipStream_t)stream, *a);
   else
-    hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a);
+    hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(a->M), dim3(512), lds, (hipStream_t)stream, *a);
   TI_LAUNCH_CHECK("latent_prep_kernel");
   return TI_OK;
 }
 
 extern "C" int ti_latent_attn_splits(int M, int heads, int max_seq) {
-  // about one workgroup per CU, none with less than one 64-key block
+  // about two workgroups per CU, none with less than one 64-key block
   const int wgs = M * ((heads + 15) / 16), cap = std::max(1, (max_seq + 63) / 64);
-  return std::max(1, std::min({cap, 64, (256 + wgs - 1) / std::max(1, wgs)}));
+  return std::max(1, std::min({cap, ti::kMaxSplits, (512 + wgs - 1) / std::max(1, wgs)}));
 }
 
 extern "C" int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t stream) {
   using namespace ti;
-  if (!a || !a->qa || !a->q || !a->cache || !a->pos || !a->sink || !a->out || a->M < 1 || a->M > 65535 || a->heads < 1 ||
-      a->splits < 1 || !dtype_ok(a->dtype) || (a->splits > 1 && (!a->part_o || !a->part_ml)))
+  if (!a || !a->qa || !a->q || !a->cache || !a->pos || !a->sink || (!a->out && a->splits < 2) || a->M < 1 || a->M > 65535 ||
+      a->heads < 1 || a->splits < 1 || a->splits > kMaxSplits || !dtype_ok(a->dtype) || (a->splits > 1 && (!a->part_o || !a->part_ml)))
     return ti_set_error(TI_ERR_ARG, "ti_latent_attn_decode: bad arguments");
   const int kt = a->dtype == TI_DT_BF16 ? 32 : 16, lim = a->dtype == TI_DT_BF16 ? 2048 : 1024;
   if (a->lat_p < kt || a->lat_p % kt || a->rot_p < kt || a->rot_p % kt || a->seq_p % 128 || a->ldqr % (kt / 4) || a->qr_off % (kt / 4))
@@ -441,8 +545,24 @@ extern "C" int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t s
   if (a->lat_p > lim || (a->lat_p + a->rot_p) / kt * 1024 > 140000)
     return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_decode: latent size %d (at most %d)", a->lat_p, lim);
   hipStream_t s = (hipStream_t)stream;
-  if (a->dtype == TI_DT_BF16) return launch_decode<bf16, 16>(*a, s);
-  return launch_decode<float, 16>(*a, s);
+  if (a->dtype == TI_DT_BF16) return launch_decode<bf16>(*a, s);
+  return launch_decode<float>(*a, s);
+}
+
+extern "C" int ti_latent_attn_out(const ti_latent_out_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->part_o || !a->part_ml || !a->sink || !a->w || !a->gate || !a->out || a->M < 1 || a->heads < 1 || a->heads > 65535 ||
+      a->splits < 1 || a->splits > kMaxSplits || a->vdim < 1 || !dtype_ok(a->dtype))
+    return ti_set_error(TI_ERR_ARG, "ti_latent_attn_out: bad arguments");
+  const int kt = a->dtype == TI_DT_BF16 ? 32 : 16;
+  if (a->lat_p < kt || a->lat_p % kt || a->w_batch % (kt / 4) || a->ldo < a->heads * a->vdim)
+    return ti_set_error(TI_ERR_ARG, "ti_latent_attn_out: lat_p %d ldo %d", a->lat_p, a->ldo);
+  const size_t lds = (size_t)a->lat_p / kt * 1024 + (size_t)256 * (kt / 4) * 4;
+  const dim3 grid(((a->vdim + 15) / 16 + 1) / 2, a->heads, (a->M + 15) / 16);
+  if (a->dtype == TI_DT_BF16) hipLaunchKernelGGL(latent_out_kernel<bf16>, grid, dim3(256), lds, (hipStream_t)stream, *a);
+  else hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), lds, (hipStream_t)stream, *a);
+  TI_LAUNCH_CHECK("latent_out_kernel");
+  return TI_OK;
 }
 
 extern "C" int ti_latent_attn_prefill(const ti_latent_prefill_args* a, ti_stream_t stream) {

@@ -73,15 +73,134 @@ __global__ __launch_bounds__(512) void rownorm_kernel(const ti_rownorm_args a) {
   }
 }
 
+// The same with H % 4 == 0 and H <= 4 * TH * NC: each thread holds NC float4 of the row in registers and
+// every load (residual, sublayer output, both norms' weights) is in flight before the first reduction.
+template <class T, int TH, int NC>
+__global__ __launch_bounds__(TH) void rownorm_vec_kernel(const ti_rownorm_args a) {
+  typedef typename El<T>::Q Q;
+  __shared__ float red[TH / 64];
+  const int m = blockIdx.x, tid = threadIdx.x, H4 = a.H >> 2;
+  const bool ln = a.kind == TI_NORM_LAYER, add = a.y || a.parts;
+  f32x4* x = (f32x4*)(a.x + (size_t)m * a.H);
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  f32x4 v[NC], y[NC], pw[NC], pb[NC], w[NC], b[NC], z[NC];
+  bool live[NC];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = min(tid + c * TH, H4 - 1);
+    live[c] = tid + c * TH < H4;
+    v[c] = x[i];
+    y[c] = a.y ? *(const f32x4*)(a.y + (size_t)m * a.ldy + 4 * i) : zero;
+    pw[c] = add && a.post_w ? *(const f32x4*)(a.post_w + 4 * i) : zero;
+    pb[c] = add && a.post_w && ln ? *(const f32x4*)(a.post_b + 4 * i) : zero;
+    w[c] = a.xn ? *(const f32x4*)(a.w + 4 * i) : zero;
+    b[c] = a.xn && ln ? *(const f32x4*)(a.b + 4 * i) : zero;
+    z[c] = a.cat ? *(const f32x4*)(a.x0 + (size_t)m * a.H + 4 * i) : zero;
+  }
+  if (a.parts) {
+    const T* p = (const T*)a.parts + (size_t)m * a.top * a.ldy;
+    for (int k0 = 0; k0 < a.top; k0 += 4) {
+      Q q[4][NC];
+      float pk[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int k = min(k0 + u, a.top - 1);
+        pk[u] = k0 + u < a.top ? a.part_w[(size_t)m * a.top + k] : 0.0f;
+#pragma unroll
+        for (int c = 0; c < NC; ++c) q[u][c] = *(const Q*)(p + (size_t)k * a.ldy + 4 * min(tid + c * TH, H4 - 1));
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (k0 + u < a.top)
+#pragma unroll
+          for (int c = 0; c < NC; ++c)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) y[c][e] = fmaf(pk[u], (float)q[u][c][e], y[c][e]);
+    }
+  }
+  // mean and inverse deviation of the row held in r
+  auto stats = [&](const f32x4* r) -> float2 {
+    float mean = 0.0f;
+    if (ln) {
+      float s = 0.0f;
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+        if (live[c]) s += (r[c][0] + r[c][1]) + (r[c][2] + r[c][3]);
+      mean = block_sum(s, red) / (float)a.H;
+    }
+    float q = 0.0f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+      if (live[c])
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float d = r[c][e] - mean;
+          q = fmaf(d, d, q);
+        }
+    return make_float2(mean, 1.0f / sqrtf(block_sum(q, red) / (float)a.H + a.eps));
+  };
+  if (add) {
+    float2 st = make_float2(0.0f, 1.0f);
+    if (a.post_w) st = stats(y);
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[c][e] += a.post_w ? (y[c][e] - st.x) * st.y * pw[c][e] + pb[c][e] : y[c][e];
+      if (live[c]) x[tid + c * TH] = v[c];
+    }
+  }
+  if (a.cat) {
+    T* cr = (T*)a.cat + (size_t)m * a.ldc;
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+      if (live[c]) {
+        *(Q*)(cr + 4 * (tid + c * TH)) = quad<T>(v[c]);
+        *(Q*)(cr + a.H + 4 * (tid + c * TH)) = quad<T>(z[c]);
+      }
+  }
+  if (a.xn) {
+    const float2 st = stats(v);
+    T* o = (T*)a.xn + (size_t)m * a.ldn;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      f32x4 r;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) r[e] = (v[c][e] - st.x) * st.y * w[c][e] + b[c][e];
+      if (live[c]) *(Q*)(o + 4 * (tid + c * TH)) = quad<T>(r);
+    }
+  }
+}
+
+template <class T>
+void launch_rownorm(const ti_rownorm_args& a, hipStream_t s) {
+  const bool vec = a.H % 4 == 0 && a.H <= 8192 && a.ldy % 4 == 0 && a.ldn % 4 == 0 && a.ldc % 4 == 0;
+  if (vec && a.H <= 1024) hipLaunchKernelGGL((rownorm_vec_kernel<T, 256, 1>), dim3(a.M), dim3(256), 0, s, a);
+  else if (vec && a.H <= 2048) hipLaunchKernelGGL((rownorm_vec_kernel<T, 512, 1>), dim3(a.M), dim3(512), 0, s, a);
+  else if (vec && a.H <= 4096) hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 1>), dim3(a.M), dim3(1024), 0, s, a);
+  else if (vec) hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 2>), dim3(a.M), dim3(1024), 0, s, a);
+  else hipLaunchKernelGGL(rownorm_kernel<T>, dim3(a.M), dim3(a.H <= 1024 ? 256 : 512), (size_t)a.H * 4, s, a);
+}
+
 // ------------------------------------------------------------------ expert routing
 constexpr int kMaxE = 1024, kMaxTop = 64;
 
-// One wave per row: softmax over the experts, the top scores by repeated maximum.  Lane l holds
-// experts l, l + 64, ...; a key orders by score, then by lower index.
+// One wave per row: softmax over the experts, the top scores (lowest index first among equals).
+// Repeated maxima; E <= 64: lane l holds expert l, more experts: lane l holds experts l, l + 64, ...
 __device__ __forceinline__ void route_row(const ti_route_args& a, int m) {
   constexpr int PER = kMaxE / 64;
   const int lane = threadIdx.x & 63;
   const float* z = a.logits + (size_t)m * a.ld;
+  if (a.E <= 64) {
+    float score;
+    route_top64(z, a.E, a.top, score, [&](int k, int e) {
+      if (lane == e) {
+        a.idx[(size_t)m * a.top + k] = e;
+        a.wgt[(size_t)m * a.top + k] = score;
+      }
+      return true;
+    });
+    return;
+  }
   float s[PER];
   float mx = -INFINITY;
 #pragma unroll
@@ -197,12 +316,8 @@ extern "C" int ti_rownorm(const ti_rownorm_args* a, ti_stream_t stream) {
       (a->xn && (!a->w || a->ldn < a->H || (a->kind == TI_NORM_LAYER && !a->b))) ||
       (a->cat && (!a->x0 || a->ldc < 2 * a->H)))
     return ti_set_error(TI_ERR_ARG, "ti_rownorm: inconsistent arguments");
-  const int threads = a->H <= 1024 ? 256 : 512;
-  const size_t lds = (size_t)a->H * 4;
-  if (a->dtype == TI_DT_BF16)
-    hipLaunchKernelGGL(rownorm_kernel<bf16>, dim3(a->M), dim3(threads), lds, (hipStream_t)stream, *a);
-  else
-    hipLaunchKernelGGL(rownorm_kernel<float>, dim3(a->M), dim3(threads), lds, (hipStream_t)stream, *a);
+  if (a->dtype == TI_DT_BF16) launch_rownorm<bf16>(*a, (hipStream_t)stream);
+  else launch_rownorm<float>(*a, (hipStream_t)stream);
   TI_LAUNCH_CHECK("rownorm_kernel");
   return TI_OK;
 }
@@ -222,7 +337,7 @@ extern "C" int ti_route(const ti_route_args* a, ti_stream_t stream) {
   if (a->tile_rows && (!a->list || !a->tiles || !a->n_tiles || a->tile_rows < 1))
     return ti_set_error(TI_ERR_ARG, "ti_route: list / tiles");
   hipStream_t s = (hipStream_t)stream;
-  if (a->tile_rows && a->M <= 64) {
+  if (a->tile_rows && a->M <= 16) {
     hipLaunchKernelGGL(route_both_kernel, dim3(1), dim3(1024), 0, s, *a);
   } else {
     hipLaunchKernelGGL(route_kernel, dim3((a->M + 3) / 4), dim3(256), 0, s, *a);
