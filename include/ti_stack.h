@@ -75,19 +75,13 @@ typedef struct ti_dense_args {
   int32_t advance;
   /* grouped products (experts): tile t covers entries [first, first + rows) of expert e's list */
   int32_t tile_rows;           /* 0 = not grouped; 16 or 64: rows a tile holds at most; 1: tile t is
-                                  entry t alone, expert tiles[t] (or the routed one, below)   */
+                                  entry t alone, of expert tiles[t]                           */
   int32_t max_tiles;           /* tiles launched; those at or past *n_tiles return at once   */
   const int32_t* tiles;        /* device [max_tiles][4] = expert, first, rows, -             */
   const int32_t* n_tiles;      /* device                                                     */
   const int32_t* rows_in;      /* entry p reads activation row (rows_in ? rows_in[p] : p) / row_div */
   const int32_t* rows_out;     /* nullable: entry p writes output row rows_out[p]            */
   int32_t row_div;
-  /* tile_rows 1: entry t = (row t / top, choice t % top) routed here from fp32 logits [.][route_e],
-   * route_e <= 64 (ti_route's choice), recorded in route_idx / route_wgt [max_tiles] */
-  int32_t route_e, top;
-  const float* route_logits;
-  int32_t* route_idx;
-  float* route_wgt;
 } ti_dense_args;
 int ti_dense(const ti_dense_args* a, ti_stream_t s);
 size_t ti_dense_args_bytes(void);
@@ -114,14 +108,21 @@ typedef struct ti_rownorm_args {
   void* cat;                   /* nullable T [M][ldc]: [x ; x0]                              */
   float eps;
   int32_t M, H, ldy, ldn, ldc, top, kind, dtype;
+  /* nullable: also route the normalised row (ti_route's choice) with fragment-ordered router weights
+   * [route_e][H], where ti_rownorm_routes(H, route_e) */
+  const void* route_w;
+  int32_t* route_idx;          /* [M][route_top] */
+  float* route_wgt;
+  int32_t route_e, route_top;
 } ti_rownorm_args;
 int ti_rownorm(const ti_rownorm_args* a, ti_stream_t s);
+int ti_rownorm_routes(int H, int E);
 
 /* ------------------------------------------------------------------- expert routing
  * logits fp32 [M][ld]: softmax over E experts, the `top` largest scores (lowest index first among
  * equals), not renormalised: idx [M][top], wgt [M][top].  Then the (row, expert) entries grouped by
  * expert: list[p] = row * top + k, and tiles of at most tile_rows entries of one expert.
- * E <= 1024, top <= min(E, 64).  tile_rows 0: idx / wgt only. */
+ * E <= 1024, top <= min(E, 64).  tile_rows 0: idx / wgt only; logits NULL: grouping of a given idx only. */
 typedef struct ti_route_args {
   const float* logits;
   int32_t ld, M, E, top;

@@ -94,14 +94,14 @@ class DenseArgs(C.Structure):
          ("gate", C.c_void_p), ("gate_ld", C.c_int32), ("key_blocks", C.c_int32), ("argmax", C.c_void_p),
          ("step_ctr", C.c_void_p), ("advance", C.c_int32), ("tile_rows", C.c_int32), ("max_tiles", C.c_int32),
          ("tiles", C.c_void_p), ("n_tiles", C.c_void_p), ("rows_in", C.c_void_p), ("rows_out", C.c_void_p),
-         ("row_div", C.c_int32), ("route_e", C.c_int32), ("top", C.c_int32), ("route_logits", C.c_void_p),
-         ("route_idx", C.c_void_p), ("route_wgt", C.c_void_p)]
+         ("row_div", C.c_int32)]
 
 
 class RownormArgs(C.Structure):
     """ti_rownorm_args (include/ti_stack.h)."""
     _fields_ = [(n, C.c_void_p) for n in ("x", "y", "parts", "part_w", "post_w", "post_b", "w", "b", "xn", "x0", "cat")] + \
-        [("eps", C.c_float)] + [(n, C.c_int32) for n in ("M", "H", "ldy", "ldn", "ldc", "top", "kind", "dtype")]
+        [("eps", C.c_float)] + [(n, C.c_int32) for n in ("M", "H", "ldy", "ldn", "ldc", "top", "kind", "dtype")] + \
+        [(n, C.c_void_p) for n in ("route_w", "route_idx", "route_wgt")] + [("route_e", C.c_int32), ("route_top", C.c_int32)]
 
 
 class RouteArgs(C.Structure):
@@ -135,7 +135,7 @@ EXPORTED = [
     "ti_qkv_attn_xchg_bytes", "ti_qkv_attn_supported", "ti_qkv_attn_error_offset",
     "ti_engine_create_stack", "ti_engine_weight_count", "ti_engine_weight_info", "ti_engine_set_weight", "ti_engine_load",
     "ti_engine_describe", "ti_engine_prefill", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
-    "ti_stack_convert", "ti_stack_fill", "ti_dense", "ti_dense_args_bytes", "ti_rownorm", "ti_route", "ti_route_max_tiles",
+    "ti_stack_convert", "ti_stack_fill", "ti_dense", "ti_dense_args_bytes", "ti_rownorm", "ti_rownorm_routes", "ti_route", "ti_route_max_tiles",
     "ti_latent_prep", "ti_latent_prepare", "ti_latent_attn_decode", "ti_latent_attn_splits", "ti_latent_attn_prefill", "ti_latent_attn_out",
 ]
 

@@ -10,6 +10,7 @@
 //             head with the gate); prompt chunks: keys / values expanded into fragments + chunk attention
 //   dense     output projection
 //   rownorm   residual += post-norm, pre-norm of the feed-forward
+//             (decode-sized row counts: with the router product and the choice of experts)
 //   dense     router; route; dense grouped gate/up with SiLU * up; dense grouped down
 #include "stack.hpp"
 
@@ -562,12 +563,18 @@ int StackModel::attention(const StackLayer& L, const StackRun& run, const StackR
   return dense(L.o, attn_, ldat, M, y_, c.width, TI_DE_F32, {});
 }
 
+// Decode-sized row counts route inside the feed-forward's pre-norm launch.
+bool StackModel::fused_router(const StackLayer& L, int M) const {
+  return M <= 64 && ti_rownorm_routes(c.width, L.c.experts);
+}
+
 int StackModel::experts(const StackLayer& L, int M) {
   const ti_stack_layer& k = L.c;
   const int W = c.width, ldx = kpad(W), ldact = kpad(k.ff);
-  TI_TRY(dense(L.router, xn_, ldx, M, zr_, k.experts, TI_DE_F32, {}));
+  const bool routed = fused_router(L, M);   // idx_ / wgt_ written by the norm's launch
+  if (!routed) TI_TRY(dense(L.router, xn_, ldx, M, zr_, k.experts, TI_DE_F32, {}));
   ti_route_args ra{};
-  ra.logits = zr_;
+  ra.logits = routed ? nullptr : zr_;
   ra.ld = k.experts;
   ra.M = M;
   ra.E = k.experts;
@@ -580,22 +587,13 @@ int StackModel::experts(const StackLayer& L, int M) {
   ti_dense_args g{};
   g.w_batch = (int64_t)up(2 * k.ff, 16) * L.gu.kp;
   g.row_div = k.top;
-  // few rows: every (row, choice) entry is a tile of its own (an expert two rows share is read twice);
-  // with at most 64 experts the gate / up launch also does the routing
+  // few rows: every (row, choice) entry is a tile of its own (an expert two rows share is read twice)
   const bool direct = M == 1 || (long)M * k.top * 2 <= k.experts;
   if (direct) {
     g.tile_rows = 1;
     g.max_tiles = M * k.top;
     g.tiles = idx_;
-    if (k.experts <= 64) {
-      g.route_logits = zr_;
-      g.route_e = k.experts;
-      g.top = k.top;
-      g.route_idx = idx_;
-      g.route_wgt = wgt_;
-    } else {
-      TI_TRY(ti_route(&ra, s_));
-    }
+    if (!routed) TI_TRY(ti_route(&ra, s_));
   } else {
     ra.tile_rows = M <= 64 ? 16 : 64;
     TI_TRY(ti_route(&ra, s_));
@@ -608,7 +606,6 @@ int StackModel::experts(const StackLayer& L, int M) {
   TI_TRY(dense(L.gu, xn_, ldx, M, act_, ldact, TI_DE_SWIGLU, g));
   g.rows_in = nullptr;
   g.row_div = 1;
-  g.route_logits = nullptr;
   if (!direct) g.rows_out = list_;
   g.w_batch = (int64_t)up(W, 16) * L.down.kp;
   return dense(L.down, act_, ldact, M, parts_, W, TI_DE_T, g);
@@ -622,7 +619,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
   const float* post = nullptr;
   bool parts = false;
   int top = 0;
-  auto rownorm = [&](const float* pre, void* cat) -> int {
+  auto rownorm = [&](const float* pre, void* cat, const StackLayer* route = nullptr) -> int {
     if (!post && !pre && !cat) return TI_OK;
     ti_rownorm_args n{};
     n.x = r.h;
@@ -654,6 +651,13 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
     n.H = W;
     n.kind = TI_NORM_LAYER;
     n.dtype = c.dtype;
+    if (route) {
+      n.route_w = route->router.p;
+      n.route_idx = idx_;
+      n.route_wgt = wgt_;
+      n.route_e = route->c.experts;
+      n.route_top = route->c.top;
+    }
     post = nullptr;
     return ti_rownorm(&n, s_);
   };
@@ -670,7 +674,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
     post = L.n1b;
     parts = false;
     if (L.c.mlp == TI_MLP_MOE) {
-      TI_TRY(rownorm(L.n2, nullptr));
+      TI_TRY(rownorm(L.n2, nullptr, fused_router(L, M) ? &L : nullptr));
       TI_TRY(experts(L, M));
       post = L.n2b;
       parts = true;

@@ -110,6 +110,7 @@ class StackModel {
            size_t elem_off = 0);
   int dense(const StackPack& w, const void* a, int lda, int M, void* out, int ldo, int epi, ti_dense_args extra);
   int attention(const StackLayer& L, const StackRun& run, const StackRows& r);
+  bool fused_router(const StackLayer& L, int M) const;
   int experts(const StackLayer& L, int M);
 };
 

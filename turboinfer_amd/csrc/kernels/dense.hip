@@ -128,20 +128,7 @@ __device__ __forceinline__ bool dense_span(const ti_dense_args& a, int y, DenseS
   if (a.tile_rows == 1) {
     s.first = y;
     s.rows = 1;
-    if (a.route_logits) {   // every wave finds the row's k-th expert itself; one workgroup records it
-      const int m = y / a.top, k = y - m * a.top;
-      float score;
-      route_top64(a.route_logits + (size_t)m * a.route_e, a.route_e, k + 1, score, [&](int i, int x) {
-        e = x;
-        return i < k;
-      });
-      if (blockIdx.x == 0 && (int)threadIdx.x == e) {
-        a.route_idx[y] = e;
-        a.route_wgt[y] = score;
-      }
-    } else {
-      e = a.tiles[y];
-    }
+    e = a.tiles[y];
     e = __builtin_amdgcn_readfirstlane(e);
   } else if (a.tile_rows) {
     if (y >= *a.n_tiles) return false;
@@ -433,11 +420,9 @@ extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
     return ti_set_error(TI_ERR_ARG, "ti_dense: lda %d < K %d or batch %d", a->lda, a->K, a->batch);
   if (a->tile_rows && ((a->tile_rows != 1 && a->tile_rows != 16 && a->tile_rows != 64) || a->max_tiles < 1 || a->max_tiles > 65535 ||
                        a->batch != 1 || a->epi > TI_DE_SWIGLU || (a->rows_in && a->row_div < 1) ||
-                       (a->tile_rows == 1 ? (!a->tiles && !a->route_logits) || a->rows_in || a->rows_out
-                                          : !a->tiles || !a->n_tiles || a->route_logits)))
+                       !a->tiles ||
+                       (a->tile_rows == 1 ? a->rows_in || a->rows_out : !a->n_tiles)))
     return ti_set_error(TI_ERR_ARG, "ti_dense: grouped arguments");
-  if (a->route_logits && (!a->route_idx || !a->route_wgt || a->route_e < 1 || a->route_e > 64 || a->top < 1 || a->top > a->route_e))
-    return ti_set_error(TI_ERR_ARG, "ti_dense: routing arguments");
   if (!a->tile_rows && (a->rows_in || a->rows_out)) return ti_set_error(TI_ERR_ARG, "ti_dense: row lists need grouped tiles");
   switch (a->epi) {
     case TI_DE_F32: case TI_DE_T: break;

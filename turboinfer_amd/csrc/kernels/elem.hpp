@@ -42,6 +42,13 @@ __device__ __forceinline__ f32x4 mma(f32x4 a, f32x4 b, f32x4 c) {
   return c;
 }
 
+// ti_stack_kpad of the element type
+template <class T>
+__host__ __device__ __forceinline__ int ti_kpad(int K) {
+  constexpr int u = 2 * El<T>::KT;
+  return (K + u - 1) / u * u;
+}
+
 template <class T>
 __device__ __forceinline__ typename El<T>::Q quad(f32x4 v) {
   typename El<T>::Q q;
@@ -50,13 +57,21 @@ __device__ __forceinline__ typename El<T>::Q quad(f32x4 v) {
   return q;
 }
 
+// LDS hand-off between the waves of a workgroup that leaves their global loads in flight (a plain
+// __syncthreads() may wait for them).
+__device__ __forceinline__ void lds_sync() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
 // block-wide sum of one float per thread; every thread gets it.  red: one float per wave.
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = group_sum<64>(v);
   const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  __syncthreads();   // red may still be read from the previous sum
+  lds_sync();   // red may still be read from the previous sum
   if ((threadIdx.x & 63) == 0) red[wave] = v;
-  __syncthreads();
+  lds_sync();
   float s = 0.0f;
   for (int i = 0; i < nw; ++i) s += red[i];
   return s;
@@ -71,21 +86,22 @@ __device__ __forceinline__ float wave_max(float v) {
   return xor32_max(xor16_max(v));
 }
 
-// Routing of one row over E <= 64 experts by one wave: the lane's softmax score (lane = expert), and
-// take(score) in turn for the best, second best, ... (lowest index first among equals) of `top`
-// choices; take returns false to stop.  NaN logits: expert 0.
-template <class F>
-__device__ __forceinline__ void route_top64(const float* z, int E, int top, float& score, F take) {
+// Routing of one row over E <= 64 experts by one wave, lane l holding expert l's logit v: softmax over
+// the experts, the `top` largest scores (lowest index first among equals) to idx / wgt.  NaN logits:
+// expert 0.
+__device__ __forceinline__ void route_top64(float v, int E, int top, int32_t* idx, float* wgt) {
   const int lane = threadIdx.x & 63;
-  const float v = lane < E ? z[lane] : -INFINITY;
-  const float mx = wave_max(v);
+  const float mx = wave_max(lane < E ? v : -INFINITY);
   float p = lane < E ? expf(v - mx) : -1.0f;
-  score = p / group_sum<64>(lane < E ? p : 0.0f);
+  const float score = p / group_sum<64>(lane < E ? p : 0.0f);
   for (int k = 0; k < top; ++k) {
     const unsigned long long best = __ballot(p == wave_max(p) && p >= 0.0f);
     const int e = best ? __builtin_ctzll(best) : 0;
-    if (!take(k, e)) return;
-    if (lane == e) p = -1.0f;
+    if (lane == e) {
+      idx[k] = e;
+      wgt[k] = score;
+      p = -1.0f;
+    }
   }
 }
 

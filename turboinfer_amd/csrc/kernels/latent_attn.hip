@@ -75,7 +75,7 @@ __device__ __forceinline__ void mma_values(f32x4* acc, const f32x4* vin, f32x4 p
 template <class T, int GPW>
 __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_attn_args a) {
   typedef typename El<T>::V V;
-  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, KB = 64, NVB = KB / KT, PLD = KB + 16 / (int)sizeof(T), NKU = 18;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, KB = 64, NVB = KB / KT, PLD = KB + 16 / (int)sizeof(T), NKU = 18, NQ = 5;
   extern __shared__ char lds[];
   const int split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
@@ -85,13 +85,13 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
   float* sm = (float*)(pb + 16 * PLD);              // [4][16] wave maxima, then [4][16] wave sums
   const int pos = a.pos[m], head = ht * 16 + col;
   const T* cache = (const T*)a.cache + (size_t)m * a.slot_stride;
-  for (int kt = wave; kt < nkt; kt += 4) {
+  auto load_q = [&](int kt) -> V {
     V v = {};
-    if (head < a.heads)
+    if (head < a.heads && kt < nkt)
       v = kt < lkt ? *(const V*)((const T*)a.qa + ((size_t)m * a.heads + head) * a.lat_p + kt * KT + g * VEC)
                    : *(const V*)((const T*)a.q + ((size_t)m * a.heads + head) * a.ldqr + a.qr_off + (kt - lkt) * KT + g * VEC);
-    qf[kt * 64 + lane] = v;
-  }
+    return v;
+  };
   f32x4 o[GPW][VEC];
 #pragma unroll
   for (int i = 0; i < GPW; ++i)
@@ -99,28 +99,46 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
     for (int c = 0; c < VEC; ++c) o[i][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float mr = -INFINITY, lr = 0.0f;
   const int nb = (pos + KB) / KB, bps = (nb + a.splits - 1) / a.splits, b0 = split * bps, b1 = min(nb, b0 + bps);
-  __syncthreads();
+  V k[NKU], vin[GPW == 1 ? NVB : 1][VEC];
+  auto load_k = [&](int b, int kt0) {
+    const V* kp = (const V*)(cache + (size_t)(b * KB + wave * 16 + col) * cw) + g;
+#pragma unroll
+    for (int u = 0; u < NKU; ++u) k[u] = kp[min(kt0 + u, nkt - 1) * 4];
+  };
+  auto load_v = [&](int b) {   // (dims past the latent: clamped, not stored)
+    if constexpr (GPW == 1) {
+      const T* vd = cache + (size_t)(b * KB + g * VEC) * cw + min(wave * 16 * VEC + col * VEC, a.lat_p - VEC);
+#pragma unroll
+      for (int kb = 0; kb < NVB; ++kb)
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) vin[kb][j] = *(const V*)(vd + (size_t)(kb * KT + j) * cw);
+    }
+  };
+  {
+    V q0[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) q0[i] = load_q(wave + 4 * i);
+    if (b0 < b1) {
+      load_k(b0, 0);
+      load_v(b0);
+    }
+#pragma unroll
+    for (int i = 0; i < NQ; ++i)
+      if (wave + 4 * i < nkt) qf[(wave + 4 * i) * 64 + lane] = q0[i];
+    for (int kt = wave + 4 * NQ; kt < nkt; kt += 4) qf[kt * 64 + lane] = load_q(kt);
+  }
+  lds_sync();
   for (int b = b0; b < b1; ++b) {
     const int k0 = b * KB + wave * 16;
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
-    const V* kp = (const V*)(cache + (size_t)(k0 + col) * cw) + g;
     const T* vp = cache + (size_t)(b * KB + g * VEC) * cw;
-    V vin[GPW == 1 ? NVB : 1][VEC];
     for (int kt0 = 0; kt0 < nkt; kt0 += NKU) {
-      V k[NKU];
-#pragma unroll
-      for (int u = 0; u < NKU; ++u) k[u] = kp[min(kt0 + u, nkt - 1) * 4];
-      if (GPW == 1 && kt0 == 0) {   // (dims past the latent: clamped, not stored)
-        const T* vd = vp + min(wave * 16 * VEC + col * VEC, a.lat_p - VEC);
-#pragma unroll
-        for (int kb = 0; kb < NVB; ++kb)
-#pragma unroll
-          for (int j = 0; j < VEC; ++j) vin[kb][j] = *(const V*)(vd + (size_t)(kb * KT + j) * cw);
-      }
+      if (kt0) load_k(b, kt0);
 #pragma unroll
       for (int u = 0; u < NKU; ++u)
         if (kt0 + u < nkt) s = mma(k[u], qf[(kt0 + u) * 64 + lane], s);
     }
+    if (b + 1 < b1) load_k(b + 1, 0);   // the next block's keys fly through the softmax and the sums
     float mx = -INFINITY;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -129,7 +147,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
     }
     mx = xor32_max(xor16_max(mx));
     if (lane < 16) sm[wave * 16 + col] = mx;
-    __syncthreads();
+    lds_sync();
     const float mn = fmaxf(fmaxf(mr, fmaxf(sm[col], sm[16 + col])), fmaxf(sm[32 + col], sm[48 + col]));
     const float alpha = expf(mr - mn);   // (every block holds a visible key: mn is finite)
     mr = mn;
@@ -141,7 +159,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
       lr += p[r];
     }
     *(typename El<T>::Q*)(pb + col * PLD + wave * 16 + 4 * g) = quad<T>(p);
-    __syncthreads();
+    lds_sync();
 #pragma unroll
     for (int i = 0; i < GPW; ++i) {
       const int gi = wave + 4 * i;
@@ -162,6 +180,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
         }
       }
     }
+    if (b + 1 < b1) load_v(b + 1);
   }
   lr = lane_xor<16>(lr) + lr;
   lr = lane_xor<32>(lr) + lr;
@@ -198,41 +217,39 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
   }
 }
 
-// The splits' rows merged and carried through the value up-projection in one launch: grid (pairs of 16
-// value dims, heads, tiles of 16 rows).  The merged rows go to LDS in operand fragments: a thread sums
-// one 16-byte piece over a share of the splits (groups of threads share a piece when there are few),
-// then the waves split k.
-constexpr int kMaxSplits = 64;
-template <class T>
-__global__ __launch_bounds__(256) void latent_out_kernel(const ti_latent_out_args a) {
+// The splits' rows merged and carried through the value up-projection in one launch: grid (groups of
+// NTW 16-dim value tiles, heads, tiles of 4 rows).  The merged rows go to LDS in operand fragments: a
+// thread sums one 16-byte piece over a share of the splits (SG threads share a piece when there are
+// few); then the 8 waves split the value tiles and k.
+constexpr int kMaxSplits = 64, kOutRows = 4;
+template <class T, int NTW>
+__global__ __launch_bounds__(512) void latent_out_kernel(const ti_latent_out_args a) {
   typedef typename El<T>::V V;
-  constexpr int KT = El<T>::KT, VEC = El<T>::VEC;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, KP = 8 / NTW;
   extern __shared__ char lds[];
-  __shared__ float wt[16][kMaxSplits];
-  __shared__ f32x4 red[4][2][64];
-  const int h = blockIdx.y, m0 = blockIdx.z * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int rows = min(16, a.M - m0), S = a.splits, nk = a.lat_p / KT, NT = (a.vdim + 15) >> 4, nt0 = blockIdx.x * 2;
+  __shared__ float wt[kOutRows][kMaxSplits];
+  __shared__ f32x4 red[8][64];
+  const int h = blockIdx.y, m0 = blockIdx.z * kOutRows, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int rows = min(kOutRows, a.M - m0), S = a.splits, nk = a.lat_p / KT, NT = (a.vdim + 15) >> 4;
+  const int nt = blockIdx.x * NTW + wave % NTW, kpart = wave / NTW;
   const int C = a.lat_p / VEC;   // pieces per row
   V* xf = (V*)lds;               // [nk][64]
-  float* part = (float*)(lds + (size_t)nk * 1024);   // [256][VEC] partial pieces
-  const V* w0 = (const V*)a.w + ((size_t)h * (a.w_batch / VEC)) + (size_t)nt0 * nk * 64 + lane;
-  const V* w1 = nt0 + 1 < NT ? w0 + (size_t)nk * 64 : w0;
-  for (int m = wave; m < rows; m += 4) {
+  float* part = (float*)(lds + (size_t)nk * 1024);   // [512][VEC] partial pieces
+  if (wave < rows) {
     float mx = -INFINITY, l = 0.0f;
     if (lane < S) {
-      const float2 ml = *(const float2*)(a.part_ml + (((size_t)(m0 + m) * S + lane) * a.heads + h) * 2);
+      const float2 ml = *(const float2*)(a.part_ml + (((size_t)(m0 + wave) * S + lane) * a.heads + h) * 2);
       mx = ml.x;
       l = ml.y;
     }
     const float sink = a.sink[h], mm = fmaxf(wave_max(mx), sink), e = l > 0.0f ? l * expf(mx - mm) : 0.0f;
-    wt[m][lane] = e / (group_sum<64>(e) + expf(sink - mm));
+    wt[wave][lane] = e / (group_sum<64>(e) + expf(sink - mm));
   }
   __syncthreads();
   const size_t sstride = (size_t)a.heads * a.lat_p;
-  // pieces in batches of 256 / SG threads' worth, SG threads per piece
   int SG = 1;
-  while (SG < 8 && rows * C * SG * 2 <= 256 && SG * 2 <= S) SG *= 2;
-  const int per = 256 / SG, ss = (S + SG - 1) / SG, sg = tid / per;
+  while (SG < 8 && rows * C * SG * 2 <= 512 && SG * 2 <= S) SG *= 2;
+  const int per = 512 / SG, ss = (S + SG - 1) / SG, sg = tid / per;
   for (int p0 = 0; p0 < rows * C; p0 += per) {
     const int p = p0 + tid % per;
     const bool live = p < rows * C;
@@ -267,22 +284,27 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const ti_latent_out_arg
       xf[(c >> 2) * 64 + (c & 3) * 16 + m] = o;
     }
   }
+  const V* wp = (const V*)a.w + (size_t)h * (a.w_batch / VEC) + (size_t)min(nt, NT - 1) * nk * 64 + lane;
   __syncthreads();
-  f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
   const int slot = (lane & 48) + min(lane & 15, rows - 1);
-  for (int kt = wave; kt < nk; kt += 4) {
-    const V wa = w0[(size_t)kt * 64], wb = w1[(size_t)kt * 64], x = xf[kt * 64 + slot];
-    acc[0] = mma(wa, x, acc[0]);
-    acc[1] = mma(wb, x, acc[1]);
+  for (int kt = kpart; kt < nk; kt += 4 * KP) {
+    V w[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) w[u] = wp[(size_t)min(kt + u * KP, nk - 1) * 64];
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      if (kt + u * KP < nk) acc = mma(w[u], xf[(kt + u * KP) * 64 + slot], acc);
   }
-  red[wave][0][lane] = acc[0];
-  red[wave][1][lane] = acc[1];
+  red[wave][lane] = acc;
   __syncthreads();
-  if (wave < 2 && (lane & 15) < rows && nt0 + wave < NT) {
+  if (kpart == 0 && (lane & 15) < rows && nt < NT) {
     const int m = lane & 15;
-    const f32x4 v = (red[0][wave][lane] + red[1][wave][lane]) + (red[2][wave][lane] + red[3][wave][lane]);
+    f32x4 v = acc;
+#pragma unroll
+    for (int k = 1; k < KP; ++k) v += red[k * NTW + wave][lane];
     const float gt = a.gate[(size_t)(m0 + m) * a.heads + h];
-    const int n0 = (nt0 + wave) * 16 + 4 * (lane >> 4);
+    const int n0 = nt * 16 + 4 * (lane >> 4);
     T* o = (T*)a.out + (size_t)(m0 + m) * a.ldo + (size_t)h * a.vdim + n0;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
@@ -479,7 +501,7 @@ int launch_prefill(const ti_latent_prefill_args& a, hipStream_t s) {
   const bool two = (size_t)nkt * 2 * 1024 * 4 <= 81920 && nv <= 8 && a.M > 64;
   const int mq = two ? 2 : 1;
   const size_t lds = (size_t)nkt * mq * 1024 * 4;
-  if (lds > 163840 - 1024) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_prefill: head of %d + %d dims", a.dim_p, a.rot_p);
+  if (lds > 131072) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_prefill: head of %d + %d dims", a.dim_p, a.rot_p);
   const dim3 grid((a.M + 64 * mq - 1) / (64 * mq), a.heads), blk(256);
 #define TI_LP(MQ, NV) hipLaunchKernelGGL((latent_prefill_kernel<T, MQ, NV>), grid, blk, lds, s, a)
   if (two && nv <= 4) TI_LP(2, 4);
@@ -492,15 +514,16 @@ int launch_prefill(const ti_latent_prefill_args& a, hipStream_t s) {
   return TI_OK;
 }
 
-// Kernels whose dynamic LDS can pass 64 KiB (before any graph capture).
+// Kernels whose dynamic LDS can pass 64 KiB (before any graph capture); at most 128 KiB is used.
 template <class T>
 int prepare() {
   const void* k[] = {(const void*)latent_decode_kernel<T, 1>, (const void*)latent_decode_kernel<T, 2>,
                      (const void*)latent_decode_kernel<T, 4>, (const void*)latent_prefill_kernel<T, 2, 4>,
                      (const void*)latent_prefill_kernel<T, 2, 8>, (const void*)latent_prefill_kernel<T, 1, 4>,
-                     (const void*)latent_prefill_kernel<T, 1, 8>, (const void*)latent_out_kernel<T>, (const void*)latent_prefill_kernel<T, 1, 16>};
+                     (const void*)latent_prefill_kernel<T, 1, 8>, (const void*)latent_out_kernel<T, 2>,
+                     (const void*)latent_out_kernel<T, 4>, (const void*)latent_out_kernel<T, 8>, (const void*)latent_prefill_kernel<T, 1, 16>};
   for (const void* f : k)
-    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, f == (const void*)latent_out_kernel<T> ? 131072 : 163840 - 1024), "latent attention LDS");
+    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 131072), "latent attention LDS");
   return TI_OK;
 }
 
@@ -529,9 +552,9 @@ extern "C" int ti_latent_prep(const ti_latent_prep_args* a, ti_stream_t stream) 
 }
 
 extern "C" int ti_latent_attn_splits(int M, int heads, int max_seq) {
-  // about two workgroups per CU, none with less than one 64-key block
+  // one or two workgroups per CU (splits cost a merge), none with less than one 64-key block
   const int wgs = M * ((heads + 15) / 16), cap = std::max(1, (max_seq + 63) / 64);
-  return std::max(1, std::min({cap, ti::kMaxSplits, (512 + wgs - 1) / std::max(1, wgs)}));
+  return std::max(1, std::min({cap, ti::kMaxSplits, ((M == 1 ? 512 : 256) + wgs - 1) / std::max(1, wgs)}));
 }
 
 extern "C" int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t stream) {
@@ -542,7 +565,7 @@ extern "C" int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t s
   const int kt = a->dtype == TI_DT_BF16 ? 32 : 16, lim = a->dtype == TI_DT_BF16 ? 2048 : 1024;
   if (a->lat_p < kt || a->lat_p % kt || a->rot_p < kt || a->rot_p % kt || a->seq_p % 128 || a->ldqr % (kt / 4) || a->qr_off % (kt / 4))
     return ti_set_error(TI_ERR_ARG, "ti_latent_attn_decode: lat_p %d rot_p %d seq_p %d", a->lat_p, a->rot_p, a->seq_p);
-  if (a->lat_p > lim || (a->lat_p + a->rot_p) / kt * 1024 > 140000)
+  if (a->lat_p > lim || (a->lat_p + a->rot_p) / kt * 1024 > 122880)
     return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_decode: latent size %d (at most %d)", a->lat_p, lim);
   hipStream_t s = (hipStream_t)stream;
   if (a->dtype == TI_DT_BF16) return launch_decode<bf16>(*a, s);
@@ -557,10 +580,18 @@ extern "C" int ti_latent_attn_out(const ti_latent_out_args* a, ti_stream_t strea
   const int kt = a->dtype == TI_DT_BF16 ? 32 : 16;
   if (a->lat_p < kt || a->lat_p % kt || a->w_batch % (kt / 4) || a->ldo < a->heads * a->vdim)
     return ti_set_error(TI_ERR_ARG, "ti_latent_attn_out: lat_p %d ldo %d", a->lat_p, a->ldo);
-  const size_t lds = (size_t)a->lat_p / kt * 1024 + (size_t)256 * (kt / 4) * 4;
-  const dim3 grid(((a->vdim + 15) / 16 + 1) / 2, a->heads, (a->M + 15) / 16);
-  if (a->dtype == TI_DT_BF16) hipLaunchKernelGGL(latent_out_kernel<bf16>, grid, dim3(256), lds, (hipStream_t)stream, *a);
-  else hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), lds, (hipStream_t)stream, *a);
+  const size_t lds = (size_t)a->lat_p / kt * 1024 + (size_t)512 * (kt / 4) * 4;
+  const int nt = (a->vdim + 15) / 16, z = (a->M + kOutRows - 1) / kOutRows;
+  hipStream_t s = (hipStream_t)stream;
+  // fewer value tiles per workgroup (the merge repeated) only while the chip is not filled
+  auto launch = [&]<int NTW>() {
+    const dim3 grid((nt + NTW - 1) / NTW, a->heads, z);
+    if (a->dtype == TI_DT_BF16) hipLaunchKernelGGL((latent_out_kernel<bf16, NTW>), grid, dim3(512), lds, s, *a);
+    else hipLaunchKernelGGL((latent_out_kernel<float, NTW>), grid, dim3(512), lds, s, *a);
+  };
+  if ((long)a->heads * z * nt <= 512) launch.template operator()<2>();
+  else if ((long)a->heads * z * nt <= 1024) launch.template operator()<4>();
+  else launch.template operator()<8>();
   TI_LAUNCH_CHECK("latent_out_kernel");
   return TI_OK;
 }

@@ -75,10 +75,18 @@ __global__ __launch_bounds__(512) void rownorm_kernel(const ti_rownorm_args a) {
 
 // The same with H % 4 == 0 and H <= 4 * TH * NC: each thread holds NC float4 of the row in registers and
 // every load (residual, sublayer output, both norms' weights) is in flight before the first reduction.
-template <class T, int TH, int NC>
+// ROUTE: the same workgroup multiplies the normalised row with the router's weights (its first
+// fragments in flight through the norms) and picks the row's experts.
+template <class T, int TH, int NC, bool ROUTE>
 __global__ __launch_bounds__(TH) void rownorm_vec_kernel(const ti_rownorm_args a) {
   typedef typename El<T>::Q Q;
+  typedef typename El<T>::V V;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, NW = TH / 64, PF = 4;
   __shared__ float red[TH / 64];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int nk = ROUTE ? ti_kpad<T>(a.H) / KT : 0, nt = ROUTE ? (a.route_e + 15) >> 4 : 0;
+  const V* rw = (const V*)a.route_w + lane;
+  V rf[ROUTE ? PF : 1][4];
   const int m = blockIdx.x, tid = threadIdx.x, H4 = a.H >> 2;
   const bool ln = a.kind == TI_NORM_LAYER, add = a.y || a.parts;
   f32x4* x = (f32x4*)(a.x + (size_t)m * a.H);
@@ -117,6 +125,12 @@ __global__ __launch_bounds__(TH) void rownorm_vec_kernel(const ti_rownorm_args a
 #pragma unroll
             for (int e = 0; e < 4; ++e) y[c][e] = fmaf(pk[u], (float)q[u][c][e], y[c][e]);
     }
+  }
+  if constexpr (ROUTE) {   // (behind the row's own loads, in flight through the norms)
+#pragma unroll
+    for (int i = 0; i < PF; ++i)
+#pragma unroll
+      for (int t = 0; t < 4; ++t) rf[i][t] = rw[((size_t)min(t, nt - 1) * nk + min(wave + i * NW, nk - 1)) * 64];
   }
   // mean and inverse deviation of the row held in r
   auto stats = [&](const f32x4* r) -> float2 {
@@ -167,18 +181,65 @@ __global__ __launch_bounds__(TH) void rownorm_vec_kernel(const ti_rownorm_args a
 #pragma unroll
       for (int e = 0; e < 4; ++e) r[e] = (v[c][e] - st.x) * st.y * w[c][e] + b[c][e];
       if (live[c]) *(Q*)(o + 4 * (tid + c * TH)) = quad<T>(r);
+      if constexpr (ROUTE) {   // (the row's k padding: zeros)
+        extern __shared__ float row[];
+        if (4 * (tid + c * TH) < nk * KT) *(Q*)((T*)row + 4 * (tid + c * TH)) = live[c] ? quad<T>(r) : quad<T>(zero);
+      }
+    }
+    if constexpr (ROUTE) {
+      extern __shared__ float row[];
+      __shared__ float zr[NW][64];
+      lds_sync();
+      f32x4 acc[4] = {zero, zero, zero, zero};
+      const T* xr = (const T*)row + (lane >> 4) * VEC;   // every operand column is this row
+#pragma unroll
+      for (int i = 0; i < PF; ++i)
+        if (wave + i * NW < nk) {
+          const V x = *(const V*)(xr + (wave + i * NW) * KT);
+#pragma unroll
+          for (int t = 0; t < 4; ++t) acc[t] = mma(rf[i][t], x, acc[t]);
+        }
+      for (int kt = wave + PF * NW; kt < nk; kt += NW) {
+        const V x = *(const V*)(xr + kt * KT);
+#pragma unroll
+        for (int t = 0; t < 4; ++t) acc[t] = mma(rw[((size_t)min(t, nt - 1) * nk + kt) * 64], x, acc[t]);
+      }
+      if ((lane & 15) == 0)
+#pragma unroll
+        for (int t = 0; t < 4; ++t) *(f32x4*)&zr[wave][t * 16 + 4 * (lane >> 4)] = acc[t];
+      lds_sync();
+      if (wave == 0) {
+        float zl = 0.0f;
+#pragma unroll
+        for (int w = 0; w < NW; ++w) zl += zr[w][lane];
+        route_top64(zl, a.route_e, a.route_top, a.route_idx + (size_t)m * a.route_top, a.route_wgt + (size_t)m * a.route_top);
+      }
     }
   }
 }
 
 template <class T>
-void launch_rownorm(const ti_rownorm_args& a, hipStream_t s) {
+int launch_rownorm(const ti_rownorm_args& a, hipStream_t s) {
   const bool vec = a.H % 4 == 0 && a.H <= 8192 && a.ldy % 4 == 0 && a.ldn % 4 == 0 && a.ldc % 4 == 0;
-  if (vec && a.H <= 1024) hipLaunchKernelGGL((rownorm_vec_kernel<T, 256, 1>), dim3(a.M), dim3(256), 0, s, a);
-  else if (vec && a.H <= 2048) hipLaunchKernelGGL((rownorm_vec_kernel<T, 512, 1>), dim3(a.M), dim3(512), 0, s, a);
-  else if (vec && a.H <= 4096) hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 1>), dim3(a.M), dim3(1024), 0, s, a);
-  else if (vec) hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 2>), dim3(a.M), dim3(1024), 0, s, a);
-  else hipLaunchKernelGGL(rownorm_kernel<T>, dim3(a.M), dim3(a.H <= 1024 ? 256 : 512), (size_t)a.H * 4, s, a);
+  if (a.route_w) {
+    if (!vec) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_rownorm: routing needs H %% 4 == 0, H <= 8192");
+    const size_t lds = (size_t)ti_kpad<T>(a.H) * sizeof(T);
+    if (a.H <= 1024) hipLaunchKernelGGL((rownorm_vec_kernel<T, 512, 1, true>), dim3(a.M), dim3(512), lds, s, a);
+    else if (a.H <= 4096) hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 1, true>), dim3(a.M), dim3(1024), lds, s, a);
+    else hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 2, true>), dim3(a.M), dim3(1024), lds, s, a);
+  } else if (vec && a.H <= 1024) {
+    hipLaunchKernelGGL((rownorm_vec_kernel<T, 256, 1, false>), dim3(a.M), dim3(256), 0, s, a);
+  } else if (vec && a.H <= 2048) {
+    hipLaunchKernelGGL((rownorm_vec_kernel<T, 512, 1, false>), dim3(a.M), dim3(512), 0, s, a);
+  } else if (vec && a.H <= 4096) {
+    hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 1, false>), dim3(a.M), dim3(1024), 0, s, a);
+  } else if (vec) {
+    hipLaunchKernelGGL((rownorm_vec_kernel<T, 1024, 2, false>), dim3(a.M), dim3(1024), 0, s, a);
+  } else {
+    hipLaunchKernelGGL(rownorm_kernel<T>, dim3(a.M), dim3(a.H <= 1024 ? 256 : 512), (size_t)a.H * 4, s, a);
+  }
+  TI_LAUNCH_CHECK("rownorm_kernel");
+  return TI_OK;
 }
 
 // ------------------------------------------------------------------ expert routing
@@ -191,14 +252,7 @@ __device__ __forceinline__ void route_row(const ti_route_args& a, int m) {
   const int lane = threadIdx.x & 63;
   const float* z = a.logits + (size_t)m * a.ld;
   if (a.E <= 64) {
-    float score;
-    route_top64(z, a.E, a.top, score, [&](int k, int e) {
-      if (lane == e) {
-        a.idx[(size_t)m * a.top + k] = e;
-        a.wgt[(size_t)m * a.top + k] = score;
-      }
-      return true;
-    });
+    route_top64(lane < a.E ? z[lane] : 0.0f, a.E, a.top, a.idx + (size_t)m * a.top, a.wgt + (size_t)m * a.top);
     return;
   }
   float s[PER];
@@ -298,7 +352,8 @@ __global__ __launch_bounds__(256) void route_kernel(const ti_route_args a) {
 __global__ __launch_bounds__(1024) void route_group_kernel(const ti_route_args a) { route_group(a); }
 // few rows: both steps in one workgroup
 __global__ __launch_bounds__(1024) void route_both_kernel(const ti_route_args a) {
-  for (int m = threadIdx.x >> 6; m < a.M; m += 16) route_row(a, m);
+  if (a.logits)
+    for (int m = threadIdx.x >> 6; m < a.M; m += 16) route_row(a, m);
   __threadfence_block();
   __syncthreads();
   route_group(a);
@@ -316,11 +371,13 @@ extern "C" int ti_rownorm(const ti_rownorm_args* a, ti_stream_t stream) {
       (a->xn && (!a->w || a->ldn < a->H || (a->kind == TI_NORM_LAYER && !a->b))) ||
       (a->cat && (!a->x0 || a->ldc < 2 * a->H)))
     return ti_set_error(TI_ERR_ARG, "ti_rownorm: inconsistent arguments");
-  if (a->dtype == TI_DT_BF16) launch_rownorm<bf16>(*a, (hipStream_t)stream);
-  else launch_rownorm<float>(*a, (hipStream_t)stream);
-  TI_LAUNCH_CHECK("rownorm_kernel");
-  return TI_OK;
+  if (a->route_w && (!a->xn || !a->route_idx || !a->route_wgt || a->route_e < 1 || a->route_e > 64 || a->route_top < 1 ||
+                     a->route_top > a->route_e))
+    return ti_set_error(TI_ERR_ARG, "ti_rownorm: routing arguments");
+  return a->dtype == TI_DT_BF16 ? launch_rownorm<bf16>(*a, (hipStream_t)stream) : launch_rownorm<float>(*a, (hipStream_t)stream);
 }
+
+extern "C" int ti_rownorm_routes(int H, int E) { return H % 4 == 0 && H <= 8192 && E >= 1 && E <= 64; }
 
 extern "C" int ti_route_max_tiles(int M, int E, int top, int tile_rows) {
   if (M < 1 || E < 1 || top < 1 || tile_rows < 1) return 0;
@@ -331,8 +388,8 @@ extern "C" int ti_route_max_tiles(int M, int E, int top, int tile_rows) {
 
 extern "C" int ti_route(const ti_route_args* a, ti_stream_t stream) {
   using namespace ti;
-  if (!a || !a->logits || !a->idx || !a->wgt || a->M < 1 || a->E < 1 || a->E > kMaxE || a->top < 1 || a->top > kMaxTop ||
-      a->top > a->E || a->ld < a->E)
+  if (!a || (!a->logits && !a->tile_rows) || !a->idx || !a->wgt || a->M < 1 || a->E < 1 || a->E > kMaxE || a->top < 1 || a->top > kMaxTop ||
+      a->top > a->E || (a->logits && a->ld < a->E))
     return ti_set_error(TI_ERR_ARG, "ti_route: bad arguments (1 <= top <= experts <= %d, top <= %d)", kMaxE, kMaxTop);
   if (a->tile_rows && (!a->list || !a->tiles || !a->n_tiles || a->tile_rows < 1))
     return ti_set_error(TI_ERR_ARG, "ti_route: list / tiles");
@@ -340,7 +397,7 @@ extern "C" int ti_route(const ti_route_args* a, ti_stream_t stream) {
   if (a->tile_rows && a->M <= 16) {
     hipLaunchKernelGGL(route_both_kernel, dim3(1), dim3(1024), 0, s, *a);
   } else {
-    hipLaunchKernelGGL(route_kernel, dim3((a->M + 3) / 4), dim3(256), 0, s, *a);
+    if (a->logits) hipLaunchKernelGGL(route_kernel, dim3((a->M + 3) / 4), dim3(256), 0, s, *a);
     if (a->tile_rows) hipLaunchKernelGGL(route_group_kernel, dim3(1), dim3(1024), 0, s, *a);
   }
   TI_LAUNCH_CHECK("route_kernel");
