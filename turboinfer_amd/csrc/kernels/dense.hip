@@ -6,9 +6,9 @@
 //   * dense_skinny_kernel (M <= 64): HBM-bound weight streaming.  One workgroup per 16 output columns,
 //     its waves split k; each weight fragment is one contiguous KiB read once and multiplied with up
 //     to 4 row tiles; the waves' partial sums meet in LDS.
-//   * dense_tile_kernel (more rows): 4 waves as 2 x 2 over a BM x BN tile, activations staged through
-//     double-buffered LDS in fragment order, weight fragments straight from L2 into registers one
-//     k-stage (128 bytes) ahead.
+//   * dense_tile_kernel (more rows): 4 waves side by side over a BM x BN tile, activations staged through
+//     double-buffered LDS in fragment order, each wave's weight fragments straight from L2 into
+//     registers; both 2 or 4 k-stages (128 bytes each) ahead of their use.
 // Both take independent batches (per-head products) or grouped tiles (experts: a tile is up to
 // tile_rows entries of one expert's list, rows gathered and scattered through the list).
 #include <algorithm>
@@ -22,22 +22,33 @@ __device__ __forceinline__ unsigned long long logit_key(float v, int n) {
 }
 
 // Four consecutive output columns n0.. of row m (out row mo); rows >= rows are padding.
-template <class T>
+template <class T, int EPI>
 __device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, int m, int mo, int rows, int n0, f32x4 v) {
   constexpr int VEC = El<T>::VEC, KT = El<T>::KT;
   const bool live = m < rows;
-  switch (a.epi) {
+  switch (EPI) {
     case TI_DE_F32: {
       if (!live) return;
       float* o = (float*)a.out + (size_t)batch * a.o_batch + (size_t)mo * a.ldo + n0;
+      if (a.add)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] += a.add[min(n0 + i, a.N - 1)];
+      if (n0 + 4 <= a.N && ((a.ldo | a.o_batch) & 3) == 0) {
+        *(f32x4*)o = v;
+        return;
+      }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (n0 + i < a.N) o[i] = a.add ? v[i] + a.add[n0 + i] : v[i];
+        if (n0 + i < a.N) o[i] = v[i];
       return;
     }
     case TI_DE_T: {
       if (!live) return;
       T* o = (T*)a.out + (size_t)batch * a.o_batch + (size_t)mo * a.ldo + n0;
+      if (n0 + 4 <= a.N && ((a.ldo | a.o_batch) & 3) == 0) {
+        *(typename El<T>::Q*)o = quad<T>(v);
+        return;
+      }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
         if (n0 + i < a.N) o[i] = (T)v[i];
@@ -149,7 +160,7 @@ __device__ __forceinline__ int row_in(const ti_dense_args& a, int p) {
 }
 __device__ __forceinline__ int row_out(const ti_dense_args& a, int p) { return a.rows_out ? a.rows_out[p] : p; }
 
-template <class T, int MT, int W>
+template <class T, int MT, int W, int EPI>
 __global__ __launch_bounds__(64 * W) void dense_skinny_kernel(const ti_dense_args a) {
   typedef typename El<T>::V V;
   constexpr int KT = El<T>::KT, VEC = El<T>::VEC, U = 8;
@@ -201,19 +212,20 @@ __global__ __launch_bounds__(64 * W) void dense_skinny_kernel(const ti_dense_arg
 #pragma unroll
     for (int w = 1; w < W; ++w) v += red[w][mt][lane];
     const int m = z0 + mt * 16 + (lane & 15), n0 = nt * 16 + 4 * (lane >> 4);
-    if (a.epi == TI_DE_LOGITS)
+    if constexpr (EPI == TI_DE_LOGITS)
       dense_argmax(a, m, sp.rows, n0, v, lane, nt);
     else
-      dense_store<T>(a, sp.batch, m, m < sp.rows ? row_out(a, sp.first + m) : 0, sp.rows, n0, v);
+      dense_store<T, EPI>(a, sp.batch, m, m < sp.rows ? row_out(a, sp.first + m) : 0, sp.rows, n0, v);
   }
-  if (a.epi == TI_DE_LOGITS && a.step_ctr && nt == 0 && blockIdx.z == 0 && tid == 0) *a.step_ctr += a.advance;
+  if (EPI == TI_DE_LOGITS && a.step_ctr && nt == 0 && blockIdx.z == 0 && tid == 0) *a.step_ctr += a.advance;
 }
 
-template <class T, int BM, int BN, bool VF>
-__global__ __launch_bounds__(256) void dense_tile_kernel(const ti_dense_args a, int m_tiles, int n_tiles) {
+template <class T, int BM, int BN, int D, int EPI>
+__global__ __launch_bounds__(256, BM * BN > 16384 ? 1 : 2) void dense_tile_kernel(const ti_dense_args a, int m_tiles, int n_tiles) {
   typedef typename El<T>::V V;
-  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, FM = BM / 32, FN = BN / 32;
-  __shared__ V as[2][BM / 16 * 2][64];
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, FM = BM / 16, FN = BN / 64, NA = BM / 32;
+  constexpr bool VF = EPI == TI_DE_VFRAG;
+  __shared__ V as[2][FM * 2][64];
   DenseSpan sp;
   if (!dense_span(a, blockIdx.y, sp, sizeof(T))) return;
   // consecutive workgroups go to the 8 XCDs in turn: give each XCD a contiguous run of tiles, row
@@ -222,11 +234,11 @@ __global__ __launch_bounds__(256) void dense_tile_kernel(const ti_dense_args a, 
   const int id = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
   if (id >= total) return;
   const int mtile = id % m_tiles, ntile = id / m_tiles, m_base = mtile * BM;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave & 1, wn = wave >> 1;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int nk = a.K / KT, nst = nk >> 1, NT = (a.N + 15) >> 4;
-  const V* ap[FM];
+  const V* ap[NA];
 #pragma unroll
-  for (int i = 0; i < FM; ++i) {
+  for (int i = 0; i < NA; ++i) {
     const int f = i * 4 + wave;   // fragment (row tile f >> 1, k-tile f & 1) of the stage
     const int p = sp.first + min(m_base + (f >> 1) * 16 + (lane & 15), sp.rows - 1);
     ap[i] = (const V*)((const T*)a.a + (size_t)sp.batch * a.a_batch + (size_t)row_in(a, p) * a.lda) + (f & 1) * (KT / VEC) +
@@ -235,111 +247,150 @@ __global__ __launch_bounds__(256) void dense_tile_kernel(const ti_dense_args a, 
   const V* wp[FN];
 #pragma unroll
   for (int j = 0; j < FN; ++j)
-    wp[j] = (const V*)sp.w + (size_t)min(ntile * (BN / 16) + wn * FN + j, NT - 1) * nk * 64 + lane;
+    wp[j] = (const V*)sp.w + (size_t)min(ntile * (BN / 16) + wave * FN + j, NT - 1) * nk * 64 + lane;
   f32x4 acc[FM][FN];
 #pragma unroll
   for (int i = 0; i < FM; ++i)
 #pragma unroll
     for (int j = 0; j < FN; ++j) acc[i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  V ar[FM], wc[FN][2], wx[FN][2];
+  // rings of D stages in registers: weights of stage s in set s % D, activations likewise until they
+  // move to LDS one stage before their use
+  V ar[D][NA], w[D][FN][2];
+  auto load_a = [&](V (&d)[NA], int s) {
 #pragma unroll
-  for (int i = 0; i < FM; ++i) ar[i] = ap[i][0];
-#pragma unroll
-  for (int j = 0; j < FN; ++j) {
-    wc[j][0] = wp[j][0];
-    wc[j][1] = wp[j][64];
-  }
-#pragma unroll
-  for (int i = 0; i < FM; ++i) as[0][i * 4 + wave][lane] = ar[i];
-  __syncthreads();
-  for (int s = 0; s < nst; ++s) {
-    const int nx = min(s + 1, nst - 1);
-#pragma unroll
-    for (int i = 0; i < FM; ++i) ar[i] = ap[i][nx * 2 * (KT / VEC)];
+    for (int i = 0; i < NA; ++i) d[i] = ap[i][min(s, nst - 1) * 2 * (KT / VEC)];
+  };
+  auto load_w = [&](V (&d)[FN][2], int s) {
 #pragma unroll
     for (int j = 0; j < FN; ++j) {
-      wx[j][0] = wp[j][(size_t)nx * 128];
-      wx[j][1] = wp[j][(size_t)nx * 128 + 64];
+      d[j][0] = wp[j][(size_t)min(s, nst - 1) * 128];
+      d[j][1] = wp[j][(size_t)min(s, nst - 1) * 128 + 64];
     }
+  };
+  auto store_a = [&](int buf, const V (&d)[NA]) {
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-      V af[FM];
+    for (int i = 0; i < NA; ++i) as[buf][i * 4 + wave][lane] = d[i];
+  };
+  // s % 4 == B.  A stage's operand reads all go out first (left alone, the scheduler keeps two in
+  // flight and waits for LDS between products), the hand-over of the next stage's activations next.
+  auto stage = [&]<int B>(int s) {
+    V af[2][FM];
 #pragma unroll
-      for (int i = 0; i < FM; ++i) af[i] = as[s & 1][(wm * FM + i) * 2 + kk][lane];
+    for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+      for (int i = 0; i < FM; ++i) af[kk][i] = as[B & 1][i * 2 + kk][lane];
+    __builtin_amdgcn_sched_barrier(0);
+    store_a((B + 1) & 1, ar[(B + 1) % D]);
+    load_a(ar[(B + 1) % D], s + 1 + D);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk)
 #pragma unroll
       for (int i = 0; i < FM; ++i)
 #pragma unroll
-        for (int j = 0; j < FN; ++j) acc[i][j] = VF ? mma(af[i], wc[j][kk], acc[i][j]) : mma(wc[j][kk], af[i], acc[i][j]);
-    }
+        for (int j = 0; j < FN; ++j)
+          acc[i][j] = VF ? mma(af[kk][i], w[B % D][j][kk], acc[i][j]) : mma(w[B % D][j][kk], af[kk][i], acc[i][j]);
+    load_w(w[B % D], s + D);
+    lds_sync();
+  };
+  load_a(ar[0], 0);
 #pragma unroll
-    for (int i = 0; i < FM; ++i) as[(s + 1) & 1][i * 4 + wave][lane] = ar[i];
-#pragma unroll
-    for (int j = 0; j < FN; ++j) {
-      wc[j][0] = wx[j][0];
-      wc[j][1] = wx[j][1];
+  for (int d = 0; d < D; ++d) {
+    load_w(w[d], d);
+    if (d == 0) {
+      store_a(0, ar[0]);
+      load_a(ar[0], D);
+    } else {
+      load_a(ar[d], d);
     }
-    __syncthreads();
+  }
+  lds_sync();
+  for (int s = 0; s < nst; s += 4) {
+    stage.template operator()<0>(s);
+    if (s + 1 < nst) stage.template operator()<1>(s + 1);
+    if (s + 2 < nst) stage.template operator()<2>(s + 2);
+    if (s + 3 < nst) stage.template operator()<3>(s + 3);
   }
 #pragma unroll
   for (int i = 0; i < FM; ++i) {
-    const int mt = m_base + (wm * FM + i) * 16;
+    const int mt = m_base + i * 16;
     const int m = mt + (lane & 15);
     const int mo = m < sp.rows ? row_out(a, sp.first + m) : 0;
 #pragma unroll
     for (int j = 0; j < FN; ++j) {
-      const int nt = ntile * (BN / 16) + wn * FN + j;
+      const int nt = ntile * (BN / 16) + wave * FN + j;
       if (nt >= NT) continue;
-      if (VF)
+      if constexpr (VF)
         dense_store_v<T>(a, mt + 4 * (lane >> 4), nt * 16 + (lane & 15), acc[i][j]);
-      else if (a.epi == TI_DE_LOGITS)
+      else if constexpr (EPI == TI_DE_LOGITS)
         dense_argmax(a, m, sp.rows, nt * 16 + 4 * (lane >> 4), acc[i][j], lane, nt);
       else
-        dense_store<T>(a, sp.batch, m, mo, sp.rows, nt * 16 + 4 * (lane >> 4), acc[i][j]);
+        dense_store<T, EPI>(a, sp.batch, m, mo, sp.rows, nt * 16 + 4 * (lane >> 4), acc[i][j]);
     }
   }
-  if (a.epi == TI_DE_LOGITS && a.step_ctr && id == 0 && tid == 0) *a.step_ctr += a.advance;
+  if (EPI == TI_DE_LOGITS && a.step_ctr && id == 0 && tid == 0) *a.step_ctr += a.advance;
 }
 
-template <class T, int MT>
+template <class T, int MT, int EPI>
 int launch_skinny(const ti_dense_args& a, hipStream_t s) {
   const int NT = (a.N + 15) / 16, y = a.tile_rows ? a.max_tiles : a.batch, nk = a.K / El<T>::KT;
   const int z = a.tile_rows ? 1 : (a.M + 16 * MT - 1) / (16 * MT);
   if (nk >= 32)
-    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 8>), dim3(NT, y, z), dim3(512), 0, s, a);
+    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 8, EPI>), dim3(NT, y, z), dim3(512), 0, s, a);
   else
-    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 4>), dim3(NT, y, z), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((dense_skinny_kernel<T, MT, 4, EPI>), dim3(NT, y, z), dim3(256), 0, s, a);
   TI_LAUNCH_CHECK("dense_skinny_kernel");
   return TI_OK;
 }
 
-template <class T, int BM, int BN, bool VF>
+template <class T, int BM, int BN, int D, int EPI>
 int launch_tile(const ti_dense_args& a, hipStream_t s) {
   const int mt = a.tile_rows ? 1 : (a.M + BM - 1) / BM, nt = (a.N + BN - 1) / BN, per = (mt * nt + 7) / 8;
-  hipLaunchKernelGGL((dense_tile_kernel<T, BM, BN, VF>), dim3(per * 8, a.tile_rows ? a.max_tiles : a.batch), dim3(256), 0, s,
-                     a, mt, nt);
+  hipLaunchKernelGGL((dense_tile_kernel<T, BM, BN, D, EPI>), dim3(per * 8, a.tile_rows ? a.max_tiles : a.batch), dim3(256), 0,
+                     s, a, mt, nt);
   TI_LAUNCH_CHECK("dense_tile_kernel");
   return TI_OK;
 }
 
+// up to 64 rows: as many row tiles per workgroup as still leave two workgroups per CU
+template <class T, int EPI>
+int skinny(const ti_dense_args& a, hipStream_t s) {
+  const long g = (long)((a.N + 15) / 16) * a.batch;
+  const int mt = (a.M + 15) / 16;
+  if (a.tile_rows || mt == 1 || g < 256) return launch_skinny<T, 1, EPI>(a, s);
+  if (mt == 2 || g < 512) return launch_skinny<T, 2, EPI>(a, s);
+  return launch_skinny<T, 4, EPI>(a, s);
+}
+
+// more rows: the largest tile that still gives every CU a workgroup
+template <class T, int EPI>
+int tiled(const ti_dense_args& a, hipStream_t s) {
+  auto wgs = [&](int bm, int bn) { return (long)((a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn) * a.batch; };
+  if (wgs(128, 256) >= 256) return launch_tile<T, 128, 256, 2, EPI>(a, s);
+  if (wgs(128, 128) >= 256) return launch_tile<T, 128, 128, 2, EPI>(a, s);
+  if (wgs(64, 128) >= 256) return launch_tile<T, 64, 128, 4, EPI>(a, s);
+  return launch_tile<T, 64, 64, 4, EPI>(a, s);
+}
+
 template <class T>
 int dispatch_dense(const ti_dense_args& a, hipStream_t s) {
-  if (a.epi == TI_DE_VFRAG) return launch_tile<T, 128, 64, true>(a, s);
-  if (a.epi == TI_DE_KFRAG) return launch_tile<T, 128, 64, false>(a, s);
-  if (a.tile_rows == 1 || a.tile_rows == 16) return launch_skinny<T, 1>(a, s);
-  if (a.tile_rows == 64) return launch_tile<T, 64, 64, false>(a, s);
-  // up to 64 rows: as many row tiles per workgroup as still leave two workgroups per CU
-  if (a.M <= 64) {
-    const long g = (long)((a.N + 15) / 16) * a.batch;
-    const int mt = (a.M + 15) / 16;
-    if (mt == 1 || g < 256) return launch_skinny<T, 1>(a, s);
-    if (mt == 2 || g < 512) return launch_skinny<T, 2>(a, s);
-    return launch_skinny<T, 4>(a, s);
+  const bool few = a.tile_rows == 1 || a.tile_rows == 16 || (!a.tile_rows && a.M <= 64);
+  switch (a.epi) {
+    case TI_DE_F32: return few ? skinny<T, TI_DE_F32>(a, s) : tiled<T, TI_DE_F32>(a, s);
+    case TI_DE_ROPE: return few ? skinny<T, TI_DE_ROPE>(a, s) : tiled<T, TI_DE_ROPE>(a, s);
+    case TI_DE_LOGITS: return few ? skinny<T, TI_DE_LOGITS>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_LOGITS>(a, s);
+    case TI_DE_GATE: return few ? skinny<T, TI_DE_GATE>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_GATE>(a, s);
+    case TI_DE_SWIGLU:
+      if (few) return skinny<T, TI_DE_SWIGLU>(a, s);
+      return launch_tile<T, 64, 256, 2, TI_DE_SWIGLU>(a, s);
+    case TI_DE_T:
+      if (few) return skinny<T, TI_DE_T>(a, s);
+      if (a.tile_rows) return launch_tile<T, 64, 256, 2, TI_DE_T>(a, s);
+      return launch_tile<T, 64, 64, 4, TI_DE_T>(a, s);
+    // (every row of a 128-row tile is written by the fragment epilogues)
+    case TI_DE_KFRAG: return launch_tile<T, 128, 128, 2, TI_DE_KFRAG>(a, s);
+    default: return launch_tile<T, 128, 128, 2, TI_DE_VFRAG>(a, s);
   }
-  // the largest tile that still gives every CU a workgroup
-  auto wgs = [&](int bm, int bn) { return (long)((a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn) * a.batch; };
-  if (wgs(128, 128) >= 256) return launch_tile<T, 128, 128, false>(a, s);
-  if (wgs(128, 64) >= 256) return launch_tile<T, 128, 64, false>(a, s);
-  return launch_tile<T, 64, 64, false>(a, s);
 }
 
 template <class T>
@@ -418,7 +469,7 @@ extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
     return ti_set_error(TI_ERR_ARG, "ti_dense: K %d / lda %d not padded", a->K, a->lda);
   if ((!a->tile_rows && !a->rows_in && a->lda < a->K) || a->batch > 65535)
     return ti_set_error(TI_ERR_ARG, "ti_dense: lda %d < K %d or batch %d", a->lda, a->K, a->batch);
-  if (a->tile_rows && ((a->tile_rows != 1 && a->tile_rows != 16 && a->tile_rows != 64) || a->max_tiles < 1 || a->max_tiles > 65535 ||
+  if (a->tile_rows && (a->epi == TI_DE_F32 || (a->tile_rows != 1 && a->tile_rows != 16 && a->tile_rows != 64) || a->max_tiles < 1 || a->max_tiles > 65535 ||
                        a->batch != 1 || a->epi > TI_DE_SWIGLU || (a->rows_in && a->row_div < 1) ||
                        !a->tiles ||
                        (a->tile_rows == 1 ? a->rows_in || a->rows_out : !a->n_tiles)))
