@@ -74,7 +74,7 @@ typedef struct ti_dense_args {
   int32_t* step_ctr;           /* TI_DE_LOGITS, nullable: += advance once                    */
   int32_t advance;
   /* grouped products (experts): tile t covers entries [first, first + rows) of expert e's list */
-  int32_t tile_rows;           /* 0 = not grouped; 16 or 64: rows a tile holds at most; 1: tile t is
+  int32_t tile_rows;           /* 0 = not grouped; 16, 64 or 128: rows a tile holds; 1: tile t is
                                   entry t alone, of expert tiles[t]                           */
   int32_t max_tiles;           /* tiles launched; those at or past *n_tiles return at once   */
   const int32_t* tiles;        /* device [max_tiles][4] = expert, first, rows, -             */

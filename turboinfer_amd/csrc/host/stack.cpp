@@ -595,7 +595,7 @@ int StackModel::experts(const StackLayer& L, int M) {
     g.tiles = idx_;
     if (!routed) TI_TRY(ti_route(&ra, s_));
   } else {
-    ra.tile_rows = M <= 64 ? 16 : 64;
+    ra.tile_rows = M <= 64 ? 16 : (long)M * k.top >= 96L * k.experts ? 128 : 64;
     TI_TRY(ti_route(&ra, s_));
     g.tile_rows = ra.tile_rows;
     g.max_tiles = ti_route_max_tiles(M, k.experts, k.top, ra.tile_rows);

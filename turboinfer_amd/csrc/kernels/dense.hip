@@ -226,14 +226,26 @@ __global__ __launch_bounds__(256, BM * BN > 16384 ? 1 : 2) void dense_tile_kerne
   constexpr int KT = El<T>::KT, VEC = El<T>::VEC, FM = BM / 16, FN = BN / 64, NA = BM / 32;
   constexpr bool VF = EPI == TI_DE_VFRAG;
   __shared__ V as[2][FM * 2][64];
-  DenseSpan sp;
-  if (!dense_span(a, blockIdx.y, sp, sizeof(T))) return;
-  // consecutive workgroups go to the 8 XCDs in turn: give each XCD a contiguous run of tiles, row
-  // tiles fastest, so the weight columns a run shares stay in that XCD's L2
-  const int total = m_tiles * n_tiles, per = (total + 7) >> 3;
+  // Consecutive workgroups go to the 8 XCDs in turn; each XCD gets a contiguous run of the work list,
+  // ordered so that neighbours share weight columns (its L2 holds them once): row tiles fastest, for
+  // grouped products 4 tiles (mostly one expert's) fastest, then the columns.
+  const int list = a.tile_rows ? (*a.n_tiles + 3) / 4 * 4 * n_tiles : m_tiles * n_tiles, per = (list + 7) >> 3;
   const int id = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
-  if (id >= total) return;
-  const int mtile = id % m_tiles, ntile = id / m_tiles, m_base = mtile * BM;
+  if ((int)(blockIdx.x >> 3) >= per || id >= list) return;
+  int mtile, ntile, y;
+  if (a.tile_rows) {
+    const int b = id / (4 * n_tiles), r = id - b * 4 * n_tiles;
+    mtile = 0;
+    ntile = r >> 2;
+    y = b * 4 + (r & 3);
+  } else {
+    mtile = id % m_tiles;
+    ntile = id / m_tiles;
+    y = blockIdx.y;
+  }
+  const int m_base = mtile * BM;
+  DenseSpan sp;
+  if (!dense_span(a, y, sp, sizeof(T))) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int nk = a.K / KT, nst = nk >> 1, NT = (a.N + 15) >> 4;
   const V* ap[NA];
@@ -345,8 +357,9 @@ int launch_skinny(const ti_dense_args& a, hipStream_t s) {
 
 template <class T, int BM, int BN, int D, int EPI>
 int launch_tile(const ti_dense_args& a, hipStream_t s) {
-  const int mt = a.tile_rows ? 1 : (a.M + BM - 1) / BM, nt = (a.N + BN - 1) / BN, per = (mt * nt + 7) / 8;
-  hipLaunchKernelGGL((dense_tile_kernel<T, BM, BN, D, EPI>), dim3(per * 8, a.tile_rows ? a.max_tiles : a.batch), dim3(256), 0,
+  const int mt = (a.M + BM - 1) / BM, nt = (a.N + BN - 1) / BN;
+  const int list = a.tile_rows ? (a.max_tiles + 3) / 4 * 4 * nt : mt * nt;
+  hipLaunchKernelGGL((dense_tile_kernel<T, BM, BN, D, EPI>), dim3((list + 7) / 8 * 8, a.tile_rows ? 1 : a.batch), dim3(256), 0,
                      s, a, mt, nt);
   TI_LAUNCH_CHECK("dense_tile_kernel");
   return TI_OK;
@@ -362,14 +375,21 @@ int skinny(const ti_dense_args& a, hipStream_t s) {
   return launch_skinny<T, 4, EPI>(a, s);
 }
 
-// more rows: the largest tile that still gives every CU a workgroup
+// More rows: the tile whose rounds over the 256 CUs cost least, by the time of one round of each tile
+// (us at K 2048, measured).
 template <class T, int EPI>
 int tiled(const ti_dense_args& a, hipStream_t s) {
-  auto wgs = [&](int bm, int bn) { return (long)((a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn) * a.batch; };
-  if (wgs(128, 256) >= 256) return launch_tile<T, 128, 256, 2, EPI>(a, s);
-  if (wgs(128, 128) >= 256) return launch_tile<T, 128, 128, 2, EPI>(a, s);
-  if (wgs(64, 128) >= 256) return launch_tile<T, 64, 128, 4, EPI>(a, s);
-  return launch_tile<T, 64, 64, 4, EPI>(a, s);
+  auto cost = [&](int bm, int bn, float us) {
+    const long wgs = (long)((a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn) * a.batch;
+    return (float)((wgs + 255) / 256) * us;
+  };
+  const float c[4] = {cost(128, 256, 37.f), cost(64, 256, 27.f), cost(64, 128, 15.f), cost(32, 128, 11.5f)};
+  switch (std::min_element(c, c + 4) - c) {
+    case 0: return launch_tile<T, 128, 256, 2, EPI>(a, s);
+    case 1: return launch_tile<T, 64, 256, 2, EPI>(a, s);
+    case 2: return launch_tile<T, 64, 128, 4, EPI>(a, s);
+    default: return launch_tile<T, 32, 128, 4, EPI>(a, s);
+  }
 }
 
 template <class T>
@@ -382,9 +402,11 @@ int dispatch_dense(const ti_dense_args& a, hipStream_t s) {
     case TI_DE_GATE: return few ? skinny<T, TI_DE_GATE>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_GATE>(a, s);
     case TI_DE_SWIGLU:
       if (few) return skinny<T, TI_DE_SWIGLU>(a, s);
+      if (a.tile_rows == 128) return launch_tile<T, 128, 256, 2, TI_DE_SWIGLU>(a, s);
       return launch_tile<T, 64, 256, 2, TI_DE_SWIGLU>(a, s);
     case TI_DE_T:
       if (few) return skinny<T, TI_DE_T>(a, s);
+      if (a.tile_rows == 128) return launch_tile<T, 128, 256, 2, TI_DE_T>(a, s);
       if (a.tile_rows) return launch_tile<T, 64, 256, 2, TI_DE_T>(a, s);
       return launch_tile<T, 64, 64, 4, TI_DE_T>(a, s);
     // (every row of a 128-row tile is written by the fragment epilogues)
@@ -469,9 +491,9 @@ extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
     return ti_set_error(TI_ERR_ARG, "ti_dense: K %d / lda %d not padded", a->K, a->lda);
   if ((!a->tile_rows && !a->rows_in && a->lda < a->K) || a->batch > 65535)
     return ti_set_error(TI_ERR_ARG, "ti_dense: lda %d < K %d or batch %d", a->lda, a->K, a->batch);
-  if (a->tile_rows && (a->epi == TI_DE_F32 || (a->tile_rows != 1 && a->tile_rows != 16 && a->tile_rows != 64) || a->max_tiles < 1 || a->max_tiles > 65535 ||
-                       a->batch != 1 || a->epi > TI_DE_SWIGLU || (a->rows_in && a->row_div < 1) ||
-                       !a->tiles ||
+  const bool rows_ok = a->tile_rows == 1 || a->tile_rows == 16 || a->tile_rows == 64 || a->tile_rows == 128;
+  if (a->tile_rows && (a->epi == TI_DE_F32 || a->epi > TI_DE_SWIGLU || !rows_ok || a->max_tiles < 1 || a->max_tiles > 65535 ||
+                       a->batch != 1 || (a->rows_in && a->row_div < 1) || !a->tiles ||
                        (a->tile_rows == 1 ? a->rows_in || a->rows_out : !a->n_tiles)))
     return ti_set_error(TI_ERR_ARG, "ti_dense: grouped arguments");
   if (!a->tile_rows && (a->rows_in || a->rows_out)) return ti_set_error(TI_ERR_ARG, "ti_dense: row lists need grouped tiles");
