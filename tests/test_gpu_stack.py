@@ -165,6 +165,22 @@ def test_long_prompt_over_chunks(ti):
     close(step, ref[2600:], "next token")
 
 
+def test_long_prompt_of_many_heads(ti):
+    """Enough row blocks for the 32-row attention tiles, value sizes of 4, 8 and 16 tiles (the last in
+    16-row tiles), in one portion and in two that start inside a key block."""
+    from stack_models import config, mixer
+    cfg = config(60, 40, [(mixer(17, 20, 12, 20, 24, 28), None), (mixer(18, 36, 6, 68, 20, 40), None),
+                          (mixer(17, 12, 8, 132, 16, 24), None)])
+    w = random_weights(cfg, 11)
+    t = tokens(cfg, 1030, 12)
+    ref = S.forward(t, f64(w), cfg)
+    e = engine(ti, cfg, w, max_seq=1030, max_batch=2)
+    close(e.prefill(0, t, 0, range(len(t))), ref, "whole")
+    e.prefill(1, t[:21])
+    close(e.prefill(1, t[21:], 21, range(len(t) - 21)), ref[21:], "second portion")
+    e.close()
+
+
 def needle_model():
     """One layer, one head of width 8, whose attention weight is decided by the token's embedding: token
     1 is the query, token 2 the key it looks for (score far above the others), token 0 the rest."""

@@ -9,7 +9,8 @@
 //     the MFMA columns, the weighted sum a second one over the latent part.  Keys are split over
 //     workgroups (splits) and over the waves of each.
 //   * latent_prefill_kernel: prompt chunks, keys and values expanded per head into MFMA fragments
-//     (dense.hip TI_DE_KFRAG / TI_DE_VFRAG); a wave owns 16 or 32 query rows of one head.
+//     (dense.hip TI_DE_KFRAG / TI_DE_VFRAG); a workgroup owns 16 or 32 query rows of one head, its waves
+//     split the keys.
 // Scores, softmax and sums are fp32; the softmax denominator holds exp(sink) of the head once.
 #include <algorithm>
 
@@ -361,25 +362,27 @@ __device__ __forceinline__ void pv_block(f32x4& acc, const f32x4* vf, const f32x
   for (int t = 0; t < 4; ++t) acc = mma(vf[t], p[t], acc);
 }
 
-// Grid (row blocks of 4 * 16 * MQ, heads); a wave owns 16 * MQ rows.  The last row blocks (most keys)
-// start first.
+// A workgroup owns 16 * MQ rows of one head; its 4 waves take the 64-key blocks in turn and merge their
+// sums at the end.  Each XCD gets a contiguous run of the (head, row block) list, so a head's keys and
+// values stay in one L2; a head's last row blocks (most keys) start first.
 template <class T, int MQ, int NV>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(const ti_latent_prefill_args a) {
+__global__ __launch_bounds__(256, NV > 8 ? 2 : 3) void latent_prefill_kernel(const ti_latent_prefill_args a, int row_blocks) {
   typedef typename El<T>::V V;
   constexpr int KT = El<T>::KT, VEC = El<T>::VEC, VB = 64 / KT;
   extern __shared__ char lds[];
-  const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
-  const int row0 = ((int)(gridDim.x - 1 - blockIdx.x) * 4 + wave) * 16 * MQ;
-  if (row0 >= a.M) return;   // (no barrier below: waves are independent)
+  __shared__ float ml[2][4][MQ * 16];   // the waves' maxima, sums
+  const int list = row_blocks * a.heads, per = (list + 7) >> 3;
+  const int id = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
+  if ((int)(blockIdx.x >> 3) >= per || id >= list) return;
+  const int h = id / row_blocks, row0 = (row_blocks - 1 - id % row_blocks) * 16 * MQ;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
   const int dkt = a.dim_p / KT, rkt = a.rot_p / KT, nkt = dkt + rkt, cw = a.lat_p + a.rot_p, nv = a.vdim_p >> 4;
-  V* qf = (V*)lds + (size_t)wave * nkt * MQ * 64;
-  for (int kt = 0; kt < nkt; ++kt)
-#pragma unroll
-    for (int q = 0; q < MQ; ++q) {
-      const int m = min(row0 + q * 16 + col, a.M - 1);
-      qf[(kt * MQ + q) * 64 + lane] =
-          *(const V*)((const T*)a.q + ((size_t)m * a.heads + h) * (a.dim_p + a.rot_p) + kt * KT + g * VEC);
-    }
+  V* qf = (V*)lds;
+  for (int i = wave; i < nkt * MQ; i += 4) {
+    const int m = min(row0 + i % MQ * 16 + col, a.M - 1);
+    qf[i * 64 + lane] = *(const V*)((const T*)a.q + ((size_t)m * a.heads + h) * (a.dim_p + a.rot_p) + i / MQ * KT + g * VEC);
+  }
+  __syncthreads();
   const V* kf = (const V*)a.kfrag + (size_t)h * a.key_blocks * dkt * 64 + lane;
   const V* vf = (const V*)a.vfrag + (size_t)h * nv * (a.key_blocks * 16 / KT) * 64 + lane;
   const V* rp = (const V*)((const T*)a.cache + a.lat_p + (size_t)col * cw) + g;
@@ -387,13 +390,13 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const ti_latent_pre
   float mr[MQ], lr[MQ];
 #pragma unroll
   for (int q = 0; q < MQ; ++q) {
-    mr[q] = a.sink[h];   // the sink: weight exp(sink - max), no value
-    lr[q] = g == 0 ? 1.0f : 0.0f;
+    mr[q] = a.sink[h];   // the sink: weight exp(sink - max), no value; counted by one wave
+    lr[q] = wave == 0 && g == 0 ? 1.0f : 0.0f;
 #pragma unroll
     for (int v = 0; v < NV; ++v) o[q][v] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
-  const int last = a.pos0 + min(row0 + 16 * MQ, a.M) - 1;   // the wave's last position
-  for (int k0 = 0; k0 <= last; k0 += 64) {
+  const int last = a.pos0 + min(row0 + 16 * MQ, a.M) - 1;   // the rows' last position
+  for (int k0 = wave * 64; k0 <= last; k0 += 256) {
     f32x4 s[MQ][4];
 #pragma unroll
     for (int q = 0; q < MQ; ++q)
@@ -461,20 +464,44 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const ti_latent_pre
   }
 #pragma unroll
   for (int q = 0; q < MQ; ++q) {
-    const int m = row0 + q * 16 + col;
     float l = lr[q];
     l += lane_xor<16>(l);
     l += lane_xor<32>(l);
-    if (m >= a.M) continue;
-    const float sc = a.gate[(size_t)m * a.heads + h] / l;
-    T* out = (T*)a.out + (size_t)m * a.ldo + (size_t)h * a.vdim;
+    if (lane < 16) {
+      ml[0][wave][q * 16 + col] = mr[q];
+      ml[1][wave][q * 16 + col] = l;
+    }
+  }
+  __syncthreads();   // (and the last reads of qf)
+  f32x4* ob = (f32x4*)lds;   // [4][NV][64]
 #pragma unroll
-    for (int v = 0; v < NV; ++v)
+  for (int q = 0; q < MQ; ++q) {
+    const int m = row0 + q * 16 + col;
+    float mx = ml[0][0][q * 16 + col], l = 0.0f;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = v * 16 + 4 * g + r;
-        if (d < a.vdim) out[d] = (T)(o[q][v][r] * sc);
+    for (int w = 1; w < 4; ++w) mx = fmaxf(mx, ml[0][w][q * 16 + col]);
+#pragma unroll
+    for (int w = 0; w < 4; ++w) l += ml[1][w][q * 16 + col] * expf(ml[0][w][q * 16 + col] - mx);
+    const float f = expf(mr[q] - mx);
+#pragma unroll
+    for (int v = 0; v < NV; ++v) ob[(wave * NV + v) * 64 + lane] = o[q][v] * f;
+    __syncthreads();
+    if (m < a.M) {
+      const float sc = a.gate[(size_t)m * a.heads + h] / l;
+      T* out = (T*)a.out + (size_t)m * a.ldo + (size_t)h * a.vdim;
+#pragma unroll
+      for (int v0 = 0; v0 < NV; v0 += 4) {
+        const int v = v0 + wave, d = v * 16 + 4 * g;
+        if (d >= a.vdim) continue;
+        f32x4 x = ob[v * 64 + lane];
+#pragma unroll
+        for (int w = 1; w < 4; ++w) x += ob[(w * NV + v) * 64 + lane];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (d + r < a.vdim) out[d + r] = (T)(x[r] * sc);
       }
+    }
+    if (q + 1 < MQ) __syncthreads();
   }
 }
 
@@ -498,12 +525,13 @@ int launch_decode(const ti_latent_attn_args& a, hipStream_t s) {
 template <class T>
 int launch_prefill(const ti_latent_prefill_args& a, hipStream_t s) {
   const int nkt = (a.dim_p + a.rot_p) / El<T>::KT, nv = a.vdim_p / 16;
-  const bool two = (size_t)nkt * 2 * 1024 * 4 <= 81920 && nv <= 8 && a.M > 64;
-  const int mq = two ? 2 : 1;
-  const size_t lds = (size_t)nkt * mq * 1024 * 4;
+  // 32-row blocks where they still give every CU two workgroups
+  const bool two = nkt <= 32 && nv <= 8 && (long)((a.M + 31) / 32) * a.heads >= 512;
+  const int mq = two ? 2 : 1, rb = (a.M + 16 * mq - 1) / (16 * mq), nvp = nv <= 4 ? 4 : nv <= 8 ? 8 : 16;
+  const size_t lds = (size_t)std::max(nkt * mq, 4 * nvp) * 1024;
   if (lds > 131072) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_latent_attn_prefill: head of %d + %d dims", a.dim_p, a.rot_p);
-  const dim3 grid((a.M + 64 * mq - 1) / (64 * mq), a.heads), blk(256);
-#define TI_LP(MQ, NV) hipLaunchKernelGGL((latent_prefill_kernel<T, MQ, NV>), grid, blk, lds, s, a)
+  const dim3 grid((unsigned)(((long)rb * a.heads + 7) / 8 * 8)), blk(256);
+#define TI_LP(MQ, NV) hipLaunchKernelGGL((latent_prefill_kernel<T, MQ, NV>), grid, blk, lds, s, a, rb)
   if (two && nv <= 4) TI_LP(2, 4);
   else if (two) TI_LP(2, 8);
   else if (nv <= 4) TI_LP(1, 4);
