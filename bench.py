@@ -186,7 +186,7 @@ def stack_bench(args) -> int:
     model at equal size: the same width, vocabulary, layer runs, heads of 128, and a dense feed-forward as
     wide as the experts a token uses, fp16 weights (as many bytes per weight).  Both in this process, on
     one GPU, timed in turn: decode is the replayed step graph at position kv - 1, prefill one prompt of
-    --prompt tokens to its last logits, each the best of --steps / 3 repetitions."""
+    --stack-prompts tokens to its last logits, each the best of --steps / 3 repetitions."""
     import numpy as np
     import turboinfer_amd as T
     T.init(0)
