@@ -42,10 +42,18 @@ typedef struct ti_engine_config {
 
 /* ---------------------------------------------------------------- layer-stack models
  * A model given layer by layer (config.json "layers"), each with its own sizes, run in order with an
- * optional looped range (config.json "loop").  Every loop pass of a layer is a run with its own cache.
- * Each sublayer is x += post_norm(f(pre_norm(x))). */
-enum ti_mixer { TI_MIX_LATENT = 0 };        /* latent attention (ti_stack.h)                     */
-enum ti_mlp { TI_MLP_NONE = 0, TI_MLP_MOE = 1 };
+ * optional looped range (config.json "loop").  Every loop pass of a layer is a run with its own cache or
+ * state.  Each sublayer is x += post_norm(f(pre_norm(x))) or x += post_norm(f(x)) (ti_norm_place). */
+enum ti_mixer {
+  TI_MIX_LATENT = 0,       /* latent attention (ti_stack.h)                                          */
+  TI_MIX_GQA = 1,          /* grouped-query attention: norms of the whole query and key projections,
+                              a gate per output element                                              */
+  TI_MIX_SSD = 2,          /* Mamba-2: short convolution, state-space recurrence, gate before the norm */
+  TI_MIX_RGLRU = 3         /* Griffin's recurrent block: short convolution, real-gated linear
+                              recurrent unit, GELU branch                                            */
+};
+enum ti_mlp { TI_MLP_NONE = 0, TI_MLP_MOE = 1, TI_MLP_DENSE = 2 /* down(gelu(up x)), exact GELU */ };
+enum ti_norm_place { TI_PLACE_SANDWICH = 0, TI_PLACE_POST = 1 };
 typedef struct ti_stack_layer {
   int32_t mixer;
   int32_t heads, dim, rot_dim, vdim, q_rank, kv_rank;
@@ -53,6 +61,15 @@ typedef struct ti_stack_layer {
   float rot_base, scale;
   int32_t mlp;
   int32_t experts, top, ff;
+  /* TI_MIX_GQA: heads, dim, vdim, scale above; sink: one is added to the softmax's denominator;
+   * queries times 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) (temp_every 0: not) */
+  int32_t kv_heads;
+  int32_t kv_shared, kv_from;   /* kv_shared: keys and values are those of layer kv_from (< this one) */
+  int32_t sink_one;
+  float temp_coef, temp_every;
+  /* TI_MIX_SSD: heads, vdim above; TI_MIX_RGLRU: mix_width, blocks; both: conv taps */
+  int32_t conv, state, groups, norm_groups;
+  int32_t mix_width, blocks;
 } ti_stack_layer;
 typedef struct ti_stack_config {
   int32_t vocab, width, layers;
@@ -60,6 +77,11 @@ typedef struct ti_stack_config {
   float eps, emb_scale;
   int32_t dtype;           /* ti_dtype: bf16 weights / activations / cache, or everything fp32       */
   int32_t max_seq, max_batch, device;
+  int32_t norm_kind;       /* ti_norm_kind of every norm                                             */
+  int32_t norm_place;
+  int32_t bigram_buckets;  /* > 0: a bigram table is added to the embedding (ti_hip.h ti_step_args)  */
+  int32_t bigram_mul_prev, bigram_mul_cur;
+  int32_t sinusoid;        /* nonzero: a sinusoidal position vector is added too                     */
 } ti_stack_config;
 
 enum ti_slot {
@@ -83,11 +105,15 @@ int ti_engine_set_weight(ti_engine* e, const char* name, const float* data, int 
 /* Build an engine from a model folder (config.json + model.safetensors): the architecture key of
  * config.json picks the model class.  max_seq KV slots per stream, max_batch streams. */
 int ti_engine_load(const char* dir, int dtype, int max_seq, int max_batch, int device, ti_engine** out);
+/* A layer-stack engine of a config.json text, its weights not set. */
+int ti_engine_create_config(const char* config_json, int dtype, int max_seq, int max_batch, int device, ti_engine** out);
 /* Sizes of an engine (a layer-stack engine reports runs as layers and its first layer's heads). */
 int ti_engine_describe(ti_engine* e, ti_engine_config* out);
 /* Prompt tokens [0, n) of stream `slot` at positions pos0 + i through the prefill path; want lists
  * n_want places (ascending) whose next-token logits [n_want][vocab] are returned.  layers_out
- * (nullable, layer-stack engines): the residual after every layer run, [runs][n][width]. */
+ * (nullable, layer-stack engines): the residual after every layer run, [runs][n][width].
+ * A model with recurrent layers goes on only where a slot's state stands: pos0 is 0 (the state starts
+ * anew) or the number of tokens the slot has run; the same holds for steps and generation. */
 int ti_engine_prefill(ti_engine* e, int slot, const int32_t* tokens, int n, int pos0, const int32_t* want, int n_want,
                       float* logits, float* layers_out);
 int ti_engine_get_stream(ti_engine* e, void** stream);
@@ -196,6 +222,9 @@ int ti_engine_set_qkv_attn(ti_engine* e, int on, int* active);
 /* One decode step: token[s] at position pos[s] for each stream; logits [n][vocab] to host
  * (used for non-greedy sampling and per-step parity). */
 int ti_engine_step(ti_engine* e, int n_streams, const int32_t* tokens, const int32_t* pos, float* logits);
+/* The same over chosen stream slots (layer-stack engines): row s is slot slots[s], each at most once; the
+ * other slots' caches and states stay as they are. */
+int ti_engine_step_slots(ti_engine* e, int n, const int32_t* slots, const int32_t* tokens, const int32_t* pos, float* logits);
 
 /* reference_compat step (compat engines): placeholder row offset, logits [vocab] to host. */
 int ti_engine_compat_step(ti_engine* e, int placeholder_offset, float* logits);

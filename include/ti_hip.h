@@ -406,6 +406,20 @@ typedef struct ti_step_args {
   int32_t emb_kind;                  /* 0: fp16 table (above); 1: bf16, 2: fp32, both scaled by emb_scale */
   float emb_scale;
   float* h0;                         /* nullable [M][hidden]: a second copy of the embedding row (emb_kind > 0) */
+  /* emb_kind > 0: further terms of the row, each nullable.
+   * bigram: a table of the same element type, row (previous token * mul_prev + token * mul_cur) mod
+   * buckets, row `buckets` for a sequence's first token.  hist [slots][hist_ld] records the tokens by
+   * position (the previous token is read there, in a chunk's later rows from in_tokens).
+   * pe_hi / pe_lo: sinusoidal position vectors in two tables [.][pe_ld], of the positions 256 k and
+   * 0..255, sine at even and cosine at odd entries. */
+  const void* bigram;
+  int32_t buckets, mul_prev, mul_cur, hist_ld;
+  int32_t* hist;
+  const int32_t* slot;               /* nullable [M]: stream slot of row m (NULL: m) */
+  int32_t chunk, slot0;              /* chunk: rows are consecutive positions of slot slot0 */
+  const float* pe_hi;
+  const float* pe_lo;
+  int32_t pe_ld;
 } ti_step_args;
 int ti_step_begin(const ti_step_args* a, ti_stream_t s);
 

@@ -48,9 +48,18 @@ enum ti_dense_epi {
   TI_DE_LOGITS,      /* out fp32 + greedy argmax keys (ti_hip.h TI_EPI_LOGITS_ARGMAX)        */
   TI_DE_KFRAG,       /* rows are keys, columns (head, head_w): key fragments of every head,
                         out T [head][key / 16][head_w / KT][64][VEC]                         */
-  TI_DE_VFRAG        /* rows are keys, columns (head, head_w): transposed value fragments,
+  TI_DE_VFRAG,       /* rows are keys, columns (head, head_w): transposed value fragments,
                         out T [head][head_w / 16][key / KT][64][VEC] (ti_latent_attn_prefill) */
+  TI_DE_ACT,         /* v += add[n] (nullable); columns n < act_cols through `act`; columns n < t_cols
+                        to out T [m][n], the others to out2 fp32 [m][n - t_cols]             */
+  TI_DE_LRU          /* gates of a real-gated linear recurrent unit, one batch per diagonal block:
+                        columns (2j, 2j + 1) = (recurrence, input) gate of the block's channel j.
+                        log a = -sigmoid(r) * lru_rate, b = sqrt(1 - a^2) * sigmoid(i) * u;
+                        lru_state NULL: out fp32 [m][channel][2] = (a, b); else the step itself:
+                        S = a S + b in the row's slot (S = 0 before position 0) and
+                        out T [m][channel] = S * lru_y[m][channel]                           */
 };
+enum ti_act { TI_ACT_NONE = 0, TI_ACT_GELU_TANH, TI_ACT_GELU_ERF };
 
 typedef struct ti_dense_args {
   const void* w;               /* fragment-ordered weights                                   */
@@ -82,6 +91,16 @@ typedef struct ti_dense_args {
   const int32_t* rows_in;      /* entry p reads activation row (rows_in ? rows_in[p] : p) / row_div */
   const int32_t* rows_out;     /* nullable: entry p writes output row rows_out[p]            */
   int32_t row_div;
+  /* TI_DE_ACT */
+  int32_t act, act_cols, t_cols, ld2;
+  float* out2;
+  /* TI_DE_LRU: batch b's columns are channels [b * N / 2, +N / 2); u is the product's own activation
+   * row (element [m][b * a_batch + j] of `a`), add [batch * N] the gates' biases in column order */
+  const float* lru_rate;       /* [channels] 8 * softplus(lambda)                            */
+  float* lru_state;            /* nullable [slots][channels]                                 */
+  const void* lru_y;           /* T [M][lru_ldy]                                             */
+  int32_t lru_ldy;
+  const int32_t* slot;         /* nullable [M]: stream slot of row m (NULL: m)               */
 } ti_dense_args;
 int ti_dense(const ti_dense_args* a, ti_stream_t s);
 size_t ti_dense_args_bytes(void);
@@ -90,7 +109,7 @@ size_t ti_dense_args_bytes(void);
  * One row per workgroup:
  *   y' = post_w ? norm(y; post_w, post_b) : y           (y: fp32 rows, or the weighted expert outputs
  *   x  = x + y'                                          sum_k part_w[m][k] * parts[m * top + k])
- *   xn = T(norm(x; w, b))  and / or  cat = T([x ; x0])
+ *   xn = T(norm(x; w, b)) (w NULL: T(x))  and / or  cat = T([x ; x0])
  * Any of the three parts may be absent.  kind 0: layer norm (x - mean) / sqrt(var + eps) * w + b;
  * kind 1: RMS norm x / sqrt(mean(x^2) + eps) * w (b ignored). */
 enum ti_norm_kind { TI_NORM_LAYER = 0, TI_NORM_RMS = 1 };
@@ -101,9 +120,9 @@ typedef struct ti_rownorm_args {
   const float* part_w;         /* [M][top]                                                   */
   const float* post_w;
   const float* post_b;
-  const float* w;              /* nullable: no xn                                            */
+  const float* w;              /* nullable: xn without a norm                                */
   const float* b;
-  void* xn;                    /* T [M][ldn]                                                 */
+  void* xn;                    /* nullable T [M][ldn]                                        */
   const float* x0;             /* with cat: [M][H]                                           */
   void* cat;                   /* nullable T [M][ldc]: [x ; x0]                              */
   float eps;
@@ -159,6 +178,7 @@ typedef struct ti_latent_prep_args {
   float* gate;
   float eps;
   int32_t dtype;
+  const int32_t* slot;         /* nullable [M]: stream slot of row m (NULL: m)               */
 } ti_latent_prep_args;
 int ti_latent_prep(const ti_latent_prep_args* a, ti_stream_t s);
 
@@ -185,6 +205,7 @@ typedef struct ti_latent_attn_args {
   void* part_o;
   float* part_ml;
   int32_t M, heads, lat_p, rot_p, splits, seq_p, dtype;
+  const int32_t* slot;         /* nullable [M]: stream slot of row m (NULL: m)               */
 } ti_latent_attn_args;
 int ti_latent_attn_decode(const ti_latent_attn_args* a, ti_stream_t s);
 /* Merge of the splits, value up-projection and head gate: out T [M][ldo], head h's vdim values at
@@ -217,6 +238,137 @@ typedef struct ti_latent_prefill_args {
   int32_t M, pos0, heads, dim_p, rot_p, lat_p, vdim, vdim_p, key_blocks, ldo, dtype;
 } ti_latent_prefill_args;
 int ti_latent_attn_prefill(const ti_latent_prefill_args* a, ti_stream_t s);
+
+/* ------------------------------------------------------------------- grouped-query attention
+ * A stream slot's cache holds, per key/value head, blocks of 64 positions, each a run of MFMA fragments:
+ *   [key tile 4][dim_p / KT][64][VEC] keys, then [vdim_p / 16][64 / KT][64][VEC] values, transposed
+ * (value fragment element t * 4 + r of lane group g is position t * 16 + 4 g + r of its KT span).
+ * dim_p = dim rounded up to KT, vdim_p to 16; ti_gqa_block_elems elements a block.
+ *
+ * ti_gqa_prep: per row, from the fused projection a32 [M][lda] fp32 (queries at 0, keys at k_off, values
+ * at v_off; k_off < 0: no keys and values, the layer reads another's cache):
+ *   q T [M][heads][dim_p] = rms_norm(all query rows; q_w) * (q_scale ? q_scale[pos] : 1)
+ *   cache position pos[m] = rms_norm(all key rows; k_w), values. */
+typedef struct ti_gqa_prep_args {
+  const float* a32;
+  int32_t lda, M, heads, kv_heads, dim, vdim, k_off, v_off;
+  const float* q_w;
+  const float* k_w;
+  const float* q_scale;        /* nullable [position]                                        */
+  const int32_t* pos;
+  const int32_t* slot;         /* nullable [M]: stream slot of row m (NULL: m)               */
+  void* q;
+  void* cache;
+  int64_t slot_stride;         /* elements; 0: all rows share one slot (prompt chunk)        */
+  int32_t seq_p;               /* positions a slot holds, a multiple of 64                   */
+  float eps;
+  int32_t dtype;
+} ti_gqa_prep_args;
+int ti_gqa_prep(const ti_gqa_prep_args* a, ti_stream_t s);
+int ti_gqa_block_elems(int dtype, int dim, int vdim);
+
+/* Attention of rows [0, M) over cache positions [0, pos[m]] of their slots: scores * scale, softmax whose
+ * denominator also holds exp(sink[h]) (sink NULL: not), values, times sigmoid(gate[m][h * vdim + d])
+ * (gate NULL: 1); out T [M][ldo].  Query head h reads key/value head h / (heads / kv_heads).
+ * ti_gqa_decode: any rows; keys split over `splits` (ti_gqa_splits) workgroups, more than one: part_o fp32
+ * [M][splits][heads][vdim_p] and part_ml fp32 [M][splits][heads][2] are merged by a second launch.
+ * ti_gqa_prefill: consecutive positions pos0 + m of one slot (slot_stride 0). */
+typedef struct ti_gqa_attn_args {
+  const void* q;
+  const void* cache;
+  int64_t slot_stride;
+  const int32_t* pos;
+  const int32_t* slot;
+  const float* sink;
+  const float* gate;
+  void* out;
+  float* part_o;
+  float* part_ml;
+  float scale;
+  int32_t M, pos0, heads, kv_heads, dim, vdim, seq_p, splits, ldg, ldo, dtype;
+} ti_gqa_attn_args;
+int ti_gqa_decode(const ti_gqa_attn_args* a, ti_stream_t s);
+int ti_gqa_prefill(const ti_gqa_attn_args* a, ti_stream_t s);
+int ti_gqa_splits(int M, int heads, int kv_heads, int max_seq);
+/* Once per process and device, before a capture: lifts the LDS limit of the kernels of this and the
+ * next section. */
+int ti_recurrent_prepare(void);
+
+/* ------------------------------------------------------------------- short convolution
+ * Causal convolution per channel: y[c] = b[c] + sum_j w[c][j] x[position - (taps - 1) + j][c], zeros before
+ * position 0, through `act` (TI_CONV_*).  A slot's last inputs live in a ring [taps][channels] T, position p
+ * at place p % taps.  chunk: rows are consecutive positions of slot `slot0`, earlier inputs come from the
+ * ring, which is left as it is (ti_ssd_norm / ti_lru_scan write it); else every row is its own slot's next
+ * token and enters the ring.
+ * Output place of channel c: c for c < c0, else o0 + (c - c0) / bw * bwp + (c - c0) % bw; the places a
+ * section of bw channels leaves free are zeroed. */
+enum ti_conv_act { TI_CONV_LINEAR = 0, TI_CONV_SILU = 1 };
+typedef struct ti_conv_args {
+  const void* x;               /* T [M][ldx]                                                 */
+  void* ring;                  /* T [slots][taps][channels]                                  */
+  const float* w;              /* [channels][taps]                                           */
+  const float* b;
+  void* out;                   /* T [M][ldo]                                                 */
+  const int32_t* pos;
+  const int32_t* slot;
+  int32_t M, channels, taps, act, ldx, ldo, c0, o0, bw, bwp, chunk, slot0, dtype;
+} ti_conv_args;
+int ti_conv(const ti_conv_args* a, ti_stream_t s);
+
+/* ------------------------------------------------------------------- state-space recurrence (SSD)
+ * dt = softplus(dt_raw + dt_bias); S = exp(-exp(a_log) dt) S + dt B x^T; y = S^T C + D x, per head, fp32.
+ * A slot's state is [heads][vdim][np] fp32, np = state rounded up to 4; zero before position 0.
+ * ti_ssd_step: one token per row, each row its own slot; x, B, C come from the raw projection
+ * [z inner | x inner | B groups * state | C groups * state] T through the short convolution (SiLU), whose
+ * ring it advances.
+ * ti_ssd_scan: a prompt chunk of slot `slot0`; x, B, C come convolved from ti_conv's output: x at 0, B of
+ * group g at o0 + g * nk, C behind all B, nk = state rounded up to KT. */
+typedef struct ti_ssd_args {
+  const void* a;               /* step: T [M][lda] raw projection; scan: T [M][lda] convolved */
+  const float* dt;             /* [M][heads] raw                                             */
+  const float* dt_bias;
+  const float* a_log;
+  const float* d;
+  const float* conv_w;         /* step: [channels][taps]                                     */
+  const float* conv_b;
+  void* ring;
+  float* state;
+  float* y;                    /* [M][ldy]                                                   */
+  const int32_t* pos;
+  const int32_t* slot;
+  int32_t M, heads, vdim, state_n, groups, taps, lda, ldy, o0, slot0, dtype;
+} ti_ssd_args;
+int ti_ssd_step(const ti_ssd_args* a, ti_stream_t s);
+int ti_ssd_scan(const ti_ssd_args* a, ti_stream_t s);
+
+/* Gate before the norm: v = y * silu(z), RMS norm in `groups` equal parts, times w; out T [M][ldo].
+ * ring non-NULL (prompt chunk): the last taps - 1 rows' convolution inputs (raw + inner) enter it. */
+typedef struct ti_ssd_norm_args {
+  const float* y;              /* [M][ldy]                                                   */
+  const void* raw;             /* T [M][lda], z at 0                                         */
+  const float* w;
+  void* out;
+  void* ring;
+  const int32_t* pos;
+  float eps;
+  int32_t M, inner, groups, lda, ldy, ldo, channels, taps, slot0, dtype;
+} ti_ssd_norm_args;
+int ti_ssd_norm(const ti_ssd_norm_args* a, ti_stream_t s);
+
+/* ------------------------------------------------------------------- linear recurrence over a chunk
+ * S = a S + b per channel over the rows of a prompt chunk (TI_DE_LRU pairs), out T [m][c] = S * y[m][c];
+ * the slot's state [channels] fp32 (zero before position 0) and convolution ring (inputs x) are advanced. */
+typedef struct ti_lru_scan_args {
+  const float* ab;             /* [M][channels][2]                                           */
+  const void* y;               /* T [M][ldy]                                                 */
+  const void* x;               /* T [M][ldy]                                                 */
+  void* out;                   /* T [M][ldo]                                                 */
+  float* state;                /* [slots][channels]                                          */
+  void* ring;
+  const int32_t* pos;
+  int32_t M, channels, taps, ldy, ldo, slot0, dtype;
+} ti_lru_scan_args;
+int ti_lru_scan(const ti_lru_scan_args* a, ti_stream_t s);
 
 /* Seeded uniform(-scale, scale) elements of `dtype` (synthetic weights and caches). */
 int ti_stack_fill(uint64_t seed, uint32_t tid, uint64_t n, float scale, int dtype, void* out, ti_stream_t s);

@@ -12,6 +12,7 @@ loudly with TiError.
 from __future__ import annotations
 
 import ctypes as C
+import json
 import os
 import subprocess
 
@@ -68,21 +69,30 @@ class EngineConfig(C.Structure):
 
 
 DT_BF16, DT_F32 = 0, 1              # ti_dtype (include/ti_stack.h)
-MLP_NONE, MLP_MOE = 0, 1            # ti_mlp (include/ti_engine.h)
-(DE_F32, DE_T, DE_SWIGLU, DE_ROPE, DE_GATE, DE_LOGITS, DE_KFRAG, DE_VFRAG) = range(8)
+MIX_LATENT, MIX_GQA, MIX_SSD, MIX_RGLRU = range(4)   # ti_mixer (include/ti_engine.h)
+MLP_NONE, MLP_MOE, MLP_DENSE = range(3)              # ti_mlp
+PLACE_SANDWICH, PLACE_POST = 0, 1                    # ti_norm_place
+(DE_F32, DE_T, DE_SWIGLU, DE_ROPE, DE_GATE, DE_LOGITS, DE_KFRAG, DE_VFRAG, DE_ACT,
+ DE_LRU) = range(10)
+ACT_NONE, ACT_GELU_TANH, ACT_GELU_ERF = range(3)
 NORM_LAYER, NORM_RMS = 0, 1
 
 
 class StackLayer(C.Structure):
     """ti_stack_layer (include/ti_engine.h)."""
     _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "rot_dims")] + \
-        [("rot_base", C.c_float), ("scale", C.c_float)] + [(n, C.c_int32) for n in ("mlp", "experts", "top", "ff")]
+        [("rot_base", C.c_float), ("scale", C.c_float)] + \
+        [(n, C.c_int32) for n in ("mlp", "experts", "top", "ff", "kv_heads", "kv_shared", "kv_from", "sink_one")] + \
+        [("temp_coef", C.c_float), ("temp_every", C.c_float)] + \
+        [(n, C.c_int32) for n in ("conv", "state", "groups", "norm_groups", "mix_width", "blocks")]
 
 
 class StackConfig(C.Structure):
     """ti_stack_config (include/ti_engine.h)."""
     _fields_ = [(n, C.c_int32) for n in ("vocab", "width", "layers", "loop_start", "loop_stop", "loop_times")] + \
-        [("eps", C.c_float), ("emb_scale", C.c_float)] + [(n, C.c_int32) for n in ("dtype", "max_seq", "max_batch", "device")]
+        [("eps", C.c_float), ("emb_scale", C.c_float)] + \
+        [(n, C.c_int32) for n in ("dtype", "max_seq", "max_batch", "device", "norm_kind", "norm_place", "bigram_buckets",
+                                  "bigram_mul_prev", "bigram_mul_cur", "sinusoid")]
 
 
 class DenseArgs(C.Structure):
@@ -94,7 +104,9 @@ class DenseArgs(C.Structure):
          ("gate", C.c_void_p), ("gate_ld", C.c_int32), ("key_blocks", C.c_int32), ("argmax", C.c_void_p),
          ("step_ctr", C.c_void_p), ("advance", C.c_int32), ("tile_rows", C.c_int32), ("max_tiles", C.c_int32),
          ("tiles", C.c_void_p), ("n_tiles", C.c_void_p), ("rows_in", C.c_void_p), ("rows_out", C.c_void_p),
-         ("row_div", C.c_int32)]
+         ("row_div", C.c_int32)] + [(n, C.c_int32) for n in ("act", "act_cols", "t_cols", "ld2")] + \
+        [("out2", C.c_void_p), ("lru_rate", C.c_void_p), ("lru_state", C.c_void_p), ("lru_y", C.c_void_p),
+         ("lru_ldy", C.c_int32), ("slot", C.c_void_p)]
 
 
 class RownormArgs(C.Structure):
@@ -134,7 +146,9 @@ EXPORTED = [
     "ti_qkv_attn_partials", "ti_qkv_attn_part_o_elems", "ti_qkv_attn_part_ml_elems", "ti_engine_set_qkv_attn",
     "ti_qkv_attn_xchg_bytes", "ti_qkv_attn_supported", "ti_qkv_attn_error_offset",
     "ti_engine_create_stack", "ti_engine_weight_count", "ti_engine_weight_info", "ti_engine_set_weight", "ti_engine_load",
-    "ti_engine_describe", "ti_engine_prefill", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
+    "ti_engine_describe", "ti_engine_prefill", "ti_engine_create_config", "ti_engine_step_slots",
+    "ti_gqa_prep", "ti_gqa_block_elems", "ti_gqa_decode", "ti_gqa_prefill", "ti_gqa_splits", "ti_recurrent_prepare", "ti_conv",
+    "ti_ssd_step", "ti_ssd_scan", "ti_ssd_norm", "ti_lru_scan", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
     "ti_stack_convert", "ti_stack_fill", "ti_dense", "ti_dense_args_bytes", "ti_rownorm", "ti_rownorm_routes", "ti_route", "ti_route_max_tiles",
     "ti_latent_prep", "ti_latent_prepare", "ti_latent_attn_decode", "ti_latent_attn_splits", "ti_latent_attn_prefill", "ti_latent_attn_out",
 ]
@@ -265,6 +279,8 @@ def lib() -> C.CDLL:
             L.ti_engine_weight_info.argtypes = [vp, i32, C.c_char_p, i32, C.POINTER(C.c_int), C.POINTER(C.c_int)]
             L.ti_engine_set_weight.argtypes = [vp, C.c_char_p, vp, i32, i32]
             L.ti_engine_load.argtypes = [C.c_char_p, i32, i32, i32, i32, C.POINTER(vp)]
+            L.ti_engine_create_config.argtypes = [C.c_char_p, i32, i32, i32, i32, C.POINTER(vp)]
+            L.ti_engine_step_slots.argtypes = [vp, i32, vp, vp, vp, vp]
             L.ti_engine_describe.argtypes = [vp, C.POINTER(EngineConfig)]
             L.ti_engine_prefill.argtypes = [vp, i32, vp, i32, i32, vp, i32, vp, vp]
             L.ti_stack_kpad.argtypes = [i32, i32]
@@ -447,21 +463,10 @@ class Engine:
 
     @classmethod
     def stack(cls, config: dict, dtype="bfloat16", max_seq=2048, max_batch=1, device=0) -> "Engine":
-        """Layer-stack engine (ti_engine_create_stack) of a config.json-shaped dictionary, weights not set."""
-        lp = config.get("loop") or {}
-        c = StackConfig(config["vocab"], config["width"], len(config["layers"]), lp.get("start", 0), lp.get("stop", 0),
-                        lp.get("times", 0), config["norm"]["eps"], config["embedding"]["scale"],
-                        {"bfloat16": DT_BF16, "float32": DT_F32}[dtype], max_seq, max_batch, device)
-        ls = (StackLayer * len(config["layers"]))()
-        for d, l in zip(ls, config["layers"]):
-            m, f = l["mixer"], l.get("mlp")
-            for k in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "scale"):
-                setattr(d, k, m[k])
-            d.rot_dims, d.rot_base = m["rot"].get("dims", m["rot_dim"]), m["rot"]["base"]
-            if f:
-                d.mlp, d.experts, d.top, d.ff = MLP_MOE, f["router"]["experts"], f["router"]["top"], f["expert"]["ff"]
+        """Layer-stack engine of a config.json-shaped dictionary, weights not set (ti_engine_create_config)."""
         h = C.c_void_p()
-        check(lib().ti_engine_create_stack(C.byref(c), ls, C.byref(h)))
+        check(lib().ti_engine_create_config(json.dumps(config).encode(), {"bfloat16": DT_BF16, "float32": DT_F32}[dtype],
+                                            max_seq, max_batch, device, C.byref(h)))
         return cls._adopt(h)
 
     def weights(self):
@@ -608,6 +613,13 @@ class Engine:
         p = np.ascontiguousarray(pos, np.int32)
         logits = np.zeros((t.size, self.cfg.vocab), np.float32)
         check(lib().ti_engine_step(self.h, t.size, _ptr(t), _ptr(p), _ptr(logits)))
+        return logits
+
+    def step_slots(self, slots, tokens, pos):
+        """One token of each of the given stream slots (ti_engine_step_slots); the other slots are left alone."""
+        s, t, p = (np.ascontiguousarray(x, np.int32) for x in (slots, tokens, pos))
+        logits = np.zeros((t.size, self.cfg.vocab), np.float32)
+        check(lib().ti_engine_step_slots(self.h, t.size, _ptr(s), _ptr(t), _ptr(p), _ptr(logits)))
         return logits
 
     def compat_step(self, offset):

@@ -37,10 +37,52 @@ void read_latent_attention(const Json& m, ti_stack_layer& L) {
   L.rot_dims = m["rot"].has("dims") ? m["rot"]["dims"].integer() : L.rot_dim;
 }
 
+// "attention": grouped-query attention with one added to the softmax's denominator.
+void read_attention(const Json& m, ti_stack_layer& L) {
+  L.mixer = TI_MIX_GQA;
+  L.heads = m["heads"].integer();
+  L.kv_heads = m["kv_heads"].integer();
+  L.dim = m["dim"].integer();
+  L.vdim = m["vdim"].integer();
+  L.scale = (float)m["scale"].number();
+  L.sink_one = 1;
+  if (m.has("q_temp") && !m["q_temp"].is_null()) {
+    L.temp_coef = (float)m["q_temp"]["coef"].number();
+    L.temp_every = (float)m["q_temp"]["every"].number();
+    if (!(L.temp_every > 0.0f)) throw std::runtime_error("config.json: q_temp.every must be positive");
+  }
+  if (m.has("kv_from") && !m["kv_from"].is_null()) {
+    L.kv_shared = 1;
+    L.kv_from = m["kv_from"].integer();
+  }
+}
+
+void read_mamba2(const Json& m, ti_stack_layer& L) {
+  L.mixer = TI_MIX_SSD;
+  L.heads = m["heads"].integer();
+  L.vdim = m["vdim"].integer();
+  L.state = m["state"].integer();
+  L.groups = m["groups"].integer();
+  L.norm_groups = m["norm_groups"].integer();
+  L.conv = m["conv"].integer();
+}
+
+void read_rglru(const Json& m, ti_stack_layer& L) {
+  L.mixer = TI_MIX_RGLRU;
+  L.mix_width = m["width"].integer();
+  L.blocks = m["blocks"].integer();
+  L.conv = m["conv"].integer();
+}
+
 void read_mlp(const Json& m, ti_stack_layer& L) {
   L.mlp = TI_MLP_NONE;
   if (m.is_null()) return;
   const std::string kind = m["kind"].string();
+  if (kind == "dense") {
+    L.mlp = TI_MLP_DENSE;
+    L.ff = m["ff"].integer();
+    return;
+  }
   if (kind != "moe") throw std::runtime_error("config.json: feed-forward kind \"" + kind + "\" is not supported");
   L.mlp = TI_MLP_MOE;
   L.experts = m["router"]["experts"].integer();
@@ -63,6 +105,7 @@ StackSpec gegepel_spec(const Json& j) {
     if (type != "latent_attention") throw std::runtime_error("config.json: layer type \"" + type + "\" is not supported");
     read_latent_attention(e["mixer"], L);
     read_mlp(e.has("mlp") ? e["mlp"] : Json(), L);
+    if (L.mlp == TI_MLP_DENSE) throw std::runtime_error("config.json: feed-forward kind \"dense\" is not supported");
     s.layers.push_back(L);
   }
   c.layers = (int)s.layers.size();
@@ -74,8 +117,39 @@ StackSpec gegepel_spec(const Json& j) {
   return s;
 }
 
+// Nogitar: attention, Mamba-2 and RG-LRU layers in any order, RMS norms behind the sublayers only, a bigram
+// table and sinusoidal position vectors in the embedding.
+StackSpec nogitar_spec(const Json& j) {
+  StackSpec s;
+  ti_stack_config& c = s.cfg;
+  c.vocab = j["vocab"].integer();
+  c.width = j["width"].integer();
+  c.eps = (float)j["norm"]["eps"].number();
+  c.emb_scale = (float)j["embedding"]["scale"].number();
+  const Json& b = j["embedding"]["bigram"];
+  c.bigram_buckets = b["buckets"].integer();
+  c.bigram_mul_prev = b["mul_prev"].integer();
+  c.bigram_mul_cur = b["mul_cur"].integer();
+  if (c.bigram_buckets < 1) throw std::runtime_error("config.json: bigram.buckets must be positive");
+  c.sinusoid = 1;
+  c.norm_kind = TI_NORM_RMS;
+  c.norm_place = TI_PLACE_POST;
+  for (const Json& e : j["layers"].array()) {
+    ti_stack_layer L{};
+    const std::string type = e["type"].string();
+    if (type == "attention") read_attention(e["mixer"], L);
+    else if (type == "mamba2") read_mamba2(e["mixer"], L);
+    else if (type == "rglru") read_rglru(e["mixer"], L);
+    else throw std::runtime_error("config.json: layer type \"" + type + "\" is not supported");
+    read_mlp(e.has("mlp") ? e["mlp"] : Json(), L);
+    s.layers.push_back(L);
+  }
+  c.layers = (int)s.layers.size();
+  return s;
+}
+
 const std::map<std::string, StackSpec (*)(const Json&)>& registry() {
-  static const std::map<std::string, StackSpec (*)(const Json&)> r = {{"Gegepel", gegepel_spec}};
+  static const std::map<std::string, StackSpec (*)(const Json&)> r = {{"Gegepel", gegepel_spec}, {"Nogitar", nogitar_spec}};
   return r;
 }
 
@@ -177,18 +251,20 @@ model::ModelData load_model_dir(const std::string& path) {
   md.vocab_size = (size_t)s.cfg.vocab;
   md.hidden_size = (size_t)s.cfg.width;
   md.num_layers = s.layers.size();
-  if (!s.layers.empty()) {
-    md.num_heads = (size_t)s.layers[0].heads;
-    md.intermediate_size = (size_t)s.layers[0].ff;
-    md.rope_theta = s.layers[0].rot_base;
+  for (auto l = s.layers.rbegin(); l != s.layers.rend(); ++l) {   // (the first layer that has the part decides)
+    if (l->mixer == TI_MIX_LATENT || l->mixer == TI_MIX_GQA) {
+      md.num_heads = (size_t)l->heads;
+      md.rope_theta = l->rot_base;
+    }
+    if (l->mlp != TI_MLP_NONE) md.intermediate_size = (size_t)l->ff;
   }
   md.extra_params["config.json"] = text;
   read_safetensors(fs::is_directory(path) ? dir / "model.safetensors" : fs::path(path), m);
   return m;
 }
 
-ti_engine* build_stack_engine(const model::ModelData& m, int dtype, int max_seq, int max_batch, int device) {
-  StackSpec s = stack_spec(m.get_config_param("config.json"));
+ti_engine* create_stack_engine(const std::string& config_json, int dtype, int max_seq, int max_batch, int device) {
+  StackSpec s = stack_spec(config_json);
   s.cfg.dtype = dtype;
   s.cfg.max_seq = max_seq;
   s.cfg.max_batch = max_batch;
@@ -196,6 +272,11 @@ ti_engine* build_stack_engine(const model::ModelData& m, int dtype, int max_seq,
   if (s.layers.empty()) throw std::runtime_error("config.json: no layers");
   ti_engine* e = nullptr;
   check(ti_engine_create_stack(&s.cfg, s.layers.data(), &e), "ti_engine_create_stack");
+  return e;
+}
+
+ti_engine* build_stack_engine(const model::ModelData& m, int dtype, int max_seq, int max_batch, int device) {
+  ti_engine* e = create_stack_engine(m.get_config_param("config.json"), dtype, max_seq, max_batch, device);
   try {
     const int n = ti_engine_weight_count(e);
     for (int i = 0; i < n; ++i) {
@@ -205,8 +286,10 @@ ti_engine* build_stack_engine(const model::ModelData& m, int dtype, int max_seq,
       const core::Tensor* t = m.get_tensor(name);
       if (!t) throw std::runtime_error("the checkpoint lacks tensor " + std::string(name));
       const auto& d = t->shape().dimensions();
-      const size_t tr = d.empty() ? 0 : d[0], tc = d.size() > 1 ? d[1] : 1;
-      if (tr != (size_t)rows || tc != (size_t)cols || d.size() > 2)
+      size_t tr = d.empty() ? 0 : d[0];   // rows: every dimension but the last (block-diagonal weights have three)
+      for (size_t q = 1; q + 1 < d.size(); ++q) tr *= d[q];
+      const size_t tc = d.size() > 1 ? d.back() : 1;
+      if (tr != (size_t)rows || tc != (size_t)cols || d.size() > 3)
         throw std::runtime_error("tensor " + std::string(name) + " has the wrong shape (expected " + std::to_string(rows) +
                                  " x " + std::to_string(cols) + ")");
       if (t->dtype() == core::DataType::kFloat32) {
@@ -235,6 +318,17 @@ extern "C" int ti_engine_load(const char* dir, int dtype, int max_seq, int max_b
     *out = turboinfer::api::build_stack_engine(turboinfer::api::load_model_dir(dir), dtype, max_seq, max_batch, device);
   } catch (const std::exception& ex) {
     return ti_set_error(TI_ERR_ARG, "ti_engine_load(%s): %s", dir, ex.what());
+  }
+  return TI_OK;
+}
+
+extern "C" int ti_engine_create_config(const char* config_json, int dtype, int max_seq, int max_batch, int device, ti_engine** out) {
+  if (!config_json || !out) return ti_set_error(TI_ERR_ARG, "ti_engine_create_config: null");
+  *out = nullptr;
+  try {
+    *out = turboinfer::api::create_stack_engine(config_json, dtype, max_seq, max_batch, device);
+  } catch (const std::exception& ex) {
+    return ti_set_error(TI_ERR_ARG, "ti_engine_create_config: %s", ex.what());
   }
   return TI_OK;
 }

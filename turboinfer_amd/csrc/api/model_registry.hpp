@@ -26,6 +26,8 @@ StackSpec stack_spec(const std::string& config_json);
 model::ModelData load_model_dir(const std::string& path);
 bool is_model_dir(const std::string& path);
 
+/// The device engine of a config.json text, weights not set; the caller owns it.
+ti_engine* create_stack_engine(const std::string& config_json, int dtype, int max_seq, int max_batch, int device);
 /// The device engine of a ModelData whose architecture is registered; the caller owns it.
 ti_engine* build_stack_engine(const model::ModelData& m, int dtype, int max_seq, int max_batch, int device);
 

@@ -79,6 +79,9 @@ uint16_t host_half(float f) {
 struct ti_engine {
   ti_engine_config c{};
   std::unique_ptr<ti_host::StackModel> stack;   // layer-stack models; NULL: llama (the members below)
+  std::vector<int> state_pos;   // recurrent layer-stack models: tokens each slot's state has run
+  int32_t* row_slot = nullptr;  // layer-stack steps over chosen slots (ti_engine_step_slots): slot of each row
+  bool slots_on = false;
   hipStream_t s = nullptr;
   std::vector<void*> allocs;
   std::vector<DevLayer> layer;
@@ -399,7 +402,28 @@ void step_embedding(ti_engine* e, ti_step_args& sa) {
   sa.emb = static_cast<const uint16_t*>(e->stack->emb);
   sa.emb_kind = k.dtype == TI_DT_BF16 ? 1 : 2;
   sa.emb_scale = k.emb_scale;
-  sa.h0 = e->stack->h0;
+  sa.h0 = k.loop_times > 0 ? e->stack->h0 : nullptr;
+  if (e->stack->bigram) {
+    sa.bigram = e->stack->bigram;
+    sa.buckets = k.bigram_buckets;
+    sa.mul_prev = k.bigram_mul_prev;
+    sa.mul_cur = k.bigram_mul_cur;
+    sa.hist = e->stack->hist;
+    sa.hist_ld = e->stack->seq_p;
+  }
+  sa.pe_hi = e->stack->pe_hi;
+  sa.pe_lo = e->stack->pe_lo;
+  sa.pe_ld = e->stack->pe_ld;
+}
+
+// Models whose layers carry a state go on only where a slot's state stands.
+int state_at(ti_engine* e, int slot, int pos) {
+  if (!e->stack || !e->stack->recurrent || pos == 0 || pos == e->state_pos[slot]) return TI_OK;
+  return ti_set_error(TI_ERR_ARG, "engine: stream slot %d holds the state after %d tokens, not after %d (a recurrent model cannot go back)",
+                      slot, e->state_pos[slot], pos);
+}
+void state_set(ti_engine* e, int slot, int pos) {
+  if (!e->state_pos.empty()) e->state_pos[slot] = pos;
 }
 
 // Final norm + lm_head + argmax of n residual rows x (first token after a prefill, wanted prompt rows).
@@ -434,8 +458,10 @@ int enqueue_step(ti_engine* e, int M, int advance) {
   sa.base_pos = e->base_pos;
   sa.step_ctr = e->step_ctr;
   if (e->stack) {
+    sa.slot = e->slots_on ? e->row_slot : nullptr;
     TI_TRY(ti_step_begin(&sa, e->s));
     ti_host::StackRows r;
+    r.slots = sa.slot;
     r.M = M;
     r.pos = e->pos;
     r.h = e->h;
@@ -627,6 +653,8 @@ static bool prefill_attn_on() {
 
 int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base, float* layers_out = nullptr, int layers_stride = 0) {
   const ti_engine_config& c = e->c;
+  TI_TRY(state_at(e, m, base + t0));
+  state_set(e, m, base + t0 + rows);
   ++e->n_prefill_chunks;
   std::vector<int32_t> bp(rows);
   for (int j = 0; j < rows; ++j) bp[j] = base + t0 + j;
@@ -647,6 +675,8 @@ int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base, float* laye
   sa.pos = e->pos;
   sa.base_pos = e->pf_base;
   sa.step_ctr = e->pf_zero;
+  sa.chunk = e->stack != nullptr;
+  sa.slot0 = m;
   TI_TRY(ti_step_begin(&sa, e->s));
   if (e->stack) {
     TI_TRY(e->stack->ready());
@@ -709,7 +739,7 @@ int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base, float* laye
 }
 
 int get_graph(ti_engine* e, int M, int advance, hipGraphExec_t* out) {
-  auto key = std::make_pair(M, advance | (e->samp_on ? 2 : 0));
+  auto key = std::make_pair(M, advance | (e->samp_on ? 2 : 0) | (e->slots_on ? 4 : 0));
   auto it = e->graphs.find(key);
   if (it != e->graphs.end()) {
     *out = it->second;
@@ -865,14 +895,21 @@ int ti_engine_create_stack(const ti_stack_config* cfg, const ti_stack_layer* lay
   DeviceScope bind_(cfg->device);
   TI_TRY(ti_init(cfg->device));
   TI_TRY(ti_latent_prepare());
+  TI_TRY(ti_recurrent_prepare());
   auto e = std::make_unique<ti_engine>();
   ti_engine_config& c = e->c;
   c.vocab = cfg->vocab;
   c.hidden = cfg->width;
-  c.heads = c.kv_heads = layers[0].heads;
-  c.head_dim = layers[0].dim + layers[0].rot_dim;
-  c.inter = layers[0].mlp == TI_MLP_MOE ? layers[0].ff * layers[0].top : 0;
-  c.rope_theta = layers[0].rot_base;
+  for (int i = cfg->layers; i-- > 0;) {   // (the first layer that has the part decides)
+    const ti_stack_layer& l = layers[i];
+    if (l.mixer == TI_MIX_LATENT || l.mixer == TI_MIX_GQA) {
+      c.heads = l.heads;
+      c.kv_heads = l.mixer == TI_MIX_GQA ? l.kv_heads : l.heads;
+      c.head_dim = l.dim + l.rot_dim;
+      c.rope_theta = l.rot_base;
+    }
+    if (l.mlp != TI_MLP_NONE) c.inter = l.mlp == TI_MLP_MOE ? l.ff * l.top : l.ff;
+  }
   c.eps = cfg->eps;
   c.bits = 16;
   c.max_seq = cfg->max_seq;
@@ -900,6 +937,8 @@ int ti_engine_create_stack(const ti_stack_config* cfg, const ti_stack_layer* lay
   TI_TRY(e->alloc_t(&e->base_pos, (size_t)B));
   TI_TRY(e->alloc_t(&e->step_ctr, (size_t)1));
   TI_TRY(e->alloc_t(&e->n_in, (size_t)B));
+  TI_TRY(e->alloc_t(&e->row_slot, (size_t)B));
+  if (e->stack->recurrent) e->state_pos.assign((size_t)B, 0);
   TI_TRY(ensure_io(e.get(), 8, 8));
   const std::vector<int32_t> ones((size_t)R, 1);
   TI_TRY(ti_memcpy_h2d(e->pf_ones, ones.data(), ones.size() * 4, e->s));
@@ -1132,7 +1171,10 @@ int ti_engine_fill_kv(ti_engine* e, int stream, int n, uint64_t seed) {
   DeviceScope bind_(e);
   if (stream < 0 || stream >= e->c.max_batch || n < 0 || n > e->c.max_seq)
     return ti_set_error(TI_ERR_ARG, "ti_engine_fill_kv: stream %d n %d", stream, n);
-  if (e->stack) return e->stack->fill_kv(stream, n, seed);
+  if (e->stack) {
+    state_set(e, stream, n);
+    return e->stack->fill_kv(stream, n, seed);
+  }
   for (int l = 0; l < e->c.layers; ++l) {
     DevLayer& L = e->layer[l];
     TI_TRY(ti_fill_kv_uniform(seed, tid_kv(l, 0), n, e->c.kv_heads, e->c.head_dim, e->c.max_seq,
@@ -1198,6 +1240,7 @@ int ti_engine_generate(ti_engine* e, int n, const int32_t* prompts, const int32_
       TI_TRY(enqueue_head(e, n, n > 1 ? e->h_last : e->h + (size_t)(last_rows - 1) * c.hidden));
     }
   }
+  for (int m = 0; m < n; ++m) TI_TRY(state_at(e, m, base[m] + s0));
   TI_TRY(ti_memcpy_h2d(e->step_ctr, &s0, 4, e->s));
   std::vector<int32_t> outd((size_t)n * e->out_cap);
   std::vector<unsigned long long> am;
@@ -1242,6 +1285,7 @@ int ti_engine_generate(ti_engine* e, int n, const int32_t* prompts, const int32_
     }
   }
   for (int m = 0; m < n; ++m) {
+    state_set(e, m, base[m] + ran);
     bool stopped = false;
     for (int t = 0; t < max_new; ++t) {
       const int32_t tok = stopped ? -1 : token_at(m, t, ran);
@@ -1384,7 +1428,12 @@ std::vector<float> beam_top_p(const std::vector<float>& probs, float p) {
 // Copy slot `src`'s cache positions [0, n) into slot `dst`, every layer, K and V.
 int fork_slot(ti_engine* e, int src, int dst, int n) {
   const ti_engine_config& c = e->c;
-  if (e->stack) return e->stack->fork(src, dst, n);
+  if (e->stack) {
+    if (e->stack->recurrent && e->state_pos[src] != n)
+      return ti_set_error(TI_ERR_ARG, "engine: slot %d holds the state after %d tokens, not %d", src, e->state_pos[src], n);
+    state_set(e, dst, n);
+    return e->stack->fork(src, dst, n);
+  }
   return ti_kv_copy_slots(e->kv_tab, 2 * c.layers, (int64_t)src * e->kv_stride, (int64_t)dst * e->kv_stride,
                           c.kv_heads, (int64_t)c.max_seq * c.head_dim, (int64_t)n * c.head_dim, e->s);
 }
@@ -1591,6 +1640,10 @@ int ti_engine_serve(ti_engine* e, int n_req, const int32_t* prompts, const int32
     TI_TRY(ti_memcpy_h2d(e->base_pos, base.data(), (size_t)B * 4, e->s));
     const int32_t zero = 0;
     TI_TRY(ti_memcpy_h2d(e->step_ctr, &zero, 4, e->s));
+    for (int m = 0; m < B; ++m) {
+      TI_TRY(state_at(e, m, base[m]));
+      state_set(e, m, base[m] + S);
+    }
     TI_TRY(run_steps(e, B, 1, S));
     TI_TRY(ti_memcpy_d2h(outd.data(), e->out_tokens, outd.size() * 4, e->s));
     TI_TRY(read_argmax(e, B, am));   // synchronises the stream
@@ -1636,26 +1689,53 @@ int ti_engine_set_prefill(ti_engine* e, int rows) {
   return TI_OK;
 }
 
-int ti_engine_step(ti_engine* e, int n, const int32_t* tokens, const int32_t* pos, float* logits) {
-  if (!e || !tokens || !pos) return ti_set_error(TI_ERR_ARG, "ti_engine_step: null");
-  DeviceScope bind_(e);
+static int step_rows(ti_engine* e, int n, const int32_t* slots, const int32_t* tokens, const int32_t* pos, float* logits) {
   const ti_engine_config& c = e->c;
-  if (c.compat) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_step: compat engine");
-  if (n < 1 || n > c.max_batch) return ti_set_error(TI_ERR_ARG, "ti_engine_step: n=%d", n);
-  for (int m = 0; m < n; ++m)
+  for (int m = 0; m < n; ++m) {
     if (pos[m] < 0 || pos[m] >= c.max_seq) return ti_set_error(TI_ERR_ARG, "ti_engine_step: pos %d", pos[m]);
+    TI_TRY(state_at(e, slots ? slots[m] : m, pos[m]));
+  }
   TI_TRY(ensure_io(e, 1, 1));
   std::vector<int32_t> in((size_t)n * e->in_cap, 0), one(n, 1);
   for (int m = 0; m < n; ++m) in[(size_t)m * e->in_cap] = tokens[m];
   TI_TRY(ti_memcpy_h2d(e->in_tokens, in.data(), in.size() * 4, e->s));
   TI_TRY(ti_memcpy_h2d(e->n_in, one.data(), (size_t)n * 4, e->s));
   TI_TRY(ti_memcpy_h2d(e->base_pos, pos, (size_t)n * 4, e->s));
+  if (slots) TI_TRY(ti_memcpy_h2d(e->row_slot, slots, (size_t)n * 4, e->s));
   TI_TRY(ti_memset(e->step_ctr, 0, 4, e->s));
-  TI_TRY(run_steps(e, n, 1, 1));
+  e->slots_on = slots != nullptr;
+  const int rc = run_steps(e, n, 1, 1);
+  e->slots_on = false;
+  TI_TRY(rc);
+  for (int m = 0; m < n; ++m) state_set(e, slots ? slots[m] : m, pos[m] + 1);
   TI_TRY(ti_stream_sync(e->s));
   if (logits) TI_TRY(ti_memcpy_d2h(logits, e->logits, (size_t)n * c.vocab * 4, e->s));
   if (n == 1) TI_TRY(qa_fault_check(e));
   return TI_OK;
+}
+
+int ti_engine_step(ti_engine* e, int n, const int32_t* tokens, const int32_t* pos, float* logits) {
+  if (!e || !tokens || !pos) return ti_set_error(TI_ERR_ARG, "ti_engine_step: null");
+  DeviceScope bind_(e);
+  const ti_engine_config& c = e->c;
+  if (c.compat) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_step: compat engine");
+  if (n < 1 || n > c.max_batch) return ti_set_error(TI_ERR_ARG, "ti_engine_step: n=%d", n);
+  return step_rows(e, n, nullptr, tokens, pos, logits);
+}
+
+int ti_engine_step_slots(ti_engine* e, int n, const int32_t* slots, const int32_t* tokens, const int32_t* pos, float* logits) {
+  if (!e || !slots || !tokens || !pos) return ti_set_error(TI_ERR_ARG, "ti_engine_step_slots: null");
+  DeviceScope bind_(e);
+  const ti_engine_config& c = e->c;
+  if (!e->stack) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_engine_step_slots: layer-stack engines only");
+  if (n < 1 || n > c.max_batch) return ti_set_error(TI_ERR_ARG, "ti_engine_step_slots: n=%d", n);
+  std::vector<char> used((size_t)c.max_batch, 0);
+  for (int m = 0; m < n; ++m) {
+    if (slots[m] < 0 || slots[m] >= c.max_batch || used[slots[m]])
+      return ti_set_error(TI_ERR_ARG, "ti_engine_step_slots: slot %d", slots[m]);
+    used[slots[m]] = 1;
+  }
+  return step_rows(e, n, slots, tokens, pos, logits);
 }
 
 int ti_engine_compat_step(ti_engine* e, int placeholder_offset, float* logits) {

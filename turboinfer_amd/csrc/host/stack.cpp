@@ -9,9 +9,12 @@
 //   attention decode rows: carried into latent space (dense per head, split attention, merge, dense per
 //             head with the gate); prompt chunks: keys / values expanded into fragments + chunk attention
 //   dense     output projection
+//             (grouped-query attention, SSD and RG-LRU layers: stack_mixers.cpp)
 //   rownorm   residual += post-norm, pre-norm of the feed-forward
 //             (decode-sized row counts: with the router product and the choice of experts)
 //   dense     router; route; dense grouped gate/up with SiLU * up; dense grouped down
+//             (dense feed-forward: up with GELU, down)
+// Models with post-norms only have the element-type copy of the residual in the pre-norms' place.
 #include "stack.hpp"
 
 #include <algorithm>
@@ -50,6 +53,53 @@ int pair_place(int j, int rot_dims) {
 
 std::string lname(int l, const char* t) { return "l" + std::to_string(l) + "." + t; }
 
+int check_latent(const ti_stack_config& c, const ti_stack_layer& L, int i) {
+  if (L.heads < 1 || L.dim < 1 || L.rot_dim < 2 || L.rot_dim % 2 || L.vdim < 1 || L.q_rank < 1 || L.kv_rank < 1 ||
+      L.rot_dims < 0 || L.rot_dims > L.rot_dim || L.rot_dims % 2 || !(L.rot_base > 0.0f))
+    return ti_set_error(TI_ERR_ARG, "layer %d: latent attention sizes", i);
+  const int lim = c.dtype == TI_DT_BF16 ? 2048 : 1024;
+  if (L.vdim > 256 || ti_stack_kpad(c.dtype, L.kv_rank) > lim)
+    return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: vdim %d (at most 256), kv_rank %d (at most %d)", i, L.vdim, L.kv_rank, lim);
+  if (L.q_rank + L.kv_rank + L.rot_dim + L.heads > 15996)
+    return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: q_rank + kv_rank + rot_dim + heads > 15996", i);
+  return TI_OK;
+}
+
+int check_mixer(const ti_stack_config& c, const ti_stack_layer* l, int i) {
+  const ti_stack_layer& L = l[i];
+  switch (L.mixer) {
+    case TI_MIX_LATENT: return check_latent(c, L, i);
+    case TI_MIX_GQA:
+      if (L.heads < 1 || L.kv_heads < 1 || L.heads % L.kv_heads || L.dim < 1 || L.vdim < 1 || L.temp_every < 0.0f)
+        return ti_set_error(TI_ERR_ARG, "layer %d: attention sizes (heads %d, kv_heads %d, dim %d, vdim %d)", i, L.heads,
+                            L.kv_heads, L.dim, L.vdim);
+      if (L.vdim > 256 || L.dim > 1024 || (L.heads + L.kv_heads) * L.dim > 32768)
+        return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: dim %d (at most 1024), vdim %d (at most 256)", i, L.dim, L.vdim);
+      if (L.kv_shared) {
+        const ti_stack_layer* K = L.kv_from >= 0 && L.kv_from < i ? l + L.kv_from : nullptr;
+        if (!K || K->mixer != TI_MIX_GQA || K->kv_shared || K->heads != L.heads || K->kv_heads != L.kv_heads || K->dim != L.dim ||
+            K->vdim != L.vdim || c.loop_times > 0)
+          return ti_set_error(TI_ERR_ARG, "layer %d: cannot share the keys and values of layer %d", i, L.kv_from);
+      }
+      return TI_OK;
+    case TI_MIX_SSD:
+      if (L.heads < 1 || L.vdim < 1 || L.state < 1 || L.groups < 1 || L.heads % L.groups || L.norm_groups < 1 ||
+          L.heads * L.vdim % L.norm_groups || L.conv < 1)
+        return ti_set_error(TI_ERR_ARG, "layer %d: SSD sizes (heads %d, vdim %d, state %d, groups %d, norm_groups %d, conv %d)", i,
+                            L.heads, L.vdim, L.state, L.groups, L.norm_groups, L.conv);
+      if (L.state > 256 || L.heads * L.vdim > 32768 || L.conv > 64)
+        return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: state %d (at most 256), heads * vdim %d (at most 32768), conv %d (at most 64)",
+                            i, L.state, L.heads * L.vdim, L.conv);
+      return TI_OK;
+    case TI_MIX_RGLRU:
+      if (L.mix_width < 1 || L.blocks < 1 || L.mix_width % L.blocks || L.conv < 1)
+        return ti_set_error(TI_ERR_ARG, "layer %d: RG-LRU sizes (width %d, blocks %d, conv %d)", i, L.mix_width, L.blocks, L.conv);
+      if (L.conv > 64) return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: conv %d (at most 64)", i, L.conv);
+      return TI_OK;
+    default: return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: mixer %d", i, L.mixer);
+  }
+}
+
 }  // namespace
 
 StackModel::~StackModel() {
@@ -57,7 +107,7 @@ StackModel::~StackModel() {
 }
 
 int StackModel::alloc(void** p, size_t bytes) {
-  TI_TRY(ti_malloc(p, bytes));
+  TI_TRY(ti_malloc(p, std::max<size_t>(bytes, 16)));
   allocs_.push_back(*p);
   if (bytes) S_HIP(hipMemsetAsync(*p, 0, bytes, s_), "hipMemsetAsync(alloc)");
   return TI_OK;
@@ -78,18 +128,14 @@ int StackModel::check(const ti_stack_config& c, const ti_stack_layer* l) {
   if (c.dtype != TI_DT_BF16 && c.dtype != TI_DT_F32) return ti_set_error(TI_ERR_ARG, "ti_engine_create_stack: dtype %d", c.dtype);
   if (c.loop_times < 0 || (c.loop_times > 0 && (c.loop_start < 0 || c.loop_stop > c.layers || c.loop_start >= c.loop_stop)))
     return ti_set_error(TI_ERR_ARG, "ti_engine_create_stack: loop [%d, %d) x %d", c.loop_start, c.loop_stop, c.loop_times);
+  if ((c.norm_kind != TI_NORM_LAYER && c.norm_kind != TI_NORM_RMS) || (c.norm_place != TI_PLACE_SANDWICH && c.norm_place != TI_PLACE_POST))
+    return ti_set_error(TI_ERR_ARG, "ti_engine_create_stack: norm kind %d, place %d", c.norm_kind, c.norm_place);
+  if (c.bigram_buckets < 0) return ti_set_error(TI_ERR_ARG, "ti_engine_create_stack: %d bigram buckets", c.bigram_buckets);
   for (int i = 0; i < c.layers; ++i) {
     const ti_stack_layer& L = l[i];
-    if (L.mixer != TI_MIX_LATENT) return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: mixer %d", i, L.mixer);
-    if (L.heads < 1 || L.dim < 1 || L.rot_dim < 2 || L.rot_dim % 2 || L.vdim < 1 || L.q_rank < 1 || L.kv_rank < 1 ||
-        L.rot_dims < 0 || L.rot_dims > L.rot_dim || L.rot_dims % 2 || !(L.rot_base > 0.0f))
-      return ti_set_error(TI_ERR_ARG, "layer %d: latent attention sizes", i);
-    const int lim = c.dtype == TI_DT_BF16 ? 2048 : 1024;
-    if (L.vdim > 256 || ti_stack_kpad(c.dtype, L.kv_rank) > lim)
-      return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: vdim %d (at most 256), kv_rank %d (at most %d)", i, L.vdim, L.kv_rank, lim);
-    if (L.q_rank + L.kv_rank + L.rot_dim + L.heads > 15996)
-      return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: q_rank + kv_rank + rot_dim + heads > 15996", i);
-    if (L.mlp != TI_MLP_NONE && L.mlp != TI_MLP_MOE) return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: feed-forward %d", i, L.mlp);
+    TI_TRY(check_mixer(c, l, i));
+    if (L.mlp == TI_MLP_DENSE && L.ff < 1) return ti_set_error(TI_ERR_ARG, "layer %d: ff %d", i, L.ff);
+    if (L.mlp != TI_MLP_NONE && L.mlp != TI_MLP_MOE && L.mlp != TI_MLP_DENSE) return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: feed-forward %d", i, L.mlp);
     if (L.mlp == TI_MLP_MOE && (L.experts < 1 || L.experts > 1024 || L.top < 1 || L.top > L.experts || L.top > 64 || L.ff < 1))
       return ti_set_error(TI_ERR_ARG, "layer %d: %d experts, top %d, ff %d", i, L.experts, L.top, L.ff);
   }
@@ -107,28 +153,32 @@ int StackModel::add_weight(const std::string& name, int rows, int cols) {
 int StackModel::alloc_layer(StackLayer& L) {
   const ti_stack_layer& k = L.c;
   const int kt = c.dtype == TI_DT_BF16 ? 32 : 16, W = c.width;
-  L.dim_p = kpad(k.dim);
-  L.rot_p = up(k.rot_dim, kt);
-  L.lat_p = kpad(k.kv_rank);
-  L.vdim_p = up(k.vdim, 16);
-  L.na = k.q_rank + k.kv_rank + k.rot_dim + k.heads;
-  TI_TRY(alloc_pack(L.a, L.na, W));
-  TI_TRY(alloc_pack(L.uq, k.heads * (L.dim_p + L.rot_p), k.q_rank));
-  TI_TRY(alloc_pack(L.ukt, L.lat_p, k.dim, k.heads));
-  TI_TRY(alloc_pack(L.uk, k.heads * L.dim_p, k.kv_rank));
-  TI_TRY(alloc_pack(L.uv, k.heads * L.vdim_p, k.kv_rank));
-  TI_TRY(alloc_pack(L.o, W, k.heads * k.vdim));
-  TI_TRY(alloc_t(&L.n1, (size_t)2 * W));
-  TI_TRY(alloc_t(&L.n1b, (size_t)2 * W));
-  TI_TRY(alloc_t(&L.q_norm, (size_t)k.q_rank));
-  TI_TRY(alloc_t(&L.c_norm, (size_t)k.kv_rank));
-  TI_TRY(alloc_t(&L.sink, (size_t)k.heads));
+  if (k.mixer == TI_MIX_LATENT) {
+    L.dim_p = kpad(k.dim);
+    L.rot_p = up(k.rot_dim, kt);
+    L.lat_p = kpad(k.kv_rank);
+    L.vdim_p = up(k.vdim, 16);
+    L.na = k.q_rank + k.kv_rank + k.rot_dim + k.heads;
+    TI_TRY(alloc_pack(L.a, L.na, W));
+    TI_TRY(alloc_pack(L.uq, k.heads * (L.dim_p + L.rot_p), k.q_rank));
+    TI_TRY(alloc_pack(L.ukt, L.lat_p, k.dim, k.heads));
+    TI_TRY(alloc_pack(L.uk, k.heads * L.dim_p, k.kv_rank));
+    TI_TRY(alloc_pack(L.uv, k.heads * L.vdim_p, k.kv_rank));
+    TI_TRY(alloc_pack(L.o, W, k.heads * k.vdim));
+    TI_TRY(alloc_t(&L.q_norm, (size_t)k.q_rank));
+    TI_TRY(alloc_t(&L.c_norm, (size_t)k.kv_rank));
+    TI_TRY(alloc_t(&L.sink, (size_t)k.heads));
+  } else {
+    TI_TRY(alloc_mixer(L));
+  }
+  for (float** n : {&L.n1, &L.n1b, &L.n2, &L.n2b}) TI_TRY(alloc_t(n, (size_t)2 * W));   // weight, bias
   if (k.mlp == TI_MLP_MOE) {
     TI_TRY(alloc_pack(L.router, k.experts, W));
     TI_TRY(alloc_pack(L.gu, 2 * k.ff, W, k.experts));
     TI_TRY(alloc_pack(L.down, W, k.ff, k.experts));
-    TI_TRY(alloc_t(&L.n2, (size_t)2 * W));
-    TI_TRY(alloc_t(&L.n2b, (size_t)2 * W));
+  } else if (k.mlp == TI_MLP_DENSE) {
+    TI_TRY(alloc_pack(L.up, k.ff, W));
+    TI_TRY(alloc_pack(L.down, W, k.ff));
   }
   return TI_OK;
 }
@@ -147,6 +197,7 @@ int StackModel::create(const ti_stack_config& cfg, const ti_stack_layer* l, int 
     StackLayer& L = layer[i];
     L.c = l[i];
     TI_TRY(alloc_layer(L));
+    if (L.c.mixer != TI_MIX_LATENT) continue;
     float*& t = tables[std::make_tuple(L.rot_p, L.c.rot_dim, L.c.rot_dims, L.c.rot_base)];
     if (!t) {
       const int pairs = L.rot_p / 2, turn = L.c.rot_dims / 2;
@@ -169,16 +220,35 @@ int StackModel::create(const ti_stack_config& cfg, const ti_stack_layer* l, int 
   for (int t = 0; t < c.loop_times; ++t)
     for (int i = l0; i < l1; ++i) add_run(i, i == l0 ? t : -1);
   for (int i = l1; i < c.layers; ++i) add_run(i, -1);
-  for (auto& r : run) {
-    const StackLayer& L = layer[r.layer];
-    const size_t b = (size_t)c.max_batch * seq_p * (L.lat_p + L.rot_p) * esize();
-    kv_bytes += b;
-    TI_TRY(alloc(&r.cache, b));
-  }
+  for (auto& r : run) TI_TRY(alloc_run(r));
   // the checkpoint's tensors
   TI_TRY(alloc(&emb, (size_t)c.vocab * W * esize()));
   weight_bytes += (size_t)c.vocab * W * esize();
   add_weight("embed", c.vocab, W);
+  if (c.bigram_buckets > 0) {
+    const size_t n = (size_t)(c.bigram_buckets + 1) * W;
+    TI_TRY(alloc(&bigram, n * esize()));
+    weight_bytes += n * esize();
+    TI_TRY(alloc_t(&hist, (size_t)c.max_batch * seq_p));
+    add_weight("bigram", c.bigram_buckets + 1, W);
+  }
+  if (c.sinusoid) {
+    pe_ld = up(W, 2);
+    const int hi = up(seq_p, 256) / 256;
+    std::vector<float> t((size_t)std::max(hi, 256) * pe_ld);
+    auto fill = [&](float** dst, int n, int step) -> int {
+      for (int p = 0; p < n; ++p)
+        for (int e = 0; e < pe_ld; ++e) {
+          const double a = (double)p * step * std::pow(10000.0, -2.0 * (e / 2) / W);
+          t[(size_t)p * pe_ld + e] = (float)(e % 2 ? std::cos(a) : std::sin(a));
+        }
+      TI_TRY(alloc_t(dst, (size_t)n * pe_ld));
+      TI_TRY(ti_memcpy_h2d(*dst, t.data(), (size_t)n * pe_ld * 4, s_));
+      return ti_stream_sync(s_);
+    };
+    TI_TRY(fill(&pe_hi, hi, 256));
+    TI_TRY(fill(&pe_lo, 256, 1));
+  }
   if (c.loop_times > 0) {
     add_weight("loop.in", W, 2 * W);
     add_weight("loop.step", c.loop_times, W);
@@ -187,23 +257,30 @@ int StackModel::create(const ti_stack_config& cfg, const ti_stack_layer* l, int 
   }
   for (int i = 0; i < c.layers; ++i) {
     const ti_stack_layer& k = layer[i].c;
-    const bool ml = k.mlp == TI_MLP_MOE;
     for (const char* n : {"norm1", "norm1b", "norm2", "norm2b"}) {
-      if (n[4] == '2' && !ml) continue;
+      if ((n[4] == '2' && k.mlp == TI_MLP_NONE) || (n[5] && c.norm_place == TI_PLACE_POST)) continue;
       add_weight(lname(i, n), W, 1);
-      add_weight(lname(i, n) + ".b", W, 1);
+      if (c.norm_kind == TI_NORM_LAYER) add_weight(lname(i, n) + ".b", W, 1);
     }
-    add_weight(lname(i, "mix.dq"), k.q_rank, W);
-    add_weight(lname(i, "mix.dq.norm"), k.q_rank, 1);
-    add_weight(lname(i, "mix.uq"), k.heads * (k.dim + k.rot_dim), k.q_rank);
-    add_weight(lname(i, "mix.dkv"), k.kv_rank + k.rot_dim, W);
-    add_weight(lname(i, "mix.dkv.norm"), k.kv_rank, 1);
-    add_weight(lname(i, "mix.uk"), k.heads * k.dim, k.kv_rank);
-    add_weight(lname(i, "mix.uv"), k.heads * k.vdim, k.kv_rank);
-    add_weight(lname(i, "mix.sink"), k.heads, 1);
-    add_weight(lname(i, "mix.g"), k.heads, W);
-    add_weight(lname(i, "mix.o"), W, k.heads * k.vdim);
-    if (!ml) continue;
+    if (k.mixer == TI_MIX_LATENT) {
+      add_weight(lname(i, "mix.dq"), k.q_rank, W);
+      add_weight(lname(i, "mix.dq.norm"), k.q_rank, 1);
+      add_weight(lname(i, "mix.uq"), k.heads * (k.dim + k.rot_dim), k.q_rank);
+      add_weight(lname(i, "mix.dkv"), k.kv_rank + k.rot_dim, W);
+      add_weight(lname(i, "mix.dkv.norm"), k.kv_rank, 1);
+      add_weight(lname(i, "mix.uk"), k.heads * k.dim, k.kv_rank);
+      add_weight(lname(i, "mix.uv"), k.heads * k.vdim, k.kv_rank);
+      add_weight(lname(i, "mix.sink"), k.heads, 1);
+      add_weight(lname(i, "mix.g"), k.heads, W);
+      add_weight(lname(i, "mix.o"), W, k.heads * k.vdim);
+    } else {
+      TI_TRY(add_mixer_weights(i));
+    }
+    if (k.mlp == TI_MLP_DENSE) {
+      add_weight(lname(i, "mlp.up"), k.ff, W);
+      add_weight(lname(i, "mlp.down"), W, k.ff);
+    }
+    if (k.mlp != TI_MLP_MOE) continue;
     add_weight(lname(i, "mlp.router"), k.experts, W);
     for (int e = 0; e < k.experts; ++e) {
       const std::string p = lname(i, "mlp.e") + std::to_string(e);
@@ -213,7 +290,7 @@ int StackModel::create(const ti_stack_config& cfg, const ti_stack_layer* l, int 
     }
   }
   add_weight("final.norm", W, 1);
-  add_weight("final.norm.b", W, 1);
+  if (c.norm_kind == TI_NORM_LAYER) add_weight("final.norm.b", W, 1);
   add_weight("head", c.vocab, W);
   TI_TRY(alloc_t(&final_norm_, (size_t)2 * W));
   TI_TRY(alloc_pack(head_, c.vocab, W));
@@ -228,18 +305,27 @@ int StackModel::alloc_work() {
   size_t cq = 0, q = 0, qa = 0, at = 0, a32 = 0, hd = 0, E = 1, n = 0, act = 0, kf = 0, vf = 0, po = 0, pml = 0, tiles = 1;
   for (const auto& L : layer) {
     const ti_stack_layer& k = L.c;
-    cq = std::max<size_t>(cq, kpad(k.q_rank));
-    q = std::max<size_t>(q, (size_t)k.heads * (L.dim_p + L.rot_p));
-    qa = std::max<size_t>(qa, (size_t)k.heads * L.lat_p);
-    at = std::max<size_t>(at, kpad(k.heads * k.vdim));
-    a32 = std::max<size_t>(a32, up(L.na, 4));
-    hd = std::max<size_t>(hd, k.heads);
-    kf = std::max<size_t>(kf, (size_t)k.heads * seq_p * L.dim_p);
-    vf = std::max<size_t>(vf, (size_t)k.heads * seq_p * L.vdim_p);
-    for (int M = 1; M <= dec_rows; ++M) {
-      const size_t ms = (size_t)M * ti_latent_attn_splits(M, k.heads, c.max_seq) * k.heads;
-      po = std::max(po, ms * L.lat_p);
-      pml = std::max(pml, ms * 2);
+    if (k.mlp == TI_MLP_DENSE) act = std::max(act, R * kpad(k.ff));
+    if (k.mixer == TI_MIX_LATENT) {
+      cq = std::max<size_t>(cq, kpad(k.q_rank));
+      q = std::max<size_t>(q, (size_t)k.heads * (L.dim_p + L.rot_p));
+      qa = std::max<size_t>(qa, (size_t)k.heads * L.lat_p);
+      at = std::max<size_t>(at, kpad(k.heads * k.vdim));
+      a32 = std::max<size_t>(a32, up(L.na, 4));
+      hd = std::max<size_t>(hd, k.heads);
+      kf = std::max<size_t>(kf, (size_t)k.heads * seq_p * L.dim_p);
+      vf = std::max<size_t>(vf, (size_t)k.heads * seq_p * L.vdim_p);
+      for (int M = 1; M <= dec_rows; ++M) {
+        const size_t ms = (size_t)M * ti_latent_attn_splits(M, k.heads, c.max_seq) * k.heads;
+        po = std::max(po, ms * L.lat_p);
+        pml = std::max(pml, ms * 2);
+      }
+    } else {
+      at = std::max<size_t>(at, kpad(k.mixer == TI_MIX_RGLRU ? k.mix_width : k.heads * k.vdim));
+      if (k.mixer == TI_MIX_GQA) {
+        q = std::max<size_t>(q, (size_t)k.heads * up(k.dim, 32));
+        a32 = std::max<size_t>(a32, up(L.na, 4));
+      }
     }
     if (k.mlp == TI_MLP_MOE) {
       E = std::max<size_t>(E, k.experts);
@@ -265,8 +351,8 @@ int StackModel::alloc_work() {
   TI_TRY(alloc_t(&y_, R * W));
   TI_TRY(alloc_t(&h0, R * W));
   if (c.loop_times > 0) TI_TRY(alloc(&cat_, R * kpad(2 * W) * es));
+  if (act) TI_TRY(alloc(&act_, act * es));
   if (n) {
-    TI_TRY(alloc(&act_, act * es));
     TI_TRY(alloc(&parts_, n * W * es));
     TI_TRY(alloc_t(&zr_, R * E));
     TI_TRY(alloc_t(&wgt_, n));
@@ -275,7 +361,7 @@ int StackModel::alloc_work() {
     TI_TRY(alloc_t(&tiles_, tiles * 4));
     TI_TRY(alloc_t(&n_tiles_, (size_t)1));
   }
-  return TI_OK;
+  return alloc_mixer_work();
 }
 
 // ------------------------------------------------------------------ weights
@@ -302,6 +388,7 @@ int StackModel::set_device(const std::string& name, const float* d, int rows, in
   wt.set = true;
   if (name == "embed") return ti_stack_convert(d, (uint64_t)rows * cols, c.dtype, emb, s_);
   if (name == "head") return pack(head_, d, W, 1, rows, nullptr);
+  if (name == "bigram") return ti_stack_convert(d, (uint64_t)rows * cols, c.dtype, bigram, s_);
   if (name == "loop.in") return pack(loop_in_, d, 2 * W, 1, rows, nullptr);
   if (name == "loop.step") return vec(loop_step_);
   if (name == "final.norm") return vec(final_norm_);
@@ -314,6 +401,11 @@ int StackModel::set_device(const std::string& name, const float* d, int rows, in
   for (const auto& n : norms) {
     if (t == n.first) return vec(n.second);
     if (t == std::string(n.first) + ".b") return vec(n.second + W);
+  }
+  if (k.mixer != TI_MIX_LATENT || k.mlp == TI_MLP_DENSE) {
+    bool known = true;
+    TI_TRY(set_mixer_weight(L, t, d, rows, cols, known));
+    if (known) return TI_OK;
   }
   if (t == "mix.dq") {
     const auto m = range(rows, 0);
@@ -400,22 +492,41 @@ int StackModel::fill_kv(int stream, int n, uint64_t seed) {
   uint32_t tid = 0x200000u;
   for (auto& r : run) {
     const StackLayer& L = layer[r.layer];
-    const size_t cw = L.lat_p + L.rot_p;
-    TI_TRY(ti_stack_fill(seed, tid++, (uint64_t)n * cw, 1.0f, c.dtype,
-                         static_cast<char*>(r.cache) + (size_t)stream * seq_p * cw * esize(), s_));
+    const size_t es = esize();
+    char* cache = static_cast<char*>(r.cache) + (size_t)stream * r.cache_slot;
+    if (r.own_cache && L.c.mixer == TI_MIX_LATENT) {
+      TI_TRY(ti_stack_fill(seed, tid++, (uint64_t)n * (r.cache_slot / seq_p / es), 1.0f, c.dtype, cache, s_));
+    } else if (r.own_cache) {
+      const size_t head = r.cache_slot / L.c.kv_heads, used = head / seq_p * up(n, 64);
+      for (int h = 0; h < L.c.kv_heads; ++h) TI_TRY(ti_stack_fill(seed, tid++, used / es, 1.0f, c.dtype, cache + h * head, s_));
+    }
+    if (r.ring)
+      TI_TRY(ti_stack_fill(seed, tid++, r.ring_slot / es, 1.0f, c.dtype, static_cast<char*>(r.ring) + (size_t)stream * r.ring_slot, s_));
+    if (r.state)
+      TI_TRY(ti_stack_fill(seed, tid++, r.state_slot / 4, 1.0f, TI_DT_F32, r.state + (size_t)stream * (r.state_slot / 4), s_));
   }
+  if (hist) TI_TRY(ti_memset(hist + (size_t)stream * seq_p, 0, (size_t)seq_p * 4, s_));
   return ti_stream_sync(s_);
 }
 
 int StackModel::fork(int src, int dst, int n) {
   if (src == dst) return TI_OK;
+  auto copy = [&](void* base, size_t slot, size_t off, size_t bytes) -> int {
+    char* b = static_cast<char*>(base);
+    return ti_memcpy_d2d(b + (size_t)dst * slot + off, b + (size_t)src * slot + off, bytes, s_);
+  };
   for (auto& r : run) {
     const StackLayer& L = layer[r.layer];
-    const size_t cw = (size_t)(L.lat_p + L.rot_p) * esize();
-    char* b = static_cast<char*>(r.cache);
-    TI_TRY(ti_memcpy_d2d(b + (size_t)dst * seq_p * cw, b + (size_t)src * seq_p * cw, (size_t)n * cw, s_));
+    if (r.own_cache && L.c.mixer == TI_MIX_LATENT) {
+      TI_TRY(copy(r.cache, r.cache_slot, 0, r.cache_slot / seq_p * n));
+    } else if (r.own_cache) {
+      const size_t head = r.cache_slot / L.c.kv_heads;
+      for (int h = 0; h < L.c.kv_heads; ++h) TI_TRY(copy(r.cache, r.cache_slot, h * head, head / seq_p * up(n, 64)));
+    }
+    if (r.ring) TI_TRY(copy(r.ring, r.ring_slot, 0, r.ring_slot));
+    if (r.state) TI_TRY(copy(r.state, r.state_slot, 0, r.state_slot));
   }
-  return TI_OK;
+  return hist ? copy(hist, (size_t)seq_p * 4, 0, (size_t)n * 4) : TI_OK;
 }
 
 // ------------------------------------------------------------------ forward
@@ -465,6 +576,7 @@ int StackModel::attention(const StackLayer& L, const StackRun& run, const StackR
   p.gate = gate_;
   p.eps = c.eps;
   p.dtype = c.dtype;
+  p.slot = r.slots;
   TI_TRY(ti_latent_prep(&p, s_));
   ti_dense_args dq{};
   dq.rope_cs = L.rope;
@@ -529,6 +641,7 @@ int StackModel::attention(const StackLayer& L, const StackRun& run, const StackR
     f.splits = ti_latent_attn_splits(M, k.heads, c.max_seq);
     f.seq_p = seq_p;
     f.dtype = c.dtype;
+    f.slot = r.slots;
     if (f.splits > 1) {
       f.out = nullptr;
       TI_TRY(ti_latent_attn_decode(&f, s_));
@@ -565,7 +678,7 @@ int StackModel::attention(const StackLayer& L, const StackRun& run, const StackR
 
 // Decode-sized row counts route inside the feed-forward's pre-norm launch.
 bool StackModel::fused_router(const StackLayer& L, int M) const {
-  return M <= 64 && ti_rownorm_routes(c.width, L.c.experts);
+  return c.norm_place == TI_PLACE_SANDWICH && M <= 64 && ti_rownorm_routes(c.width, L.c.experts);
 }
 
 int StackModel::experts(const StackLayer& L, int M) {
@@ -619,8 +732,9 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
   const float* post = nullptr;
   bool parts = false;
   int top = 0;
-  auto rownorm = [&](const float* pre, void* cat, const StackLayer* route = nullptr) -> int {
-    if (!post && !pre && !cat) return TI_OK;
+  // pre: weights of the norm in front of the next product, NULL with `copy`: its input is the residual
+  auto rownorm = [&](const float* pre, void* cat, const StackLayer* route = nullptr, bool copy = false) -> int {
+    if (!post && !pre && !cat && !copy) return TI_OK;
     ti_rownorm_args n{};
     n.x = r.h;
     if (post) {
@@ -635,9 +749,9 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
       n.post_w = post;
       n.post_b = post + W;
     }
-    if (pre) {
+    if (pre || copy) {
       n.w = pre;
-      n.b = pre + W;
+      n.b = pre ? pre + W : nullptr;
       n.xn = xn_;
       n.ldn = kpad(W);
     }
@@ -649,7 +763,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
     n.eps = c.eps;
     n.M = M;
     n.H = W;
-    n.kind = TI_NORM_LAYER;
+    n.kind = c.norm_kind;
     n.dtype = c.dtype;
     if (route) {
       n.route_w = route->router.p;
@@ -669,15 +783,23 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
       d.add = loop_step_ + (size_t)run[i].pass * W;
       TI_TRY(dense(loop_in_, cat_, kpad(2 * W), M, r.h, W, TI_DE_F32, d));
     }
-    TI_TRY(rownorm(L.n1, nullptr));
-    TI_TRY(attention(L, run[i], r));
-    post = L.n1b;
+    const bool sandwich = c.norm_place == TI_PLACE_SANDWICH;
+    TI_TRY(rownorm(sandwich ? L.n1 : nullptr, nullptr, nullptr, !sandwich));
+    switch (L.c.mixer) {
+      case TI_MIX_GQA: TI_TRY(gqa(L, run[i], r)); break;
+      case TI_MIX_SSD: TI_TRY(ssd(L, run[i], r)); break;
+      case TI_MIX_RGLRU: TI_TRY(rglru(L, run[i], r)); break;
+      default: TI_TRY(attention(L, run[i], r));
+    }
+    post = sandwich ? L.n1b : L.n1;
     parts = false;
-    if (L.c.mlp == TI_MLP_MOE) {
-      TI_TRY(rownorm(L.n2, nullptr, fused_router(L, M) ? &L : nullptr));
-      TI_TRY(experts(L, M));
-      post = L.n2b;
-      parts = true;
+    if (L.c.mlp != TI_MLP_NONE) {
+      const bool moe = L.c.mlp == TI_MLP_MOE;
+      TI_TRY(rownorm(sandwich ? L.n2 : nullptr, nullptr, moe && fused_router(L, M) ? &L : nullptr, !sandwich));
+      if (moe) TI_TRY(experts(L, M));
+      else TI_TRY(dense_mlp(L, M));
+      post = sandwich ? L.n2b : L.n2;
+      parts = moe;
       top = L.c.top;
     }
     if (r.layers_out) {
@@ -705,7 +827,7 @@ int StackModel::head(float* h, int M, float* logits, unsigned long long* argmax)
   n.eps = c.eps;
   n.M = M;
   n.H = W;
-  n.kind = TI_NORM_LAYER;
+  n.kind = c.norm_kind;
   n.dtype = c.dtype;
   TI_TRY(ti_rownorm(&n, s_));
   ti_dense_args d{};

@@ -27,11 +27,25 @@ struct StackLayer {
   float *n1 = nullptr, *n1b = nullptr, *n2 = nullptr, *n2b = nullptr;   // [2][width]: weight, bias
   float *q_norm = nullptr, *c_norm = nullptr, *sink = nullptr;
   const float* rope = nullptr;
+  // grouped-query attention (a: [queries | keys | values | gates]), SSD (a: the in projection) and RG-LRU
+  // (a: [GELU branch | convolution input], gates: per block, rows (recurrence, input) interleaved)
+  int ka = -1, va = -1, ga = 0;            // a's rows of keys, values, gates
+  int cin = 0, o0 = 0, bwp = 0, conv_ld = 0;   // convolution channels and its output layout (ti_conv)
+  StackPack gates, up;
+  float *k_norm = nullptr, *in_b = nullptr, *conv_w = nullptr, *conv_b = nullptr, *dt_bias = nullptr, *a_log = nullptr,
+        *d_skip = nullptr, *gate_b = nullptr, *rate = nullptr;
+  const float* q_scale = nullptr;          // [position]
 };
 
 struct StackRun {             // one pass through one layer
   int layer = 0, pass = -1;   // pass >= 0: the loop entry step comes first
-  void* cache = nullptr;      // T [max_batch][seq_p][lat_p + rot_p]
+  // per stream slot (slot bytes each): positions' rows, recurrent state, convolution ring
+  void* cache = nullptr;      // latent: T [seq_p][lat_p + rot_p]; grouped-query: ti_stack.h blocks (a layer
+                              // that shares keys and values points at its source's)
+  void* ring = nullptr;       // T [taps][channels]
+  float* state = nullptr;
+  size_t cache_slot = 0, ring_slot = 0, state_slot = 0;
+  bool own_cache = false;
 };
 
 // Rows a forward call works on: decode = one row per stream slot, prompt chunk = consecutive positions
@@ -43,6 +57,7 @@ struct StackRows {
   const float* h0 = nullptr;      // device [M][width] embedding output
   bool chunk = false;
   int slot = 0, pos0 = 0;         // chunk: stream slot and first position (host)
+  const int32_t* slots = nullptr; // decode, device [M], nullable: the rows' stream slots (NULL: row m is slot m)
   float* layers_out = nullptr;    // host, nullable: residual after every run, run stride layers_stride rows
   size_t layers_stride = 0;
 };
@@ -63,6 +78,11 @@ class StackModel {
   int seq_p = 0, rows_cap = 0, dec_rows = 0;
   void* emb = nullptr;
   float* h0 = nullptr;          // [rows_cap][width]
+  void* bigram = nullptr;       // [buckets + 1][width]
+  int32_t* hist = nullptr;      // [max_batch][seq_p] tokens by position (with a bigram table)
+  float *pe_hi = nullptr, *pe_lo = nullptr;   // sinusoidal position vectors (ti_hip.h ti_step_args)
+  int pe_ld = 0;
+  bool recurrent = false;       // some layer carries a state: a slot only goes on where it stands
 
   ~StackModel();
   static int check(const ti_stack_config& c, const ti_stack_layer* l);
@@ -75,7 +95,7 @@ class StackModel {
   // all runs over `rows`; with `head` the final norm, head product and argmax of every row follow
   int forward(const StackRows& r, bool head, float* logits, unsigned long long* argmax, int32_t* step_ctr, int advance);
   int head(float* h, int M, float* logits, unsigned long long* argmax);
-  int fork(int src, int dst, int n);   // copy cache rows [0, n) of a slot
+  int fork(int src, int dst, int n);   // copy a slot's cache positions [0, n) and its states
 
  private:
   hipStream_t s_ = nullptr;
@@ -90,6 +110,10 @@ class StackModel {
   float *a32_ = nullptr, *gate_ = nullptr, *y_ = nullptr, *zr_ = nullptr, *wgt_ = nullptr, *part_ml_ = nullptr, *stage_ = nullptr;
   int32_t *idx_ = nullptr, *list_ = nullptr, *tiles_ = nullptr, *n_tiles_ = nullptr, *map_ = nullptr;
   size_t stage_elems_ = 0, map_elems_ = 0;
+  // work buffers of the grouped-query and recurrent mixers
+  void *proj_ = nullptr, *conv_ = nullptr;   // T: projections, convolution outputs
+  float *dt_ = nullptr, *ys_ = nullptr, *ab_ = nullptr, *gpart_o_ = nullptr, *gpart_ml_ = nullptr;
+  std::map<std::pair<float, float>, float*> temps_;
 
   int alloc(void** p, size_t bytes);
   template <class P>
@@ -109,6 +133,16 @@ class StackModel {
   int pack(const StackPack& w, const float* src, int64_t rs, int64_t ks, int rows, const std::vector<int32_t>* map,
            size_t elem_off = 0);
   int dense(const StackPack& w, const void* a, int lda, int M, void* out, int ldo, int epi, ti_dense_args extra);
+  int add_mixer_weights(int i);
+  int alloc_mixer(StackLayer& L);
+  int alloc_run(StackRun& r);
+  int alloc_mixer_work();
+  int host_copy(const float* dev, size_t n, std::vector<float>& out);
+  int set_mixer_weight(StackLayer& L, const std::string& t, const float* d, int rows, int cols, bool& known);
+  int gqa(const StackLayer& L, const StackRun& run, const StackRows& r);
+  int ssd(const StackLayer& L, const StackRun& run, const StackRows& r);
+  int rglru(const StackLayer& L, const StackRun& run, const StackRows& r);
+  int dense_mlp(const StackLayer& L, int M);
   int attention(const StackLayer& L, const StackRun& run, const StackRows& r);
   bool fused_router(const StackLayer& L, int M) const;
   int experts(const StackLayer& L, int M);

@@ -21,6 +21,12 @@ __device__ __forceinline__ unsigned long long logit_key(float v, int n) {
   return ((unsigned long long)float_order_key(v) << 32) | (unsigned long long)(0xFFFFFFFFu - (uint32_t)n);
 }
 
+__device__ __forceinline__ float activate(int act, float z) {
+  if (act == TI_ACT_GELU_ERF) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
+  if (act == TI_ACT_GELU_TANH) return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * fmaf(0.044715f * z * z, z, z)));
+  return z;
+}
+
 // Four consecutive output columns n0.. of row m (out row mo); rows >= rows are padding.
 template <class T, int EPI>
 __device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, int m, int mo, int rows, int n0, f32x4 v) {
@@ -90,6 +96,48 @@ __device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, i
       T* o = (T*)a.out + ((((size_t)h * a.key_blocks + (m >> 4)) * dt + d / KT) * 64 + ((d % KT) / VEC) * 16 + (m & 15)) * VEC +
              d % VEC;
       *(typename El<T>::Q*)o = quad<T>(v);
+      return;
+    }
+    case TI_DE_ACT: {
+      if (!live) return;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        if (a.add) v[i] += a.add[min(n0 + i, a.N - 1)];
+        if (n0 + i < a.act_cols) v[i] = activate(a.act, v[i]);
+      }
+      T* o = (T*)a.out + (size_t)mo * a.ldo + n0;
+      if (n0 + 4 <= a.t_cols && (a.ldo & 3) == 0) {
+        *(typename El<T>::Q*)o = quad<T>(v);
+        return;
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int n = n0 + i;
+        if (n < a.t_cols) o[i] = (T)v[i];
+        else if (n < a.N) a.out2[(size_t)mo * a.ld2 + n - a.t_cols] = v[i];
+      }
+      return;
+    }
+    case TI_DE_LRU: {
+      if (!live || n0 >= a.N) return;
+      const int per = a.N >> 1, channels = per * a.batch;
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int j = (n0 >> 1) + i, c = batch * per + j;
+        if (j >= per) return;
+        const float* gb = a.add + (size_t)batch * a.N + n0 + 2 * i;
+        const float la = -sigmoidf(v[2 * i] + gb[0]) * a.lru_rate[c];
+        const float u = (float)((const T*)a.a)[(size_t)m * a.lda + (size_t)batch * a.a_batch + j];
+        const float av = expf(la), bv = sqrtf(-expm1f(2.0f * la)) * sigmoidf(v[2 * i + 1] + gb[1]) * u;
+        if (!a.lru_state) {
+          *(float2*)((float*)a.out + ((size_t)m * channels + c) * 2) = make_float2(av, bv);
+        } else {
+          float* st = a.lru_state + (size_t)(a.slot ? a.slot[m] : m) * channels + c;
+          const float s = a.pos[m] > 0 ? fmaf(av, *st, bv) : bv;
+          *st = s;
+          ((T*)a.out)[(size_t)m * a.ldo + c] = (T)(s * (float)((const T*)a.lru_y)[(size_t)m * a.lru_ldy + c]);
+        }
+      }
       return;
     }
     default: return;
@@ -398,6 +446,8 @@ int dispatch_dense(const ti_dense_args& a, hipStream_t s) {
   switch (a.epi) {
     case TI_DE_F32: return few ? skinny<T, TI_DE_F32>(a, s) : tiled<T, TI_DE_F32>(a, s);
     case TI_DE_ROPE: return few ? skinny<T, TI_DE_ROPE>(a, s) : tiled<T, TI_DE_ROPE>(a, s);
+    case TI_DE_ACT: return few ? skinny<T, TI_DE_ACT>(a, s) : tiled<T, TI_DE_ACT>(a, s);
+    case TI_DE_LRU: return few ? skinny<T, TI_DE_LRU>(a, s) : tiled<T, TI_DE_LRU>(a, s);
     case TI_DE_LOGITS: return few ? skinny<T, TI_DE_LOGITS>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_LOGITS>(a, s);
     case TI_DE_GATE: return few ? skinny<T, TI_DE_GATE>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_GATE>(a, s);
     case TI_DE_SWIGLU:
@@ -521,6 +571,15 @@ extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
                             a->key_blocks, a->M);
       break;
     }
+    case TI_DE_ACT:
+      if (a->batch != 1 || a->t_cols < 0 || a->t_cols > a->N || (a->t_cols < a->N && !a->out2) || a->ldo < a->t_cols ||
+          a->act < TI_ACT_NONE || a->act > TI_ACT_GELU_ERF)
+        return ti_set_error(TI_ERR_ARG, "ti_dense: ACT arguments");
+      break;
+    case TI_DE_LRU:
+      if (a->N % 2 || !a->add || !a->lru_rate || (a->lru_state && (!a->lru_y || !a->pos || a->ldo < a->N / 2 * a->batch)))
+        return ti_set_error(TI_ERR_ARG, "ti_dense: LRU arguments");
+      break;
     default: return ti_set_error(TI_ERR_ARG, "ti_dense: epilogue %d", a->epi);
   }
   return a->dtype == TI_DT_BF16 ? dispatch_dense<bf16>(*a, (hipStream_t)stream) : dispatch_dense<float>(*a, (hipStream_t)stream);

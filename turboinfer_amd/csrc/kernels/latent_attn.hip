@@ -33,7 +33,7 @@ __global__ __launch_bounds__(512) void latent_prep_kernel(const ti_latent_prep_a
   const float ci = 1.0f / sqrtf(block_sum(c2, red) / (float)a.kv_rank + a.eps);
   T* cq = (T*)a.cq + (size_t)m * a.ldq;
   for (int i = tid; i < a.q_rank; i += 512) cq[i] = (T)(r[i] * qi * a.q_w[i]);
-  T* row = (T*)a.cache + (size_t)m * a.slot_stride + (size_t)pos * (a.lat_p + a.rot_p);
+  T* row = (T*)a.cache + (size_t)(a.slot ? a.slot[m] : m) * a.slot_stride + (size_t)pos * (a.lat_p + a.rot_p);
   for (int i = tid; i < a.lat_p; i += 512) row[i] = i < a.kv_rank ? (T)(r[a.lat_off + i] * ci * a.c_w[i]) : (T)0.0f;
   for (int i = tid; i < a.rot_p / 2; i += 512) {
     float u = 0.0f, v = 0.0f;
@@ -85,7 +85,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const ti_latent_a
   T* pb = (T*)(lds + (size_t)nkt * 1024);           // [16][PLD]
   float* sm = (float*)(pb + 16 * PLD);              // [4][16] wave maxima, then [4][16] wave sums
   const int pos = a.pos[m], head = ht * 16 + col;
-  const T* cache = (const T*)a.cache + (size_t)m * a.slot_stride;
+  const T* cache = (const T*)a.cache + (size_t)(a.slot ? a.slot[m] : m) * a.slot_stride;
   auto load_q = [&](int kt) -> V {
     V v = {};
     if (head < a.heads && kt < nkt)

@@ -17,7 +17,7 @@ __global__ __launch_bounds__(256) void step_begin_kernel(const ti_step_args a, u
   stamp_end(stamp, t_entry);
 }
 __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
-  __shared__ int s_tok;
+  __shared__ int s_tok, s_row;
   const int m = blockIdx.x, tid = threadIdx.x;
   // With hidden % 8 == 0 (<= 8192): the embedding row moves in 16-byte pieces, all
   // of a thread's loads in flight together; the fold weights (independent of the token) are
@@ -58,7 +58,19 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
     }
     if (tok < 0 || tok >= a.vocab) tok = 0;     // never index outside the table
     s_tok = tok;
-    a.pos[m] = a.base_pos[m] + s;
+    const int pos = a.base_pos[m] + s;
+    a.pos[m] = pos;
+    if (a.bigram) {
+      int32_t* hist = a.hist + (size_t)(a.chunk ? a.slot0 : a.slot ? a.slot[m] : m) * a.hist_ld;
+      s_row = a.buckets;
+      if (pos > 0) {   // (a chunk's rows run side by side: only its first one reads what an earlier launch wrote)
+        int prev = a.chunk && m > 0 ? a.in_tokens[m - 1] : hist[pos - 1];
+        if (prev < 0 || prev >= a.vocab) prev = 0;
+        s_row = (int)(((int64_t)prev * a.mul_prev + (int64_t)tok * a.mul_cur) % a.buckets);
+        if (s_row < 0) s_row += a.buckets;
+      }
+      hist[pos] = tok;
+    }
   }
   __syncthreads();   // every slot read before any is cleared
   if (tid < TI_ARGMAX_SLOTS) am[tid] = 0ull;
@@ -73,9 +85,21 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
   } else if (a.emb_kind) {
     const size_t r0 = (size_t)s_tok * a.hidden;
     float* h0 = a.h0 ? a.h0 + (size_t)m * a.hidden : nullptr;
+    const size_t b0 = a.bigram ? (size_t)s_row * a.hidden : 0;
+    const int pos = a.base_pos[m] + s;
+    const float* hi = a.pe_hi ? a.pe_hi + (size_t)(pos >> 8) * a.pe_ld : nullptr;
+    const float* lo = a.pe_hi ? a.pe_lo + (size_t)(pos & 255) * a.pe_ld : nullptr;
+    auto elem = [&](const void* t, size_t i) {
+      return a.emb_kind == 1 ? __builtin_bit_cast(float, (uint32_t)((const uint16_t*)t)[i] << 16) : ((const float*)t)[i];
+    };
     for (int i = tid; i < a.hidden; i += 256) {
-      const float v = a.emb_scale * (a.emb_kind == 1 ? __builtin_bit_cast(float, (uint32_t)a.emb[r0 + i] << 16)
-                                                     : ((const float*)a.emb)[r0 + i]);
+      float v = a.emb_scale * elem(a.emb, r0 + i);
+      if (a.bigram) v += elem(a.bigram, b0 + i);
+      if (hi) {   // the angles' sum: (sine, cosine) at the even and odd entry of a pair
+        const int e = i & ~1;
+        const float2 p = *(const float2*)(hi + e), q = *(const float2*)(lo + e);
+        v += (i & 1) ? p.y * q.y - p.x * q.x : fmaf(p.x, q.y, p.y * q.x);
+      }
       h[i] = v;
       if (h0) h0[i] = v;
     }
@@ -281,6 +305,9 @@ extern "C" int ti_step_begin(const ti_step_args* a, ti_stream_t stream) {
     return ti_set_error(TI_ERR_ARG, "ti_step_begin: fold_x needs fold_w, fold_ss and the embedding gather");
   if (a->emb_kind < 0 || a->emb_kind > 2 || (a->emb_kind && (a->fold_x || a->placeholder_first >= 0)) || (a->h0 && !a->emb_kind))
     return ti_set_error(TI_ERR_ARG, "ti_step_begin: emb_kind %d", a->emb_kind);
+  if ((a->bigram && (!a->emb_kind || !a->hist || a->buckets < 1)) || (a->pe_hi && (!a->emb_kind || !a->pe_lo || a->pe_ld < a->hidden || a->pe_ld % 2)) ||
+      (a->chunk && a->in_stride != 1))
+    return ti_set_error(TI_ERR_ARG, "ti_step_begin: embedding terms");
   hipLaunchKernelGGL(step_begin_kernel, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a,
                      ti_stamp_next(STAMP_BEGIN, a->M));
   TI_LAUNCH_CHECK("step_begin_kernel");

@@ -63,7 +63,10 @@ __global__ __launch_bounds__(512) void rownorm_kernel(const ti_rownorm_args a) {
       c[H + i] = (T)x0[i];
     }
   }
-  if (a.xn) {
+  if (a.xn && !a.w) {
+    T* o = (T*)a.xn + (size_t)m * a.ldn;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = (T)row[i];
+  } else if (a.xn) {
     const float2 st = row_stats(row, H, a.eps, a.kind, red);
     T* o = (T*)a.xn + (size_t)m * a.ldn;
     for (int i = threadIdx.x; i < H; i += blockDim.x) {
@@ -101,8 +104,8 @@ __global__ __launch_bounds__(TH) void rownorm_vec_kernel(const ti_rownorm_args a
     y[c] = a.y ? *(const f32x4*)(a.y + (size_t)m * a.ldy + 4 * i) : zero;
     pw[c] = add && a.post_w ? *(const f32x4*)(a.post_w + 4 * i) : zero;
     pb[c] = add && a.post_w && ln ? *(const f32x4*)(a.post_b + 4 * i) : zero;
-    w[c] = a.xn ? *(const f32x4*)(a.w + 4 * i) : zero;
-    b[c] = a.xn && ln ? *(const f32x4*)(a.b + 4 * i) : zero;
+    w[c] = a.w ? *(const f32x4*)(a.w + 4 * i) : zero;
+    b[c] = a.w && ln ? *(const f32x4*)(a.b + 4 * i) : zero;
     z[c] = a.cat ? *(const f32x4*)(a.x0 + (size_t)m * a.H + 4 * i) : zero;
   }
   if (a.parts) {
@@ -173,13 +176,14 @@ __global__ __launch_bounds__(TH) void rownorm_vec_kernel(const ti_rownorm_args a
       }
   }
   if (a.xn) {
-    const float2 st = stats(v);
+    float2 st = make_float2(0.0f, 1.0f);
+    if (a.w) st = stats(v);
     T* o = (T*)a.xn + (size_t)m * a.ldn;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       f32x4 r;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) r[e] = (v[c][e] - st.x) * st.y * w[c][e] + b[c][e];
+      for (int e = 0; e < 4; ++e) r[e] = a.w ? (v[c][e] - st.x) * st.y * w[c][e] + b[c][e] : v[c][e];
       if (live[c]) *(Q*)(o + 4 * (tid + c * TH)) = quad<T>(r);
       if constexpr (ROUTE) {   // (the row's k padding: zeros)
         extern __shared__ float row[];
@@ -368,10 +372,10 @@ extern "C" int ti_rownorm(const ti_rownorm_args* a, ti_stream_t stream) {
     return ti_set_error(TI_ERR_ARG, "ti_rownorm: bad arguments");
   if ((a->y && a->parts) || ((a->y || a->parts) && a->ldy < a->H) || (a->parts && (!a->part_w || a->top < 1)) ||
       (a->post_w && a->kind == TI_NORM_LAYER && !a->post_b) ||
-      (a->xn && (!a->w || a->ldn < a->H || (a->kind == TI_NORM_LAYER && !a->b))) ||
+      (a->w && !a->xn) || (a->xn && (a->ldn < a->H || (a->w && a->kind == TI_NORM_LAYER && !a->b))) ||
       (a->cat && (!a->x0 || a->ldc < 2 * a->H)))
     return ti_set_error(TI_ERR_ARG, "ti_rownorm: inconsistent arguments");
-  if (a->route_w && (!a->xn || !a->route_idx || !a->route_wgt || a->route_e < 1 || a->route_e > 64 || a->route_top < 1 ||
+  if (a->route_w && (!a->xn || !a->w || !a->route_idx || !a->route_wgt || a->route_e < 1 || a->route_e > 64 || a->route_top < 1 ||
                      a->route_top > a->route_e))
     return ti_set_error(TI_ERR_ARG, "ti_rownorm: routing arguments");
   return a->dtype == TI_DT_BF16 ? launch_rownorm<bf16>(*a, (hipStream_t)stream) : launch_rownorm<float>(*a, (hipStream_t)stream);
