@@ -74,16 +74,18 @@ void read_rglru(const Json& m, ti_stack_layer& L) {
   L.conv = m["conv"].integer();
 }
 
-void read_mlp(const Json& m, ti_stack_layer& L) {
+// The feed-forward of a design whose layers have this kind or none.
+void read_mlp(const Json& e, const char* design_kind, ti_stack_layer& L) {
   L.mlp = TI_MLP_NONE;
-  if (m.is_null()) return;
+  if (!e.has("mlp") || e["mlp"].is_null()) return;
+  const Json& m = e["mlp"];
   const std::string kind = m["kind"].string();
+  if (kind != design_kind) throw std::runtime_error("config.json: feed-forward kind \"" + kind + "\" is not supported");
   if (kind == "dense") {
     L.mlp = TI_MLP_DENSE;
     L.ff = m["ff"].integer();
     return;
   }
-  if (kind != "moe") throw std::runtime_error("config.json: feed-forward kind \"" + kind + "\" is not supported");
   L.mlp = TI_MLP_MOE;
   L.experts = m["router"]["experts"].integer();
   L.top = m["router"]["top"].integer();
@@ -104,8 +106,7 @@ StackSpec gegepel_spec(const Json& j) {
     const std::string type = e["type"].string();
     if (type != "latent_attention") throw std::runtime_error("config.json: layer type \"" + type + "\" is not supported");
     read_latent_attention(e["mixer"], L);
-    read_mlp(e.has("mlp") ? e["mlp"] : Json(), L);
-    if (L.mlp == TI_MLP_DENSE) throw std::runtime_error("config.json: feed-forward kind \"dense\" is not supported");
+    read_mlp(e, "moe", L);
     s.layers.push_back(L);
   }
   c.layers = (int)s.layers.size();
@@ -141,7 +142,7 @@ StackSpec nogitar_spec(const Json& j) {
     else if (type == "mamba2") read_mamba2(e["mixer"], L);
     else if (type == "rglru") read_rglru(e["mixer"], L);
     else throw std::runtime_error("config.json: layer type \"" + type + "\" is not supported");
-    read_mlp(e.has("mlp") ? e["mlp"] : Json(), L);
+    read_mlp(e, "dense", L);
     s.layers.push_back(L);
   }
   c.layers = (int)s.layers.size();
