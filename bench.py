@@ -40,6 +40,17 @@ STACKS = {
     "gegepel-4k": (32000, 4096, 4, (1, 3, 2), dict(heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512), 32, 4, 2816),
     "gegepel-1k": (32000, 1024, 8, (2, 6, 2), dict(heads=8, dim=64, rot_dim=32, vdim=64, q_rank=512, kv_rank=256), 32, 4, 768),
 }
+# layer-stack models (architecture "Nogitar"): three times [RG-LRU + feed-forward, Mamba-2, attention + feed-forward]
+# at the layer sizes of real hybrid models, the second attention sharing the first one's keys and values
+HYBRIDS = {
+    # name: (vocab, width, ff, attention, mamba2, rglru)
+    "nogitar-1k": (32000, 1024, 4096, dict(heads=8, kv_heads=2, dim=128, vdim=128),
+                   dict(heads=32, vdim=64, state=128, groups=1, norm_groups=1, conv=4), dict(width=1280, blocks=10, conv=4)),
+    "nogitar-2k": (32000, 2048, 8192, dict(heads=16, kv_heads=4, dim=128, vdim=128),
+                   dict(heads=64, vdim=64, state=128, groups=1, norm_groups=1, conv=4), dict(width=2560, blocks=10, conv=4)),
+    "nogitar-4k": (32000, 4096, 14336, dict(heads=32, kv_heads=8, dim=128, vdim=128),
+                   dict(heads=128, vdim=64, state=128, groups=8, norm_groups=8, conv=4), dict(width=4096, blocks=16, conv=4)),
+}
 MFMA_PEAK_TFS = 2500.0  # MI355X dense bf16 / fp16
 HBM_PEAK_GBS = 8000.0   # MI355X HBM3E spec peak (MI355X_MICROARCH.md, chip-level parameters)
 
@@ -173,7 +184,21 @@ def dry_run(g: "Group", args) -> int:
     return 0
 
 
+def hybrid_config(name: str) -> dict:
+    V, W, ff, at, ma, rg = HYBRIDS[name]
+    at = dict(at, scale=at["dim"] ** -0.5, q_temp=dict(coef=0.1, every=1024))
+    mlp = dict(kind="dense", ff=ff)
+    layers = []
+    for i in range(3):
+        layers += [dict(type="rglru", mixer=rg, mlp=mlp), dict(type="mamba2", mixer=ma, mlp=None),
+                   dict(type="attention", mixer=dict(at, kv_from=2) if i == 1 else at, mlp=mlp)]
+    return dict(architecture="Nogitar", vocab=V, width=W, norm=dict(eps=1e-5), layers=layers,
+                embedding=dict(scale=1.0, bigram=dict(buckets=65521, mul_prev=31337, mul_cur=1009)))
+
+
 def stack_config(name: str) -> dict:
+    if name in HYBRIDS:
+        return hybrid_config(name)
     V, W, n, (l0, l1, t), mx, E, top, ff = STACKS[name]
     mixer = dict(mx, rot=dict(base=10000.0, dims=mx["rot_dim"]), scale=(mx["dim"] + mx["rot_dim"]) ** -0.5)
     layer = dict(type="latent_attention", mixer=mixer, mlp=dict(kind="moe", expert=dict(ff=ff), router=dict(experts=E, top=top)))
@@ -182,9 +207,10 @@ def stack_config(name: str) -> dict:
 
 
 def stack_bench(args) -> int:
-    """Prefill and decode throughput of a layer-stack model (`--model gegepel-*`) beside the engine's llama
-    model at equal size: the same width, vocabulary, layer runs, heads of 128, and a dense feed-forward as
-    wide as the experts a token uses, fp16 weights (as many bytes per weight).  Both in this process, on
+    """Prefill and decode throughput of a layer-stack model (`--model gegepel-*`, `nogitar-*`) beside the
+    engine's llama model at equal size: the same width, vocabulary, layer runs, heads of 128, and a dense
+    feed-forward as wide as the experts a token uses (nogitar: as many feed-forward weights per layer that
+    has one; its heads and key/value heads), fp16 weights (as many bytes per weight).  Both in this process, on
     one GPU, timed in turn: decode is the replayed step graph at position kv - 1, prefill one prompt of
     --stack-prompts tokens to its last logits, each the best of --steps / 3 repetitions."""
     import numpy as np
@@ -192,7 +218,12 @@ def stack_bench(args) -> int:
     T.init(0)
     name, L = args.model, args.kv
     cfg = stack_config(name)
-    V, W, _, _, mx, E, top, ff = STACKS[name]
+    if name in HYBRIDS:
+        V, W, ff, at, _, _ = HYBRIDS[name]
+        heads, kv_heads, inter = at["heads"], at["kv_heads"], 2 * ff // 3 // 128 * 128
+    else:
+        V, W, _, _, _, _, top, ff = STACKS[name]
+        heads, kv_heads, inter = W // 128, W // 128, top * ff
     batches = [int(b) for b in args.stack_batches.split(",")]
     prompts = [int(p) for p in args.stack_prompts.split(",")]
     out = {"metric": "layer-stack decode / prefill tokens/s (one GPU) beside the llama engine at equal size", "value": None,
@@ -236,8 +267,7 @@ def stack_bench(args) -> int:
     e.close()
     ld = lp = None
     if not args.no_llama:
-        h = W // 128
-        e = T.Engine(V, W, runs, h, h, 128, top * ff, bits=16, max_seq=seq, max_batch=max(batches))
+        e = T.Engine(V, W, runs, heads, kv_heads, 128, inter, bits=16, max_seq=seq, max_batch=max(batches))
         e.synth(args.seed, 0.0)
         ld, lp = measure(e, runs)
         lwb = e.memory()[0]
@@ -308,8 +338,8 @@ def main() -> int:
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--batch", type=int, default=1, help="decode streams per GPU")
     ap.add_argument("--kv", type=int, default=2048, help="KV length read per step")
-    ap.add_argument("--model", default="llama2-7b", choices=sorted(MODELS) + sorted(STACKS),
-                    help="gegepel-*: the layer-stack benchmark (decode and prefill beside llama at equal size)")
+    ap.add_argument("--model", default="llama2-7b", choices=sorted(MODELS) + sorted(STACKS) + sorted(HYBRIDS),
+                    help="gegepel-*, nogitar-*: the layer-stack benchmark (decode and prefill beside llama at equal size)")
     ap.add_argument("--stack-batches", default="1,16,64", help="decode streams, layer-stack benchmark")
     ap.add_argument("--stack-prompts", default="512,2048", help="prompt lengths, layer-stack benchmark")
     ap.add_argument("--stack-dtype", default="bfloat16", choices=("bfloat16", "float32"))
@@ -324,7 +354,7 @@ def main() -> int:
                          "no engine; prints the JSON line with value null (tests)")
     args = ap.parse_args()
 
-    if args.model in STACKS:
+    if args.model in STACKS or args.model in HYBRIDS:
         if args.gpus != 1:
             print("bench.py: the layer-stack benchmark runs on one GPU", file=sys.stderr)
             return 2

@@ -420,6 +420,8 @@ typedef struct ti_step_args {
   const float* pe_hi;
   const float* pe_lo;
   int32_t pe_ld;
+  void* xn;                          /* nullable [M][xn_ld]: the row in the table's element type (emb_kind > 0) */
+  int32_t xn_ld;
 } ti_step_args;
 int ti_step_begin(const ti_step_args* a, ti_stream_t s);
 

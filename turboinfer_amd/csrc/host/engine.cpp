@@ -414,6 +414,10 @@ void step_embedding(ti_engine* e, ti_step_args& sa) {
   sa.pe_hi = e->stack->pe_hi;
   sa.pe_lo = e->stack->pe_lo;
   sa.pe_ld = e->stack->pe_ld;
+  if (k.norm_place == TI_PLACE_POST && k.loop_times == 0) {   // the first layer reads the embedding itself
+    sa.xn = e->stack->xn;
+    sa.xn_ld = e->stack->xn_ld;
+  }
 }
 
 // Models whose layers carry a state go on only where a slot's state stands.
@@ -462,6 +466,7 @@ int enqueue_step(ti_engine* e, int M, int advance) {
     TI_TRY(ti_step_begin(&sa, e->s));
     ti_host::StackRows r;
     r.slots = sa.slot;
+    r.xn_ready = sa.xn != nullptr;
     r.M = M;
     r.pos = e->pos;
     r.h = e->h;
@@ -685,6 +690,7 @@ int enqueue_prefill(ti_engine* e, int m, int t0, int rows, int base, float* laye
     r.pos = e->pos;
     r.h = e->h;
     r.h0 = e->stack->h0;
+    r.xn_ready = sa.xn != nullptr;
     r.chunk = true;
     r.slot = m;
     r.pos0 = base + t0;

@@ -336,7 +336,8 @@ int StackModel::alloc_work() {
       tiles = std::max<size_t>(tiles, (size_t)8 * k.top);
     }
   }
-  TI_TRY(alloc(&xn_, R * kpad(W) * es));
+  xn_ld = kpad(W);
+  TI_TRY(alloc(&xn, R * xn_ld * es));
   TI_TRY(alloc(&cq_, R * cq * es));
   TI_TRY(alloc(&q_, R * q * es));
   TI_TRY(alloc(&qa_, (size_t)dec_rows * qa * es));
@@ -551,7 +552,7 @@ int StackModel::attention(const StackLayer& L, const StackRun& run, const StackR
   const int ldat = kpad(k.heads * k.vdim);
   char* cache = static_cast<char*>(run.cache) + (r.chunk ? (size_t)r.slot * seq_p * cw * esize() : 0);
   const int64_t stride = r.chunk ? 0 : (int64_t)seq_p * cw;
-  TI_TRY(dense(L.a, xn_, kpad(c.width), M, a32_, lda32, TI_DE_F32, {}));
+  TI_TRY(dense(L.a, xn, kpad(c.width), M, a32_, lda32, TI_DE_F32, {}));
   ti_latent_prep_args p{};
   p.a32 = a32_;
   p.lda = lda32;
@@ -685,7 +686,7 @@ int StackModel::experts(const StackLayer& L, int M) {
   const ti_stack_layer& k = L.c;
   const int W = c.width, ldx = kpad(W), ldact = kpad(k.ff);
   const bool routed = fused_router(L, M);   // idx_ / wgt_ written by the norm's launch
-  if (!routed) TI_TRY(dense(L.router, xn_, ldx, M, zr_, k.experts, TI_DE_F32, {}));
+  if (!routed) TI_TRY(dense(L.router, xn, ldx, M, zr_, k.experts, TI_DE_F32, {}));
   ti_route_args ra{};
   ra.logits = routed ? nullptr : zr_;
   ra.ld = k.experts;
@@ -716,7 +717,7 @@ int StackModel::experts(const StackLayer& L, int M) {
     g.n_tiles = n_tiles_;
     g.rows_in = list_;
   }
-  TI_TRY(dense(L.gu, xn_, ldx, M, act_, ldact, TI_DE_SWIGLU, g));
+  TI_TRY(dense(L.gu, xn, ldx, M, act_, ldact, TI_DE_SWIGLU, g));
   g.rows_in = nullptr;
   g.row_div = 1;
   if (!direct) g.rows_out = list_;
@@ -752,7 +753,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
     if (pre || copy) {
       n.w = pre;
       n.b = pre ? pre + W : nullptr;
-      n.xn = xn_;
+      n.xn = xn;
       n.ldn = kpad(W);
     }
     if (cat) {
@@ -784,7 +785,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
       TI_TRY(dense(loop_in_, cat_, kpad(2 * W), M, r.h, W, TI_DE_F32, d));
     }
     const bool sandwich = c.norm_place == TI_PLACE_SANDWICH;
-    TI_TRY(rownorm(sandwich ? L.n1 : nullptr, nullptr, nullptr, !sandwich));
+    if (sandwich || i || !r.xn_ready) TI_TRY(rownorm(sandwich ? L.n1 : nullptr, nullptr, nullptr, !sandwich));
     switch (L.c.mixer) {
       case TI_MIX_GQA: TI_TRY(gqa(L, run[i], r)); break;
       case TI_MIX_SSD: TI_TRY(ssd(L, run[i], r)); break;
@@ -813,7 +814,7 @@ int StackModel::forward(const StackRows& r, bool with_head, float* logits, unsig
   d.argmax = argmax;
   d.step_ctr = step_ctr;
   d.advance = advance;
-  return dense(head_, xn_, kpad(W), M, logits, c.vocab, TI_DE_LOGITS, d);
+  return dense(head_, xn, kpad(W), M, logits, c.vocab, TI_DE_LOGITS, d);
 }
 
 int StackModel::head(float* h, int M, float* logits, unsigned long long* argmax) {
@@ -822,7 +823,7 @@ int StackModel::head(float* h, int M, float* logits, unsigned long long* argmax)
   n.x = h;
   n.w = final_norm_;
   n.b = final_norm_ + W;
-  n.xn = xn_;
+  n.xn = xn;
   n.ldn = kpad(W);
   n.eps = c.eps;
   n.M = M;
@@ -832,7 +833,7 @@ int StackModel::head(float* h, int M, float* logits, unsigned long long* argmax)
   TI_TRY(ti_rownorm(&n, s_));
   ti_dense_args d{};
   d.argmax = argmax;
-  return dense(head_, xn_, kpad(W), M, logits, c.vocab, TI_DE_LOGITS, d);
+  return dense(head_, xn, kpad(W), M, logits, c.vocab, TI_DE_LOGITS, d);
 }
 
 }  // namespace ti_host

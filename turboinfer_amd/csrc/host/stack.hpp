@@ -58,6 +58,7 @@ struct StackRows {
   bool chunk = false;
   int slot = 0, pos0 = 0;         // chunk: stream slot and first position (host)
   const int32_t* slots = nullptr; // decode, device [M], nullable: the rows' stream slots (NULL: row m is slot m)
+  bool xn_ready = false;          // the embedding's element-type rows are in xn already
   float* layers_out = nullptr;    // host, nullable: residual after every run, run stride layers_stride rows
   size_t layers_stride = 0;
 };
@@ -82,6 +83,8 @@ class StackModel {
   int32_t* hist = nullptr;      // [max_batch][seq_p] tokens by position (with a bigram table)
   float *pe_hi = nullptr, *pe_lo = nullptr;   // sinusoidal position vectors (ti_hip.h ti_step_args)
   int pe_ld = 0;
+  void* xn = nullptr;           // T [rows_cap][kpad(width)]: input rows of the next product
+  int xn_ld = 0;
   bool recurrent = false;       // some layer carries a state: a slot only goes on where it stands
 
   ~StackModel();
@@ -105,7 +108,7 @@ class StackModel {
   StackPack loop_in_, head_;
   float *loop_step_ = nullptr, *final_norm_ = nullptr;
   // work buffers
-  void *xn_ = nullptr, *cat_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *qa_ = nullptr, *olat_ = nullptr, *attn_ = nullptr,
+  void *cat_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *qa_ = nullptr, *olat_ = nullptr, *attn_ = nullptr,
        *act_ = nullptr, *parts_ = nullptr, *kfrag_ = nullptr, *vfrag_ = nullptr, *part_o_ = nullptr;
   float *a32_ = nullptr, *gate_ = nullptr, *y_ = nullptr, *zr_ = nullptr, *wgt_ = nullptr, *part_ml_ = nullptr, *stage_ = nullptr;
   int32_t *idx_ = nullptr, *list_ = nullptr, *tiles_ = nullptr, *n_tiles_ = nullptr, *map_ = nullptr;

@@ -1,7 +1,7 @@
 // stack_mixers.cpp -- grouped-query attention, SSD and RG-LRU layers and the dense feed-forward of the
 // layer-stack models (stack.hpp).
 //
-// Every mixer reads the rows xn_ and leaves its output product's fp32 rows in y_:
+// Every mixer reads the rows xn and leaves its output product's fp32 rows in y_:
 //   attention  dense [queries | keys | values | gates]; prep (norms, query scale, cache append); attention
 //              over the cache's fragments with the gate behind it; output product
 //   SSD        dense in projection (step sizes fp32); rows of many slots: convolution and recurrence in one
@@ -275,7 +275,7 @@ int StackModel::gqa(const StackLayer& L, const StackRun& run, const StackRows& r
   const ti_stack_layer& k = L.c;
   const int M = r.M, lda = up(L.na, 4), ldo = kpad(k.heads * k.vdim);
   char* cache = static_cast<char*>(run.cache) + (r.chunk ? (size_t)r.slot * run.cache_slot : 0);
-  TI_TRY(dense(L.a, xn_, kpad(c.width), M, a32_, lda, TI_DE_F32, {}));
+  TI_TRY(dense(L.a, xn, kpad(c.width), M, a32_, lda, TI_DE_F32, {}));
   ti_gqa_prep_args p{};
   p.a32 = a32_;
   p.lda = lda;
@@ -337,7 +337,7 @@ int StackModel::ssd(const StackLayer& L, const StackRun& run, const StackRows& r
   da.t_cols = L.na - k.heads;
   da.out2 = dt_;
   da.ld2 = k.heads;
-  TI_TRY(dense(L.a, xn_, kpad(c.width), M, proj_, lda, TI_DE_ACT, da));
+  TI_TRY(dense(L.a, xn, kpad(c.width), M, proj_, lda, TI_DE_ACT, da));
   ti_ssd_args s{};
   s.dt = dt_;
   s.dt_bias = L.dt_bias;
@@ -421,7 +421,7 @@ int StackModel::rglru(const StackLayer& L, const StackRun& run, const StackRows&
   da.act = TI_ACT_GELU_TANH;
   da.act_cols = w;
   da.t_cols = L.na;
-  TI_TRY(dense(L.a, xn_, kpad(c.width), M, proj_, lda, TI_DE_ACT, da));
+  TI_TRY(dense(L.a, xn, kpad(c.width), M, proj_, lda, TI_DE_ACT, da));
   ti_conv_args v{};
   v.x = x;
   v.ring = run.ring;
@@ -482,7 +482,7 @@ int StackModel::dense_mlp(const StackLayer& L, int M) {
   ti_dense_args d{};
   d.act = TI_ACT_GELU_ERF;
   d.act_cols = d.t_cols = L.c.ff;
-  TI_TRY(dense(L.up, xn_, kpad(c.width), M, act_, ldact, TI_DE_ACT, d));
+  TI_TRY(dense(L.up, xn, kpad(c.width), M, act_, ldact, TI_DE_ACT, d));
   return dense(L.down, act_, ldact, M, y_, c.width, TI_DE_F32, {});
 }
 

@@ -23,8 +23,21 @@ __device__ __forceinline__ unsigned long long logit_key(float v, int n) {
 
 __device__ __forceinline__ float activate(int act, float z) {
   if (act == TI_ACT_GELU_ERF) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
-  if (act == TI_ACT_GELU_TANH) return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * fmaf(0.044715f * z * z, z, z)));
+  // (1 + tanh x) / 2 is the logistic function of 2 x
+  if (act == TI_ACT_GELU_TANH) return z * fast_sigmoid(1.59576912160573072f * fmaf(0.044715f * z * z, z, z));
   return z;
+}
+
+// 1 - exp(y), y <= 0: its series near 0, where the difference would cancel.
+__device__ __forceinline__ float one_minus_exp(float y) {
+  float s = fmaf(y, 1.0f / 40320.0f, 1.0f / 5040.0f);
+  s = fmaf(y, s, 1.0f / 720.0f);
+  s = fmaf(y, s, 1.0f / 120.0f);
+  s = fmaf(y, s, 1.0f / 24.0f);
+  s = fmaf(y, s, 1.0f / 6.0f);
+  s = fmaf(y, s, 0.5f);
+  s = fmaf(y, s, 1.0f);
+  return y > -0.5f ? -y * s : 1.0f - fast_exp(y);
 }
 
 // Four consecutive output columns n0.. of row m (out row mo); rows >= rows are padding.
@@ -126,9 +139,9 @@ __device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, i
         const int j = (n0 >> 1) + i, c = batch * per + j;
         if (j >= per) return;
         const float* gb = a.add + (size_t)batch * a.N + n0 + 2 * i;
-        const float la = -sigmoidf(v[2 * i] + gb[0]) * a.lru_rate[c];
+        const float la = -fast_sigmoid(v[2 * i] + gb[0]) * a.lru_rate[c];
         const float u = (float)((const T*)a.a)[(size_t)m * a.lda + (size_t)batch * a.a_batch + j];
-        const float av = expf(la), bv = sqrtf(-expm1f(2.0f * la)) * sigmoidf(v[2 * i + 1] + gb[1]) * u;
+        const float av = fast_exp(la), bv = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * la)) * fast_sigmoid(v[2 * i + 1] + gb[1]) * u;
         if (!a.lru_state) {
           *(float2*)((float*)a.out + ((size_t)m * channels + c) * 2) = make_float2(av, bv);
         } else {

@@ -105,6 +105,11 @@ __device__ __forceinline__ void route_top64(float v, int E, int top, int32_t* id
   }
 }
 
+// exp and the logistic function through the hardware exponential and reciprocal (about an ulp each; the
+// exponential's argument rounding adds |z| * 2^-24 relative).
+__device__ __forceinline__ float fast_exp(float z) { return __builtin_amdgcn_exp2f(z * 1.44269504088896340736f); }
+__device__ __forceinline__ float fast_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + fast_exp(-z)); }
+
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 }  // namespace ti

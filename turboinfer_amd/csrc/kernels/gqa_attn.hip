@@ -65,6 +65,65 @@ __global__ __launch_bounds__(512) void gqa_prep_kernel(const ti_gqa_prep_args a)
   }
 }
 
+// The same with head and value sizes that are multiples of 4 and at most NC * 2048 projected values: a thread
+// holds its quads in registers, every load in flight before the sums.
+template <class T, int NC>
+__global__ __launch_bounds__(512) void gqa_prep_vec_kernel(const ti_gqa_prep_args a) {
+  typedef typename El<T>::Q Q;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC;
+  __shared__ float red[8];
+  const int m = blockIdx.x, tid = threadIdx.x, nq4 = a.heads * a.dim >> 2, dim_p = gqa_dim_p<T>(a.dim), vdim_p = gqa_vdim_p(a.vdim);
+  const bool kv = a.k_off >= 0;
+  const int nk4 = kv ? a.kv_heads * a.dim >> 2 : 0, n4 = nq4 + nk4 + (kv ? a.kv_heads * a.vdim >> 2 : 0);
+  const int pos = a.pos[m], slot = a.slot ? a.slot[m] : m;
+  const float* src = a.a32 + (size_t)m * a.lda;
+  f32x4 x[NC], w[NC];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = tid + 512 * c, k = i - nq4, v = k - nk4;
+    const float* s = i < nq4 ? src + 4 * i : v < 0 ? src + a.k_off + 4 * k : src + a.v_off + 4 * v;
+    const float* ws = i < nq4 ? a.q_w + 4 * i : a.k_w + 4 * k;
+    x[c] = w[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    if (i < n4) x[c] = *(const f32x4*)s;
+    if (i < nq4 + nk4) w[c] = *(const f32x4*)ws;
+  }
+  const float temp = a.q_scale ? a.q_scale[pos] : 1.0f;
+  float q2 = 0.0f, k2 = 0.0f;
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = tid + 512 * c;
+    const float s = (x[c][0] * x[c][0] + x[c][1] * x[c][1]) + (x[c][2] * x[c][2] + x[c][3] * x[c][3]);
+    if (i < nq4) q2 += s;
+    else if (i < nq4 + nk4) k2 += s;
+  }
+  const float qi = temp / sqrtf(block_sum(q2, red) / (float)(4 * nq4) + a.eps);
+  const float ki = kv ? 1.0f / sqrtf(block_sum(k2, red) / (float)(4 * nk4) + a.eps) : 0.0f;
+  const int be = 64 * (dim_p + vdim_p), p = pos & 63, nkt = dim_p / KT;
+  T* blk = (T*)a.cache + (size_t)slot * a.slot_stride + (size_t)(pos >> 6) * be;
+  const size_t hs = (size_t)(a.seq_p >> 6) * be;
+  T* q = (T*)a.q + (size_t)m * a.heads * dim_p;
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = tid + 512 * c, k = i - nq4, v = k - nk4;
+    if (i < nq4) {
+      const int h = 4 * i / a.dim, d = 4 * i - h * a.dim;
+      *(Q*)(q + h * dim_p + d) = quad<T>(x[c] * qi * w[c]);
+    } else if (v < 0) {
+      const int h = 4 * k / a.dim, d = 4 * k - h * a.dim;
+      *(Q*)(blk + h * hs + ((size_t)((p >> 4) * nkt + d / KT) * 64 + (d % KT) / VEC * 16 + (p & 15)) * VEC + d % VEC) =
+          quad<T>(x[c] * ki * w[c]);
+    } else if (i < n4) {
+      const int h = 4 * v / a.vdim, d = 4 * v - h * a.vdim;
+      T* o = blk + h * hs + 64 * dim_p + ((size_t)((d >> 4) * (64 / KT) + p / KT) * 64 + ((p & 15) >> 2) * 16 + (d & 15)) * VEC +
+             (p % KT >> 4) * 4 + (p & 3);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e * VEC] = (T)x[c][e];
+    }
+  }
+  const int pad = dim_p - a.dim;   // (the queries' k padding)
+  for (int i = tid; i < a.heads * pad; i += 512) q[i / pad * dim_p + a.dim + i % pad] = (T)0.0f;
+}
+
 // The weights' operand fragment of one KT span: row[] holds 64 positions' weights of this lane's column.
 __device__ __forceinline__ bf16x8 weight_frag(const bf16* row, int g) {
   const bf16x4 lo = *(const bf16x4*)(row + 4 * g), hi = *(const bf16x4*)(row + 16 + 4 * g);
@@ -185,7 +244,7 @@ __global__ __launch_bounds__(256, 2) void gqa_decode_kernel(const ti_gqa_attn_ar
     for (int r = 0; r < 4; ++r) {
       if (d0 + r >= a.vdim) continue;
       const int c = head * a.vdim + d0 + r;
-      const float gt = a.gate ? sigmoidf(a.gate[(size_t)m * a.ldg + c]) : 1.0f;
+      const float gt = a.gate ? fast_sigmoid(a.gate[(size_t)m * a.ldg + c]) : 1.0f;
       ((T*)a.out)[(size_t)m * a.ldo + c] = (T)(o[i][r] * inv * gt);
     }
   }
@@ -225,7 +284,7 @@ __global__ __launch_bounds__(256) void gqa_merge_kernel(const ti_gqa_attn_args a
       }
     }
     const int c = h * a.vdim + d;
-    const float gt = a.gate ? sigmoidf(a.gate[(size_t)m * a.ldg + c]) : 1.0f;
+    const float gt = a.gate ? fast_sigmoid(a.gate[(size_t)m * a.ldg + c]) : 1.0f;
     ((T*)a.out)[(size_t)m * a.ldo + c] = (T)(acc * gt);
   }
 }
@@ -378,7 +437,7 @@ __global__ __launch_bounds__(256, NV * MQ > 16 ? 1 : 2) void gqa_prefill_kernel(
         for (int r = 0; r < 4; ++r) {
           if (d + r >= a.vdim) continue;
           const int c = h * a.vdim + d + r;
-          const float gt = a.gate ? sigmoidf(a.gate[(size_t)m * a.ldg + c]) : 1.0f;
+          const float gt = a.gate ? fast_sigmoid(a.gate[(size_t)m * a.ldg + c]) : 1.0f;
           ((T*)a.out)[(size_t)m * a.ldo + c] = (T)(x[r] * inv * gt);
         }
       }
@@ -464,6 +523,19 @@ extern "C" int ti_gqa_prep(const ti_gqa_prep_args* a, ti_stream_t stream) {
       a->seq_p < 64 || a->seq_p % 64 || (a->dtype != TI_DT_BF16 && a->dtype != TI_DT_F32) || a->lda < a->heads * a->dim ||
       (a->k_off >= 0 && (!a->k_w || !a->cache || a->lda < a->k_off + a->kv_heads * a->dim || a->lda < a->v_off + a->kv_heads * a->vdim)))
     return ti_set_error(TI_ERR_ARG, "ti_gqa_prep: bad arguments");
+  const int n = (a->heads + (a->k_off >= 0 ? a->kv_heads : 0)) * a->dim + (a->k_off >= 0 ? a->kv_heads * a->vdim : 0);
+  if (((a->dim | a->vdim | a->lda) & 3) == 0 && (a->k_off < 0 || ((a->k_off | a->v_off) & 3) == 0) && n <= 4 * 2048) {
+    hipStream_t s = (hipStream_t)stream;
+    auto launch = [&]<int NC>() {
+      if (a->dtype == TI_DT_BF16) hipLaunchKernelGGL((gqa_prep_vec_kernel<bf16, NC>), dim3(a->M), dim3(512), 0, s, *a);
+      else hipLaunchKernelGGL((gqa_prep_vec_kernel<float, NC>), dim3(a->M), dim3(512), 0, s, *a);
+    };
+    if (n <= 2048) launch.template operator()<1>();
+    else if (n <= 2 * 2048) launch.template operator()<2>();
+    else launch.template operator()<4>();
+    TI_LAUNCH_CHECK("gqa_prep_vec_kernel");
+    return TI_OK;
+  }
   const size_t lds = (size_t)(a->heads + a->kv_heads) * a->dim * 4;
   if (lds > 131072) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_gqa_prep: %d + %d heads of %d", a->heads, a->kv_heads, a->dim);
   if (a->dtype == TI_DT_BF16)

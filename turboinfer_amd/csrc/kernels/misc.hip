@@ -16,6 +16,69 @@ __global__ __launch_bounds__(256) void step_begin_kernel(const ti_step_args a, u
   step_begin_body(a);
   stamp_end(stamp, t_entry);
 }
+// The embedding row of a layer-stack model: table row, bigram row and position vector, VQ entries a thread
+// and pass, two passes' loads in flight.
+struct StackRow {
+  int kind;
+  size_t tok, pair;
+  const float *hi, *lo;
+};
+template <int VQ>
+__device__ __forceinline__ void stack_row(const ti_step_args& a, const StackRow& r, int m) {
+  typedef float fv __attribute__((ext_vector_type(VQ)));
+  typedef uint16_t hv __attribute__((ext_vector_type(VQ)));
+  constexpr int U = 2;
+  auto load = [&](const void* t, size_t i) -> fv {
+    if (r.kind == 2) return *(const fv*)((const float*)t + i);
+    const hv h = *(const hv*)((const uint16_t*)t + i);
+    fv v;
+#pragma unroll
+    for (int e = 0; e < VQ; ++e) v[e] = __builtin_bit_cast(float, (uint32_t)h[e] << 16);
+    return v;
+  };
+  const int n = a.hidden / VQ;
+  for (int i0 = threadIdx.x; i0 < n; i0 += 256 * U) {
+    fv v[U], g[U];
+    float p[U][VQ + 1], q[U][VQ + 1];   // (the whole (sine, cosine) pairs)
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = min(i0 + 256 * u, n - 1) * VQ;
+      v[u] = load(a.emb, r.tok + i);
+      if (a.bigram) g[u] = load(a.bigram, r.pair + i);
+      if (r.hi)
+#pragma unroll
+        for (int e = 0; e < (VQ > 1 ? VQ : 2); ++e) {
+          p[u][e] = r.hi[(i & ~1) + e];
+          q[u][e] = r.lo[(i & ~1) + e];
+        }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (i0 + 256 * u >= n) continue;
+      const int i = (i0 + 256 * u) * VQ;
+#pragma unroll
+      for (int e = 0; e < VQ; ++e) {
+        v[u][e] *= a.emb_scale;
+        if (a.bigram) v[u][e] += g[u][e];
+        if (r.hi) {   // the angles' sum
+          const int k = e & ~1;
+          v[u][e] += ((i + e) & 1) ? p[u][k + 1] * q[u][k + 1] - p[u][k] * q[u][k] : fmaf(p[u][k], q[u][k + 1], p[u][k + 1] * q[u][k]);
+        }
+      }
+      *(fv*)(a.h + (size_t)m * a.hidden + i) = v[u];
+      if (a.h0) *(fv*)(a.h0 + (size_t)m * a.hidden + i) = v[u];
+      if (a.xn && r.kind == 2) {
+        *(fv*)((float*)a.xn + (size_t)m * a.xn_ld + i) = v[u];
+      } else if (a.xn) {
+        typedef __bf16 bv __attribute__((ext_vector_type(VQ)));
+        bv o;
+#pragma unroll
+        for (int e = 0; e < VQ; ++e) o[e] = (__bf16)v[u][e];
+        *(bv*)((__bf16*)a.xn + (size_t)m * a.xn_ld + i) = o;
+      }
+    }
+  }
+}
 __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
   __shared__ int s_tok, s_row;
   const int m = blockIdx.x, tid = threadIdx.x;
@@ -37,6 +100,15 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
   const int s = *a.step_ctr;
   const int nin = a.n_in ? a.n_in[m] : 0;
   unsigned long long* am = a.argmax + (size_t)m * TI_ARGMAX_SLOTS;
+  // the previous token, while the argmax is read (a chunk's rows run side by side: only its first one reads
+  // what an earlier launch wrote)
+  int32_t* hist = nullptr;
+  int prev = 0;
+  const int pos0 = a.bigram ? a.base_pos[m] + s : 0;
+  if (a.bigram && tid == 0) {
+    hist = a.hist + (size_t)(a.chunk ? a.slot0 : a.slot ? a.slot[m] : m) * a.hist_ld;
+    if (pos0 > 0) prev = a.chunk && m > 0 ? a.in_tokens[m - 1] : hist[pos0 - 1];
+  }
   unsigned long long key = 0ull;
   if (tid < 64) {   // row m's key = max over its slots (wave 0)
     key = tid < TI_ARGMAX_SLOTS ? am[tid] : 0ull;
@@ -58,18 +130,14 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
     }
     if (tok < 0 || tok >= a.vocab) tok = 0;     // never index outside the table
     s_tok = tok;
-    const int pos = a.base_pos[m] + s;
-    a.pos[m] = pos;
+    a.pos[m] = a.base_pos[m] + s;
     if (a.bigram) {
-      int32_t* hist = a.hist + (size_t)(a.chunk ? a.slot0 : a.slot ? a.slot[m] : m) * a.hist_ld;
-      s_row = a.buckets;
-      if (pos > 0) {   // (a chunk's rows run side by side: only its first one reads what an earlier launch wrote)
-        int prev = a.chunk && m > 0 ? a.in_tokens[m - 1] : hist[pos - 1];
-        if (prev < 0 || prev >= a.vocab) prev = 0;
-        s_row = (int)(((int64_t)prev * a.mul_prev + (int64_t)tok * a.mul_cur) % a.buckets);
-        if (s_row < 0) s_row += a.buckets;
-      }
-      hist[pos] = tok;
+      if (prev < 0 || prev >= a.vocab) prev = 0;
+      const int64_t x = (int64_t)prev * a.mul_prev + (int64_t)tok * a.mul_cur;
+      int row = x >> 32 ? (int)(x % a.buckets) : (int)((uint32_t)x % (uint32_t)a.buckets);   // (long division: slow)
+      if (row < 0) row += a.buckets;
+      s_row = pos0 > 0 ? row : a.buckets;
+      hist[pos0] = tok;
     }
   }
   __syncthreads();   // every slot read before any is cleared
@@ -83,26 +151,12 @@ __device__ __forceinline__ void step_begin_body(const ti_step_args a) {
       h[i] = 0.1f * (float)((off + (size_t)i) % 100);
     }
   } else if (a.emb_kind) {
-    const size_t r0 = (size_t)s_tok * a.hidden;
-    float* h0 = a.h0 ? a.h0 + (size_t)m * a.hidden : nullptr;
-    const size_t b0 = a.bigram ? (size_t)s_row * a.hidden : 0;
     const int pos = a.base_pos[m] + s;
-    const float* hi = a.pe_hi ? a.pe_hi + (size_t)(pos >> 8) * a.pe_ld : nullptr;
-    const float* lo = a.pe_hi ? a.pe_lo + (size_t)(pos & 255) * a.pe_ld : nullptr;
-    auto elem = [&](const void* t, size_t i) {
-      return a.emb_kind == 1 ? __builtin_bit_cast(float, (uint32_t)((const uint16_t*)t)[i] << 16) : ((const float*)t)[i];
-    };
-    for (int i = tid; i < a.hidden; i += 256) {
-      float v = a.emb_scale * elem(a.emb, r0 + i);
-      if (a.bigram) v += elem(a.bigram, b0 + i);
-      if (hi) {   // the angles' sum: (sine, cosine) at the even and odd entry of a pair
-        const int e = i & ~1;
-        const float2 p = *(const float2*)(hi + e), q = *(const float2*)(lo + e);
-        v += (i & 1) ? p.y * q.y - p.x * q.x : fmaf(p.x, q.y, p.y * q.x);
-      }
-      h[i] = v;
-      if (h0) h0[i] = v;
-    }
+    const StackRow r = {a.emb_kind, (size_t)s_tok * a.hidden, a.bigram ? (size_t)s_row * a.hidden : 0,
+                        a.pe_hi ? a.pe_hi + (size_t)(pos >> 8) * a.pe_ld : nullptr,
+                        a.pe_hi ? a.pe_lo + (size_t)(pos & 255) * a.pe_ld : nullptr};
+    if ((a.hidden & 3) == 0 && (a.xn_ld & 3) == 0) stack_row<4>(a, r, m);
+    else stack_row<1>(a, r, m);
   } else if (vec) {
     const uint16_t* e = a.emb + (size_t)s_tok * a.hidden;
     f16x8 ev[kPT];
@@ -306,7 +360,7 @@ extern "C" int ti_step_begin(const ti_step_args* a, ti_stream_t stream) {
   if (a->emb_kind < 0 || a->emb_kind > 2 || (a->emb_kind && (a->fold_x || a->placeholder_first >= 0)) || (a->h0 && !a->emb_kind))
     return ti_set_error(TI_ERR_ARG, "ti_step_begin: emb_kind %d", a->emb_kind);
   if ((a->bigram && (!a->emb_kind || !a->hist || a->buckets < 1)) || (a->pe_hi && (!a->emb_kind || !a->pe_lo || a->pe_ld < a->hidden || a->pe_ld % 2)) ||
-      (a->chunk && a->in_stride != 1))
+      (a->chunk && a->in_stride != 1) || (a->xn && (!a->emb_kind || a->xn_ld < a->hidden)))
     return ti_set_error(TI_ERR_ARG, "ti_step_begin: embedding terms");
   hipLaunchKernelGGL(step_begin_kernel, dim3(a->M), dim3(256), 0, (hipStream_t)stream, *a,
                      ti_stamp_next(STAMP_BEGIN, a->M));

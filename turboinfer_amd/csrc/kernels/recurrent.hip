@@ -15,7 +15,6 @@
 
 namespace ti {
 
-__device__ __forceinline__ float siluf(float z) { return z * sigmoidf(z); }
 __device__ __forceinline__ float softplusf(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
 // ------------------------------------------------------------------ short convolution
@@ -58,9 +57,66 @@ __global__ __launch_bounds__(256) void conv_kernel(const ti_conv_args a, int pla
       }
       if (!a.chunk) *(TV*)(ring + (size_t)(pos % a.taps) * a.channels) = cur;
 #pragma unroll
-      for (int e = 0; e < VQ; ++e) o[e] = (T)(a.act == TI_CONV_SILU ? siluf(acc[e]) : acc[e]);
+      for (int e = 0; e < VQ; ++e) o[e] = (T)(a.act == TI_CONV_SILU ? acc[e] * fast_sigmoid(acc[e]) : acc[e]);
     }
     *(TV*)((T*)a.out + (size_t)m * a.ldo + i0) = o;
+  }
+}
+
+// The same for TAPS known and 16-byte places (VEC channels): a thread slides over R rows of a chunk with all
+// their inputs in flight, or takes one row of its own slot (DEC).
+template <class T, int TAPS, bool DEC>
+__global__ __launch_bounds__(256) void conv_vec_kernel(const ti_conv_args a, int places) {
+  typedef typename El<T>::V V;
+  constexpr int VEC = El<T>::VEC, R = DEC ? 1 : 8, NX = R + TAPS - 1;
+  const int i0 = ((int)blockIdx.x * 64 + (int)(threadIdx.x & 63)) * VEC, m0 = ((int)blockIdx.y * 4 + (int)(threadIdx.x >> 6)) * R;
+  if (i0 >= places || m0 >= a.M) return;
+  int c0 = i0;
+  if (i0 >= a.c0) {
+    const int s = i0 - a.o0, r = s % a.bwp;
+    c0 = s >= 0 && r < a.bw ? a.c0 + s / a.bwp * a.bw + r : -1;
+    if (s < 0 && i0 < a.o0) return;
+  }
+  T* out = (T*)a.out + (size_t)m0 * a.ldo + i0;
+  if (c0 < 0) {
+    const V z = {};
+    for (int r = 0; r < R && m0 + r < a.M; ++r) *(V*)(out + (size_t)r * a.ldo) = z;
+    return;
+  }
+  const int pos = a.pos[m0];
+  T* ring = (T*)a.ring + (size_t)(a.chunk ? a.slot0 : a.slot ? a.slot[m0] : m0) * a.taps * a.channels + c0;
+  V x[NX];   // x[i]: the input i - (TAPS - 1) rows after m0
+#pragma unroll
+  for (int i = 0; i < NX; ++i) {
+    const int d = i - (TAPS - 1);
+    const T* src = d >= 0 || (!DEC && m0 + d >= 0) ? (const T*)a.x + (size_t)min(m0 + d, a.M - 1) * a.ldx + c0
+                                                   : ring + (size_t)(max(pos + d, 0) % TAPS) * a.channels;
+    x[i] = *(const V*)src;
+  }
+  float w[TAPS][VEC], b[VEC];
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) {
+    b[e] = a.b[c0 + e];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j][e] = a.w[(size_t)(c0 + e) * TAPS + j];
+  }
+  const V z = {};
+#pragma unroll
+  for (int i = 0; i < TAPS - 1; ++i)
+    if (pos + i - (TAPS - 1) < 0) x[i] = z;
+  if (DEC) *(V*)(ring + (size_t)(pos % TAPS) * a.channels) = x[NX - 1];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (m0 + r >= a.M) return;
+    V o;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      float acc = b[e];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) acc = fmaf(w[j][e], (float)x[r + j][e], acc);
+      o[e] = (T)(a.act == TI_CONV_SILU ? acc * fast_sigmoid(acc) : acc);
+    }
+    *(V*)(out + (size_t)r * a.ldo) = o;
   }
 }
 
@@ -110,7 +166,7 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(const ti_ssd_args a, int 
       v = fmaf(a.conv_w[(size_t)c * a.taps + a.taps - 1], (float)cur, v);
       // (the place written is read by no one: it held position pos - taps)
       if (own) ring[(size_t)(pos % a.taps) * channels + c] = cur;
-      v = (float)(T)siluf(v);
+      v = (float)(T)(v * fast_sigmoid(v));
     }
     *dst = v;
   }
@@ -157,27 +213,29 @@ constexpr int kSsdTok = 64;
 // L(t, s) = exp(cum_t - cum_s):
 //   y_t = sum_{s <= t} (C_t . B_s) L(t, s) dt_s x_s + exp(cum_t) S^T C_t + D x_t
 //   S  <- exp(cum_last) S + sum_t L(last, t) dt_t B_t x_t^T
-// Wave w owns tokens [16 w, +16) of the outputs and the state tiles w, w + 4, ... of 16 state rows; the
-// accumulator of a product is the operand fragment of the next one (scores, state).
-template <class T, int NTW>
-__global__ __launch_bounds__(256, 1) void ssd_scan_kernel(const ti_ssd_args a) {
+// Waves 0..3 carry the state (tiles w, w + 4, ... of 16 state rows): its share of every token's output, then
+// its update.  Waves 4..7 own 16 tokens each: their scores within the block and the output.  Accumulators
+// are the operand fragments of the next product (scores, state).  The next block is loaded during a block
+// and staged at its end (DB: into the other buffer); wave 4, which has the fewest scores, prepares its
+// step sizes and decays.
+template <class T, int NTW, bool DB>
+__global__ __launch_bounds__(512, 1) void ssd_scan_kernel(const ti_ssd_args a) {
   typedef typename El<T>::V V;
-  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, PF = 4, XLD = kSsdTok + 4;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, PF = 2, XLD = kSsdTok + 4, TH = 512;
   extern __shared__ char lds[];
   const int N = a.state_n, nk = (N + KT - 1) / KT * KT, ld = nk + 16 / (int)sizeof(T), np = (N + 3) & ~3, nt = (N + 15) >> 4;
-  T* Bs = (T*)lds;                       // [64][ld]
-  T* Cs = Bs + kSsdTok * ld;             // [64][ld]
-  float* xt = (float*)(Cs + kSsdTok * ld);   // [16][XLD] values, transposed
-  f32x4* red = (f32x4*)(xt + 16 * XLD);  // [4][4][64] the waves' state outputs
-  double* cum = (double*)(red + 16 * 64);
-  float* dts = (float*)(cum + kSsdTok);  // [64]
-  float* wl = dts + kSsdTok;             // [64] L(last, t) dt_t
-  float* ec = wl + kSsdTok;              // [64] exp(cum_t)
+  T* bc = (T*)lds;                       // [DB ? 2 : 1][B, C][64][ld]
+  float* xts = (float*)(bc + (DB ? 4 : 2) * kSsdTok * ld);   // [2][16][XLD] values, transposed
+  f32x4* reds = (f32x4*)(xts + 2 * 16 * XLD);                // [DB ? 2 : 1][4][4][64] the state's output shares
+  double* cums = (double*)(reds + (DB ? 2 : 1) * 16 * 64);   // [2][64]
+  float* coef = (float*)(cums + 2 * kSsdTok);                // [2][3][64] dt, L(last, t) dt_t, exp(cum_t)
   const int h = blockIdx.y, p0 = blockIdx.x * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
   const int grp = h / (a.heads / a.groups);
+  const bool sw = wave < 4;
+  const int w4 = wave & 3;
   const T* src = (const T*)a.a;
   const T* bsrc = src + a.o0 + (size_t)grp * nk;
-  const T* csrc = bsrc + (size_t)a.groups * nk;
+  const size_t c_off = (size_t)a.groups * nk;
   const int ppr = nk / VEC, pieces = kSsdTok * ppr;   // 16-byte pieces per row, per block
   const float A = -expf(a.a_log[h]), bias = a.dt_bias[h], D = a.d[h];
   float* state = a.state + (((size_t)a.slot0 * a.heads + h) * a.vdim + p0) * np;
@@ -187,153 +245,234 @@ __global__ __launch_bounds__(256, 1) void ssd_scan_kernel(const ti_ssd_args a) {
   for (int i = 0; i < NTW; ++i) {
     const int n = (wave + 4 * i) * 16 + 4 * g;
     S[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    if (a.pos[0] > 0 && prow && n < np) S[i] = *(const f32x4*)(state + (size_t)col * np + n);
+    if (sw && a.pos[0] > 0 && prow && n < np) S[i] = *(const f32x4*)(state + (size_t)col * np + n);
   }
   V rb[PF], rc[PF];
-  float rx[4], rdt = 0.0f;
+  float rx[2];
   const V vz = {};
-  auto piece = [&](const T* s, int m0, int i) -> V {
-    const int t = i / ppr, c = i - t * ppr;
-    return i < pieces && m0 + t < a.M ? *(const V*)(s + (size_t)(m0 + t) * a.lda + c * VEC) : vz;
-  };
+  int prow_[PF], pcol_[PF];
+#pragma unroll
+  for (int u = 0; u < PF; ++u) {
+    prow_[u] = (tid + u * TH) / ppr;
+    pcol_[u] = (tid + u * TH - prow_[u] * ppr) * VEC;
+  }
   auto load = [&](int m0) {
 #pragma unroll
     for (int u = 0; u < PF; ++u) {
-      rb[u] = piece(bsrc, m0, tid + u * 256);
-      rc[u] = piece(csrc, m0, tid + u * 256);
+      const bool in = prow_[u] < kSsdTok && m0 + prow_[u] < a.M;
+      const T* s = bsrc + (size_t)(m0 + prow_[u]) * a.lda + pcol_[u];
+      rb[u] = in ? *(const V*)s : vz;
+      rc[u] = in ? *(const V*)(s + c_off) : vz;
     }
-    const int m = m0 + (tid >> 2), p = p0 + (tid & 3) * 4;
+    const int m = m0 + (tid >> 3), p = p0 + (tid & 7) * 2;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) rx[e] = m < a.M && p + e < a.vdim ? (float)src[(size_t)m * a.lda + h * a.vdim + p + e] : 0.0f;
-    if (wave == 0) rdt = m0 + lane < a.M ? a.dt[(size_t)(m0 + lane) * a.heads + h] : 0.0f;
+    for (int e = 0; e < 2; ++e) rx[e] = m < a.M && p + e < a.vdim ? (float)src[(size_t)m * a.lda + h * a.vdim + p + e] : 0.0f;
   };
-  auto put = [&](T* d, int i, V v) {
-    const int t = i / ppr, c = i - t * ppr;
-    if (i < pieces) *(V*)(d + t * ld + c * VEC) = v;
+  auto stage = [&](int buf, int m0) {
+    T* B = bc + (DB ? buf : 0) * 2 * kSsdTok * ld;
+    T* C = B + kSsdTok * ld;
+#pragma unroll
+    for (int u = 0; u < PF; ++u)
+      if (prow_[u] < kSsdTok) {
+        *(V*)(B + prow_[u] * ld + pcol_[u]) = rb[u];
+        *(V*)(C + prow_[u] * ld + pcol_[u]) = rc[u];
+      }
+    for (int i = tid + PF * TH; i < pieces; i += TH) {   // (long states)
+      const int t = i / ppr, c = (i - t * ppr) * VEC;
+      const T* s = bsrc + (size_t)(m0 + t) * a.lda + c;
+      *(V*)(B + t * ld + c) = m0 + t < a.M ? *(const V*)s : vz;
+      *(V*)(C + t * ld + c) = m0 + t < a.M ? *(const V*)(s + c_off) : vz;
+    }
+#pragma unroll
+    for (int e = 0; e < 2; ++e) xts[buf * 16 * XLD + ((tid & 7) * 2 + e) * XLD + (tid >> 3)] = rx[e];
   };
+  auto steps = [&](int buf, int m0, float raw) {   // one wave: step sizes, cumulated log decays
+    const float dt = m0 + lane < a.M ? softplusf(raw + bias) : 0.0f;   // (past the end: no decay, no input)
+    double c = (double)(A * dt);
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const double v = __shfl_up(c, o, 64);
+      if (lane >= o) c += v;
+    }
+    cums[buf * kSsdTok + lane] = c;
+    float* k = coef + buf * 3 * kSsdTok;
+    k[lane] = dt;
+    k[kSsdTok + lane] = fast_exp((float)(__shfl(c, 63, 64) - c)) * dt;
+    k[2 * kSsdTok + lane] = fast_exp((float)c);
+  };
+  auto raw_dt = [&](int m0) { return m0 + lane < a.M ? a.dt[(size_t)(m0 + lane) * a.heads + h] : 0.0f; };
   load(0);
-  for (int m0 = 0; m0 < a.M; m0 += kSsdTok) {
-#pragma unroll
-    for (int u = 0; u < PF; ++u) {
-      put(Bs, tid + u * 256, rb[u]);
-      put(Cs, tid + u * 256, rc[u]);
+  if (wave == 4) steps(0, 0, raw_dt(0));
+  stage(0, 0);
+  lds_sync();
+  for (int m0 = 0, buf = 0; m0 < a.M; m0 += kSsdTok, buf ^= 1) {
+    const T* Bs = bc + (DB ? buf : 0) * 2 * kSsdTok * ld;
+    const T* Cs = Bs + kSsdTok * ld;
+    const float *xt = xts + buf * 16 * XLD, *dts = coef + buf * 3 * kSsdTok, *wl = dts + kSsdTok, *ec = wl + kSsdTok;
+    const double* cum = cums + buf * kSsdTok;
+    f32x4* red = reds + (DB ? buf : 0) * 16 * 64;
+    const bool more = m0 + kSsdTok < a.M;
+    float rdt = 0.0f;
+    if (more) {
+      load(m0 + kSsdTok);
+      if (wave == 4) rdt = raw_dt(m0 + kSsdTok);
     }
-    for (int i = tid + PF * 256; i < pieces; i += 256) {   // (long states)
-      put(Bs, i, piece(bsrc, m0, i));
-      put(Cs, i, piece(csrc, m0, i));
-    }
-#pragma unroll
-    for (int e = 0; e < 4; ++e) xt[((tid & 3) * 4 + e) * XLD + (tid >> 2)] = rx[e];
-    if (wave == 0) {
-      const float dt = m0 + lane < a.M ? softplusf(rdt + bias) : 0.0f;   // (past the end: no decay, no input)
-      double c = (double)(A * dt);
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const double v = __shfl_up(c, o, 64);
-        if (lane >= o) c += v;
-      }
-      cum[lane] = c;
-      dts[lane] = dt;
-      wl[lane] = expf((float)(__shfl(c, 63, 64) - c)) * dt;
-      ec[lane] = expf((float)c);
-    }
-    lds_sync();
-    if (m0 + kSsdTok < a.M) load(m0 + kSsdTok);
-    // the carried state's share of every token, over this wave's state rows
-    f32x4 yi[4];
-#pragma unroll
-    for (int t = 0; t < 4; ++t) yi[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int i = 0; i < NTW; ++i) {
-      const int tile = wave + 4 * i;
-      if (tile < nt)
-#pragma unroll
-        for (int t = 0; t < 4; ++t) yi[t] = mma(S[i], widen4(Cs + (t * 16 + col) * ld + tile * 16 + 4 * g), yi[t]);
-    }
-#pragma unroll
-    for (int t = 0; t < 4; ++t) red[(wave * 4 + t) * 64 + lane] = yi[t];
-    // scores of this wave's tokens with the block's earlier ones, decayed, times their inputs
+    const int tok = w4 * 16 + col;
     f32x4 y = {0.f, 0.f, 0.f, 0.f};
-    const int tok = wave * 16 + col;
-    const double ct = cum[tok];
-    for (int st = 0; st <= wave; ++st) {
-      f32x4 sc = {0.f, 0.f, 0.f, 0.f};
-      for (int k = 0; k < nk; k += KT)
-        sc = mma(*(const V*)(Bs + (st * 16 + col) * ld + k + g * VEC), *(const V*)(Cs + tok * ld + k + g * VEC), sc);
+    float et = 0.0f;
+    if (sw) {
+      // the carried state's share of every token, over this wave's state rows
+      f32x4 yi[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int s = st * 16 + 4 * g + r;
-        sc[r] = s <= tok ? sc[r] * expf((float)(ct - cum[s])) * dts[s] : 0.0f;
+      for (int t = 0; t < 4; ++t) yi[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < NTW; ++i) {
+        const int tile = w4 + 4 * i;
+        if (tile >= nt) continue;
+        f32x4 c[4];
+#pragma unroll
+        for (int t = 0; t < 4; ++t) c[t] = widen4(Cs + (t * 16 + col) * ld + tile * 16 + 4 * g);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int t = 0; t < 4; ++t) yi[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(S[i][r], c[t][r], yi[t], 0, 0, 0);
       }
-      y = mma(*(const f32x4*)(xt + col * XLD + st * 16 + 4 * g), sc, y);
-    }
-    // the state over the block
-    const float last = ec[kSsdTok - 1];
-    f32x4 wx[4];
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      const f32x4 w = *(const f32x4*)(wl + t * 16 + 4 * g), x = *(const f32x4*)(xt + col * XLD + t * 16 + 4 * g);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) wx[t][r] = w[r] * x[r];
-    }
-#pragma unroll
-    for (int i = 0; i < NTW; ++i) {
-      const int tile = wave + 4 * i;
-      if (tile >= nt) continue;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) S[i][r] *= last;
+      for (int t = 0; t < 4; ++t) red[(w4 * 4 + t) * 64 + lane] = yi[t];
+      // the state over the block
+      const float last = ec[kSsdTok - 1];
+      f32x4 wx[4];
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        f32x4 b;
+        const f32x4 w = *(const f32x4*)(wl + t * 16 + 4 * g), x = *(const f32x4*)(xt + col * XLD + t * 16 + 4 * g);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) b[r] = (float)Bs[(t * 16 + 4 * g + r) * ld + tile * 16 + col];
-        S[i] = mma(b, wx[t], S[i]);
+        for (int r = 0; r < 4; ++r) wx[t][r] = w[r] * x[r];
+      }
+#pragma unroll
+      for (int i = 0; i < NTW; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[i][r] *= last;
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        f32x4 b[NTW];
+#pragma unroll
+        for (int i = 0; i < NTW; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) b[i][r] = (float)Bs[(t * 16 + 4 * g + r) * ld + min(w4 + 4 * i, nt - 1) * 16 + col];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int i = 0; i < NTW; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(b[i][r], wx[t][r], S[i], 0, 0, 0);
+      }
+    } else {
+      // scores of this wave's tokens with the block's earlier ones, decayed, times their inputs
+      const double ct = cum[tok];
+      et = ec[tok];
+      for (int st = 0; st <= w4; ++st) {
+        f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+        for (int k = 0; k < nk; k += KT)
+          sc = mma(*(const V*)(Bs + (st * 16 + col) * ld + k + g * VEC), *(const V*)(Cs + tok * ld + k + g * VEC), sc);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int s = st * 16 + 4 * g + r;
+          sc[r] = s <= tok ? sc[r] * fast_exp((float)(ct - cum[s])) * dts[s] : 0.0f;
+        }
+        y = mma(*(const f32x4*)(xt + col * XLD + st * 16 + 4 * g), sc, y);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) y[r] = fmaf(D, xt[(4 * g + r) * XLD + tok], y[r]);
+      if (wave == 4 && more) steps(buf ^ 1, m0 + kSsdTok, rdt);
+    }
+    if (DB && more) stage(buf ^ 1, m0 + kSsdTok);
+    lds_sync();
+    if (!sw && m0 + tok < a.M) {   // out: this wave's tokens, dimensions 4 g + r
+      f32x4 z = red[w4 * 64 + lane];
+#pragma unroll
+      for (int w = 1; w < 4; ++w) z += red[(w * 4 + w4) * 64 + lane];
+      float* o = a.y + (size_t)(m0 + tok) * a.ldy + h * a.vdim + p0 + 4 * g;
+      f32x4 v;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] = fmaf(et, z[r], y[r]);
+      if (p0 + 4 * g + 4 <= a.vdim && ((a.ldy | a.vdim) & 3) == 0) {
+        *(f32x4*)o = v;
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (p0 + 4 * g + r < a.vdim) o[r] = v[r];
       }
     }
-    lds_sync();
-    // out: tokens this wave's, dimensions 4 g + r
-    f32x4 z = red[wave * 64 + lane];
-#pragma unroll
-    for (int w = 1; w < 4; ++w) z += red[(w * 4 + wave) * 64 + lane];
-    if (m0 + tok < a.M) {
-      float* o = a.y + (size_t)(m0 + tok) * a.ldy + h * a.vdim + p0 + 4 * g;
-      const float e = ec[tok];
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (p0 + 4 * g + r < a.vdim) o[r] = fmaf(e, z[r], y[r]) + D * xt[(4 * g + r) * XLD + tok];
+    if (!DB && more) {
+      stage(buf ^ 1, m0 + kSsdTok);
+      lds_sync();
     }
-    lds_sync();   // (the block's LDS is free)
   }
+  if (!sw) return;
 #pragma unroll
   for (int i = 0; i < NTW; ++i) {
-    const int n = (wave + 4 * i) * 16 + 4 * g;
+    const int n = (w4 + 4 * i) * 16 + 4 * g;
     if (prow && n < np) *(f32x4*)(state + (size_t)col * np + n) = S[i];
   }
 }
 
 // ------------------------------------------------------------------ gate and norm
+// Grid (groups, rows).
+__device__ __forceinline__ float gated(float y, float z) { return y * z * fast_sigmoid(z); }
+template <class T>
+__device__ __forceinline__ void ssd_ring(const ti_ssd_norm_args& a, int m, const T* raw) {
+  if (!a.ring || blockIdx.x || m < a.M - (a.taps - 1)) return;
+  T* ring = (T*)a.ring + ((size_t)a.slot0 * a.taps + a.pos[m] % a.taps) * a.channels;
+  for (int i = threadIdx.x; i < a.channels; i += blockDim.x) ring[i] = raw[a.inner + i];
+}
 template <class T>
 __global__ __launch_bounds__(512) void ssd_norm_kernel(const ti_ssd_norm_args a) {
   extern __shared__ float v[];
   __shared__ float red[8];
-  const int m = blockIdx.x, tid = threadIdx.x, per = a.inner / a.groups;
-  const float* y = a.y + (size_t)m * a.ldy;
+  const int m = blockIdx.y, tid = threadIdx.x, per = a.inner / a.groups, i0 = blockIdx.x * per;
+  const float* y = a.y + (size_t)m * a.ldy + i0;
   const T* raw = (const T*)a.raw + (size_t)m * a.lda;
-  T* out = (T*)a.out + (size_t)m * a.ldo;
-  for (int gr = 0; gr < a.groups; ++gr) {
-    float q = 0.0f;
-    for (int i = gr * per + tid; i < (gr + 1) * per; i += 512) {
-      const float x = y[i] * siluf((float)raw[i]);
-      v[i] = x;
-      q = fmaf(x, x, q);
+  T* out = (T*)a.out + (size_t)m * a.ldo + i0;
+  float q = 0.0f;
+  for (int i = tid; i < per; i += 512) {
+    v[i] = gated(y[i], (float)raw[i0 + i]);
+    q = fmaf(v[i], v[i], q);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)per + a.eps);
+  for (int i = tid; i < per; i += 512) out[i] = (T)(v[i] * inv * a.w[i0 + i]);
+  ssd_ring<T>(a, m, raw);
+}
+// Groups of a multiple of 4 values, at most 4 * TH * NC: held in registers, every load in flight at once.
+template <class T, int TH, int NC>
+__global__ __launch_bounds__(TH) void ssd_norm_vec_kernel(const ti_ssd_norm_args a) {
+  typedef typename El<T>::Q Q;
+  __shared__ float red[TH / 64];
+  const int m = blockIdx.y, tid = threadIdx.x, per = a.inner / a.groups, i0 = blockIdx.x * per, n4 = per >> 2;
+  const T* raw = (const T*)a.raw + (size_t)m * a.lda;
+  const f32x4 *y = (const f32x4*)(a.y + (size_t)m * a.ldy + i0), *w = (const f32x4*)(a.w + i0);
+  f32x4 v[NC], wv[NC];
+  Q z[NC];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = min(tid + c * TH, n4 - 1);
+    v[c] = y[i];
+    z[c] = *(const Q*)(raw + i0 + 4 * i);
+    wv[c] = w[i];
+  }
+  float q = 0.0f;
+#pragma unroll
+  for (int c = 0; c < NC; ++c)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v[c][e] = gated(v[c][e], (float)z[c][e]);
+      if (tid + c * TH < n4) q = fmaf(v[c][e], v[c][e], q);
     }
-    const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)per + a.eps);
-    for (int i = gr * per + tid; i < (gr + 1) * per; i += 512) out[i] = (T)(v[i] * inv * a.w[i]);
+  const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)per + a.eps);
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[c][e] *= inv * wv[c][e];
+    if (tid + c * TH < n4) *(Q*)((T*)a.out + (size_t)m * a.ldo + i0 + 4 * (tid + c * TH)) = quad<T>(v[c]);
   }
-  if (a.ring && m >= a.M - (a.taps - 1)) {
-    T* ring = (T*)a.ring + ((size_t)a.slot0 * a.taps + a.pos[m] % a.taps) * a.channels;
-    for (int i = tid; i < a.channels; i += 512) ring[i] = raw[a.inner + i];
-  }
+  ssd_ring<T>(a, m, raw);
 }
 
 // ------------------------------------------------------------------ gated linear recurrence over a chunk
@@ -404,8 +543,22 @@ template <class T>
 int launch_conv(const ti_conv_args& a, hipStream_t s) {
   const int sections = a.c0 < a.channels ? (a.channels - a.c0) / a.bw : 0, places = sections ? a.o0 + sections * a.bwp : a.channels;
   const int rb = (a.M + kConvRows - 1) / kConvRows;
-  const bool vec = ((a.channels | a.ldx | a.ldo | a.c0) & 3) == 0 && (!sections || ((a.o0 | a.bw | a.bwp) & 3) == 0);
-  if (vec && sizeof(T) * 4 <= 16)
+  const int all = a.channels | a.ldx | a.ldo | a.c0 | (sections ? a.o0 | a.bw | a.bwp : 0);
+  constexpr int VEC = El<T>::VEC;
+  if (all % VEC == 0 && a.taps >= 2 && a.taps <= 4) {
+    const int rows = a.chunk ? 8 : 1;
+    const dim3 grid((places / VEC + 63) / 64, (a.M + 4 * rows - 1) / (4 * rows)), blk(256);
+#define TI_CV(TAPS)                                                                                   \
+  if (a.chunk) hipLaunchKernelGGL((conv_vec_kernel<T, TAPS, false>), grid, blk, 0, s, a, places);     \
+  else hipLaunchKernelGGL((conv_vec_kernel<T, TAPS, true>), grid, blk, 0, s, a, places)
+    if (a.taps == 2) TI_CV(2);
+    else if (a.taps == 3) TI_CV(3);
+    else TI_CV(4);
+#undef TI_CV
+    TI_LAUNCH_CHECK("conv_vec_kernel");
+    return TI_OK;
+  }
+  if (all % 4 == 0)
     hipLaunchKernelGGL((conv_kernel<T, 4>), dim3((places / 4 + 255) / 256, rb), dim3(256), 0, s, a, places);
   else
     hipLaunchKernelGGL((conv_kernel<T, 1>), dim3((places + 255) / 256, rb), dim3(256), 0, s, a, places);
@@ -429,30 +582,53 @@ int launch_ssd_step(const ti_ssd_args& a, hipStream_t s) {
   return TI_OK;
 }
 
+constexpr size_t kSsdLds = 163840 - 1024;
+
 template <class T>
-size_t ssd_scan_lds(int N) {
+size_t ssd_scan_lds(int N, bool db) {
   const int kt = El<T>::KT, nk = (N + kt - 1) / kt * kt;
-  return (size_t)2 * kSsdTok * (nk * sizeof(T) + 16) + 16 * (kSsdTok + 4) * 4 + 16 * 64 * 16 + kSsdTok * 8 + 3 * kSsdTok * 4;
+  return (size_t)(db ? 4 : 2) * kSsdTok * (nk * sizeof(T) + 16) + 2 * 16 * (kSsdTok + 4) * 4 + (db ? 2 : 1) * 16 * 64 * 16 +
+         2 * kSsdTok * 8 + 2 * 3 * kSsdTok * 4;
 }
 
 template <class T>
 int launch_ssd_scan(const ti_ssd_args& a, hipStream_t s) {
-  const dim3 grid((a.vdim + 15) / 16, a.heads), blk(256);
-  const size_t lds = ssd_scan_lds<T>(a.state_n);
+  const dim3 grid((a.vdim + 15) / 16, a.heads), blk(512);
+  const bool db = ssd_scan_lds<T>(a.state_n, true) <= kSsdLds;
+  const size_t lds = ssd_scan_lds<T>(a.state_n, db);
   const int nt = (a.state_n + 15) / 16;
-  if (nt <= 4) hipLaunchKernelGGL((ssd_scan_kernel<T, 1>), grid, blk, lds, s, a);
-  else if (nt <= 8) hipLaunchKernelGGL((ssd_scan_kernel<T, 2>), grid, blk, lds, s, a);
-  else hipLaunchKernelGGL((ssd_scan_kernel<T, 4>), grid, blk, lds, s, a);
+#define TI_SS(NTW)                                                                       \
+  if (db) hipLaunchKernelGGL((ssd_scan_kernel<T, NTW, true>), grid, blk, lds, s, a);     \
+  else hipLaunchKernelGGL((ssd_scan_kernel<T, NTW, false>), grid, blk, lds, s, a)
+  if (nt <= 4) TI_SS(1);
+  else if (nt <= 8) TI_SS(2);
+  else TI_SS(4);
+#undef TI_SS
   TI_LAUNCH_CHECK("ssd_scan_kernel");
   return TI_OK;
 }
 
 template <class T>
 int recurrent_prepare() {
-  const void* k[] = {(const void*)ssd_scan_kernel<T, 1>, (const void*)ssd_scan_kernel<T, 2>, (const void*)ssd_scan_kernel<T, 4>,
+  const void* k[] = {(const void*)ssd_scan_kernel<T, 1, true>,  (const void*)ssd_scan_kernel<T, 2, true>,
+                     (const void*)ssd_scan_kernel<T, 4, true>,  (const void*)ssd_scan_kernel<T, 1, false>,
+                     (const void*)ssd_scan_kernel<T, 2, false>, (const void*)ssd_scan_kernel<T, 4, false>,
                      (const void*)ssd_norm_kernel<T>};
   for (const void* f : k)
-    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 163840 - 1024), "recurrent kernels' LDS");
+    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kSsdLds), "recurrent kernels' LDS");
+  return TI_OK;
+}
+
+template <class T>
+int launch_ssd_norm(const ti_ssd_norm_args& a, hipStream_t s) {
+  const int per = a.inner / a.groups;
+  const dim3 grid(a.groups, a.M);
+  const bool vec = ((per | a.ldy | a.lda | a.ldo) & 3) == 0 && per <= 8192;
+  if (vec && per <= 1024) hipLaunchKernelGGL((ssd_norm_vec_kernel<T, 256, 1>), grid, dim3(256), 0, s, a);
+  else if (vec && per <= 4096) hipLaunchKernelGGL((ssd_norm_vec_kernel<T, 512, 2>), grid, dim3(512), 0, s, a);
+  else if (vec) hipLaunchKernelGGL((ssd_norm_vec_kernel<T, 1024, 2>), grid, dim3(1024), 0, s, a);
+  else hipLaunchKernelGGL(ssd_norm_kernel<T>, grid, dim3(512), (size_t)per * 4, s, a);
+  TI_LAUNCH_CHECK("ssd_norm_kernel");
   return TI_OK;
 }
 
@@ -514,18 +690,12 @@ extern "C" int ti_ssd_scan(const ti_ssd_args* a, ti_stream_t stream) {
 
 extern "C" int ti_ssd_norm(const ti_ssd_norm_args* a, ti_stream_t stream) {
   using namespace ti;
-  if (!a || !a->y || !a->raw || !a->w || !a->out || a->M < 1 || a->inner < 1 || a->groups < 1 || a->inner % a->groups ||
+  if (!a || !a->y || !a->raw || !a->w || !a->out || a->M < 1 || a->M > 65535 || a->inner < 1 || a->groups < 1 || a->inner % a->groups ||
       a->ldy < a->inner || a->ldo < a->inner || a->lda < a->inner + (a->ring ? a->channels : 0) || (a->ring && !a->pos) ||
       !rec_dtype(a->dtype))
     return ti_set_error(TI_ERR_ARG, "ti_ssd_norm: bad arguments");
   if (a->inner > 32768) return ti_set_error(TI_ERR_UNSUPPORTED, "ti_ssd_norm: %d values (at most 32768)", a->inner);
-  const size_t lds = (size_t)a->inner * 4;
-  if (a->dtype == TI_DT_BF16)
-    hipLaunchKernelGGL(ssd_norm_kernel<bf16>, dim3(a->M), dim3(512), lds, (hipStream_t)stream, *a);
-  else
-    hipLaunchKernelGGL(ssd_norm_kernel<float>, dim3(a->M), dim3(512), lds, (hipStream_t)stream, *a);
-  TI_LAUNCH_CHECK("ssd_norm_kernel");
-  return TI_OK;
+  return a->dtype == TI_DT_BF16 ? launch_ssd_norm<bf16>(*a, (hipStream_t)stream) : launch_ssd_norm<float>(*a, (hipStream_t)stream);
 }
 
 extern "C" int ti_lru_scan(const ti_lru_scan_args* a, ti_stream_t stream) {
