@@ -460,7 +460,7 @@ int dispatch_dense(const ti_dense_args& a, hipStream_t s) {
     case TI_DE_F32: return few ? skinny<T, TI_DE_F32>(a, s) : tiled<T, TI_DE_F32>(a, s);
     case TI_DE_ROPE: return few ? skinny<T, TI_DE_ROPE>(a, s) : tiled<T, TI_DE_ROPE>(a, s);
     case TI_DE_ACT: return few ? skinny<T, TI_DE_ACT>(a, s) : tiled<T, TI_DE_ACT>(a, s);
-    case TI_DE_LRU: return few ? skinny<T, TI_DE_LRU>(a, s) : tiled<T, TI_DE_LRU>(a, s);
+    case TI_DE_LRU: return few ? skinny<T, TI_DE_LRU>(a, s) : launch_tile<T, 64, 128, 4, TI_DE_LRU>(a, s);   // (short k: the epilogue decides)
     case TI_DE_LOGITS: return few ? skinny<T, TI_DE_LOGITS>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_LOGITS>(a, s);
     case TI_DE_GATE: return few ? skinny<T, TI_DE_GATE>(a, s) : launch_tile<T, 64, 64, 4, TI_DE_GATE>(a, s);
     case TI_DE_SWIGLU:

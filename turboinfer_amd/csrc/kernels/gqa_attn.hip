@@ -133,7 +133,7 @@ __device__ __forceinline__ f32x4 weight_frag(const float* row, int g) { return *
 
 // Grid (splits, kv heads * tiles of 16 query heads, rows).
 template <class T, int NVW>
-__global__ __launch_bounds__(256, 2) void gqa_decode_kernel(const ti_gqa_attn_args a) {
+__global__ __launch_bounds__(256, NVW > 2 || sizeof(T) > 2 ? 2 : 4) void gqa_decode_kernel(const ti_gqa_attn_args a) {
   typedef typename El<T>::V V;
   constexpr int KT = El<T>::KT, VEC = El<T>::VEC, VB = 64 / KT, PLD = 64 + 16 / (int)sizeof(T), NKU = 8;
   extern __shared__ char lds[];
@@ -547,9 +547,9 @@ extern "C" int ti_gqa_prep(const ti_gqa_prep_args* a, ti_stream_t stream) {
 }
 
 extern "C" int ti_gqa_splits(int M, int heads, int kv_heads, int max_seq) {
-  // two workgroups per CU (splits cost a merge), none with less than one 64-position block
+  // four workgroups per CU (splits cost a merge), none with less than one 64-position block
   const int rep = heads / std::max(1, kv_heads), wgs = M * kv_heads * ((rep + 15) / 16), cap = std::max(1, (max_seq + 63) / 64);
-  return std::max(1, std::min({cap, ti::kGqaSplits, (512 + wgs - 1) / std::max(1, wgs)}));
+  return std::max(1, std::min({cap, ti::kGqaSplits, (1024 + wgs - 1) / std::max(1, wgs)}));
 }
 
 extern "C" int ti_gqa_decode(const ti_gqa_attn_args* a, ti_stream_t stream) {

@@ -201,11 +201,29 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(const ti_ssd_args a, int 
 }
 
 // ------------------------------------------------------------------ SSD over a prompt chunk
-__device__ __forceinline__ f32x4 widen4(const bf16* p) {
-  const bf16x4 v = *(const bf16x4*)p;
-  return (f32x4){(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+// Running sums over the lanes of a wave (inclusive): within rows of 16 by lane shifts, then the rows' totals.
+template <int N>
+__device__ __forceinline__ double row_shift(double v) {   // lane l - N of the row; 0 before its start
+  const uint64_t u = __builtin_bit_cast(uint64_t, v);
+  const uint32_t lo = __builtin_amdgcn_update_dpp(0u, (uint32_t)u, 0x110 + N, 0xf, 0xf, true);
+  const uint32_t hi = __builtin_amdgcn_update_dpp(0u, (uint32_t)(u >> 32), 0x110 + N, 0xf, 0xf, true);
+  return __builtin_bit_cast(double, (uint64_t)hi << 32 | lo);
 }
-__device__ __forceinline__ f32x4 widen4(const float* p) { return *(const f32x4*)p; }
+template <int L>
+__device__ __forceinline__ double lane_value(double v) {
+  const uint64_t u = __builtin_bit_cast(uint64_t, v);
+  const uint32_t lo = __builtin_amdgcn_readlane((uint32_t)u, L), hi = __builtin_amdgcn_readlane((uint32_t)(u >> 32), L);
+  return __builtin_bit_cast(double, (uint64_t)hi << 32 | lo);
+}
+__device__ __forceinline__ double wave_prefix(double v) {
+  v += row_shift<1>(v);
+  v += row_shift<2>(v);
+  v += row_shift<4>(v);
+  v += row_shift<8>(v);
+  const double a = lane_value<15>(v), b = a + lane_value<31>(v), c = b + lane_value<47>(v);
+  const int row = (int)(threadIdx.x & 63) >> 4;
+  return v + (row == 0 ? 0.0 : row == 1 ? a : row == 2 ? b : c);
+}
 
 constexpr int kSsdTok = 64;
 
@@ -213,24 +231,26 @@ constexpr int kSsdTok = 64;
 // L(t, s) = exp(cum_t - cum_s):
 //   y_t = sum_{s <= t} (C_t . B_s) L(t, s) dt_s x_s + exp(cum_t) S^T C_t + D x_t
 //   S  <- exp(cum_last) S + sum_t L(last, t) dt_t B_t x_t^T
-// Waves 0..3 carry the state (tiles w, w + 4, ... of 16 state rows): its share of every token's output, then
+// Waves 0..3 carry the state, 16 * NTW of its rows each, tile i holding every NTW-th from the i-th (a lane's
+// rows are 4 * NTW consecutive ones, its operands of all tiles come in one read): its share of every token's output, then
 // its update.  Waves 4..7 own 16 tokens each: their scores within the block and the output.  Accumulators
-// are the operand fragments of the next product (scores, state).  The next block is loaded during a block
-// and staged at its end (DB: into the other buffer); wave 4, which has the fewest scores, prepares its
-// step sizes and decays.
+// are the operand fragments of the next product (scores, state).  Waves 4..7 also load the next block and
+// stage it at the end of this one (DB: into the other buffer); wave 4, which has the fewest scores, prepares
+// its step sizes and decays.
 template <class T, int NTW, bool DB>
 __global__ __launch_bounds__(512, 1) void ssd_scan_kernel(const ti_ssd_args a) {
   typedef typename El<T>::V V;
-  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, PF = 2, XLD = kSsdTok + 4, TH = 512;
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, PF = NTW * 16 / VEC < 4 ? NTW * 16 / VEC : 4, XLD = kSsdTok + 4, TH = 256;
   extern __shared__ char lds[];
-  const int N = a.state_n, nk = (N + KT - 1) / KT * KT, ld = nk + 16 / (int)sizeof(T), np = (N + 3) & ~3, nt = (N + 15) >> 4;
+  const int N = a.state_n, nk = (N + KT - 1) / KT * KT, np = (N + 3) & ~3;
+  constexpr int LN = 64 * NTW, ld = LN + 16 / (int)sizeof(T);   // (places past nk stay 0)
   T* bc = (T*)lds;                       // [DB ? 2 : 1][B, C][64][ld]
   float* xts = (float*)(bc + (DB ? 4 : 2) * kSsdTok * ld);   // [2][16][XLD] values, transposed
   f32x4* reds = (f32x4*)(xts + 2 * 16 * XLD);                // [DB ? 2 : 1][4][4][64] the state's output shares
-  double* cums = (double*)(reds + (DB ? 2 : 1) * 16 * 64);   // [2][64]
-  float* coef = (float*)(cums + 2 * kSsdTok);                // [2][3][64] dt, L(last, t) dt_t, exp(cum_t)
-  const int h = blockIdx.y, p0 = blockIdx.x * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
-  const int grp = h / (a.heads / a.groups);
+  // [2][5][64]: cum_t / ln 2 in two floats, dt, L(last, t) dt_t, exp(cum_t)
+  float* coef = (float*)(reds + (DB ? 2 : 1) * 16 * 64);
+  const int h = blockIdx.y, p0 = blockIdx.x * 16, tid = threadIdx.x, lane = tid & 63, col = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), grp = h / (a.heads / a.groups);
   const bool sw = wave < 4;
   const int w4 = wave & 3;
   const T* src = (const T*)a.a;
@@ -240,83 +260,88 @@ __global__ __launch_bounds__(512, 1) void ssd_scan_kernel(const ti_ssd_args a) {
   const float A = -expf(a.a_log[h]), bias = a.dt_bias[h], D = a.d[h];
   float* state = a.state + (((size_t)a.slot0 * a.heads + h) * a.vdim + p0) * np;
   const bool prow = p0 + col < a.vdim;
-  f32x4 S[NTW];   // tile i: state rows n0 + 4 g + r, value dimension col
+  const int n0 = 16 * NTW * (wave & 3);   // this wave's state rows
+  f32x4 S[NTW];   // S[i][r]: state row n0 + NTW (4 g + r) + i, value dimension col
 #pragma unroll
-  for (int i = 0; i < NTW; ++i) {
-    const int n = (wave + 4 * i) * 16 + 4 * g;
-    S[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    if (sw && a.pos[0] > 0 && prow && n < np) S[i] = *(const f32x4*)(state + (size_t)col * np + n);
+  for (int q = 0; q < NTW; ++q) {
+    const int n = n0 + 4 * NTW * g + 4 * q;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    if (sw && a.pos[0] > 0 && prow && n < np) v = *(const f32x4*)(state + (size_t)col * np + n);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) S[(4 * q + e) % NTW][(4 * q + e) / NTW] = v[e];
   }
-  V rb[PF], rc[PF];
-  float rx[2];
-  const V vz = {};
+  for (int i = tid; i < (DB ? 4 : 2) * kSsdTok * (LN - nk); i += 512)
+    bc[i / (LN - nk) * ld + nk + i % (LN - nk)] = (T)0.0f;
+  // Rows past the end repeat the last one: their step size is 0, so nothing of them is kept.  (The values
+  // past a head's last dimension are its row's next elements; their results are not stored.)
+  struct Regs {   // a block on its way
+    V b[PF], c[PF];
+    T x[4];
+  } reg;
   int prow_[PF], pcol_[PF];
 #pragma unroll
   for (int u = 0; u < PF; ++u) {
-    prow_[u] = (tid + u * TH) / ppr;
-    pcol_[u] = (tid + u * TH - prow_[u] * ppr) * VEC;
+    prow_[u] = ((tid & 255) + u * TH) / ppr;
+    pcol_[u] = ((tid & 255) + u * TH - prow_[u] * ppr) * VEC;
   }
-  auto load = [&](int m0) {
+  const T* xsrc = src + h * a.vdim + p0 + (tid & 3) * 4;
+  auto load = [&](Regs& d, int m0) {
 #pragma unroll
     for (int u = 0; u < PF; ++u) {
-      const bool in = prow_[u] < kSsdTok && m0 + prow_[u] < a.M;
-      const T* s = bsrc + (size_t)(m0 + prow_[u]) * a.lda + pcol_[u];
-      rb[u] = in ? *(const V*)s : vz;
-      rc[u] = in ? *(const V*)(s + c_off) : vz;
+      const T* s = bsrc + (size_t)min(m0 + prow_[u], a.M - 1) * a.lda + pcol_[u];
+      d.b[u] = *(const V*)s;
+      d.c[u] = *(const V*)(s + c_off);
     }
-    const int m = m0 + (tid >> 3), p = p0 + (tid & 7) * 2;
+    const T* x = xsrc + (size_t)min(m0 + ((tid & 255) >> 2), a.M - 1) * a.lda;
 #pragma unroll
-    for (int e = 0; e < 2; ++e) rx[e] = m < a.M && p + e < a.vdim ? (float)src[(size_t)m * a.lda + h * a.vdim + p + e] : 0.0f;
+    for (int e = 0; e < 4; ++e) d.x[e] = x[e];
   };
-  auto stage = [&](int buf, int m0) {
+  auto stage = [&](const Regs& d, int buf, int m0) {
     T* B = bc + (DB ? buf : 0) * 2 * kSsdTok * ld;
     T* C = B + kSsdTok * ld;
 #pragma unroll
     for (int u = 0; u < PF; ++u)
       if (prow_[u] < kSsdTok) {
-        *(V*)(B + prow_[u] * ld + pcol_[u]) = rb[u];
-        *(V*)(C + prow_[u] * ld + pcol_[u]) = rc[u];
+        *(V*)(B + prow_[u] * ld + pcol_[u]) = d.b[u];
+        *(V*)(C + prow_[u] * ld + pcol_[u]) = d.c[u];
       }
-    for (int i = tid + PF * TH; i < pieces; i += TH) {   // (long states)
+    for (int i = (tid & 255) + PF * TH; i < pieces; i += TH) {   // (long states)
       const int t = i / ppr, c = (i - t * ppr) * VEC;
-      const T* s = bsrc + (size_t)(m0 + t) * a.lda + c;
-      *(V*)(B + t * ld + c) = m0 + t < a.M ? *(const V*)s : vz;
-      *(V*)(C + t * ld + c) = m0 + t < a.M ? *(const V*)(s + c_off) : vz;
+      const T* s = bsrc + (size_t)min(m0 + t, a.M - 1) * a.lda + c;
+      *(V*)(B + t * ld + c) = *(const V*)s;
+      *(V*)(C + t * ld + c) = *(const V*)(s + c_off);
     }
 #pragma unroll
-    for (int e = 0; e < 2; ++e) xts[buf * 16 * XLD + ((tid & 7) * 2 + e) * XLD + (tid >> 3)] = rx[e];
+    for (int e = 0; e < 4; ++e) xts[buf * 16 * XLD + ((tid & 3) * 4 + e) * XLD + ((tid & 255) >> 2)] = (float)d.x[e];
   };
   auto steps = [&](int buf, int m0, float raw) {   // one wave: step sizes, cumulated log decays
     const float dt = m0 + lane < a.M ? softplusf(raw + bias) : 0.0f;   // (past the end: no decay, no input)
-    double c = (double)(A * dt);
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const double v = __shfl_up(c, o, 64);
-      if (lane >= o) c += v;
-    }
-    cums[buf * kSsdTok + lane] = c;
-    float* k = coef + buf * 3 * kSsdTok;
-    k[lane] = dt;
-    k[kSsdTok + lane] = fast_exp((float)(__shfl(c, 63, 64) - c)) * dt;
-    k[2 * kSsdTok + lane] = fast_exp((float)c);
+    const double c = wave_prefix((double)(A * dt) * 1.4426950408889634), last = lane_value<63>(c);
+    float* k = coef + buf * 5 * kSsdTok;
+    const float hi = (float)c;
+    k[lane] = hi;
+    k[kSsdTok + lane] = (float)(c - hi);
+    k[2 * kSsdTok + lane] = dt;
+    k[3 * kSsdTok + lane] = __builtin_amdgcn_exp2f((float)(last - c)) * dt;
+    k[4 * kSsdTok + lane] = __builtin_amdgcn_exp2f(hi);
   };
-  auto raw_dt = [&](int m0) { return m0 + lane < a.M ? a.dt[(size_t)(m0 + lane) * a.heads + h] : 0.0f; };
-  load(0);
+  auto raw_dt = [&](int m0) { return a.dt[(size_t)min(m0 + lane, a.M - 1) * a.heads + h]; };
+  if (!sw) {
+    load(reg, 0);
+    stage(reg, 0, 0);
+  }
   if (wave == 4) steps(0, 0, raw_dt(0));
-  stage(0, 0);
   lds_sync();
   for (int m0 = 0, buf = 0; m0 < a.M; m0 += kSsdTok, buf ^= 1) {
     const T* Bs = bc + (DB ? buf : 0) * 2 * kSsdTok * ld;
     const T* Cs = Bs + kSsdTok * ld;
-    const float *xt = xts + buf * 16 * XLD, *dts = coef + buf * 3 * kSsdTok, *wl = dts + kSsdTok, *ec = wl + kSsdTok;
-    const double* cum = cums + buf * kSsdTok;
+    const float *xt = xts + buf * 16 * XLD, *ch = coef + buf * 5 * kSsdTok, *cl = ch + kSsdTok, *dts = cl + kSsdTok, *wl = dts + kSsdTok,
+                *ec = wl + kSsdTok;
     f32x4* red = reds + (DB ? buf : 0) * 16 * 64;
     const bool more = m0 + kSsdTok < a.M;
     float rdt = 0.0f;
-    if (more) {
-      load(m0 + kSsdTok);
-      if (wave == 4) rdt = raw_dt(m0 + kSsdTok);
-    }
+    if (more && !sw) load(reg, m0 + kSsdTok);
+    if (more && wave == 4) rdt = raw_dt(m0 + kSsdTok);
     const int tok = w4 * 16 + col;
     f32x4 y = {0.f, 0.f, 0.f, 0.f};
     float et = 0.0f;
@@ -325,18 +350,15 @@ __global__ __launch_bounds__(512, 1) void ssd_scan_kernel(const ti_ssd_args a) {
       f32x4 yi[4];
 #pragma unroll
       for (int t = 0; t < 4; ++t) yi[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      typedef T TN __attribute__((ext_vector_type(4 * NTW), aligned(4 * NTW * sizeof(T) < 16 ? 4 * NTW * sizeof(T) : 16)));
+      TN c[4];
 #pragma unroll
-      for (int i = 0; i < NTW; ++i) {
-        const int tile = w4 + 4 * i;
-        if (tile >= nt) continue;
-        f32x4 c[4];
+      for (int t = 0; t < 4; ++t) c[t] = *(const TN*)(Cs + (t * 16 + col) * ld + n0 + 4 * NTW * g);
 #pragma unroll
-        for (int t = 0; t < 4; ++t) c[t] = widen4(Cs + (t * 16 + col) * ld + tile * 16 + 4 * g);
+      for (int k = 0; k < 4 * NTW; ++k)
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-#pragma unroll
-          for (int t = 0; t < 4; ++t) yi[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(S[i][r], c[t][r], yi[t], 0, 0, 0);
-      }
+        for (int t = 0; t < 4; ++t)
+          yi[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(S[k % NTW][k / NTW], (float)c[t][k], yi[t], 0, 0, 0);
 #pragma unroll
       for (int t = 0; t < 4; ++t) red[(w4 * 4 + t) * 64 + lane] = yi[t];
       // the state over the block
@@ -354,36 +376,66 @@ __global__ __launch_bounds__(512, 1) void ssd_scan_kernel(const ti_ssd_args a) {
         for (int r = 0; r < 4; ++r) S[i][r] *= last;
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        f32x4 b[NTW];
+        typedef T TB __attribute__((ext_vector_type(NTW)));
+        TB b[4];
 #pragma unroll
-        for (int i = 0; i < NTW; ++i)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) b[i][r] = (float)Bs[(t * 16 + 4 * g + r) * ld + min(w4 + 4 * i, nt - 1) * 16 + col];
+        for (int r = 0; r < 4; ++r) b[r] = *(const TB*)(Bs + (t * 16 + 4 * g + r) * ld + n0 + NTW * col);
 #pragma unroll
         for (int r = 0; r < 4; ++r)
 #pragma unroll
-          for (int i = 0; i < NTW; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(b[i][r], wx[t][r], S[i], 0, 0, 0);
+          for (int i = 0; i < NTW; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32((float)b[r][i], wx[t][r], S[i], 0, 0, 0);
       }
     } else {
       // scores of this wave's tokens with the block's earlier ones, decayed, times their inputs
-      const double ct = cum[tok];
       et = ec[tok];
-      for (int st = 0; st <= w4; ++st) {
-        f32x4 sc = {0.f, 0.f, 0.f, 0.f};
-        for (int k = 0; k < nk; k += KT)
-          sc = mma(*(const V*)(Bs + (st * 16 + col) * ld + k + g * VEC), *(const V*)(Cs + tok * ld + k + g * VEC), sc);
+      // (two or all four tiles of earlier tokens side by side; those past the wave's own tokens are masked)
+      const float th = ch[tok], tl = cl[tok];
+      f32x4 y2 = {0.f, 0.f, 0.f, 0.f};
+      auto scores = [&]<int NS>() {
+        f32x4 sc[NS];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int s = st * 16 + 4 * g + r;
-          sc[r] = s <= tok ? sc[r] * fast_exp((float)(ct - cum[s])) * dts[s] : 0.0f;
+        for (int i = 0; i < NS; ++i) sc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        const T *crow = Cs + tok * ld + g * VEC, *brow = Bs + col * ld + g * VEC;
+        constexpr int UF = 2;
+        for (int k = 0; k < nk; k += UF * KT) {
+          V cf[UF], bf[UF][NS];
+#pragma unroll
+          for (int f = 0; f < UF; ++f) {
+            const int kf = min(k + f * KT, LN - KT);   // (past nk: zeros)
+            cf[f] = *(const V*)(crow + kf);
+#pragma unroll
+            for (int i = 0; i < NS; ++i) bf[f][i] = *(const V*)(brow + i * 16 * ld + kf);
+          }
+#pragma unroll
+          for (int f = 0; f < UF; ++f)
+#pragma unroll
+            for (int i = 0; i < NS; ++i) sc[i] = mma(bf[f][i], cf[f], sc[i]);
         }
-        y = mma(*(const f32x4*)(xt + col * XLD + st * 16 + 4 * g), sc, y);
-      }
+#pragma unroll
+        for (int i = 0; i < NS; ++i) {
+          const int s0 = i * 16 + 4 * g;
+          const f32x4 sh = *(const f32x4*)(ch + s0), sl = *(const f32x4*)(cl + s0), d = *(const f32x4*)(dts + s0);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const float e = __builtin_amdgcn_exp2f((th - sh[r]) + (tl - sl[r]));
+            sc[i][r] = s0 + r <= tok ? sc[i][r] * (e * d[r]) : 0.0f;
+          }
+        }
+#pragma unroll
+        for (int i = 0; i < NS; ++i) {
+          const f32x4 x = *(const f32x4*)(xt + col * XLD + i * 16 + 4 * g);
+          if (i & 1) y2 = mma(x, sc[i], y2);
+          else y = mma(x, sc[i], y);
+        }
+      };
+      if (w4 < 2) scores.template operator()<2>();
+      else scores.template operator()<4>();
+      y += y2;
 #pragma unroll
       for (int r = 0; r < 4; ++r) y[r] = fmaf(D, xt[(4 * g + r) * XLD + tok], y[r]);
       if (wave == 4 && more) steps(buf ^ 1, m0 + kSsdTok, rdt);
     }
-    if (DB && more) stage(buf ^ 1, m0 + kSsdTok);
+    if (DB && more && !sw) stage(reg, buf ^ 1, m0 + kSsdTok);
     lds_sync();
     if (!sw && m0 + tok < a.M) {   // out: this wave's tokens, dimensions 4 g + r
       f32x4 z = red[w4 * 64 + lane];
@@ -402,15 +454,18 @@ __global__ __launch_bounds__(512, 1) void ssd_scan_kernel(const ti_ssd_args a) {
       }
     }
     if (!DB && more) {
-      stage(buf ^ 1, m0 + kSsdTok);
+      if (!sw) stage(reg, buf ^ 1, m0 + kSsdTok);
       lds_sync();
     }
   }
   if (!sw) return;
 #pragma unroll
-  for (int i = 0; i < NTW; ++i) {
-    const int n = (w4 + 4 * i) * 16 + 4 * g;
-    if (prow && n < np) *(f32x4*)(state + (size_t)col * np + n) = S[i];
+  for (int q = 0; q < NTW; ++q) {
+    const int n = n0 + 4 * NTW * g + 4 * q;
+    f32x4 v;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = S[(4 * q + e) % NTW][(4 * q + e) / NTW];
+    if (prow && n < np) *(f32x4*)(state + (size_t)col * np + n) = v;
   }
 }
 
@@ -476,64 +531,56 @@ __global__ __launch_bounds__(TH) void ssd_norm_vec_kernel(const ti_ssd_norm_args
 }
 
 // ------------------------------------------------------------------ gated linear recurrence over a chunk
-// 16 channels x 64 segments of the rows: every segment's product and end value from zero, one scan over
-// the segments, then the segments again from their start values.
+// 16 channels x 64 segments of at most LEN rows, held in registers: every segment's product and end value
+// from zero, one scan over the segments, then the segments again from their start values.
 constexpr int kLruSeg = 64;
-template <class T>
-__global__ __launch_bounds__(1024) void lru_scan_kernel(const ti_lru_scan_args a) {
+template <class T, int LEN>
+__global__ __launch_bounds__(1024) void lru_scan_kernel(const ti_lru_scan_args a, int row0, int rows) {
   __shared__ float sa[kLruSeg][16], sb[kLruSeg][16];
   const int tid = threadIdx.x, ch = tid & 15, seg = tid >> 4, c = blockIdx.x * 16 + ch, cc = min(c, a.channels - 1);
-  const int len = (a.M + kLruSeg - 1) / kLruSeg, r0 = seg * len, r1 = min(a.M, r0 + len);
+  const int len = (rows + kLruSeg - 1) / kLruSeg, end = row0 + rows, r0 = row0 + seg * len, n = min(end - r0, len);
   const float2* ab = (const float2*)a.ab + cc;
-  constexpr int U = 8;
+  const T* y = (const T*)a.y + cc;
+  float2 v[LEN];
+  T yv[LEN];
+#pragma unroll
+  for (int u = 0; u < LEN; ++u) v[u] = ab[(size_t)min(r0 + u, end - 1) * a.channels];
+#pragma unroll
+  for (int u = 0; u < LEN; ++u) yv[u] = y[(size_t)min(r0 + u, end - 1) * a.ldy];
   float pa = 1.0f, pb = 0.0f;
-  for (int r = r0; r < r1; r += U) {
-    float2 v[U];
 #pragma unroll
-    for (int u = 0; u < U; ++u) v[u] = ab[(size_t)min(r + u, a.M - 1) * a.channels];
-#pragma unroll
-    for (int u = 0; u < U; ++u)
-      if (r + u < r1) {
-        pa *= v[u].x;
-        pb = fmaf(v[u].x, pb, v[u].y);
-      }
-  }
+  for (int u = 0; u < LEN; ++u)
+    if (u < n) {
+      pa *= v[u].x;
+      pb = fmaf(v[u].x, pb, v[u].y);
+    }
   sa[seg][ch] = pa;
   sb[seg][ch] = pb;
-  __syncthreads();
+  lds_sync();
   float* st = a.state + (size_t)a.slot0 * a.channels + cc;
   if (seg == 0) {   // sb becomes every segment's start value
-    float s = a.pos[0] > 0 ? *st : 0.0f;
+    float s = a.pos[row0] > 0 ? *st : 0.0f;
+#pragma unroll 16
     for (int k = 0; k < kLruSeg; ++k) {
-      const float x = sa[k][ch], y = sb[k][ch];
+      const float x = sa[k][ch], e = sb[k][ch];
       sb[k][ch] = s;
-      s = fmaf(x, s, y);
+      s = fmaf(x, s, e);
     }
     if (c < a.channels) *st = s;
   }
-  __syncthreads();
+  lds_sync();
   if (c >= a.channels) return;
   float s = sb[seg][ch];
-  const T* y = (const T*)a.y + c;
   T* out = (T*)a.out + c;
-  for (int r = r0; r < r1; r += U) {
-    float2 v[U];
-    T yv[U];
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      v[u] = ab[(size_t)min(r + u, a.M - 1) * a.channels];
-      yv[u] = y[(size_t)min(r + u, a.M - 1) * a.ldy];
+  for (int u = 0; u < LEN; ++u)
+    if (u < n) {
+      s = fmaf(v[u].x, s, v[u].y);
+      out[(size_t)(r0 + u) * a.ldo] = (T)(s * (float)yv[u]);
     }
-#pragma unroll
-    for (int u = 0; u < U; ++u)
-      if (r + u < r1) {
-        s = fmaf(v[u].x, s, v[u].y);
-        out[(size_t)(r + u) * a.ldo] = (T)(s * (float)yv[u]);
-      }
-  }
   const int back = seg;   // the last taps - 1 rows' inputs enter the ring
-  if (back < a.taps - 1 && a.M - 1 - back >= 0) {
-    const int m = a.M - 1 - back;
+  if (back < a.taps - 1 && rows - 1 - back >= 0) {
+    const int m = end - 1 - back;
     ((T*)a.ring)[((size_t)a.slot0 * a.taps + a.pos[m] % a.taps) * a.channels + c] = ((const T*)a.x)[(size_t)m * a.ldy + c];
   }
 }
@@ -585,23 +632,22 @@ int launch_ssd_step(const ti_ssd_args& a, hipStream_t s) {
 constexpr size_t kSsdLds = 163840 - 1024;
 
 template <class T>
-size_t ssd_scan_lds(int N, bool db) {
-  const int kt = El<T>::KT, nk = (N + kt - 1) / kt * kt;
-  return (size_t)(db ? 4 : 2) * kSsdTok * (nk * sizeof(T) + 16) + 2 * 16 * (kSsdTok + 4) * 4 + (db ? 2 : 1) * 16 * 64 * 16 +
-         2 * kSsdTok * 8 + 2 * 3 * kSsdTok * 4;
+size_t ssd_scan_lds(int ntw, bool db) {
+  return (size_t)(db ? 4 : 2) * kSsdTok * (64 * ntw * sizeof(T) + 16) + 2 * 16 * (kSsdTok + 4) * 4 + (db ? 2 : 1) * 16 * 64 * 16 +
+         2 * 5 * kSsdTok * 4;
 }
 
 template <class T>
 int launch_ssd_scan(const ti_ssd_args& a, hipStream_t s) {
   const dim3 grid((a.vdim + 15) / 16, a.heads), blk(512);
-  const bool db = ssd_scan_lds<T>(a.state_n, true) <= kSsdLds;
-  const size_t lds = ssd_scan_lds<T>(a.state_n, db);
-  const int nt = (a.state_n + 15) / 16;
+  const int ntw = a.state_n <= 64 ? 1 : a.state_n <= 128 ? 2 : 4;
+  const bool db = ssd_scan_lds<T>(ntw, true) <= kSsdLds;
+  const size_t lds = ssd_scan_lds<T>(ntw, db);
 #define TI_SS(NTW)                                                                       \
   if (db) hipLaunchKernelGGL((ssd_scan_kernel<T, NTW, true>), grid, blk, lds, s, a);     \
   else hipLaunchKernelGGL((ssd_scan_kernel<T, NTW, false>), grid, blk, lds, s, a)
-  if (nt <= 4) TI_SS(1);
-  else if (nt <= 8) TI_SS(2);
+  if (ntw == 1) TI_SS(1);
+  else if (ntw == 2) TI_SS(2);
   else TI_SS(4);
 #undef TI_SS
   TI_LAUNCH_CHECK("ssd_scan_kernel");
@@ -629,6 +675,20 @@ int launch_ssd_norm(const ti_ssd_norm_args& a, hipStream_t s) {
   else if (vec) hipLaunchKernelGGL((ssd_norm_vec_kernel<T, 1024, 2>), grid, dim3(1024), 0, s, a);
   else hipLaunchKernelGGL(ssd_norm_kernel<T>, grid, dim3(512), (size_t)per * 4, s, a);
   TI_LAUNCH_CHECK("ssd_norm_kernel");
+  return TI_OK;
+}
+
+template <class T>
+int launch_lru_scan(const ti_lru_scan_args& a, hipStream_t s) {
+  const dim3 grid((a.channels + 15) / 16), blk(1024);
+  for (int r = 0; r < a.M; r += 32 * kLruSeg) {
+    const int rows = std::min(a.M - r, 32 * kLruSeg), len = (rows + kLruSeg - 1) / kLruSeg;
+    if (len <= 4) hipLaunchKernelGGL((lru_scan_kernel<T, 4>), grid, blk, 0, s, a, r, rows);
+    else if (len <= 8) hipLaunchKernelGGL((lru_scan_kernel<T, 8>), grid, blk, 0, s, a, r, rows);
+    else if (len <= 16) hipLaunchKernelGGL((lru_scan_kernel<T, 16>), grid, blk, 0, s, a, r, rows);
+    else hipLaunchKernelGGL((lru_scan_kernel<T, 32>), grid, blk, 0, s, a, r, rows);
+  }
+  TI_LAUNCH_CHECK("lru_scan_kernel");
   return TI_OK;
 }
 
@@ -703,11 +763,5 @@ extern "C" int ti_lru_scan(const ti_lru_scan_args* a, ti_stream_t stream) {
   if (!a || !a->ab || !a->y || !a->x || !a->out || !a->state || !a->ring || !a->pos || a->M < 1 || a->channels < 1 || a->taps < 1 ||
       a->taps > kLruSeg || a->ldy < a->channels || a->ldo < a->channels || !rec_dtype(a->dtype))
     return ti_set_error(TI_ERR_ARG, "ti_lru_scan: bad arguments");
-  const dim3 grid((a->channels + 15) / 16), blk(1024);
-  if (a->dtype == TI_DT_BF16)
-    hipLaunchKernelGGL(lru_scan_kernel<bf16>, grid, blk, 0, (hipStream_t)stream, *a);
-  else
-    hipLaunchKernelGGL(lru_scan_kernel<float>, grid, blk, 0, (hipStream_t)stream, *a);
-  TI_LAUNCH_CHECK("lru_scan_kernel");
-  return TI_OK;
+  return a->dtype == TI_DT_BF16 ? launch_lru_scan<bf16>(*a, (hipStream_t)stream) : launch_lru_scan<float>(*a, (hipStream_t)stream);
 }
