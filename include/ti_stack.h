@@ -52,12 +52,10 @@ enum ti_dense_epi {
                         out T [head][head_w / 16][key / KT][64][VEC] (ti_latent_attn_prefill) */
   TI_DE_ACT,         /* v += add[n] (nullable); columns n < act_cols through `act`; columns n < t_cols
                         to out T [m][n], the others to out2 fp32 [m][n - t_cols]             */
-  TI_DE_LRU          /* gates of a real-gated linear recurrent unit, one batch per diagonal block:
-                        columns (2j, 2j + 1) = (recurrence, input) gate of the block's channel j.
-                        log a = -sigmoid(r) * lru_rate, b = sqrt(1 - a^2) * sigmoid(i) * u;
-                        lru_state NULL: out fp32 [m][channel][2] = (a, b); else the step itself:
-                        S = a S + b in the row's slot (S = 0 before position 0) and
-                        out T [m][channel] = S * lru_y[m][channel]                           */
+  TI_DE_LRU          /* gates of a real-gated linear recurrent unit over a prompt chunk, one batch per
+                        diagonal block: columns (2j, 2j + 1) = (recurrence, input) gate of the block's
+                        channel j.  log a = -sigmoid(r) * lru_rate, b = sqrt(1 - a^2) * sigmoid(i) * u;
+                        out fp32 [m][channel][2] = (a, b) (ti_lru_scan)                      */
 };
 enum ti_act { TI_ACT_NONE = 0, TI_ACT_GELU_TANH, TI_ACT_GELU_ERF };
 
@@ -97,10 +95,6 @@ typedef struct ti_dense_args {
   /* TI_DE_LRU: batch b's columns are channels [b * N / 2, +N / 2); u is the product's own activation
    * row (element [m][b * a_batch + j] of `a`), add [batch * N] the gates' biases in column order */
   const float* lru_rate;       /* [channels] 8 * softplus(lambda)                            */
-  float* lru_state;            /* nullable [slots][channels]                                 */
-  const void* lru_y;           /* T [M][lru_ldy]                                             */
-  int32_t lru_ldy;
-  const int32_t* slot;         /* nullable [M]: stream slot of row m (NULL: m)               */
 } ti_dense_args;
 int ti_dense(const ti_dense_args* a, ti_stream_t s);
 size_t ti_dense_args_bytes(void);
@@ -295,23 +289,21 @@ int ti_gqa_splits(int M, int heads, int kv_heads, int max_seq);
 int ti_recurrent_prepare(void);
 
 /* ------------------------------------------------------------------- short convolution
- * Causal convolution per channel: y[c] = b[c] + sum_j w[c][j] x[position - (taps - 1) + j][c], zeros before
- * position 0, through `act` (TI_CONV_*).  A slot's last inputs live in a ring [taps][channels] T, position p
- * at place p % taps.  chunk: rows are consecutive positions of slot `slot0`, earlier inputs come from the
- * ring, which is left as it is (ti_ssd_norm / ti_lru_scan write it); else every row is its own slot's next
- * token and enters the ring.
+ * Causal convolution per channel over a prompt chunk (rows: consecutive positions of slot `slot0`):
+ * y[c] = b[c] + sum_j w[j][c] x[position - (taps - 1) + j][c], zeros before position 0, through `act`
+ * (TI_CONV_*).  A slot's last inputs live in a ring [taps][channels] T, position p at place p % taps; the
+ * chunk's first rows read it, and it is left as it is (ti_ssd_norm / ti_lru_scan write it).
  * Output place of channel c: c for c < c0, else o0 + (c - c0) / bw * bwp + (c - c0) % bw; the places a
  * section of bw channels leaves free are zeroed. */
 enum ti_conv_act { TI_CONV_LINEAR = 0, TI_CONV_SILU = 1 };
 typedef struct ti_conv_args {
   const void* x;               /* T [M][ldx]                                                 */
-  void* ring;                  /* T [slots][taps][channels]                                  */
-  const float* w;              /* [channels][taps]                                           */
+  const void* ring;            /* T [slots][taps][channels]                                  */
+  const float* w;              /* [taps][channels]                                           */
   const float* b;
   void* out;                   /* T [M][ldo]                                                 */
   const int32_t* pos;
-  const int32_t* slot;
-  int32_t M, channels, taps, act, ldx, ldo, c0, o0, bw, bwp, chunk, slot0, dtype;
+  int32_t M, channels, taps, act, ldx, ldo, c0, o0, bw, bwp, slot0, dtype;
 } ti_conv_args;
 int ti_conv(const ti_conv_args* a, ti_stream_t s);
 
@@ -329,7 +321,7 @@ typedef struct ti_ssd_args {
   const float* dt_bias;
   const float* a_log;
   const float* d;
-  const float* conv_w;         /* step: [channels][taps]                                     */
+  const float* conv_w;         /* step: [taps][channels]                                     */
   const float* conv_b;
   void* ring;
   float* state;
@@ -369,6 +361,28 @@ typedef struct ti_lru_scan_args {
   int32_t M, channels, taps, ldy, ldo, slot0, dtype;
 } ti_lru_scan_args;
 int ti_lru_scan(const ti_lru_scan_args* a, ti_stream_t s);
+
+/* One token per row of a gated linear recurrent unit, each row its own slot: the row's convolution (inputs
+ * x and the ring, which it advances), the block-diagonal gate products and the step S = a S + b of TI_DE_LRU,
+ * out T [m][c] = S * y[m][c].  gates: fragment-ordered [blocks][2 * width / blocks] rows (recurrence, input)
+ * per channel; gate_b in the same order. */
+typedef struct ti_lru_step_args {
+  const void* x;               /* T [M][ldx]                                                 */
+  const void* y;               /* T [M][ldx]                                                 */
+  void* ring;
+  const float* conv_w;         /* [taps][channels]                                           */
+  const float* conv_b;
+  const void* gates;
+  const float* gate_b;
+  const float* lru_rate;       /* [channels]                                                 */
+  float* state;                /* [slots][channels]                                          */
+  void* out;                   /* T [M][ldo]                                                 */
+  const int32_t* pos;
+  const int32_t* slot;         /* nullable [M]: stream slot of row m (NULL: m)               */
+  int32_t M, channels, blocks, taps, ldx, ldo, dtype;
+} ti_lru_step_args;
+int ti_lru_step(const ti_lru_step_args* a, ti_stream_t s);
+int ti_lru_step_max_block(int dtype);   /* most channels a block may have */
 
 /* Seeded uniform(-scale, scale) elements of `dtype` (synthetic weights and caches). */
 int ti_stack_fill(uint64_t seed, uint32_t tid, uint64_t n, float scale, int dtype, void* out, ti_stream_t s);

@@ -120,7 +120,7 @@ def test_argument_errors(ti_host):
     assert L.ti_rownorm(C.byref(n), None) == 1
     assert L.ti_gqa_block_elems(T.DT_BF16, 20, 28) == 64 * (32 + 32)
     assert L.ti_gqa_block_elems(T.DT_F32, 20, 28) == 64 * (32 + 32) and L.ti_gqa_block_elems(T.DT_F32, 16, 9) == 64 * 32
-    for f in ("ti_gqa_prep", "ti_gqa_decode", "ti_gqa_prefill", "ti_conv", "ti_ssd_step", "ti_ssd_scan", "ti_ssd_norm", "ti_lru_scan"):
+    for f in ("ti_gqa_prep", "ti_gqa_decode", "ti_gqa_prefill", "ti_conv", "ti_ssd_step", "ti_ssd_scan", "ti_ssd_norm", "ti_lru_scan", "ti_lru_step"):
         assert getattr(L, f)(None, None) == 1 and f in L.ti_last_error().decode()
     assert 1 <= L.ti_gqa_splits(1, 32, 4, 4096) <= 64 and L.ti_gqa_splits(512, 32, 4, 4096) == 1
     assert "l3.mix.k" not in shapes(MIXED) and "l1.mix.k" in shapes(MIXED)

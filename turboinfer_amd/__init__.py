@@ -105,8 +105,7 @@ class DenseArgs(C.Structure):
          ("step_ctr", C.c_void_p), ("advance", C.c_int32), ("tile_rows", C.c_int32), ("max_tiles", C.c_int32),
          ("tiles", C.c_void_p), ("n_tiles", C.c_void_p), ("rows_in", C.c_void_p), ("rows_out", C.c_void_p),
          ("row_div", C.c_int32)] + [(n, C.c_int32) for n in ("act", "act_cols", "t_cols", "ld2")] + \
-        [("out2", C.c_void_p), ("lru_rate", C.c_void_p), ("lru_state", C.c_void_p), ("lru_y", C.c_void_p),
-         ("lru_ldy", C.c_int32), ("slot", C.c_void_p)]
+        [("out2", C.c_void_p), ("lru_rate", C.c_void_p)]
 
 
 class RownormArgs(C.Structure):
@@ -148,7 +147,7 @@ EXPORTED = [
     "ti_engine_create_stack", "ti_engine_weight_count", "ti_engine_weight_info", "ti_engine_set_weight", "ti_engine_load",
     "ti_engine_describe", "ti_engine_prefill", "ti_engine_create_config", "ti_engine_step_slots",
     "ti_gqa_prep", "ti_gqa_block_elems", "ti_gqa_decode", "ti_gqa_prefill", "ti_gqa_splits", "ti_recurrent_prepare", "ti_conv",
-    "ti_ssd_step", "ti_ssd_scan", "ti_ssd_norm", "ti_lru_scan", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
+    "ti_ssd_step", "ti_ssd_scan", "ti_ssd_norm", "ti_lru_scan", "ti_lru_step", "ti_lru_step_max_block", "ti_stack_kpad", "ti_stack_weight_bytes", "ti_stack_pack",
     "ti_stack_convert", "ti_stack_fill", "ti_dense", "ti_dense_args_bytes", "ti_rownorm", "ti_rownorm_routes", "ti_route", "ti_route_max_tiles",
     "ti_latent_prep", "ti_latent_prepare", "ti_latent_attn_decode", "ti_latent_attn_splits", "ti_latent_attn_prefill", "ti_latent_attn_out",
 ]

@@ -94,7 +94,9 @@ int check_mixer(const ti_stack_config& c, const ti_stack_layer* l, int i) {
     case TI_MIX_RGLRU:
       if (L.mix_width < 1 || L.blocks < 1 || L.mix_width % L.blocks || L.conv < 1)
         return ti_set_error(TI_ERR_ARG, "layer %d: RG-LRU sizes (width %d, blocks %d, conv %d)", i, L.mix_width, L.blocks, L.conv);
-      if (L.conv > 64) return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: conv %d (at most 64)", i, L.conv);
+      if (L.conv > 64 || L.mix_width / L.blocks > ti_lru_step_max_block(c.dtype))
+        return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: conv %d (at most 64), blocks of %d (at most %d)", i, L.conv,
+                            L.mix_width / L.blocks, ti_lru_step_max_block(c.dtype));
       return TI_OK;
     default: return ti_set_error(TI_ERR_UNSUPPORTED, "layer %d: mixer %d", i, L.mixer);
   }

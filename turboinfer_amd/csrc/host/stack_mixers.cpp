@@ -6,9 +6,9 @@
 //              over the cache's fragments with the gate behind it; output product
 //   SSD        dense in projection (step sizes fp32); rows of many slots: convolution and recurrence in one
 //              launch; prompt chunks: convolution, block scan; gated norm; output product
-//   RG-LRU     dense [GELU branch | convolution input]; convolution; per-block gate product whose epilogue
-//              makes the recurrence's coefficients (rows of many slots: and the step itself; prompt
-//              chunks: a scan follows); output product
+//   RG-LRU     dense [GELU branch | convolution input]; rows of many slots: convolution, gate products and
+//              the recurrence's step in one launch; prompt chunks: convolution, per-block gate product whose
+//              epilogue makes the recurrence's coefficients, scan; output product
 #include <algorithm>
 #include <cmath>
 
@@ -223,7 +223,14 @@ int StackModel::set_mixer_weight(StackLayer& L, const std::string& t, const floa
   if (t == "mlp.down" && k.mlp == TI_MLP_DENSE) return pack(L.down, d, k.ff, 1, rows, nullptr);
   if (k.mixer != TI_MIX_LATENT) {
     if (t == "mix.o") return pack(L.o, d, cols, 1, rows, nullptr);
-    if (t == "mix.conv") return vec(L.conv_w);
+    if (t == "mix.conv") {   // [channels][taps] -> [taps][channels]
+      std::vector<float> v, o(n);
+      TI_TRY(host_copy(d, n, v));
+      for (int i = 0; i < rows; ++i)
+        for (int j = 0; j < cols; ++j) o[(size_t)j * rows + i] = v[(size_t)i * cols + j];
+      TI_TRY(ti_memcpy_h2d(L.conv_w, o.data(), n * 4, s_));
+      return ti_stream_sync(s_);
+    }
     if (t == "mix.conv.b") return vec(L.conv_b);
   }
   if (k.mixer == TI_MIX_GQA) {
@@ -374,7 +381,6 @@ int StackModel::ssd(const StackLayer& L, const StackRun& run, const StackRows& r
     v.o0 = L.o0;
     v.bw = k.state;
     v.bwp = L.bwp;
-    v.chunk = 1;
     v.slot0 = r.slot;
     v.dtype = c.dtype;
     TI_TRY(ti_conv(&v, s_));
@@ -422,6 +428,30 @@ int StackModel::rglru(const StackLayer& L, const StackRun& run, const StackRows&
   da.act_cols = w;
   da.t_cols = L.na;
   TI_TRY(dense(L.a, xn, kpad(c.width), M, proj_, lda, TI_DE_ACT, da));
+  if (!r.chunk) {
+    ti_lru_step_args t{};
+    t.x = x;
+    t.y = proj_;
+    t.ring = run.ring;
+    t.conv_w = L.conv_w;
+    t.conv_b = L.conv_b;
+    t.gates = L.gates.p;
+    t.gate_b = L.gate_b;
+    t.lru_rate = L.rate;
+    t.state = run.state;
+    t.out = attn_;
+    t.pos = r.pos;
+    t.slot = r.slots;
+    t.M = M;
+    t.channels = w;
+    t.blocks = k.blocks;
+    t.taps = k.conv;
+    t.ldx = lda;
+    t.ldo = ldo;
+    t.dtype = c.dtype;
+    TI_TRY(ti_lru_step(&t, s_));
+    return dense(L.o, attn_, ldo, M, y_, c.width, TI_DE_F32, {});
+  }
   ti_conv_args v{};
   v.x = x;
   v.ring = run.ring;
@@ -429,7 +459,6 @@ int StackModel::rglru(const StackLayer& L, const StackRun& run, const StackRows&
   v.b = L.conv_b;
   v.out = conv_;
   v.pos = r.pos;
-  v.slot = r.slots;
   v.M = M;
   v.channels = w;
   v.taps = k.conv;
@@ -438,7 +467,6 @@ int StackModel::rglru(const StackLayer& L, const StackRun& run, const StackRows&
   v.ldo = L.conv_ld;
   v.bw = bw;
   v.bwp = L.bwp;
-  v.chunk = r.chunk;
   v.slot0 = r.slot;
   v.dtype = c.dtype;
   TI_TRY(ti_conv(&v, s_));
@@ -448,32 +476,23 @@ int StackModel::rglru(const StackLayer& L, const StackRun& run, const StackRows&
   g.a_batch = L.bwp;
   g.add = L.gate_b;
   g.lru_rate = L.rate;
-  if (!r.chunk) {
-    g.lru_state = run.state;
-    g.lru_y = proj_;
-    g.lru_ldy = lda;
-    g.pos = r.pos;
-    g.slot = r.slots;
-    TI_TRY(dense(L.gates, conv_, L.conv_ld, M, attn_, ldo, TI_DE_LRU, g));
-  } else {
-    TI_TRY(dense(L.gates, conv_, L.conv_ld, M, ab_, 2 * w, TI_DE_LRU, g));
-    ti_lru_scan_args s{};
-    s.ab = ab_;
-    s.y = proj_;
-    s.x = x;
-    s.out = attn_;
-    s.state = run.state;
-    s.ring = run.ring;
-    s.pos = r.pos;
-    s.M = M;
-    s.channels = w;
-    s.taps = k.conv;
-    s.ldy = lda;
-    s.ldo = ldo;
-    s.slot0 = r.slot;
-    s.dtype = c.dtype;
-    TI_TRY(ti_lru_scan(&s, s_));
-  }
+  TI_TRY(dense(L.gates, conv_, L.conv_ld, M, ab_, 2 * w, TI_DE_LRU, g));
+  ti_lru_scan_args s{};
+  s.ab = ab_;
+  s.y = proj_;
+  s.x = x;
+  s.out = attn_;
+  s.state = run.state;
+  s.ring = run.ring;
+  s.pos = r.pos;
+  s.M = M;
+  s.channels = w;
+  s.taps = k.conv;
+  s.ldy = lda;
+  s.ldo = ldo;
+  s.slot0 = r.slot;
+  s.dtype = c.dtype;
+  TI_TRY(ti_lru_scan(&s, s_));
   return dense(L.o, attn_, ldo, M, y_, c.width, TI_DE_F32, {});
 }
 

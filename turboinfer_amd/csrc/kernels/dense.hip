@@ -28,18 +28,6 @@ __device__ __forceinline__ float activate(int act, float z) {
   return z;
 }
 
-// 1 - exp(y), y <= 0: its series near 0, where the difference would cancel.
-__device__ __forceinline__ float one_minus_exp(float y) {
-  float s = fmaf(y, 1.0f / 40320.0f, 1.0f / 5040.0f);
-  s = fmaf(y, s, 1.0f / 720.0f);
-  s = fmaf(y, s, 1.0f / 120.0f);
-  s = fmaf(y, s, 1.0f / 24.0f);
-  s = fmaf(y, s, 1.0f / 6.0f);
-  s = fmaf(y, s, 0.5f);
-  s = fmaf(y, s, 1.0f);
-  return y > -0.5f ? -y * s : 1.0f - fast_exp(y);
-}
-
 // Four consecutive output columns n0.. of row m (out row mo); rows >= rows are padding.
 template <class T, int EPI>
 __device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, int m, int mo, int rows, int n0, f32x4 v) {
@@ -139,17 +127,8 @@ __device__ __forceinline__ void dense_store(const ti_dense_args& a, int batch, i
         const int j = (n0 >> 1) + i, c = batch * per + j;
         if (j >= per) return;
         const float* gb = a.add + (size_t)batch * a.N + n0 + 2 * i;
-        const float la = -fast_sigmoid(v[2 * i] + gb[0]) * a.lru_rate[c];
         const float u = (float)((const T*)a.a)[(size_t)m * a.lda + (size_t)batch * a.a_batch + j];
-        const float av = fast_exp(la), bv = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * la)) * fast_sigmoid(v[2 * i + 1] + gb[1]) * u;
-        if (!a.lru_state) {
-          *(float2*)((float*)a.out + ((size_t)m * channels + c) * 2) = make_float2(av, bv);
-        } else {
-          float* st = a.lru_state + (size_t)(a.slot ? a.slot[m] : m) * channels + c;
-          const float s = a.pos[m] > 0 ? fmaf(av, *st, bv) : bv;
-          *st = s;
-          ((T*)a.out)[(size_t)m * a.ldo + c] = (T)(s * (float)((const T*)a.lru_y)[(size_t)m * a.lru_ldy + c]);
-        }
+        *(float2*)((float*)a.out + ((size_t)m * channels + c) * 2) = lru_coef(v[2 * i] + gb[0], v[2 * i + 1] + gb[1], a.lru_rate[c], u);
       }
       return;
     }
@@ -590,7 +569,7 @@ extern "C" int ti_dense(const ti_dense_args* a, ti_stream_t stream) {
         return ti_set_error(TI_ERR_ARG, "ti_dense: ACT arguments");
       break;
     case TI_DE_LRU:
-      if (a->N % 2 || !a->add || !a->lru_rate || (a->lru_state && (!a->lru_y || !a->pos || a->ldo < a->N / 2 * a->batch)))
+      if (a->N % 2 || !a->add || !a->lru_rate)
         return ti_set_error(TI_ERR_ARG, "ti_dense: LRU arguments");
       break;
     default: return ti_set_error(TI_ERR_ARG, "ti_dense: epilogue %d", a->epi);

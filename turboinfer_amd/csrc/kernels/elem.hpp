@@ -110,6 +110,24 @@ __device__ __forceinline__ void route_top64(float v, int E, int top, int32_t* id
 __device__ __forceinline__ float fast_exp(float z) { return __builtin_amdgcn_exp2f(z * 1.44269504088896340736f); }
 __device__ __forceinline__ float fast_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + fast_exp(-z)); }
 
+// 1 - exp(y), y <= 0: its series near 0, where the difference would cancel.
+__device__ __forceinline__ float one_minus_exp(float y) {
+  float s = fmaf(y, 1.0f / 40320.0f, 1.0f / 5040.0f);
+  s = fmaf(y, s, 1.0f / 720.0f);
+  s = fmaf(y, s, 1.0f / 120.0f);
+  s = fmaf(y, s, 1.0f / 24.0f);
+  s = fmaf(y, s, 1.0f / 6.0f);
+  s = fmaf(y, s, 0.5f);
+  s = fmaf(y, s, 1.0f);
+  return y > -0.5f ? -y * s : 1.0f - fast_exp(y);
+}
+
+// A gated linear recurrence's coefficients (a, b) from its gates' logits r and i, rate and input u.
+__device__ __forceinline__ float2 lru_coef(float r, float i, float rate, float u) {
+  const float la = -fast_sigmoid(r) * rate;
+  return make_float2(fast_exp(la), __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * la)) * fast_sigmoid(i) * u);
+}
+
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 }  // namespace ti

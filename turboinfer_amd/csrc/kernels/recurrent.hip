@@ -1,13 +1,14 @@
 // recurrent.hip -- recurrent mixers of the layer-stack models (ti_stack.h): short causal convolutions, the
 // state-space recurrence (SSD) and the gated linear recurrence over prompt chunks and single tokens.
 //
-//   * conv_kernel: convolution over rows and the slot's ring of earlier inputs.
+//   * conv_kernel: convolution over a prompt chunk and the slot's ring of earlier inputs.
 //   * ssd_step_kernel: one token per row: convolution, step size, state update and output of a slice of
 //     one head; the state is streamed once (read, update, write).
 //   * ssd_scan_kernel: a prompt chunk in blocks of 64 tokens: scores C B^T under the decay mask, the state
 //     carried in MFMA accumulators; products that involve decays or the state are fp32 MFMA.
 //   * ssd_norm_kernel: SiLU gate and grouped RMS norm.
 //   * lru_scan_kernel: S = a S + b per channel, the chunk cut into 64 segments scanned side by side.
+//   * lru_step_kernel: one token per row: convolution, gate products, state update.
 // Step sizes, decays, states and sums are fp32 (cumulated log decays fp64).
 #include <algorithm>
 
@@ -41,21 +42,19 @@ __global__ __launch_bounds__(256) void conv_kernel(const ti_conv_args a, int pla
       for (int e = 0; e < VQ; ++e) o[e] = (T)0.0f;
     } else {
       const int pos = a.pos[m];
-      T* ring = (T*)a.ring + (size_t)(a.chunk ? a.slot0 : a.slot ? a.slot[m] : m) * a.taps * a.channels + c0;
+      const T* ring = (const T*)a.ring + (size_t)a.slot0 * a.taps * a.channels + c0;
       float acc[VQ];
 #pragma unroll
       for (int e = 0; e < VQ; ++e) acc[e] = a.b[c0 + e];
-      TV cur;
       for (int back = a.taps - 1; back >= 0; --back) {
         const int p = pos - back;
         if (p < 0) continue;
-        const T* src = back == 0 || (a.chunk && m >= back) ? (const T*)a.x + (size_t)(m - back) * a.ldx + c0
-                                                           : ring + (size_t)(p % a.taps) * a.channels;
-        cur = *(const TV*)src;
+        const T* src = m >= back ? (const T*)a.x + (size_t)(m - back) * a.ldx + c0
+                                 : ring + (size_t)(p % a.taps) * a.channels;
+        const TV cur = *(const TV*)src;
 #pragma unroll
-        for (int e = 0; e < VQ; ++e) acc[e] = fmaf(a.w[(size_t)(c0 + e) * a.taps + a.taps - 1 - back], (float)cur[e], acc[e]);
+        for (int e = 0; e < VQ; ++e) acc[e] = fmaf(a.w[(size_t)(a.taps - 1 - back) * a.channels + c0 + e], (float)cur[e], acc[e]);
       }
-      if (!a.chunk) *(TV*)(ring + (size_t)(pos % a.taps) * a.channels) = cur;
 #pragma unroll
       for (int e = 0; e < VQ; ++e) o[e] = (T)(a.act == TI_CONV_SILU ? acc[e] * fast_sigmoid(acc[e]) : acc[e]);
     }
@@ -63,12 +62,12 @@ __global__ __launch_bounds__(256) void conv_kernel(const ti_conv_args a, int pla
   }
 }
 
-// The same for TAPS known and 16-byte places (VEC channels): a thread slides over R rows of a chunk with all
-// their inputs in flight, or takes one row of its own slot (DEC).
-template <class T, int TAPS, bool DEC>
+// The same for TAPS known and 16-byte places (VEC channels): a thread slides over R rows with all their inputs
+// in flight.
+template <class T, int TAPS>
 __global__ __launch_bounds__(256) void conv_vec_kernel(const ti_conv_args a, int places) {
   typedef typename El<T>::V V;
-  constexpr int VEC = El<T>::VEC, R = DEC ? 1 : 8, NX = R + TAPS - 1;
+  constexpr int VEC = El<T>::VEC, R = 8, NX = R + TAPS - 1;
   const int i0 = ((int)blockIdx.x * 64 + (int)(threadIdx.x & 63)) * VEC, m0 = ((int)blockIdx.y * 4 + (int)(threadIdx.x >> 6)) * R;
   if (i0 >= places || m0 >= a.M) return;
   int c0 = i0;
@@ -84,27 +83,24 @@ __global__ __launch_bounds__(256) void conv_vec_kernel(const ti_conv_args a, int
     return;
   }
   const int pos = a.pos[m0];
-  T* ring = (T*)a.ring + (size_t)(a.chunk ? a.slot0 : a.slot ? a.slot[m0] : m0) * a.taps * a.channels + c0;
+  const T* ring = (const T*)a.ring + (size_t)a.slot0 * TAPS * a.channels + c0;
   V x[NX];   // x[i]: the input i - (TAPS - 1) rows after m0
 #pragma unroll
   for (int i = 0; i < NX; ++i) {
     const int d = i - (TAPS - 1);
-    const T* src = d >= 0 || (!DEC && m0 + d >= 0) ? (const T*)a.x + (size_t)min(m0 + d, a.M - 1) * a.ldx + c0
-                                                   : ring + (size_t)(max(pos + d, 0) % TAPS) * a.channels;
+    const T* src = m0 + d >= 0 ? (const T*)a.x + (size_t)min(m0 + d, a.M - 1) * a.ldx + c0
+                               : ring + (size_t)(max(pos + d, 0) % TAPS) * a.channels;
     x[i] = *(const V*)src;
   }
-  float w[TAPS][VEC], b[VEC];
+  typedef float FV __attribute__((ext_vector_type(VEC), aligned(16)));
+  const FV b = *(const FV*)(a.b + c0);
+  FV w[TAPS];
 #pragma unroll
-  for (int e = 0; e < VEC; ++e) {
-    b[e] = a.b[c0 + e];
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) w[j][e] = a.w[(size_t)(c0 + e) * TAPS + j];
-  }
+  for (int j = 0; j < TAPS; ++j) w[j] = *(const FV*)(a.w + (size_t)j * a.channels + c0);
   const V z = {};
 #pragma unroll
   for (int i = 0; i < TAPS - 1; ++i)
     if (pos + i - (TAPS - 1) < 0) x[i] = z;
-  if (DEC) *(V*)(ring + (size_t)(pos % TAPS) * a.channels) = x[NX - 1];
 #pragma unroll
   for (int r = 0; r < R; ++r) {
     if (m0 + r >= a.M) return;
@@ -162,8 +158,8 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(const ti_ssd_args a, int 
       const T cur = raw[c];
       for (int back = a.taps - 1; back > 0; --back)
         if (pos >= back)
-          v = fmaf(a.conv_w[(size_t)c * a.taps + a.taps - 1 - back], (float)ring[(size_t)((pos - back) % a.taps) * channels + c], v);
-      v = fmaf(a.conv_w[(size_t)c * a.taps + a.taps - 1], (float)cur, v);
+          v = fmaf(a.conv_w[(size_t)(a.taps - 1 - back) * channels + c], (float)ring[(size_t)((pos - back) % a.taps) * channels + c], v);
+      v = fmaf(a.conv_w[(size_t)(a.taps - 1) * channels + c], (float)cur, v);
       // (the place written is read by no one: it held position pos - taps)
       if (own) ring[(size_t)(pos % a.taps) * channels + c] = cur;
       v = (float)(T)(v * fast_sigmoid(v));
@@ -585,6 +581,92 @@ __global__ __launch_bounds__(1024) void lru_scan_kernel(const ti_lru_scan_args a
   }
 }
 
+// ------------------------------------------------------------------ gated linear recurrence, one token per row
+// Grid (groups of 4 tiles of 16 gate columns = 8 channels, blocks, tiles of 16 rows).  Every workgroup makes
+// its rows' convolution of the whole block in LDS, while the first weight fragments, the states and the
+// epilogue's operands are in flight; each wave multiplies its tile and steps its channels' states.  VQ:
+// channels a thread convolves at a time.
+template <class T, int VQ>
+__global__ __launch_bounds__(256) void lru_step_kernel(const ti_lru_step_args a) {
+  typedef typename El<T>::V V;
+  typedef T TV __attribute__((ext_vector_type(VQ)));
+  typedef float FV __attribute__((ext_vector_type(VQ), aligned(VQ > 1 ? 16 : 4)));
+  constexpr int KT = El<T>::KT, VEC = El<T>::VEC, PF = 8;
+  extern __shared__ char lds[];
+  const int blk = blockIdx.y, m0 = blockIdx.z * 16, rows = min(16, a.M - m0), bw = a.channels / a.blocks, tiles = (2 * bw + 15) >> 4;
+  const int kp = ti_kpad<T>(bw), nk = kp / KT, ld = kp + VEC, c0 = blk * bw;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nt = blockIdx.x * 4 + wave;
+  T* us = (T*)lds;   // [16][ld]
+  const V* wp = (const V*)a.gates + ((size_t)blk * tiles + min(nt, tiles - 1)) * nk * 64 + lane;
+  V wf[PF];
+#pragma unroll
+  for (int u = 0; u < PF; ++u) wf[u] = wp[(size_t)min(u, nk - 1) * 64];
+  // this lane's results: row r, channels j0 and j0 + 1 of the block
+  const int r = min(lane & 15, rows - 1), m = m0 + r, j0 = nt * 8 + 2 * (lane >> 4);
+  const int rpos = a.pos[m], rslot = a.slot ? a.slot[m] : m;
+  float rb[2], ib[2], rate[2], st[2];
+  T y[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int c = c0 + min(j0 + i, bw - 1);
+    rb[i] = a.gate_b[2 * c];
+    ib[i] = a.gate_b[2 * c + 1];
+    rate[i] = a.lru_rate[c];
+    st[i] = a.state[(size_t)rslot * a.channels + c];
+    y[i] = ((const T*)a.y)[(size_t)m * a.ldx + c];
+  }
+  for (int i = tid; i < rows * (kp / VQ); i += 256) {
+    const int q = i / (kp / VQ), c = (i - q * (kp / VQ)) * VQ, mq = m0 + q;
+    TV o;
+#pragma unroll
+    for (int e = 0; e < VQ; ++e) o[e] = (T)0.0f;
+    if (c < bw) {   // (bw is a multiple of VQ)
+      const int pos = a.pos[mq], ch = c0 + c;
+      T* ring = (T*)a.ring + (size_t)(a.slot ? a.slot[mq] : mq) * a.taps * a.channels + ch;
+      const TV cur = *(const TV*)((const T*)a.x + (size_t)mq * a.ldx + ch);
+      FV acc = *(const FV*)(a.conv_b + ch);
+      for (int b0 = a.taps - 1; b0 >= 0; b0 -= 4) {   // four taps' loads in flight
+        TV v[4];
+        FV w[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const int back = max(b0 - u, 0);
+          v[u] = cur;
+          if (back && pos >= back) v[u] = *(const TV*)(ring + (size_t)((pos - back) % a.taps) * a.channels);
+          w[u] = *(const FV*)(a.conv_w + (size_t)(a.taps - 1 - back) * a.channels + ch);
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (b0 - u >= 0 && pos >= b0 - u)
+#pragma unroll
+            for (int e = 0; e < VQ; ++e) acc[e] = fmaf(w[u][e], (float)v[u][e], acc[e]);
+      }
+      // (the place written is read by no one: it held position pos - taps)
+      if (blockIdx.x == 0) *(TV*)(ring + (size_t)(pos % a.taps) * a.channels) = cur;
+#pragma unroll
+      for (int e = 0; e < VQ; ++e) o[e] = (T)acc[e];
+    }
+    *(TV*)(us + q * ld + c) = o;
+  }
+  lds_sync();
+  const V* up = (const V*)(us + r * ld + (lane >> 4) * VEC);
+  f32x4 g = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int u = 0; u < PF; ++u)
+    if (u < nk) g = mma(wf[u], up[u * (KT / VEC)], g);
+  for (int kt = PF; kt < nk; ++kt) g = mma(wp[(size_t)kt * 64], up[kt * (KT / VEC)], g);
+  if ((lane & 15) >= rows || nt >= tiles) return;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int j = j0 + i, c = c0 + j;
+    if (j >= bw) return;
+    const float2 k = lru_coef(g[2 * i] + rb[i], g[2 * i + 1] + ib[i], rate[i], (float)us[r * ld + j]);
+    const float s = rpos > 0 ? fmaf(k.x, st[i], k.y) : k.y;
+    a.state[(size_t)rslot * a.channels + c] = s;
+    ((T*)a.out)[(size_t)m * a.ldo + c] = (T)(s * (float)y[i]);
+  }
+}
+
 // ------------------------------------------------------------------ launchers
 template <class T>
 int launch_conv(const ti_conv_args& a, hipStream_t s) {
@@ -593,15 +675,10 @@ int launch_conv(const ti_conv_args& a, hipStream_t s) {
   const int all = a.channels | a.ldx | a.ldo | a.c0 | (sections ? a.o0 | a.bw | a.bwp : 0);
   constexpr int VEC = El<T>::VEC;
   if (all % VEC == 0 && a.taps >= 2 && a.taps <= 4) {
-    const int rows = a.chunk ? 8 : 1;
-    const dim3 grid((places / VEC + 63) / 64, (a.M + 4 * rows - 1) / (4 * rows)), blk(256);
-#define TI_CV(TAPS)                                                                                   \
-  if (a.chunk) hipLaunchKernelGGL((conv_vec_kernel<T, TAPS, false>), grid, blk, 0, s, a, places);     \
-  else hipLaunchKernelGGL((conv_vec_kernel<T, TAPS, true>), grid, blk, 0, s, a, places)
-    if (a.taps == 2) TI_CV(2);
-    else if (a.taps == 3) TI_CV(3);
-    else TI_CV(4);
-#undef TI_CV
+    const dim3 grid((places / VEC + 63) / 64, (a.M + 31) / 32), blk(256);
+    if (a.taps == 2) hipLaunchKernelGGL((conv_vec_kernel<T, 2>), grid, blk, 0, s, a, places);
+    else if (a.taps == 3) hipLaunchKernelGGL((conv_vec_kernel<T, 3>), grid, blk, 0, s, a, places);
+    else hipLaunchKernelGGL((conv_vec_kernel<T, 4>), grid, blk, 0, s, a, places);
     TI_LAUNCH_CHECK("conv_vec_kernel");
     return TI_OK;
   }
@@ -660,8 +737,11 @@ int recurrent_prepare() {
                      (const void*)ssd_scan_kernel<T, 4, true>,  (const void*)ssd_scan_kernel<T, 1, false>,
                      (const void*)ssd_scan_kernel<T, 2, false>, (const void*)ssd_scan_kernel<T, 4, false>,
                      (const void*)ssd_norm_kernel<T>};
+  const void* step[] = {(const void*)lru_step_kernel<T, 1>, (const void*)lru_step_kernel<T, El<T>::VEC>};
   for (const void* f : k)
     TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kSsdLds), "recurrent kernels' LDS");
+  for (const void* f : step)   // (16 rows of ti_lru_step_max_block inputs; the kernel's own LDS beside them)
+    TI_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 16 * (4096 + 8) * 2), "recurrent kernels' LDS");
   return TI_OK;
 }
 
@@ -692,6 +772,18 @@ int launch_lru_scan(const ti_lru_scan_args& a, hipStream_t s) {
   return TI_OK;
 }
 
+template <class T>
+int launch_lru_step(const ti_lru_step_args& a, hipStream_t s) {
+  constexpr int VEC = El<T>::VEC;
+  const int bw = a.channels / a.blocks;
+  const dim3 grid((2 * bw + 63) / 64, a.blocks, (a.M + 15) / 16), blk(256);
+  const size_t lds = (size_t)16 * (ti_kpad<T>(bw) + VEC) * sizeof(T);
+  if ((bw | a.ldx) % VEC == 0) hipLaunchKernelGGL((lru_step_kernel<T, VEC>), grid, blk, lds, s, a);
+  else hipLaunchKernelGGL((lru_step_kernel<T, 1>), grid, blk, lds, s, a);
+  TI_LAUNCH_CHECK("lru_step_kernel");
+  return TI_OK;
+}
+
 int gqa_prepare_all();   // gqa_attn.hip
 
 inline bool rec_dtype(int dt) { return dt == TI_DT_BF16 || dt == TI_DT_F32; }
@@ -703,6 +795,8 @@ extern "C" int ti_recurrent_prepare(void) {
   if (!rc) rc = ti::recurrent_prepare<ti::bf16>();
   return rc ? rc : ti::recurrent_prepare<float>();
 }
+
+extern "C" int ti_lru_step_max_block(int dtype) { return dtype == TI_DT_BF16 ? 4096 : 2048; }
 
 extern "C" int ti_conv(const ti_conv_args* a, ti_stream_t stream) {
   using namespace ti;
@@ -764,4 +858,15 @@ extern "C" int ti_lru_scan(const ti_lru_scan_args* a, ti_stream_t stream) {
       a->taps > kLruSeg || a->ldy < a->channels || a->ldo < a->channels || !rec_dtype(a->dtype))
     return ti_set_error(TI_ERR_ARG, "ti_lru_scan: bad arguments");
   return a->dtype == TI_DT_BF16 ? launch_lru_scan<bf16>(*a, (hipStream_t)stream) : launch_lru_scan<float>(*a, (hipStream_t)stream);
+}
+
+extern "C" int ti_lru_step(const ti_lru_step_args* a, ti_stream_t stream) {
+  using namespace ti;
+  if (!a || !a->x || !a->y || !a->ring || !a->conv_w || !a->conv_b || !a->gates || !a->gate_b || !a->lru_rate || !a->state || !a->out ||
+      !a->pos || a->M < 1 || a->channels < 1 || a->blocks < 1 || a->blocks > 65535 || a->channels % a->blocks || a->taps < 1 ||
+      a->ldx < a->channels || a->ldo < a->channels || !rec_dtype(a->dtype))
+    return ti_set_error(TI_ERR_ARG, "ti_lru_step: bad arguments");
+  if (a->channels / a->blocks > ti_lru_step_max_block(a->dtype))
+    return ti_set_error(TI_ERR_UNSUPPORTED, "ti_lru_step: blocks of %d channels", a->channels / a->blocks);
+  return a->dtype == TI_DT_BF16 ? launch_lru_step<bf16>(*a, (hipStream_t)stream) : launch_lru_step<float>(*a, (hipStream_t)stream);
 }
