@@ -125,6 +125,24 @@ def test_many_streams(ti, streams):
     e.close()
 
 
+def test_steps_over_chosen_slots(ti):
+    """Rows in any order of slots, some slots left out: their caches stay as they are."""
+    cfg, w = model("mixed")
+    lens = [20, 65, 7]
+    seqs = [tokens(cfg, n + 8, 70 + n) for n in lens]
+    refs = [reference("mixed", s) for s in seqs]
+    e = engine(ti, cfg, w)
+    for i, (s, n) in enumerate(zip(seqs, lens)):
+        e.prefill(i + 1, s[:n])
+    at = list(lens)
+    for live in ([2, 0], [1], [0, 1, 2], [2, 1], [0]):
+        got = e.step_slots([i + 1 for i in live], [seqs[i][at[i]] for i in live], [at[i] for i in live])
+        for r, i in enumerate(live):
+            close(got[r : r + 1], refs[i][at[i]][None], f"slot {i + 1} position {at[i]}")
+            at[i] += 1
+    e.close()
+
+
 def test_slots_are_used_again(ti):
     cfg, w = model("mixed")
     e = engine(ti, cfg, w)

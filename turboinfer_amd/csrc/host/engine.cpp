@@ -1793,6 +1793,7 @@ int ti_engine_replay_prepare(ti_engine* e, int n, int kv_len, int start_token) {
   hipGraphExec_t g = nullptr;
   TI_TRY(get_graph(e, n, 0, &g));
   e->replay_M = n;
+  for (int m = 0; m < n; ++m) state_set(e, m, -1);   // (a replayed step runs at one position: the states are no sequence's)
   return ti_stream_sync(e->s);
 }
 
