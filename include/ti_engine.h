@@ -49,8 +49,8 @@ enum ti_mixer {
   TI_MIX_GQA = 1,          /* grouped-query attention: norms of the whole query and key projections,
                               a gate per output element                                              */
   TI_MIX_SSD = 2,          /* Mamba-2: short convolution, state-space recurrence, gate before the norm */
-  TI_MIX_RGLRU = 3         /* Griffin's recurrent block: short convolution, real-gated linear
-                              recurrent unit, GELU branch                                            */
+  TI_MIX_RGLRU = 3         /* RG-LRU block: short convolution, gated linear recurrence, times a GELU
+                              branch                                                                 */
 };
 enum ti_mlp { TI_MLP_NONE = 0, TI_MLP_MOE = 1, TI_MLP_DENSE = 2 /* down(gelu(up x)), exact GELU */ };
 enum ti_norm_place { TI_PLACE_SANDWICH = 0, TI_PLACE_POST = 1 };

@@ -1,8 +1,8 @@
 """Plain restatement of the recurrent layer-stack models (architecture "Nogitar").
 
 One function per mechanism, whole-sequence, token by token where the mechanism is a recurrence, no
-cache, no batching, numpy only; the checker of the engine's recurrent and grouped-query layers.  It
-shares no code with the product.  A model is a (config, weights) pair: config the parsed config.json
+cache, no batching, numpy only; what the engine's recurrent and grouped-query layers are compared with.
+It shares no code with the product.  A model is a (config, weights) pair: config the parsed config.json
 dictionary, weights a name -> float array dictionary with the checkpoint's tensor names.
 """
 from __future__ import annotations
